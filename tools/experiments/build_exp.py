@@ -39,7 +39,7 @@ def build() -> str:
     objs = []
     for src in sorted(glob.glob(os.path.join(HERE, "*.hip"))):
         obj = os.path.join(BUILD, os.path.basename(src) + ".o")
-        subprocess.run([csrc_build.HIPCC, "-x", "hip", f"--offload-arch={csrc_build.ARCH}", "-munsafe-fp-atomics",
+        subprocess.run([csrc_build.HIPCC, "-x", "hip", f"--offload-arch={csrc_build.ARCH}", "-munsafe-fp-atomics", *csrc_build.NO_PACKED_F32,
                         *common, "-I", CSRC, "-c", src, "-o", obj], check=True)
         objs.append(obj)
     bobj = os.path.join(BUILD, "exp_bindings.cpp.o")
