@@ -29,6 +29,8 @@ void launch_dual_norm_add(float* x, const void* a, const float* wa, const void* 
                           float eps, bool bf, hipStream_t stream);
 void launch_add_norm(void* out, float* x, const void* y, const float* w, int T, int W, int groups, float eps,
                      bool out_bf, bool y_bf, hipStream_t stream);
+void launch_add_layer_norm(void* out, float* x, const void* y, const float* s, const float* w, const float* b, int T,
+                           int W, float eps, bool out_bf, bool y_bf, hipStream_t stream);
 void launch_limited_glu(void* out, const void* gu, int64_t rows, int F, float limit, bool bf, hipStream_t stream);
 int gqa_key_tile(int Dk, int Dv);
 int launch_gqa_attention(void* out, const void* q, const void* kc, const void* vc, const int* block_tables,
@@ -49,7 +51,8 @@ int launch_topk_softmax(int* idx, float* wt, const float* logits, int T, int E, 
 int launch_moe_rows(void* out, float* hid, const void* h, const void* wgu, const void* wd, const int* idx,
                     const float* wt, int T, int W, int F, int top, int act, bool bf, hipStream_t stream);
 int launch_route_topk(int* idx, float* wt, const void* h, const float* wr, const float* bias, int T, int W, int E,
-                      int top, bool bf, hipStream_t stream);
+                      int top, bool sigmoid, const float* corr, int count, int keep, float scale, bool bf,
+                      hipStream_t stream);
 void launch_canon_add(void* h, float* xs, const float* x, const void* y, const void* y2, const float* nw, float eps,
                       const float* cw, float* state, int sub, int nsub, const int* row_seq, const int64_t* positions,
                       const int* start_pos, const int* slots, int T, int W, int taps, int keep, bool out_bf, bool y_bf,
@@ -72,12 +75,16 @@ int launch_delta_prep(float* five, float* vout, const void* proj, int stride, in
                       const float* cw, float* state, const float* neg_rate, const float* dt_bias, int T, int A, int G,
                       int D, int E, int taps, int keep, const int* row_seq, const int64_t* positions,
                       const int* start_pos, const int* slots, bool shift_state, bool bf, hipStream_t stream);
+int launch_gla_prep(float* out, const void* proj, int stride, int q_off, int k_off, int v_off, int a_off, int rank,
+                    const float* a2, const float* ab, float q_scale, float inv_tau, int T, int n, int nv, bool bf,
+                    hipStream_t stream);
 void launch_head_norm_gate(void* out, int out_stride, int out_off, const float* o, const float* w, int wmod, int span,
                            const void* gate, int gate_stride, int gate_off, int act, float eps, float scale, int T, int C,
                            bool out_bf, bool gate_bf, hipStream_t stream);
 int launch_state_scan(float* out, const float* q, const float* k, const float* v, const float* w, const float* a,
                       const float* b, int sq, int sk, int sv, int sw, int sa, int sb, const float* decay, float* state,
                       const int* cu_q, const int* start_pos, const int* slots, int S, int T, int A, int D, int E,
+                      const int* chunks, int n_chunks, int chunk_rows, const int* seq_chunk0, float* ws,
                       hipStream_t stream);
 
 namespace {
@@ -309,6 +316,27 @@ void add_norm(torch::Tensor out, torch::Tensor x, c10::optional<torch::Tensor> y
                   (float)eps, is_bf(out), y_bf, cur());
 }
 
+// x += y * s (y / s absent: nothing is added), out = layer norm of x
+void add_layer_norm(torch::Tensor out, torch::Tensor x, c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> s,
+                    torch::Tensor w, torch::Tensor b, double eps) {
+  chk_act(out, "out"); chk_f32(x, "x");
+  TORCH_CHECK(x.dim() == 2 && out.sizes() == x.sizes(), "add_layer_norm: shapes");
+  chk_f32(w, "w", x.size(1)); chk_f32(b, "b", x.size(1));
+  TORCH_CHECK(y.has_value() == s.has_value(), "add_layer_norm: y and its scale come together");
+  const void* yp = nullptr;
+  const float* sp = nullptr;
+  bool y_bf = false;
+  if (y.has_value()) {
+    chk_act(*y, "y"); chk_f32(*s, "s", x.size(1));
+    TORCH_CHECK(y->sizes() == x.sizes(), "add_layer_norm: y must have x's shape");
+    yp = y->data_ptr();
+    y_bf = is_bf(*y);
+    sp = s->data_ptr<float>();
+  }
+  launch_add_layer_norm(out.data_ptr(), x.data_ptr<float>(), yp, sp, w.data_ptr<float>(), b.data_ptr<float>(), x.size(0),
+                        x.size(1), (float)eps, is_bf(out), y_bf, cur());
+}
+
 void limited_glu(torch::Tensor out, torch::Tensor gu, double limit) {
   chk_act(out, "out"); chk_act(gu, "gu");
   TORCH_CHECK(gu.dim() == 2 && out.dim() == 2 && gu.size(1) == 2 * out.size(1) && gu.size(0) == out.size(0) &&
@@ -378,15 +406,20 @@ void topk_softmax(torch::Tensor idx, torch::Tensor wt, torch::Tensor logits) {
 }
 
 // wgu [E, 2F, W] (gate rows, then up rows), wd [E, W, F]; idx / wt [T, top]; hid fp32 [T, top, F] scratch
-void route_topk(torch::Tensor idx, torch::Tensor wt, torch::Tensor h, torch::Tensor wr, c10::optional<torch::Tensor> bias) {
+void route_topk(torch::Tensor idx, torch::Tensor wt, torch::Tensor h, torch::Tensor wr, c10::optional<torch::Tensor> bias,
+                bool sigmoid, c10::optional<torch::Tensor> corr, int64_t count, int64_t keep, double scale) {
   chk_act(h, "h"); chk_f32(wr, "router"); chk_i32(idx, "idx"); chk_f32(wt, "wt", idx.numel());
   TORCH_CHECK(h.dim() == 2 && wr.dim() == 2 && idx.dim() == 2 && wr.size(1) == h.size(1) && idx.size(0) == h.size(0),
               "route_topk: h [T, W], router [E, W], idx [T, top]");
   const float* bp = nullptr;
   if (bias.has_value()) { chk_f32(*bias, "bias", wr.size(0)); bp = bias->data_ptr<float>(); }
+  const float* cp = nullptr;
+  if (corr.has_value()) { chk_f32(*corr, "correction", wr.size(0)); cp = corr->data_ptr<float>(); }
   int rc = launch_route_topk(idx.data_ptr<int>(), wt.data_ptr<float>(), h.data_ptr(), wr.data_ptr<float>(), bp,
-                             (int)h.size(0), (int)h.size(1), (int)wr.size(0), (int)idx.size(1), is_bf(h), cur());
-  TORCH_CHECK(rc == 0, "route_topk: at most 512 experts, 64 choices and a row of 48 KiB (code ", rc, ")");
+                             (int)h.size(0), (int)h.size(1), (int)wr.size(0), (int)idx.size(1), sigmoid, cp, (int)count,
+                             (int)keep, (float)scale, is_bf(h), cur());
+  TORCH_CHECK(rc == 0, "route_topk: at most 512 experts, 64 choices, a row of 48 KiB, groups that divide the experts and "
+              "hold the choices (code ", rc, ")");
 }
 
 void moe_rows(torch::Tensor out, torch::Tensor hid, torch::Tensor h, torch::Tensor wgu, torch::Tensor wd, torch::Tensor idx,
@@ -601,7 +634,7 @@ const float* stream_of(const OptT& t, const char* name, int64_t T, int64_t n, in
 
 void state_scan(torch::Tensor out, torch::Tensor q, torch::Tensor k, torch::Tensor v, OptT w, OptT a, OptT b, OptT decay,
                 torch::Tensor state, torch::Tensor cu_q, torch::Tensor start_pos, torch::Tensor slots, int64_t A, int64_t D,
-                int64_t E) {
+                int64_t E, OptT chunks, OptT seq_chunk0, OptT ws, int64_t chunk_rows) {
   TORCH_CHECK(A >= 1 && D >= 1 && D <= 256 && E >= 1, "state_scan: heads, dim <= 256, vdim");
   TORCH_CHECK(q.dim() == 2, "state_scan: q [T, A * D]");
   const int64_t T = q.size(0), S = cu_q.numel() - 1;
@@ -618,10 +651,41 @@ void state_scan(torch::Tensor out, torch::Tensor q, torch::Tensor k, torch::Tens
   chk_f32(state, "state");
   TORCH_CHECK(state.dim() == 2 && state.size(1) == A * D * E, "state_scan: state [slots, A * E * D]");
   chk_i32(cu_q, "cu_q"); chk_i32(start_pos, "start_pos", S); chk_i32(slots, "slots", S);
+  const int* cp = nullptr;
+  const int* c0p = nullptr;
+  float* wsp = nullptr;
+  int n_chunks = 0;
+  if (chunks.has_value()) {
+    TORCH_CHECK(!a.has_value(), "state_scan: a recurrence that removes cannot be scanned in chunks");
+    TORCH_CHECK(seq_chunk0.has_value() && ws.has_value() && chunk_rows >= 1, "state_scan: chunks need their lists and scratch");
+    chk_i32(*chunks, "chunks"); chk_i32(*seq_chunk0, "seq_chunk0", S + 1); chk_f32(*ws, "ws");
+    TORCH_CHECK(chunks->dim() == 2 && chunks->size(1) == 2, "state_scan: chunks [n, 2]");
+    n_chunks = (int)chunks->size(0);
+    TORCH_CHECK(ws->numel() >= (int64_t)n_chunks * A * D * (E + 1), "state_scan: scratch too small");
+    cp = chunks->data_ptr<int>();
+    c0p = seq_chunk0->data_ptr<int>();
+    wsp = ws->data_ptr<float>();
+  }
   int rc = launch_state_scan(out.data_ptr<float>(), qp, kp, vp, wp, ap, bp, sq, sk, sv, sw, sa, sb,
                              opt_f32(decay, "decay", A), state.data_ptr<float>(), cu_q.data_ptr<int>(),
-                             start_pos.data_ptr<int>(), slots.data_ptr<int>(), (int)S, (int)T, (int)A, (int)D, (int)E, cur());
+                             start_pos.data_ptr<int>(), slots.data_ptr<int>(), (int)S, (int)T, (int)A, (int)D, (int)E,
+                             cp, n_chunks, (int)chunk_rows, c0p, wsp, cur());
   TORCH_CHECK(rc == 0, "state_scan: unsupported shape (code ", rc, ")");
+}
+
+// out [T, 3 A D + A E]; proj columns q_off (A D), k_off (A D), v_off (A E), a_off (rank); a2 [rank, A D]
+void gla_prep(torch::Tensor out, torch::Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off, int64_t a_off,
+              torch::Tensor a2, torch::Tensor ab, double q_scale, double inv_tau) {
+  chk_act(proj, "proj"); chk_f32(a2, "a2"); chk_f32(out, "out"); chk_f32(ab, "ab");
+  TORCH_CHECK(proj.dim() == 2 && a2.dim() == 2 && out.dim() == 2 && out.size(0) == proj.size(0), "gla_prep: ranks");
+  const int64_t T = proj.size(0), rank = a2.size(0), n = a2.size(1), nv = out.size(1) - 3 * n, N = proj.size(1);
+  TORCH_CHECK(rank >= 1 && n >= 1 && nv >= 1 && ab.numel() == n, "gla_prep: a2 [rank, heads * dim], out [T, 3 heads dim + heads vdim]");
+  TORCH_CHECK(q_off >= 0 && k_off >= 0 && v_off >= 0 && a_off >= 0 && q_off + n <= N && k_off + n <= N && v_off + nv <= N &&
+              a_off + rank <= N, "gla_prep: columns");
+  int rc = launch_gla_prep(out.data_ptr<float>(), proj.data_ptr(), (int)N, (int)q_off, (int)k_off, (int)v_off, (int)a_off,
+                           (int)rank, a2.data_ptr<float>(), ab.data_ptr<float>(), (float)q_scale, (float)inv_tau, (int)T,
+                           (int)n, (int)nv, is_bf(proj), cur());
+  TORCH_CHECK(rc == 0, "gla_prep: the low-rank path is too wide");
 }
 
 void head_norm_gate(torch::Tensor out, int64_t out_off, torch::Tensor o, torch::Tensor w, int64_t span, torch::Tensor gate,
@@ -663,6 +727,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("dual_norm_add", &dual_norm_add);
   m.def("add_norm", &add_norm, py::arg("out"), py::arg("x"), py::arg("y"), py::arg("w"), py::arg("eps"),
         py::arg("groups") = 1);
+  m.def("add_layer_norm", &add_layer_norm);
   m.def("wkv_scan", &wkv_scan, py::arg("out"), py::arg("rkvg"), py::arg("lw"), py::arg("w0"), py::arg("u"),
         py::arg("norm_w"), py::arg("eps"), py::arg("state"), py::arg("cu_q"), py::arg("start_pos"), py::arg("slots"),
         py::arg("chunks") = py::none(), py::arg("seq_chunk0") = py::none(), py::arg("ws") = py::none());
@@ -670,7 +735,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("xielu", &xielu);
   m.def("silu_glu", &silu_glu);
   m.def("topk_softmax", &topk_softmax);
-  m.def("route_topk", &route_topk);
+  m.def("route_topk", &route_topk, py::arg("idx"), py::arg("wt"), py::arg("h"), py::arg("wr"), py::arg("bias"),
+        py::arg("sigmoid") = false, py::arg("corr") = py::none(), py::arg("count") = 1, py::arg("keep") = 1,
+        py::arg("scale") = 1.0);
   m.def("moe_rows", &moe_rows, py::arg("out"), py::arg("hid"), py::arg("h"), py::arg("wgu"), py::arg("wd"), py::arg("idx"),
         py::arg("wt"), py::arg("act") = 0);
   m.def("limited_glu", &limited_glu);
@@ -682,6 +749,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("relu2", &relu2);
   m.def("removal_prep", &removal_prep);
   m.def("delta_prep", &delta_prep);
-  m.def("state_scan", &state_scan);
+  m.def("gla_prep", &gla_prep);
+  m.def("state_scan", &state_scan, py::arg("out"), py::arg("q"), py::arg("k"), py::arg("v"), py::arg("w"), py::arg("a"),
+        py::arg("b"), py::arg("decay"), py::arg("state"), py::arg("cu_q"), py::arg("start_pos"), py::arg("slots"),
+        py::arg("heads"), py::arg("dim"), py::arg("vdim"), py::arg("chunks") = py::none(),
+        py::arg("seq_chunk0") = py::none(), py::arg("ws") = py::none(), py::arg("chunk_rows") = 0);
   m.def("head_norm_gate", &head_norm_gate);
 }

@@ -4,6 +4,10 @@
 //   silu_glu         gu = (gate | up) [T, 2F] -> silu(gate) * up
 //   topk_softmax     per row of fp32 router logits: the `top` largest (lower index wins a tie) and
 //                    the softmax over those alone
+//   route_topk       router logits and the choice in one launch; either the softmax choice above, or
+//                    scores s = sigmoid(logit): the `top` largest s + correction among the experts of
+//                    the best groups (a group's value: the sum of its two largest), weights s of the
+//                    chosen over their sum, times a constant
 //   moe_rows         a few rows through their experts, two launches (the decode-step form of a
 //                    mixture of gated experts, no host round trip so a graph can hold it):
 //                    hid[t, k, :] = silu(Wg[e] h_t) * (Wu[e] h_t),  e = idx[t, k]
@@ -85,6 +89,80 @@ __global__ void __launch_bounds__(64) topk_softmax_kernel(int* __restrict__ idx,
   topk_row(idx + (size_t)t * top, wt + (size_t)t * top, logits + (size_t)t * E, E, top, threadIdx.x);
 }
 
+// The sigmoid form of the choice, one wave. sc [E]: the scores s (written here over the logits);
+// ch [E], gv [count]: scratch in LDS for the choice scores and the groups' values. Experts of groups
+// that are not kept, and experts already taken, count as minus infinity.
+RT_DEVICE void choose_sigmoid(int* __restrict__ idx, float* __restrict__ wt, float* sc, float* ch, float* gv,
+                              const float* __restrict__ corr, int E, int top, int count, int keep, float scale, int lane) {
+  auto wave_sync = [] {
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  };
+  for (int e = lane; e < E; e += 64) {
+    const float s = sigm(sc[e]);
+    sc[e] = s;
+    ch[e] = s + (corr ? corr[e] : 0.f);
+  }
+  wave_sync();
+  const int n = E / count;
+  for (int g = lane; g < count; g += 64) {
+    float a = -INFINITY, b = -INFINITY;      // the two largest
+    for (int e = g * n; e < (g + 1) * n; ++e) {
+      const float v = ch[e];
+      if (v > a) {
+        b = a;
+        a = v;
+      } else if (v > b) {
+        b = v;
+      }
+    }
+    gv[g] = n > 1 ? a + b : a;
+  }
+  wave_sync();
+  float v[kTopPerLane];
+#pragma unroll
+  for (int q = 0; q < kTopPerLane; ++q) {
+    const int e = lane + 64 * q;
+    v[q] = -INFINITY;
+    if (e < E) {
+      const int g = e / n;
+      const float mine = gv[g];
+      int better = 0;
+      if (keep < count)
+        for (int o = 0; o < count; ++o) better += (gv[o] > mine || (gv[o] == mine && o < g)) ? 1 : 0;
+      if (better < keep) v[q] = ch[e];
+    }
+  }
+  float mine = 0.f;      // lane k keeps the k-th chosen expert's score
+  int mine_e = 0;
+  for (int k = 0; k < top; ++k) {
+    float best = -INFINITY;
+    int be = 1 << 30;
+#pragma unroll
+    for (int q = 0; q < kTopPerLane; ++q)
+      if (v[q] > best) {
+        best = v[q];
+        be = lane + 64 * q;
+      }
+    const float top_v = rt::wave_max(best);
+    int cand = best == top_v ? be : 1 << 30;
+    for (int o = 32; o; o >>= 1) cand = min(cand, __shfl_xor(cand, o));
+#pragma unroll
+    for (int q = 0; q < kTopPerLane; ++q)
+      if (lane + 64 * q == cand) v[q] = -INFINITY;
+    if (lane == k) {
+      mine_e = min(cand, E - 1);     // (only NaN scores leave no candidate)
+      mine = sc[mine_e];
+    }
+  }
+  const float sum = rt::wave_sum(lane < top ? mine : 0.f) + 1e-20f;
+  if (lane < top) {
+    idx[lane] = mine_e;
+    wt[lane] = mine / sum * scale;
+  }
+}
+
 // router and choice in one launch: logits = W_router h (+ bias) in fp32 from the row in LDS — eight
 // experts at a time, every lane's weight loads of a batch in flight together (16-byte loads when the
 // row allows), wave sums, partials through LDS — then wave 0 chooses.
@@ -93,7 +171,9 @@ constexpr int kRouteBatch = 8;
 template <typename T>
 __global__ void __launch_bounds__(256) route_topk_kernel(int* __restrict__ idx, float* __restrict__ wt,
                                                          const T* __restrict__ h, const float* __restrict__ wr,
-                                                         const float* __restrict__ bias, int W, int E, int top, int vec) {
+                                                         const float* __restrict__ bias, int W, int E, int top, int vec,
+                                                         int sigmoid, const float* __restrict__ corr, int count, int keep,
+                                                         float scale) {
   extern __shared__ float4 rl4[];       // (16-byte aligned: the row is read in 16-byte pieces)
   float* rl = reinterpret_cast<float*>(rl4);
   const int Wp = (W + 3) & ~3;
@@ -136,7 +216,11 @@ __global__ void __launch_bounds__(256) route_topk_kernel(int* __restrict__ idx, 
     lg[e] = v;
   }
   __syncthreads();
-  if (wave == 0) topk_row(idx + (size_t)t * top, wt + (size_t)t * top, lg, E, top, lane);
+  if (wave != 0) return;
+  int* ir = idx + (size_t)t * top;
+  float* wr_ = wt + (size_t)t * top;
+  if (sigmoid) choose_sigmoid(ir, wr_, lg, part, part + E, corr, E, top, count, keep, scale, lane);
+  else topk_row(ir, wr_, lg, E, top, lane);
 }
 
 // R dot products at once for the whole wave: rows w, w + rs, ... (the first `ok` of them) against
@@ -310,14 +394,16 @@ int launch_topk_softmax(int* idx, float* wt, const float* logits, int T, int E, 
 }
 
 int launch_route_topk(int* idx, float* wt, const void* h, const float* wr, const float* bias, int T, int W, int E,
-                      int top, bool bf, hipStream_t stream) {
+                      int top, bool sigmoid, const float* corr, int count, int keep, float scale, bool bf,
+                      hipStream_t stream) {
   if (T <= 0) return 0;
   if (E > 64 * kTopPerLane || top > 64 || top < 1 || top > E) return -1;
+  if (sigmoid && (count < 1 || E % count || keep < 1 || keep > count || top > keep * (E / count))) return -3;
   const size_t shm = sizeof(float) * ((size_t)((W + 3) & ~3) + 5 * (size_t)E);
   if (shm > 48 * 1024) return -2;
   const int vec = (W & 3) == 0 && (reinterpret_cast<uintptr_t>(wr) & 15) == 0 ? 1 : 0;
-  if (bf) route_topk_kernel<uint16_t><<<T, 256, shm, stream>>>(idx, wt, (const uint16_t*)h, wr, bias, W, E, top, vec);
-  else route_topk_kernel<float><<<T, 256, shm, stream>>>(idx, wt, (const float*)h, wr, bias, W, E, top, vec);
+  if (bf) route_topk_kernel<uint16_t><<<T, 256, shm, stream>>>(idx, wt, (const uint16_t*)h, wr, bias, W, E, top, vec, sigmoid ? 1 : 0, corr, count, keep, scale);
+  else route_topk_kernel<float><<<T, 256, shm, stream>>>(idx, wt, (const float*)h, wr, bias, W, E, top, vec, sigmoid ? 1 : 0, corr, count, keep, scale);
   return 0;
 }
 

@@ -15,6 +15,7 @@
 //   mingru_scan       z = sigmoid(.), c = u + 1/2 | sigmoid(u); S = (1 - z) S + z c; out = S silu(g)
 //   dual_norm_add     x += (a / rms(a) * wa + b / rms(b) * wb) / 2
 //   add_norm          x += y ; out = x / rms(x) * w
+//   add_layer_norm    x += y * s (s: a number per channel) ; out = (x - mean) / sqrt(var + eps) * w + b
 //   limited_glu       g = min(gate, L), u = clamp(up, -L, L); g * sigmoid(1.702 g) * (u + 1)
 #include "../common.h"
 
@@ -337,6 +338,52 @@ __global__ void __launch_bounds__(1024) add_norm_kernel(OT* __restrict__ out, fl
   }
 }
 
+// the variance is the mean of the squared deviations (a second sum, over the entries kept in
+// registers), not E[x^2] - mean^2
+template <typename OT, typename YT>
+__global__ void __launch_bounds__(1024) add_layer_norm_kernel(OT* __restrict__ out, float* __restrict__ x,
+                                                              const YT* __restrict__ y, const float* __restrict__ s,
+                                                              const float* __restrict__ w, const float* __restrict__ b,
+                                                              int W, float eps) {
+  __shared__ float scratch[16];
+  float* xr = x + (size_t)blockIdx.x * W;
+  const YT* yr = y ? y + (size_t)blockIdx.x * W : nullptr;
+  out += (size_t)blockIdx.x * W;
+  auto sum_at = [&](int c) { return xr[c] + (yr ? DT<YT>::load(yr + c) * s[c] : 0.f); };
+  float cv[kKeep];
+  float sum = 0.f;
+  int i = 0;
+  for (int c = threadIdx.x; c < W; c += blockDim.x, ++i) {
+    const float v = sum_at(c);
+    sum += v;
+#pragma unroll
+    for (int j = 0; j < kKeep; ++j)
+      if (j == i) cv[j] = v;
+  }
+  auto kept = [&](int idx, int c) {
+    if (idx >= kKeep) return sum_at(c);
+    float v = 0.f;
+#pragma unroll
+    for (int j = 0; j < kKeep; ++j)
+      if (j == idx) v = cv[j];
+    return v;
+  };
+  const float mean = rt::block_sum(sum, scratch) / (float)W;
+  float ss = 0.f;
+  i = 0;
+  for (int c = threadIdx.x; c < W; c += blockDim.x, ++i) {
+    const float d = kept(i, c) - mean;
+    ss += d * d;
+  }
+  const float k = inv_rms(rt::block_sum(ss, scratch), W, eps);
+  i = 0;
+  for (int c = threadIdx.x; c < W; c += blockDim.x, ++i) {
+    const float v = kept(i, c);
+    if (yr) xr[c] = v;
+    DT<OT>::store(out + c, (v - mean) * k * w[c] + b[c]);
+  }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256) limited_glu_kernel(T* __restrict__ out, const T* __restrict__ gu, int64_t rows,
                                                           int F, float limit) {
@@ -484,6 +531,19 @@ void launch_add_norm(void* out, float* x, const void* y, const float* w, int T, 
     if (y_bf) RT_AN(float, uint16_t); else RT_AN(float, float);
   }
 #undef RT_AN
+}
+
+void launch_add_layer_norm(void* out, float* x, const void* y, const float* s, const float* w, const float* b, int T,
+                           int W, float eps, bool out_bf, bool y_bf, hipStream_t stream) {
+  if (T <= 0) return;
+  const int th = row_threads(W);
+#define RT_AL(OT, YT) add_layer_norm_kernel<OT, YT><<<T, th, 0, stream>>>((OT*)out, x, (const YT*)y, s, w, b, W, eps)
+  if (out_bf) {
+    if (y_bf) RT_AL(uint16_t, uint16_t); else RT_AL(uint16_t, float);
+  } else {
+    if (y_bf) RT_AL(float, uint16_t); else RT_AL(float, float);
+  }
+#undef RT_AL
 }
 
 void launch_limited_glu(void* out, const void* gu, int64_t rows, int F, float limit, bool bf, hipStream_t stream) {

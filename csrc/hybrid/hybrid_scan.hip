@@ -17,6 +17,13 @@
 // is unrolled over two operand sets), and a lane's share of q . S goes to LDS as it is: the shares
 // of a column are added when the chunk's outputs are written, as whole lines. The state is
 // kept column by column, [slot][head][E][D], so that a lane's rows are contiguous.
+//
+// Without removal streams (a, b) the effect of a chunk of tokens on the state is a product per key
+// channel, so long spans can run in three launches over chunks: (1) every chunk alone from S = 0,
+// leaving its end state and its decay product; (2) chunk by chunk, an entry of S per lane, the state
+// each chunk starts from (carry = product * carry + end state, written over the end state) and the
+// sequence's new state; (3) every chunk again from its true start state, writing the outputs. There is
+// no division by a decay product, so decays close to zero are harmless.
 #include "../common.h"
 
 namespace {
@@ -51,23 +58,28 @@ RT_DEVICE float4 load4(const float* __restrict__ row, int r, int D, bool vec) {
 
 // UNROLL: whole chunks run unrolled (prompts); without it the code is a fraction of the size, which is
 // what a launch over single rows (a decode step, cold instruction cache) is timed by
-template <int DR, bool HAS_W, bool HAS_AB, bool UNROLL>
+// MODE 0: whole spans, state in and out of the slots; 1 / 2: launch (1) / (3) of the chunked form
+template <int DR, bool HAS_W, bool HAS_AB, bool UNROLL, int MODE>
 __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
     float* __restrict__ out, const float* __restrict__ q, const float* __restrict__ k, const float* __restrict__ v,
     const float* __restrict__ w, const float* __restrict__ a, const float* __restrict__ b, int sq, int sk, int sv, int sw,
     int sa, int sb, const float* __restrict__ decay, float* __restrict__ state, const int* __restrict__ cu_q,
-    const int* __restrict__ start_pos, const int* __restrict__ slots, int A, int D, int E, int P, int lgP, int vec) {
+    const int* __restrict__ start_pos, const int* __restrict__ slots, int A, int D, int E, int P, int lgP, int vec,
+    const int* __restrict__ chunks, int chunk_rows, float* __restrict__ ws_e, float* __restrict__ ws_p) {
   extern __shared__ float4 lds4[];
-  constexpr int NS = 2 + (HAS_W ? 1 : 0) + (HAS_AB ? 2 : 0);
+  constexpr bool OUT = MODE != 1;               // q is read and outputs are written
+  constexpr int NQ = OUT ? 1 : 0;
+  constexpr int NS = NQ + 1 + (HAS_W ? 1 : 0) + (HAS_AB ? 2 : 0);
   constexpr int NL = (kTT * DR + 63) / 64;      // 16-byte loads per lane, stream and chunk (P <= 16)
   constexpr int R4 = DR / 4;
-  const int seq = blockIdx.x, head = blockIdx.y;
+  const int seq = MODE == 0 ? (int)blockIdx.x : chunks[2 * blockIdx.x], head = blockIdx.y;
   const int CB = kScanThreads >> lgP;           // columns of this workgroup
   const int Dp4 = (P * DR) >> 2;                // padded rows / 4 (a power of two)
   const int lgDp4 = lgP + (DR == 4 ? 0 : DR == 8 ? 1 : 2);
   const int cl = threadIdx.x >> lgP, part = threadIdx.x & (P - 1);
   const int col = blockIdx.z * CB + cl;
-  const int r0 = cu_q[seq], n = cu_q[seq + 1] - r0;
+  const int r0 = MODE == 0 ? cu_q[seq] : chunks[2 * blockIdx.x + 1];
+  const int n = MODE == 0 ? cu_q[seq + 1] - r0 : min(chunk_rows, cu_q[seq + 1] - r0);
   if (n <= 0) return;
   float4* str = lds4;                                             // [kTT][NS][Dp4]
   float* vs = reinterpret_cast<float*>(str + kTT * NS * Dp4);     // [kTT][CB]
@@ -75,8 +87,9 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
   const int row_lo = part * DR;
   const bool live = col < E;
   float S[DR];
-  float* sp = state + (((size_t)slots[seq] * A + head) * E + (live ? col : 0)) * D + row_lo;
-  const bool cont = start_pos[seq] > 0;
+  float* sp = (MODE == 0 ? state + (size_t)slots[seq] * A * E * D : ws_e + (size_t)blockIdx.x * A * E * D) +
+              ((size_t)head * E + (live ? col : 0)) * D + row_lo;
+  const bool cont = MODE == 0 ? start_pos[seq] > 0 : MODE == 2;
   const bool svec = (D & 3) == 0;
 #pragma unroll
   for (int i4 = 0; i4 < R4; ++i4) {
@@ -84,12 +97,15 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
     if (cont && live) t = load4(sp, i4 * 4, D - row_lo, svec);
     S[i4 * 4] = t.x; S[i4 * 4 + 1] = t.y; S[i4 * 4 + 2] = t.z; S[i4 * 4 + 3] = t.w;
   }
+  float prod[MODE == 1 ? DR : 1];               // MODE 1: product of the chunk's decays, per row
+#pragma unroll
+  for (int i = 0; i < (MODE == 1 ? DR : 1); ++i) prod[i] = 1.f;
   const float dconst = HAS_W ? 1.f : decay[head];
   const float* src[NS];
   int strides[NS];
   {
     int j = 0;
-    src[j] = q; strides[j++] = sq;
+    if (OUT) { src[j] = q; strides[j++] = sq; }
     src[j] = k; strides[j++] = sk;
     if (HAS_W) { src[j] = w; strides[j++] = sw; }
     if (HAS_AB) { src[j] = a; strides[j++] = sa; src[j] = b; strides[j++] = sb; }
@@ -156,7 +172,7 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
       float acc = 0.f;
 #pragma unroll
       for (int i4 = 0; i4 < R4; ++i4) {
-        const float4 kk = tk[i4], qq = tq[i4];
+        const float4 kk = tk[i4];
         float u0 = kk.x * vv, u1 = kk.y * vv, u2 = kk.z * vv, u3 = kk.w * vv;
         if (HAS_AB) {
           const float4 aa = ta[i4];
@@ -171,19 +187,25 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
         S[i4 * 4 + 1] = S[i4 * 4 + 1] * d1 + u1;
         S[i4 * 4 + 2] = S[i4 * 4 + 2] * d2 + u2;
         S[i4 * 4 + 3] = S[i4 * 4 + 3] * d3 + u3;
-        acc += qq.x * S[i4 * 4] + qq.y * S[i4 * 4 + 1] + qq.z * S[i4 * 4 + 2] + qq.w * S[i4 * 4 + 3];
+        if (OUT) {
+          const float4 qq = tq[i4];
+          acc += qq.x * S[i4 * 4] + qq.y * S[i4 * 4 + 1] + qq.z * S[i4 * 4 + 2] + qq.w * S[i4 * 4 + 3];
+        }
+        if (MODE == 1) {
+          prod[i4 * 4] *= d0; prod[i4 * 4 + 1] *= d1; prod[i4 * 4 + 2] *= d2; prod[i4 * 4 + 3] *= d3;
+        }
       }
-      os[tok * kScanThreads + threadIdx.x] = acc;
+      if (OUT) os[tok * kScanThreads + threadIdx.x] = acc;
     };
     auto read_tok = [&](int tok, float4* tq, float4* tk, float4* tw, float4* ta, float4* tb, float& tv) {
       const float4* qs = str + (tok * NS) * Dp4 + part * R4;
-      const float4* ks = qs + Dp4;
+      const float4* ks = qs + NQ * Dp4;
       const float4* ws = ks + Dp4;                              // HAS_W
       const float4* as = ks + (HAS_W ? 2 : 1) * Dp4;            // HAS_AB
       const float4* bs = as + Dp4;
 #pragma unroll
       for (int i4 = 0; i4 < R4; ++i4) {
-        tq[i4] = qs[i4];
+        if (OUT) tq[i4] = qs[i4];
         tk[i4] = ks[i4];
         if (HAS_W) tw[i4] = ws[i4];
         if (HAS_AB) {
@@ -213,6 +235,7 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
         step(tok, tq, tk, tw, ta, tb, tv);
       }
     }
+    if (!OUT) continue;
     __syncthreads();
     for (int i = threadIdx.x; i < nt * CB; i += kScanThreads) {
       const int tok = i / CB, c = i - tok * CB;
@@ -222,6 +245,13 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
       for (int j = 0; j < P; ++j) o += sh[j];
       if (gc < E) out[(size_t)(r0 + c0 + tok) * A * E + head * E + gc] = o;
     }
+  }
+  if (MODE == 2) return;      // the sequence's new state came out of the carry
+  if (MODE == 1 && blockIdx.z == 0 && cl == 0) {
+    float* pp = ws_p + ((size_t)blockIdx.x * A + head) * D + row_lo;
+#pragma unroll
+    for (int i = 0; i < DR; ++i)
+      if (row_lo + i < D) pp[i] = prod[MODE == 1 ? i : 0];
   }
   if (live) {
     if (svec && row_lo + DR <= D) {
@@ -236,6 +266,39 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
         if (row_lo + i < D) sp[i] = S[i];
     }
   }
+}
+
+// launch (2): grid (sequences, heads, blocks of 256 entries of S); a batch of chunks is loaded ahead of
+// the dependent chain
+constexpr int kCarryBatch = 8;
+__global__ void __launch_bounds__(256) state_carry_kernel(float* __restrict__ ws_e, const float* __restrict__ ws_p,
+                                                          float* __restrict__ state, const int* __restrict__ seq_chunk0,
+                                                          const int* __restrict__ start_pos, const int* __restrict__ slots,
+                                                          int A, int D, int E) {
+  const int s = blockIdx.x, h = blockIdx.y;
+  const int e = blockIdx.z * blockDim.x + threadIdx.x;      // entry col * D + row
+  const int DE = D * E;
+  const int k0 = seq_chunk0[s], k1 = seq_chunk0[s + 1];
+  if (e >= DE || k1 <= k0) return;
+  const int row = e % D;
+  float* st = state + ((size_t)slots[s] * A + h) * DE + e;
+  float S = start_pos[s] > 0 ? *st : 0.f;
+  for (int c0 = k0; c0 < k1; c0 += kCarryBatch) {
+    float end[kCarryBatch], pr[kCarryBatch];
+#pragma unroll
+    for (int j = 0; j < kCarryBatch; ++j) {
+      const size_t at = (size_t)min(c0 + j, k1 - 1) * A + h;
+      end[j] = ws_e[at * DE + e];
+      pr[j] = ws_p[at * D + row];
+    }
+#pragma unroll
+    for (int j = 0; j < kCarryBatch; ++j)
+      if (c0 + j < k1) {
+        ws_e[((size_t)(c0 + j) * A + h) * DE + e] = S;
+        S = pr[j] * S + end[j];
+      }
+  }
+  *st = S;
 }
 
 }  // namespace
@@ -254,8 +317,10 @@ static void scan_shape(int D, int& DR, int& P, int& lgP) {
 int launch_state_scan(float* out, const float* q, const float* k, const float* v, const float* w, const float* a,
                       const float* b, int sq, int sk, int sv, int sw, int sa, int sb, const float* decay, float* state,
                       const int* cu_q, const int* start_pos, const int* slots, int S, int T, int A, int D, int E,
+                      const int* chunks, int n_chunks, int chunk_rows, const int* seq_chunk0, float* ws,
                       hipStream_t stream) {
   if (S <= 0) return 0;
+  if (chunks != nullptr && n_chunks <= 0) return 0;
   const bool unroll = T > 2 * S;      // rows per span on average: single rows take the small kernel
   int DR, P, lgP;
   scan_shape(D, DR, P, lgP);
@@ -269,28 +334,44 @@ int launch_state_scan(float* out, const float* q, const float* k, const float* v
   auto al = [&](const float* p, int st) { return p == nullptr || ((reinterpret_cast<uintptr_t>(p) & 15) == 0 && (st & 3) == 0); };
   const int vec = (D & 3) == 0 && al(q, sq) && al(k, sk) && al(w, sw) && al(a, sa) && al(b, sb) ? 1 : 0;
   const size_t shm = sizeof(float) * (size_t)kTT * ((size_t)NS * Dp + CB + kScanThreads);
-  dim3 grid(S, A, (E + CB - 1) / CB);
+  dim3 grid(chunks != nullptr ? n_chunks : S, A, (E + CB - 1) / CB);
+  float* ws_e = ws;
+  float* ws_p = ws != nullptr ? ws + (size_t)n_chunks * A * E * D : nullptr;
 #define RT_SCAN(DRV, HW, HAB)                                                                                          \
   do {                                                                                                                 \
-    if (unroll) RT_SCAN_U(DRV, HW, HAB, true); else RT_SCAN_U(DRV, HW, HAB, false);                                    \
+    if (unroll) RT_SCAN_U(DRV, HW, HAB, true, 0); else RT_SCAN_U(DRV, HW, HAB, false, 0);                              \
   } while (0)
-#define RT_SCAN_U(DRV, HW, HAB, UN)                                                                                    \
+#define RT_SCAN_U(DRV, HW, HAB, UN, MODE)                                                                              \
   do {                                                                                                                 \
-    auto kern = state_scan_kernel<DRV, HW, HAB, UN>;                                                                   \
+    auto kern = state_scan_kernel<DRV, HW, HAB, UN, MODE>;                                                             \
     if (shm > 48 * 1024 &&                                                                                             \
         hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm) != hipSuccess)    \
       return -3;                                                                                                       \
     kern<<<grid, kScanThreads, shm, stream>>>(out, q, k, v, w, a, b, sq, sk, sv, sw, sa, sb, decay, state, cu_q,       \
-                                              start_pos, slots, A, D, E, P, lgP, vec);                                 \
+                                              start_pos, slots, A, D, E, P, lgP, vec, chunks, chunk_rows, ws_e, ws_p); \
   } while (0)
 #define RT_SCAN_DR(HW, HAB)                                                                                            \
   do {                                                                                                                 \
     if (DR == 4) RT_SCAN(4, HW, HAB); else if (DR == 8) RT_SCAN(8, HW, HAB); else RT_SCAN(16, HW, HAB);                \
   } while (0)
+#define RT_CHUNK(HW, MODE)                                                                                             \
+  do {                                                                                                                 \
+    if (DR == 4) RT_SCAN_U(4, HW, false, true, MODE); else if (DR == 8) RT_SCAN_U(8, HW, false, true, MODE);           \
+    else RT_SCAN_U(16, HW, false, true, MODE);                                                                         \
+  } while (0)
+  if (chunks != nullptr) {
+    if (has_ab) return -5;
+    if (has_w) RT_CHUNK(true, 1); else RT_CHUNK(false, 1);
+    state_carry_kernel<<<dim3(S, A, (D * E + 255) / 256), 256, 0, stream>>>(ws_e, ws_p, state, seq_chunk0, start_pos, slots,
+                                                                            A, D, E);
+    if (has_w) RT_CHUNK(true, 2); else RT_CHUNK(false, 2);
+    return 0;
+  }
   if (has_w && has_ab) RT_SCAN_DR(true, true);
   else if (!has_w) RT_SCAN_DR(false, false);
   else RT_SCAN_DR(true, false);
 #undef RT_SCAN_DR
+#undef RT_CHUNK
 #undef RT_SCAN
 #undef RT_SCAN_U
   return 0;

@@ -13,6 +13,8 @@
 //   silu_cols        fp32 silu of a column range
 //   removal_prep     r, k, v, decay, removal rate * unit key, unit key of a generalized delta rule
 //   delta_prep       short convolutions + silu, unit q / k, step size and decay of a gated delta rule
+//   gla_prep         scaled q, k, v and the decay sigmoid(low-rank path + bias)^(1 / tau) of a gated
+//                    linear attention
 //   head_norm_gate   per-head or whole-row RMS norm, weight, sigmoid / silu gate, scale
 //   relu2            relu(a)^2
 #include "../common.h"
@@ -372,6 +374,49 @@ __global__ void __launch_bounds__(1024) delta_prep_kernel(
   for (int c = threadIdx.x; c < A * E; c += blockDim.x) vout[(size_t)t * A * E + c] = z[2 * G * D + c];
 }
 
+// out [T][3 n + nv] = q * q_scale, k, decay (n = heads * dim columns each), v; a2 [rank][n] is the second
+// factor of the decay's low-rank path, read once for ROWS rows. dynamic LDS: the rows' rank inputs.
+// decay = sigmoid(z)^(1 / tau) = exp(-softplus(-z) / tau)
+template <typename T, int ROWS>
+__global__ void __launch_bounds__(1024) gla_prep_kernel(float* __restrict__ out, const T* __restrict__ proj, int stride,
+                                                        int q_off, int k_off, int v_off, int a_off, int rank,
+                                                        const float* __restrict__ a2, const float* __restrict__ ab,
+                                                        float q_scale, float inv_tau, int Tn, int n, int nv) {
+  extern __shared__ float low[];        // [ROWS][rank]
+  const int t0 = blockIdx.x * ROWS;
+  const int rows = min(ROWS, Tn - t0);
+  for (int i = threadIdx.x; i < ROWS * rank; i += blockDim.x) {
+    const int r = i / rank;
+    low[i] = r < rows ? DT<T>::load(proj + (size_t)(t0 + r) * stride + a_off + (i - r * rank)) : 0.f;
+  }
+  __syncthreads();
+  const size_t os = (size_t)3 * n + nv;
+  for (int c = threadIdx.x; c < n; c += blockDim.x) {
+    float z[ROWS];
+    const float bc = ab[c];
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) z[r] = bc;
+#pragma unroll 4
+    for (int j = 0; j < rank; ++j) {
+      const float wv = a2[(size_t)j * n + c];
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r) z[r] += wv * low[r * rank + j];
+    }
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r)
+      if (r < rows) {
+        const T* pr = proj + (size_t)(t0 + r) * stride;
+        float* o = out + (size_t)(t0 + r) * os;
+        o[c] = DT<T>::load(pr + q_off + c) * q_scale;
+        o[n + c] = DT<T>::load(pr + k_off + c);
+        o[2 * (size_t)n + c] = expf(-(fmaxf(-z[r], 0.f) + log1pf(expf(-fabsf(z[r])))) * inv_tau);
+      }
+  }
+  for (int r = 0; r < rows; ++r)
+    for (int c = threadIdx.x; c < nv; c += blockDim.x)
+      out[(size_t)(t0 + r) * os + 3 * (size_t)n + c] = DT<T>::load(proj + (size_t)(t0 + r) * stride + v_off + c);
+}
+
 // o [T, C] fp32: segments of `span` entries are divided by their RMS; wmod = entries of the weight
 template <typename OT, typename GT>
 __global__ void __launch_bounds__(kThreads) head_norm_gate_kernel(
@@ -520,6 +565,27 @@ int launch_delta_prep(float* five, float* vout, const void* proj, int stride, in
   } while (0)
   if (bf) RT_DP(uint16_t); else RT_DP(float);
 #undef RT_DP
+  return 0;
+}
+
+int launch_gla_prep(float* out, const void* proj, int stride, int q_off, int k_off, int v_off, int a_off, int rank,
+                    const float* a2, const float* ab, float q_scale, float inv_tau, int T, int n, int nv, bool bf,
+                    hipStream_t stream) {
+  if (T <= 0) return 0;
+  const int rows = T >= 256 ? 4 : 1;      // few rows: one workgroup each; many: the low-rank factor is read once for four
+  const size_t shm = sizeof(float) * (size_t)rows * rank;
+  if (shm > 48 * 1024) return -1;
+  const int m = n > nv ? n : nv;
+  const int th = m >= 1024 ? 1024 : m <= 64 ? 64 : (m + 63) / 64 * 64;
+#define RT_GP(TT, R)                                                                                                   \
+  gla_prep_kernel<TT, R><<<(T + R - 1) / R, th, shm, stream>>>(out, (const TT*)proj, stride, q_off, k_off, v_off, a_off, \
+                                                               rank, a2, ab, q_scale, inv_tau, T, n, nv)
+  if (bf) {
+    if (rows == 4) RT_GP(uint16_t, 4); else RT_GP(uint16_t, 1);
+  } else {
+    if (rows == 4) RT_GP(float, 4); else RT_GP(float, 1);
+  }
+#undef RT_GP
   return 0;
 }
 

@@ -1,5 +1,6 @@
-// L3: causal attention over the paged latent cache with a softmax sink, for any head count and
-// any latent / rotary width (fp32 FMA; the cache and queries are bf16 or fp32 as templated).
+// L3: causal attention over the paged latent cache, with or without a softmax sink and a sliding
+// window, for any head count and any latent / rotary width (fp32 FMA; the cache and queries are
+// bf16 or fp32 as templated).
 //
 // The query of every head has been folded into latent space (q_lat = q_unrotated . W_uk), so the
 // key of token t is its cached row [latent C | rotated key part R] and its value is the row's
@@ -17,7 +18,12 @@
 // tile's keys and writes (o, m, l) partials that `latent_combine_kernel` merges; the ranges
 // follow from the run-time position, so one captured launch serves every length.
 //
-// The rotary part of q is rotated here, on load, by the row's position (fp32 angles).
+// With a window (position i sees keys j with i - j < window) a workgroup starts at the key tile its
+// first row's window begins in; the mask does the rest.
+//
+// The rotary part of q is rotated here, on load, by the row's position (fp32 angles): entries 2i
+// and 2i + 1 turn by pos * base^(-2i / dims), or — with a frequency table — entries i and
+// i + dims / 2 (or 2i and 2i + 1) turn by pos * freq[i], cos and sin times a magnitude.
 #include <cstdlib>
 
 #include "../common.h"
@@ -32,20 +38,59 @@ constexpr int KT = 64;  // keys per tile: one per lane
 struct AttnArgs {
   void* out;            // [H, T, C]
   const void* q_lat;    // [H, T, C]
-  const void* q;        // [T, H, Dq]; entries rot_off.. of a head are its rotary part
+  const void* q;        // [T, H, Dq], rows q_stride apart; entries rot_off.. of a head are its rotary part
   const void* cache;    // [num_blocks, BS, Dk], Dk = C + R
   const int* block_tables;
   const int* cu_q;
   const int* start_pos;
   const int* tiles;     // [n_tiles, 2] (sequence, first row)
-  const float* sink;    // [H]
+  const float* sink;    // [H], or null: no sink
+  const float* freq;    // [rot_dims / 2] rotary frequencies, or null: base^(-2i / dims)
   float* part_o;        // [T, H, splits, C]
   float* part_ml;       // [T, H, splits, 2]
   int T, H, C, R, Dq, rot_off, BS, max_blocks, rows, num_splits, kstride, rot_dims;
   int hwin;             // heads one workgroup takes (grid.z walks the windows)
   int kt;               // keys per staged tile of the plain kernel (64, or fewer when LDS is short)
-  float scale, rot_k;
+  int q_stride;         // numbers from one row of q to the next
+  int window;           // 0: every earlier key
+  int halves;           // rotary pairs: (i, i + rot_dims / 2) instead of (2i, 2i + 1)
+  float scale, rot_k, mag;
 };
+
+// Rotary part of one query head (R entries at qr, by position posf) handed to put(entry, value),
+// lanes striding over pairs and unrotated entries.
+template <typename QT, typename F>
+RT_DEVICE void rotate_query(const AttnArgs& a, const QT* qr, float posf, int lane, F put) {
+  const int half = a.rot_dims >> 1;
+  for (int i = lane; i < a.R - half; i += 64) {
+    if (i >= half) {      // past the rotated entries
+      put(i + half, DT<QT>::load(qr + i + half));
+      continue;
+    }
+    const int iu = a.halves ? i : 2 * i, iv = a.halves ? i + half : 2 * i + 1;
+    const float u = DT<QT>::load(qr + iu), v = DT<QT>::load(qr + iv);
+    float cs, sn;
+    sincosf(posf * (a.freq ? a.freq[i] : exp2f((float)i * a.rot_k)), &sn, &cs);
+    cs *= a.mag;
+    sn *= a.mag;
+    put(iu, u * cs - v * sn);
+    put(iv, v * cs + u * sn);
+  }
+}
+
+// Keys this workgroup walks: from the tile its first row's window begins in (0 without a window)
+// to its last row, cut into num_splits ranges of whole tiles.
+RT_DEVICE void key_range(const AttnArgs& a, int pos0, int nkeys, int& kb, int& ke) {
+  const int lo = a.window > 0 ? max(0, pos0 - a.window + 1) / KT * KT : 0;
+  kb = lo;
+  ke = nkeys;
+  if (a.num_splits > 1) {
+    const int ntile = (nkeys - lo + KT - 1) / KT;
+    const int per = (ntile + a.num_splits - 1) / a.num_splits;
+    kb = min(nkeys, lo + (int)blockIdx.y * per * KT);
+    ke = min(nkeys, kb + per * KT);
+  }
+}
 
 // CPL: latent columns per lane (C <= 64 * CPL); PW: (row, head) pairs per wave
 template <typename CT, typename QT, int CPL, int PW>
@@ -73,20 +118,8 @@ __global__ void __launch_bounds__(kThreads) latent_attn_kernel(AttnArgs a) {
     const int r = p / HW, h = h0 + p - r * HW;
     const QT* ql = reinterpret_cast<const QT*>(a.q_lat) + ((size_t)h * a.T + row0 + r) * a.C;
     for (int d = lane; d < a.C; d += 64) qd[d] = DT<QT>::load(ql + d) * a.scale;
-    const QT* qr = reinterpret_cast<const QT*>(a.q) + ((size_t)(row0 + r) * a.H + h) * a.Dq + a.rot_off;
-    const float posf = (float)(pos0 + r);
-    for (int i = lane; i < (a.R + 1) / 2; i += 64) {
-      const float u = DT<QT>::load(qr + 2 * i);
-      if (2 * i + 1 >= a.R) {
-        qd[a.C + 2 * i] = u * a.scale;
-        continue;
-      }
-      const float v = DT<QT>::load(qr + 2 * i + 1);
-      float cs = 1.f, sn = 0.f;
-      if (2 * i < a.rot_dims) sincosf(posf * exp2f((float)i * a.rot_k), &sn, &cs);
-      qd[a.C + 2 * i] = (u * cs - v * sn) * a.scale;
-      qd[a.C + 2 * i + 1] = (v * cs + u * sn) * a.scale;
-    }
+    const QT* qr = reinterpret_cast<const QT*>(a.q) + (size_t)(row0 + r) * a.q_stride + (size_t)h * a.Dq + a.rot_off;
+    rotate_query(a, qr, (float)(pos0 + r), lane, [&](int d, float v) { qd[a.C + d] = v * a.scale; });
   }
   float m[PW], l[PW], o[PW][CPL];
   int qpos[PW];
@@ -101,16 +134,12 @@ __global__ void __launch_bounds__(kThreads) latent_attn_kernel(AttnArgs a) {
   }
   // ---- key range of this workgroup ----
   const int nkeys = pos0 + nrows;   // keys 0 .. last row's position
-  int kb = 0, ke = nkeys;
-  if (a.num_splits > 1) {
-    const int ntile = (nkeys + KT - 1) / KT;
-    const int per = (ntile + a.num_splits - 1) / a.num_splits;
-    kb = min(nkeys, (int)blockIdx.y * per * KT);
-    ke = min(nkeys, kb + per * KT);
-  }
+  int kb, ke;
+  key_range(a, pos0, nkeys, kb, ke);
   const int* bt = a.block_tables + (size_t)seq * a.max_blocks;
   const CT* cache = reinterpret_cast<const CT*>(a.cache);
   const int kt = a.kt;
+  const int reach = a.window > 0 ? a.window : 0x7fffffff;
   for (int k0 = kb; k0 < ke; k0 += kt) {
     __syncthreads();   // the previous tile's readers are done (and Qs is written, first time)
     // stage: wave w copies keys w, w + 4, ...; lanes stride over the row
@@ -140,7 +169,7 @@ __global__ void __launch_bounds__(kThreads) latent_attn_kernel(AttnArgs a) {
     float* pw = Ps + (size_t)wave * PW * KT;
 #pragma unroll
     for (int i = 0; i < PW; ++i) {
-      const bool vis = lane < kt && kp < ke && kp <= qpos[i];
+      const bool vis = lane < kt && kp < ke && kp <= qpos[i] && qpos[i] - kp < reach;
       const float sv = vis ? s[i] : -INFINITY;
       const float mn = fmaxf(m[i], rt::wave_max(sv));
       float p = 0.f, alpha = 1.f;
@@ -193,7 +222,7 @@ __global__ void __launch_bounds__(kThreads) latent_attn_kernel(AttnArgs a) {
         ml[1] = l[i];
       }
     } else {
-      const float sk = a.sink[h];
+      const float sk = a.sink ? a.sink[h] : -INFINITY;
       const float M = fmaxf(m[i], sk);
       const float w = __expf(m[i] - M);
       const float inv = 1.f / (l[i] * w + __expf(sk - M));
@@ -220,7 +249,7 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(OT* __restrict__ ou
   const float* ml = part_ml + ((size_t)t * H + h) * splits * 2;
   if (threadIdx.x < 64) {
     const int s = threadIdx.x;
-    const float sk = sink[h];
+    const float sk = sink ? sink[h] : -INFINITY;
     const float ms = s < splits ? ml[2 * s] : -INFINITY;
     const float M = fmaxf(rt::wave_max(ms), sk);
     const float w = s < splits ? __expf(ms - M) : 0.f;          // m = -inf (an empty split) -> 0
@@ -296,15 +325,9 @@ __global__ void __launch_bounds__(kThreads) latent_attn_mfma_kernel(AttnArgs a) 
     const int r = p / HW, hd = h0 + p - r * HW;
     const uint16_t* ql = reinterpret_cast<const uint16_t*>(a.q_lat) + ((size_t)hd * a.T + row0 + r) * C;
     for (int d = lane; d < C; d += 64) qd[d] = ql[d];
-    const uint16_t* qr = reinterpret_cast<const uint16_t*>(a.q) + ((size_t)(row0 + r) * a.H + hd) * a.Dq + a.rot_off;
-    const float posf = (float)(pos0 + r);
-    for (int i = lane; i < a.R / 2; i += 64) {
-      const float u = rt::bf2f(qr[2 * i]), v = rt::bf2f(qr[2 * i + 1]);
-      float cs = 1.f, sn = 0.f;
-      if (2 * i < a.rot_dims) sincosf(posf * exp2f((float)i * a.rot_k), &sn, &cs);
-      qd[C + 2 * i] = rt::f2bf(u * cs - v * sn);
-      qd[C + 2 * i + 1] = rt::f2bf(v * cs + u * sn);
-    }
+    const uint16_t* qr =
+        reinterpret_cast<const uint16_t*>(a.q) + (size_t)(row0 + r) * a.q_stride + (size_t)hd * a.Dq + a.rot_off;
+    rotate_query(a, qr, (float)(pos0 + r), lane, [&](int d, float v) { qd[C + d] = rt::f2bf(v); });
   }
   __syncthreads();
   rt::short8 qf[NQM];
@@ -320,14 +343,10 @@ __global__ void __launch_bounds__(kThreads) latent_attn_mfma_kernel(AttnArgs a) 
     for (int i = 0; i < 16; ++i) o[db][i] = 0.f;
   float m = -INFINITY, l = 0.f;   // m in log2 units of the scaled score
   const float sc2 = a.scale * kLog2e;
+  const int qlow = a.window > 0 ? qpos - a.window : -1;    // keys up to here are out of the window
   const int nkeys = pos0 + nrows;
-  int kb = 0, ke = nkeys;
-  if (a.num_splits > 1) {
-    const int ntile = (nkeys + KT - 1) / KT;
-    const int per = (ntile + a.num_splits - 1) / a.num_splits;
-    kb = min(nkeys, (int)blockIdx.y * per * KT);
-    ke = min(nkeys, kb + per * KT);
-  }
+  int kb, ke;
+  key_range(a, pos0, nkeys, kb, ke);
   const int* bt = a.block_tables + (size_t)seq * a.max_blocks;
   const uint16_t* cache = reinterpret_cast<const uint16_t*>(a.cache);
   const int nch = Dk >> 3;   // 16-byte chunks per cached row
@@ -382,7 +401,7 @@ __global__ void __launch_bounds__(kThreads) latent_attn_mfma_kernel(AttnArgs a) 
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       const int key = k0 + 32 * x + 16 * (i >> 3) + 8 * h + (i & 7);
-      const float v = (key < ke && key <= qpos) ? sc[i] * sc2 : -INFINITY;
+      const float v = (key < ke && key <= qpos && key > qlow) ? sc[i] * sc2 : -INFINITY;
       sc[i] = v;
       tmax = fmaxf(tmax, v);
     }
@@ -446,7 +465,7 @@ __global__ void __launch_bounds__(kThreads) latent_attn_mfma_kernel(AttnArgs a) 
       ml[1] = ltot;
     }
   } else {
-    const float sk = a.sink[hd];
+    const float sk = a.sink ? a.sink[hd] : -INFINITY;
     const float M = fmaxf(m_nat, sk);
     const float w = __expf(m_nat - M);
     const float inv = w / (ltot * w + __expf(sk - M));
@@ -537,7 +556,8 @@ int launch_latent_attention(void* out, const void* q_lat, const void* q, const v
                             const int* cu_q, const int* start_pos, const int* tiles, int n_tiles, const float* sink,
                             float* part_o, float* part_ml, int T, int H, int C, int R, int Dq, int rot_off, int BS,
                             int max_blocks, int rows, int num_splits, float scale, float rot_base, int rot_dims,
-                            bool bf, hipStream_t stream) {
+                            int q_stride, const float* freq, float mag, bool halves, int window, bool bf,
+                            hipStream_t stream) {
   if (n_tiles <= 0 || T <= 0) return 0;
   if (C > 512) return 2;
   const int Dk = C + R;
@@ -552,6 +572,7 @@ int launch_latent_attention(void* out, const void* q_lat, const void* q, const v
   a.T = T; a.H = H; a.C = C; a.R = R; a.Dq = Dq; a.rot_off = rot_off; a.BS = BS; a.max_blocks = max_blocks;
   a.rows = rows; a.num_splits = num_splits; a.rot_dims = rot_dims; a.scale = scale;
   a.rot_k = rot_dims > 0 ? (float)(-2.0 * log2((double)rot_base) / rot_dims) : 0.f;
+  a.q_stride = q_stride; a.freq = freq; a.mag = mag; a.halves = halves ? 1 : 0; a.window = window;
   a.hwin = H < pairs ? H : pairs;
   a.kt = kt;
   if (rows < 1 || rows * a.hwin > pairs) return 1;

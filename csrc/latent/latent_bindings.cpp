@@ -15,9 +15,10 @@ void launch_canon_norm(void* out, const float* x, const float* g, float eps, con
                        int W, int taps, int keep, bool out_bf, bool shift_state, hipStream_t stream);
 void launch_canon_state(const float* x, const float* g, float eps, float* conv, int sub, const int* cu_q,
                         const int* start_pos, const int* slots, int S, int W, int taps, int keep, hipStream_t stream);
-void launch_latent_prep(void* cq, const void* proj, int proj_stride, int T, int q_rank, int kv_rank, int rot_dim,
-                        const float* wq, const float* wkv, float eps, const int64_t* positions, float rot_base,
-                        int rot_dims, void* cache, const int64_t* slot_mapping, bool bf, hipStream_t stream);
+void launch_latent_prep(void* cq, const void* proj, int proj_stride, int T, int q_rank, int kv_off, int kv_rank,
+                        int rot_dim, const float* wq, const float* wkv, float eps, const int64_t* positions,
+                        float rot_base, int rot_dims, const float* freq, float mag, bool halves, void* cache,
+                        const int64_t* slot_mapping, bool bf, hipStream_t stream);
 void launch_gate_mul(void* out, const void* o, const void* proj, int proj_stride, int g_off, int T, int H, int Dv,
                      bool bf, hipStream_t stream);
 void launch_poly_norm(void* out, const void* z, const float* coef, int rows, int F, float eps, bool bf,
@@ -28,7 +29,8 @@ int launch_latent_attention(void* out, const void* q_lat, const void* q, const v
                             const int* cu_q, const int* start_pos, const int* tiles, int n_tiles, const float* sink,
                             float* part_o, float* part_ml, int T, int H, int C, int R, int Dq, int rot_off, int BS,
                             int max_blocks, int rows, int num_splits, float scale, float rot_base, int rot_dims,
-                            bool bf, hipStream_t stream);
+                            int q_stride, const float* freq, float mag, bool halves, int window, bool bf,
+                            hipStream_t stream);
 
 namespace {
 
@@ -109,29 +111,53 @@ void canon_state_update(torch::Tensor x, torch::Tensor g, double eps, torch::Ten
                      conv.size(2), cur());
 }
 
-void latent_prep(torch::Tensor cq, torch::Tensor proj, int64_t q_rank, int64_t kv_rank, int64_t rot_dim,
-                 torch::Tensor wq, torch::Tensor wkv, double eps, torch::Tensor positions, double rot_base,
-                 int64_t rot_dims, torch::Tensor cache, torch::Tensor slot_mapping) {
-  chk_act(cq, "cq"); chk_act(proj, "proj"); chk_act(cache, "cache"); chk_f32(wq, "wq"); chk_f32(wkv, "wkv");
-  TORCH_CHECK(proj.scalar_type() == cq.scalar_type() && proj.scalar_type() == cache.scalar_type(),
-              "latent_prep: proj, cq and the cache share one dtype");
+using OptT = c10::optional<torch::Tensor>;
+
+// rotary frequency table [rot_dims / 2] fp32, or none
+const float* freq_of(const OptT& freq, int64_t rot_dims, const char* who) {
+  if (!freq.has_value()) return nullptr;
+  chk_f32(*freq, "freq");
+  TORCH_CHECK(freq->numel() == rot_dims / 2, who, ": freq must hold rot_dims / 2 numbers");
+  return freq->data_ptr<float>();
+}
+
+// cq / wq absent: the layer has no query latent (q_rank 0)
+void latent_prep(OptT cq, torch::Tensor proj, int64_t q_rank, int64_t kv_off, int64_t kv_rank, int64_t rot_dim, OptT wq,
+                 torch::Tensor wkv, double eps, torch::Tensor positions, double rot_base, int64_t rot_dims, OptT freq,
+                 double mag, bool halves, torch::Tensor cache, torch::Tensor slot_mapping) {
+  chk_act(proj, "proj"); chk_act(cache, "cache"); chk_f32(wkv, "wkv");
+  TORCH_CHECK(proj.scalar_type() == cache.scalar_type(), "latent_prep: proj and the cache share one dtype");
   const int64_t T = proj.size(0);
-  TORCH_CHECK(proj.dim() == 2 && proj.size(1) >= q_rank + kv_rank + rot_dim, "latent_prep: proj too narrow");
-  TORCH_CHECK(cq.dim() == 2 && cq.size(0) == T && cq.size(1) == q_rank, "latent_prep: cq [T, q_rank]");
-  TORCH_CHECK(wq.numel() == q_rank && wkv.numel() == kv_rank, "latent_prep: norm weights");
+  TORCH_CHECK(q_rank >= 0 && kv_off >= q_rank && kv_rank >= 1 && rot_dim >= 0, "latent_prep: columns");
+  TORCH_CHECK(proj.dim() == 2 && proj.size(1) >= kv_off + kv_rank + rot_dim, "latent_prep: proj too narrow");
+  TORCH_CHECK(cq.has_value() == (q_rank > 0) && wq.has_value() == (q_rank > 0), "latent_prep: cq / wq go with a query latent");
+  if (q_rank > 0) {
+    chk_act(*cq, "cq"); chk_f32(*wq, "wq");
+    TORCH_CHECK(cq->dim() == 2 && cq->size(0) == T && cq->size(1) == q_rank && cq->scalar_type() == proj.scalar_type(),
+                "latent_prep: cq [T, q_rank]");
+    TORCH_CHECK(wq->numel() == q_rank, "latent_prep: wq");
+  }
+  TORCH_CHECK(wkv.numel() == kv_rank, "latent_prep: wkv");
   TORCH_CHECK(cache.dim() == 3 && cache.size(2) == kv_rank + rot_dim, "latent_prep: cache [blocks, BS, kv_rank + rot_dim]");
   TORCH_CHECK(rot_dims >= 0 && rot_dims <= rot_dim && rot_dims % 2 == 0, "latent_prep: rot_dims");
   chk_i64(positions, "positions", T); chk_i64(slot_mapping, "slot_mapping", T);
-  launch_latent_prep(cq.data_ptr(), proj.data_ptr(), proj.size(1), T, q_rank, kv_rank, rot_dim, wq.data_ptr<float>(),
-                     wkv.data_ptr<float>(), (float)eps, positions.data_ptr<int64_t>(), (float)rot_base, rot_dims,
-                     cache.data_ptr(), slot_mapping.data_ptr<int64_t>(), is_bf(proj), cur());
+  launch_latent_prep(q_rank > 0 ? cq->data_ptr() : nullptr, proj.data_ptr(), proj.size(1), T, q_rank, kv_off, kv_rank,
+                     rot_dim, q_rank > 0 ? wq->data_ptr<float>() : nullptr, wkv.data_ptr<float>(), (float)eps,
+                     positions.data_ptr<int64_t>(), (float)rot_base, rot_dims, freq_of(freq, rot_dims, "latent_prep"),
+                     (float)mag, halves, cache.data_ptr(), slot_mapping.data_ptr<int64_t>(), is_bf(proj), cur());
 }
 
 void latent_attention(torch::Tensor out, torch::Tensor q_lat, torch::Tensor q, int64_t rot_off, torch::Tensor cache,
                       torch::Tensor block_tables, torch::Tensor cu_q, torch::Tensor start_pos, torch::Tensor tiles,
-                      torch::Tensor sink, double scale, double rot_base, int64_t rot_dims, int64_t rows,
-                      int64_t num_splits, c10::optional<torch::Tensor> part_o, c10::optional<torch::Tensor> part_ml) {
-  chk_act(out, "out"); chk_act(q_lat, "q_lat"); chk_act(q, "q"); chk_act(cache, "cache"); chk_f32(sink, "sink");
+                      OptT sink, double scale, double rot_base, int64_t rot_dims, int64_t rows, int64_t num_splits,
+                      OptT part_o, OptT part_ml, OptT freq, double mag, bool halves, int64_t window) {
+  chk_act(out, "out"); chk_act(q_lat, "q_lat"); chk_act(cache, "cache");
+  // q may be a column range of a wider projection: heads and their entries in one piece, any row stride
+  chk(q, "q", false);
+  TORCH_CHECK(is_bf(q) || q.scalar_type() == torch::kFloat32, "q must be bf16 or fp32");
+  TORCH_CHECK(q.dim() == 3 && q.stride(2) == 1 && (q.size(1) == 1 || q.stride(1) == q.size(2)) &&
+              (q.size(0) == 1 || q.stride(0) >= q.size(1) * q.size(2)), "latent_attention: q rows must be in one piece");
+  TORCH_CHECK(window >= 0, "latent_attention: window");
   TORCH_CHECK(q_lat.scalar_type() == q.scalar_type() && q.scalar_type() == cache.scalar_type() &&
               out.scalar_type() == q.scalar_type(), "latent_attention: one dtype for q, cache and out");
   TORCH_CHECK(q_lat.dim() == 3 && q.dim() == 3 && cache.dim() == 3, "latent_attention: ranks");
@@ -139,7 +165,11 @@ void latent_attention(torch::Tensor out, torch::Tensor q_lat, torch::Tensor q, i
   const int64_t Dq = q.size(2), R = Dq - rot_off, BS = cache.size(1);
   TORCH_CHECK(q.size(0) == T && q.size(1) == H && rot_off >= 0 && R >= 0, "latent_attention: q [T, H, rot_off + R]");
   TORCH_CHECK(cache.size(2) == C + R, "latent_attention: cache rows must hold C + R = ", C + R, " numbers");
-  TORCH_CHECK(out.sizes() == q_lat.sizes() && sink.numel() == H, "latent_attention: out / sink");
+  TORCH_CHECK(out.sizes() == q_lat.sizes(), "latent_attention: out");
+  if (sink.has_value()) {
+    chk_f32(*sink, "sink");
+    TORCH_CHECK(sink->numel() == H, "latent_attention: sink [H]");
+  }
   TORCH_CHECK(rot_dims >= 0 && rot_dims <= R && rot_dims % 2 == 0, "latent_attention: rot_dims");
   chk_i32(block_tables, "block_tables"); chk_i32(cu_q, "cu_q"); chk_i32(start_pos, "start_pos", cu_q.numel() - 1);
   chk_i32(tiles, "tiles");
@@ -158,9 +188,11 @@ void latent_attention(torch::Tensor out, torch::Tensor q_lat, torch::Tensor q, i
   }
   int rc = launch_latent_attention(out.data_ptr(), q_lat.data_ptr(), q.data_ptr(), cache.data_ptr(),
                                    block_tables.data_ptr<int>(), cu_q.data_ptr<int>(), start_pos.data_ptr<int>(),
-                                   tiles.data_ptr<int>(), tiles.size(0), sink.data_ptr<float>(), po, pml, T, H, C, R, Dq,
-                                   rot_off, BS, block_tables.size(1), rows, num_splits, (float)scale, (float)rot_base,
-                                   rot_dims, is_bf(q), cur());
+                                   tiles.data_ptr<int>(), tiles.size(0), sink.has_value() ? sink->data_ptr<float>() : nullptr,
+                                   po, pml, T, H, C, R, Dq, rot_off, BS, block_tables.size(1), rows, num_splits,
+                                   (float)scale, (float)rot_base, rot_dims, (int)q.stride(0),
+                                   freq_of(freq, rot_dims, "latent_attention"), (float)mag, halves, (int)window,
+                                   is_bf(q), cur());
   TORCH_CHECK(rc == 0, "latent_attention: unsupported shape (code ", rc, ": 1 rows per tile, 2 latent wider than 512, "
               "3 cached row too wide for the LDS tile)");
 }

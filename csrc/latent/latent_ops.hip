@@ -8,7 +8,8 @@
 //   canon_norm        h = x / rms(x) * g ; out = h + sum_j w[:, j] * h_(t - taps + 1 + j)
 //                     rows ahead of a sequence's first row of this batch come from its state slot
 //   canon_state       shift a sequence's state by its rows of this batch
-//   latent_prep       query-latent norm; KV-latent norm + rotary shared key part -> paged cache row
+//   latent_prep       query-latent norm (if the layer has one); KV-latent norm + rotary shared key
+//                     part -> paged cache row
 //   gate_mul          [H, T, Dv] head-major -> [T, H * Dv], times sigmoid(gate)
 //   poly_norm         a N(z) + b N(z^2) + c N(z^3) + e,  N(u) = u / rms(u)
 //   logit_softcap     cap * tanh(scale * x / cap)
@@ -144,43 +145,54 @@ __global__ void __launch_bounds__(1024) canon_state_kernel(const float* __restri
 // the op computes the same expression)
 RT_DEVICE float rot_freq(int i, float neg2_log2base_over_dims) { return exp2f((float)i * neg2_log2base_over_dims); }
 
+// columns 0 .. q_rank of proj: the query latent (q_rank 0: none); kv_off ..: the key / value latent,
+// then the rotated key part. Rotary pairs are (2i, 2i + 1) or (`halves`) (i, i + rot_dims / 2), by
+// pos * freq[i] (freq null: base^(-2i / dims)) with cos and sin times `mag`.
 template <typename PT, typename CT, typename OT>
 __global__ void __launch_bounds__(1024) latent_prep_kernel(
-    OT* __restrict__ cq, const PT* __restrict__ proj, int proj_stride, int q_rank, int kv_rank, int rot_dim,
+    OT* __restrict__ cq, const PT* __restrict__ proj, int proj_stride, int q_rank, int kv_off, int kv_rank, int rot_dim,
     const float* __restrict__ wq, const float* __restrict__ wkv, float eps, const int64_t* __restrict__ positions,
-    float rot_k, int rot_dims, CT* __restrict__ cache, const int64_t* __restrict__ slot_mapping) {
+    float rot_k, int rot_dims, const float* __restrict__ freq, float mag, int halves, CT* __restrict__ cache,
+    const int64_t* __restrict__ slot_mapping) {
   __shared__ float scratch[16];
   const int t = blockIdx.x;
   const PT* p = proj + (size_t)t * proj_stride;
-  float sq = 0.f, sk = 0.f;
-  for (int c = threadIdx.x; c < q_rank; c += blockDim.x) {
-    const float v = DT<PT>::load(p + c);
-    sq += v * v;
+  const PT* pk = p + kv_off;
+  if (q_rank > 0) {
+    float sq = 0.f;
+    for (int c = threadIdx.x; c < q_rank; c += blockDim.x) {
+      const float v = DT<PT>::load(p + c);
+      sq += v * v;
+    }
+    const float iq = rsqrtf(rt::block_sum(sq, scratch) / q_rank + eps);
+    OT* o = cq + (size_t)t * q_rank;
+    for (int c = threadIdx.x; c < q_rank; c += blockDim.x) DT<OT>::store(o + c, DT<PT>::load(p + c) * iq * wq[c]);
   }
+  float sk = 0.f;
   for (int c = threadIdx.x; c < kv_rank; c += blockDim.x) {
-    const float v = DT<PT>::load(p + q_rank + c);
+    const float v = DT<PT>::load(pk + c);
     sk += v * v;
   }
-  const float iq = rsqrtf(rt::block_sum(sq, scratch) / q_rank + eps);
   const float ik = rsqrtf(rt::block_sum(sk, scratch) / kv_rank + eps);
-  OT* o = cq + (size_t)t * q_rank;
-  for (int c = threadIdx.x; c < q_rank; c += blockDim.x) DT<OT>::store(o + c, DT<PT>::load(p + c) * iq * wq[c]);
   CT* row = cache + (size_t)slot_mapping[t] * (kv_rank + rot_dim);
-  for (int c = threadIdx.x; c < kv_rank; c += blockDim.x)
-    DT<CT>::store(row + c, DT<PT>::load(p + q_rank + c) * ik * wkv[c]);
-  const PT* pr = p + q_rank + kv_rank;
+  for (int c = threadIdx.x; c < kv_rank; c += blockDim.x) DT<CT>::store(row + c, DT<PT>::load(pk + c) * ik * wkv[c]);
+  const PT* pr = pk + kv_rank;
+  CT* rr = row + kv_rank;
   const float posf = (float)positions[t];
-  for (int i = threadIdx.x; i < rot_dim / 2 + (rot_dim & 1); i += blockDim.x) {
-    const float u = DT<PT>::load(pr + 2 * i);
-    if (2 * i + 1 >= rot_dim) {  // odd tail entry: never rotated
-      DT<CT>::store(row + kv_rank + 2 * i, u);
+  const int half = rot_dims >> 1;
+  for (int i = threadIdx.x; i < rot_dim - half; i += blockDim.x) {
+    if (i >= half) {      // past the rotated entries
+      DT<CT>::store(rr + i + half, DT<PT>::load(pr + i + half));
       continue;
     }
-    const float v = DT<PT>::load(pr + 2 * i + 1);
-    float cs = 1.f, sn = 0.f;
-    if (2 * i < rot_dims) sincosf(posf * rot_freq(i, rot_k), &sn, &cs);
-    DT<CT>::store(row + kv_rank + 2 * i, u * cs - v * sn);
-    DT<CT>::store(row + kv_rank + 2 * i + 1, v * cs + u * sn);
+    const int iu = halves ? i : 2 * i, iv = halves ? i + half : 2 * i + 1;
+    const float u = DT<PT>::load(pr + iu), v = DT<PT>::load(pr + iv);
+    float cs, sn;
+    sincosf(posf * (freq ? freq[i] : rot_freq(i, rot_k)), &sn, &cs);
+    cs *= mag;
+    sn *= mag;
+    DT<CT>::store(rr + iu, u * cs - v * sn);
+    DT<CT>::store(rr + iv, v * cs + u * sn);
   }
 }
 
@@ -273,13 +285,19 @@ void launch_canon_state(const float* x, const float* g, float eps, float* conv, 
   RT_LAUNCH_W(canon_state_kernel, S, W, x, g, eps, conv, sub, cu_q, start_pos, slots, W, taps, keep);
 }
 
-void launch_latent_prep(void* cq, const void* proj, int proj_stride, int T, int q_rank, int kv_rank, int rot_dim,
-                        const float* wq, const float* wkv, float eps, const int64_t* positions, float rot_base,
-                        int rot_dims, void* cache, const int64_t* slot_mapping, bool bf, hipStream_t stream) {
+void launch_latent_prep(void* cq, const void* proj, int proj_stride, int T, int q_rank, int kv_off, int kv_rank,
+                        int rot_dim, const float* wq, const float* wkv, float eps, const int64_t* positions,
+                        float rot_base, int rot_dims, const float* freq, float mag, bool halves, void* cache,
+                        const int64_t* slot_mapping, bool bf, hipStream_t stream) {
   if (T <= 0) return;
-  const float rot_k = rot_dims > 0 ? -2.0f * log2f(rot_base) / (float)rot_dims : 0.f;
-  if (bf) RT_LAUNCH_W((latent_prep_kernel<uint16_t, uint16_t, uint16_t>), T, (q_rank > kv_rank ? q_rank : kv_rank), (uint16_t*)cq, (const uint16_t*)proj, proj_stride, q_rank, kv_rank, rot_dim, wq, wkv, eps, positions, rot_k, rot_dims, (uint16_t*)cache, slot_mapping);
-  else RT_LAUNCH_W((latent_prep_kernel<float, float, float>), T, (q_rank > kv_rank ? q_rank : kv_rank), (float*)cq, (const float*)proj, proj_stride, q_rank, kv_rank, rot_dim, wq, wkv, eps, positions, rot_k, rot_dims, (float*)cache, slot_mapping);
+  const float rot_k = rot_dims > 0 && freq == nullptr ? -2.0f * log2f(rot_base) / (float)rot_dims : 0.f;
+  const int W = q_rank > kv_rank ? q_rank : kv_rank;
+#define RT_LP(TT)                                                                                                      \
+  RT_LAUNCH_W((latent_prep_kernel<TT, TT, TT>), T, W, (TT*)cq, (const TT*)proj, proj_stride, q_rank, kv_off, kv_rank,  \
+              rot_dim, wq, wkv, eps, positions, rot_k, rot_dims, freq, mag, halves ? 1 : 0, (TT*)cache, slot_mapping)
+  if (bf) RT_LP(uint16_t);
+  else RT_LP(float);
+#undef RT_LP
 }
 
 void launch_gate_mul(void* out, const void* o, const void* proj, int proj_stride, int g_off, int T, int H, int Dv,

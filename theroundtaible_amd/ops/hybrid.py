@@ -208,7 +208,7 @@ def gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale: flo
 
 # ---- minGRU ---------------------------------------------------------------------------------------
 
-SCAN_CHUNK = 64          # rows per chunk of the chunked scan (csrc/hybrid/hybrid_ops.hip kScanChunk)
+SCAN_CHUNK = 64          # rows per chunk of the chunked scans (csrc/hybrid/hybrid_ops.hip kScanChunk; state_scan)
 
 
 def scan_chunks(cu_q: torch.Tensor, device=None):
@@ -265,6 +265,16 @@ def add_norm(x, y, w, eps, out_dtype, groups: int = 1) -> torch.Tensor:
         native().add_norm(out, x, y, w, float(eps), int(groups))
         return out
     return ref_add_norm(x, y, w, eps, out_dtype, groups)
+
+
+def add_layer_norm(x, y, scale, w, b, eps, out_dtype) -> torch.Tensor:
+    """x += y * scale (in place, fp32; ``scale`` [W] fp32, ``y`` may be None), returns the layer
+    norm (x - mean) / sqrt(variance + eps) * w + b of the new x."""
+    if _gpu(x):
+        out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+        native().add_layer_norm(out, x, y, scale if y is not None else None, w, b, float(eps))
+        return out
+    return ref_add_layer_norm(x, y, scale, w, b, eps, out_dtype)
 
 
 def limited_glu(gu, limit: float, out_dtype) -> torch.Tensor:
@@ -360,6 +370,22 @@ def route_topk(h, router_w, top: int, bias=None) -> Tuple[torch.Tensor, torch.Te
         native().route_topk(idx, wt, h.contiguous(), router_w, bias)
         return idx, wt
     return topk_softmax(torch.nn.functional.linear(h.float(), router_w, bias), top)
+
+
+def route_groups(h, router_w, moe, correction) -> Tuple[torch.Tensor, torch.Tensor]:
+    """Router and choice of a sigmoid-scored mixture (``moe``: :class:`MoESpec`): fp32 scores
+    s = sigmoid(``router_w`` [E, W] . ``h``); the ``moe.top`` experts with the largest
+    s + ``correction`` [E] among those of the best ``moe.group_keep`` of ``moe.groups`` equal groups
+    of neighbours (a group's value: the sum of its two largest); weights s of the chosen over
+    (their sum + 1e-20), times ``moe.scale``. One launch on the GPU."""
+    E, W = router_w.shape
+    if _gpu(h) and E <= 512 and moe.top <= 64 and (W + 4 + 5 * E) * 4 <= 48 * 1024:
+        idx = torch.empty(h.shape[0], moe.top, dtype=torch.int32, device=h.device)
+        wt = torch.empty(h.shape[0], moe.top, dtype=torch.float32, device=h.device)
+        native().route_topk(idx, wt, h.contiguous(), router_w, None, True, correction, moe.groups, moe.group_keep,
+                            float(moe.scale))
+        return idx, wt
+    return ref_route_groups(h, router_w, moe, correction)
 
 
 MOE_ROWS = 16            # steps of up to this many rows run the experts row by row (moe_rows)
@@ -548,6 +574,27 @@ def ref_add_norm(x, y, w, eps, out_dtype, groups=1):
     return (_rms(x, eps, groups) * w).to(out_dtype)
 
 
+def ref_add_layer_norm(x, y, scale, w, b, eps, out_dtype):
+    if y is not None:
+        x.add_(y.float() * scale)
+    d = x - x.mean(-1, keepdim=True)
+    return (d / torch.sqrt((d * d).mean(-1, keepdim=True) + eps) * w + b).to(out_dtype)
+
+
+def ref_route_groups(h, router_w, moe, correction):
+    s = torch.sigmoid(torch.nn.functional.linear(h.float(), router_w))
+    choice = s + correction
+    T, E = s.shape
+    if moe.group_keep < moe.groups:
+        parts = choice.view(T, moe.groups, E // moe.groups)
+        value = torch.topk(parts, min(2, parts.shape[2]), dim=-1).values.sum(-1)
+        keep = torch.zeros_like(value, dtype=torch.bool).scatter_(1, torch.topk(value, moe.group_keep, dim=-1).indices, True)
+        choice = parts.masked_fill(~keep[:, :, None], float("-inf")).reshape(T, E)
+    idx = torch.topk(choice, moe.top, dim=-1).indices
+    wt = s.gather(1, idx)
+    return idx.to(torch.int32), wt / (wt.sum(-1, keepdim=True) + 1e-20) * moe.scale
+
+
 def ref_wkv_scan(rkvg, lw, w0, u, norm_w, eps, state, cu_q, start_pos, slots, out_dtype):
     T, HD = rkvg.shape[1], rkvg.shape[2]
     H, D = u.shape
@@ -718,16 +765,45 @@ def delta_prep(proj, spec, q_off: int, b_off: int, a_off: int, conv_w, state, ne
                           start_pos, slots, shift_state)
 
 
-def state_scan(q, k, v, w, a, b, decay, state, cu_q, start_pos, slots, heads: int, dim: int, vdim: int) -> torch.Tensor:
+def gla_prep(proj, spec, q_off: int, k_off: int, v_off: int, a_off: int, a2, a_bias) -> Tuple[torch.Tensor, ...]:
+    """Inputs of a gated linear attention (``spec``: :class:`GLASpec`) from ``proj`` [T, N]: columns of
+    q and k (heads x dim), v (heads x vdim) and the input of the decay's low-rank path (``a2``
+    [rank, heads * dim] fp32 its second factor). All math fp32: q times dim^(-1/2); decay =
+    sigmoid(low . a2 + a_bias)^(1 / tau) per key channel. Returns fp32 rows (q, k, decay
+    [T, heads * dim], v [T, heads * vdim]): the (q, k, w, v) of :func:`state_scan`."""
+    n, nv = spec.heads * spec.dim, spec.heads * spec.vdim
+    if _gpu(proj):
+        out = torch.empty(proj.shape[0], 3 * n + nv, dtype=torch.float32, device=proj.device)
+        native().gla_prep(out, proj, int(q_off), int(k_off), int(v_off), int(a_off), a2, a_bias, spec.dim ** -0.5,
+                          1.0 / spec.tau)
+    else:
+        low = proj[:, a_off:a_off + a2.shape[0]].float()
+        z = low @ a2 + a_bias
+        dec = torch.exp(torch.nn.functional.logsigmoid(z) / spec.tau)
+        out = torch.cat([proj[:, q_off:q_off + n].float() * spec.dim ** -0.5, proj[:, k_off:k_off + n].float(), dec,
+                         proj[:, v_off:v_off + nv].float()], 1)
+    return out[:, :n], out[:, n:2 * n], out[:, 2 * n:3 * n], out[:, 3 * n:]
+
+
+def state_scan(q, k, v, w, a, b, decay, state, cu_q, start_pos, slots, heads: int, dim: int, vdim: int,
+               chunks=None) -> torch.Tensor:
     """Matrix-state recurrence, fp32 throughout. Per sequence and head, with the dim x vdim state S
     from ``state[slot]`` (zeros at position 0), for every token in order:
         s = b_t^T S;   S <- diag(w_t) S - a_t s^T + k_t v_t^T;   o_t = S^T q_t
     ``q, k, w, a, b`` [T, heads * dim] and ``v`` [T, heads * vdim] are fp32 rows (any row stride).
     ``w`` None: every head decays by its constant ``decay[head]``; ``a`` / ``b`` None: nothing is
     removed. Returns o [T, heads * vdim] fp32 and leaves every span's last S in ``state``
-    (``[n_slots, heads * vdim * dim]``, each head stored column by column)."""
+    (``[n_slots, heads * vdim * dim]``, each head stored column by column). ``chunks`` (GPU, without
+    a / b): :func:`scan_chunks` of this batch — spans are then scanned in chunks of ``SCAN_CHUNK``
+    rows in parallel (chunk end states and decay products, a carry pass, the outputs from each
+    chunk's true start state); the results differ from the one-launch scan by rounding only."""
     if _gpu(q):
         out = torch.empty(q.shape[0], heads * vdim, dtype=torch.float32, device=q.device)
+        if chunks is not None:
+            ws = torch.empty(chunks[0].shape[0] * heads * dim * (vdim + 1), dtype=torch.float32, device=q.device)
+            native().state_scan(out, q, k, v, w, a, b, decay, state, cu_q, start_pos, slots, int(heads), int(dim), int(vdim),
+                                chunks[0], chunks[1], ws, SCAN_CHUNK)
+            return out
         native().state_scan(out, q, k, v, w, a, b, decay, state, cu_q, start_pos, slots, int(heads), int(dim), int(vdim))
         return out
     return ref_state_scan(q, k, v, w, a, b, decay, state, cu_q, start_pos, slots, heads, dim, vdim)

@@ -1,6 +1,6 @@
 """Ops of the latent-attention model family: scalar RMS norms, input convolutions with a running
-state, the latent cache write, attention over the cached latents with a softmax sink, the output
-gate, PolyNorm and the logit soft cap.
+state, the latent cache write, attention over the cached latents (optional softmax sink, optional sliding
+window), the output gate, PolyNorm and the logit soft cap.
 
 GPU tensors go to the HIP kernels of ``theroundtaible_amd._C_latent`` (``csrc/latent/``, built
 in-tree by ``csrc/build.py``; :func:`ensure_built` compiles it on first use in a fresh checkout);
@@ -13,6 +13,7 @@ from __future__ import annotations
 
 import os
 import sys
+from dataclasses import dataclass
 from typing import Optional
 
 import torch
@@ -99,14 +100,43 @@ def canon_state_update(x, g, eps, w, conv, sub, cu_q, start_pos, slots):
     ref.canon_state_update(x, g, eps, conv[:, sub, :w.shape[1] - 1], cu_q, start_pos, slots)
 
 
-def latent_prep(proj, spec, wq, wkv, eps, positions, cache_rows, slot_mapping, out_dtype):
+@dataclass
+class RotaryTable:
+    """Rotary frequencies as a table (``freq`` [dims / 2] fp32 on the device, None: nothing is
+    rotated), the factor of cos and sin, and how entries pair up: (i, i + dims / 2) or (2i, 2i + 1)."""
+    freq: Optional[torch.Tensor]
+    mag: float
+    halves: bool
+
+
+def rotary_table(rot, device) -> RotaryTable:
+    """:class:`RotaryTable` of a ``RotarySpec`` (None: no rotation)."""
+    if rot is None or rot.dims == 0:
+        return RotaryTable(None, 1.0, False)
+    inv, mag = ref.rope_inv_freq(rot.dims, rot.base, rot.scaling)
+    return RotaryTable(inv.to(torch.float32).to(device).contiguous(), float(mag), rot.halves)
+
+
+def _rotary_args(spec, table):
+    """(rot_base, rot_dims, freq, mag, halves) of a kernel call."""
+    if table is None:
+        return float(spec.rot_base), spec.rot_dims, None, 1.0, False
+    return 1.0, 2 * table.freq.numel() if table.freq is not None else 0, table.freq, table.mag, table.halves
+
+
+def latent_prep(proj, spec, wq, wkv, eps, positions, cache_rows, slot_mapping, out_dtype, kv_off=None, table=None):
+    """See :func:`.reference.latent_prep`. ``kv_off``: the first column of the key / value latent
+    (default: right behind the query latent). A spec with ``q_rank`` 0 has no query latent: only
+    the cache row is written and None returned."""
+    kv_off = spec.q_rank if kv_off is None else kv_off
     if _gpu(proj):
-        cq = torch.empty(proj.shape[0], spec.q_rank, dtype=out_dtype, device=proj.device)
-        native().latent_prep(cq, proj, spec.q_rank, spec.kv_rank, spec.rot_dim, wq, wkv, float(eps), positions,
-                             float(spec.rot_base), spec.rot_dims, cache_rows, slot_mapping)
+        cq = torch.empty(proj.shape[0], spec.q_rank, dtype=out_dtype, device=proj.device) if spec.q_rank else None
+        base, dims, freq, mag, halves = _rotary_args(spec, table)
+        native().latent_prep(cq, proj, spec.q_rank, int(kv_off), spec.kv_rank, spec.rot_dim, wq, wkv, float(eps), positions,
+                             base, dims, freq, mag, halves, cache_rows, slot_mapping)
         return cq
     return ref.latent_prep(proj, spec.q_rank, spec.kv_rank, spec.rot_dim, wq, wkv, eps, positions, spec.rot_base,
-                           spec.rot_dims, cache_rows, slot_mapping, out_dtype)
+                           spec.rot_dims, cache_rows, slot_mapping, out_dtype, kv_off, table)
 
 
 def rows_per_tile(heads: int, kv_rank: int, rot_dim: int, dtype) -> int:
@@ -140,10 +170,12 @@ class LatentWorkspace:
 
 
 def latent_attention(q_lat, q, spec, cache_rows, block_tables, cu_q, start_pos, sink, tiles=None,
-                     num_splits: int = 1, workspace: Optional[LatentWorkspace] = None, out_dtype=None):
-    """See :func:`.reference.latent_attention`. ``tiles``: :func:`tile_map` on the device (GPU);
-    ``num_splits`` > 1 cuts every tile's keys into that many ranges merged by a second launch
-    (one row per sequence: the decode step)."""
+                     num_splits: int = 1, workspace: Optional[LatentWorkspace] = None, out_dtype=None, table=None):
+    """See :func:`.reference.latent_attention`. ``q`` [T, H, dim + rot_dim] may be a column range of
+    a wider projection; ``sink`` None: no sink; ``spec.window`` > 0: a sliding window. ``tiles``:
+    :func:`tile_map` on the device (GPU); ``num_splits`` > 1 cuts every tile's keys into that many
+    ranges merged by a second launch (one row per sequence: the decode step). ``table``: the
+    :class:`RotaryTable` of the rotated part (default: interleaved pairs of ``spec.rot_base``)."""
     out_dtype = out_dtype or q.dtype
     if _gpu(q):
         H, T, C = q_lat.shape
@@ -155,13 +187,19 @@ def latent_attention(q_lat, q, spec, cache_rows, block_tables, cu_q, start_pos, 
             tiles = tile_map(cu_q.cpu(), start_pos.cpu(), rows).to(q.device)
         if num_splits > 1 and workspace is None:
             workspace = LatentWorkspace(T, H, C, num_splits, q.device)
+        base, dims, freq, mag, halves = _rotary_args(spec, table)
         native().latent_attention(out, q_lat, q, spec.dim, cache_rows, block_tables, cu_q, start_pos, tiles, sink,
-                                  float(spec.scale), float(spec.rot_base), spec.rot_dims, rows, int(num_splits),
+                                  float(spec.scale), base, dims, rows, int(num_splits),
                                   workspace.part_o if num_splits > 1 else None,
-                                  workspace.part_ml if num_splits > 1 else None)
+                                  workspace.part_ml if num_splits > 1 else None, freq, mag, halves, int(spec.window))
         return out
     return ref.latent_attention(q_lat, q, spec.dim, cache_rows, block_tables, cu_q, start_pos, sink, spec.scale,
-                                spec.rot_base, spec.rot_dims, out_dtype)
+                                spec.rot_base, spec.rot_dims, out_dtype, table, spec.window)
+
+
+def window_splits(splits: int, window: int) -> int:
+    """Key ranges per decoded row under a sliding window: no more than the tiles it can touch."""
+    return splits if window <= 0 else max(1, min(splits, (window + KEY_TILE - 1) // KEY_TILE + 1))
 
 
 def gate_mul(o, proj, g_off, out_dtype):

@@ -79,9 +79,7 @@ def rope_inv_freq(head_dim: int, theta: float, scaling: Optional[tuple] = None) 
             return (head_dim * math.log(orig / (rot * 2 * math.pi))) / (2 * math.log(theta))
         low = max(math.floor(corr_dim(beta_fast)), 0)
         high = min(math.ceil(corr_dim(beta_slow)), head_dim - 1)
-        if low == high:
-            high += 0.001
-        ramp = ((torch.arange(head_dim // 2, dtype=torch.float64) - low) / (high - low)).clamp(0, 1)
+        ramp = ((torch.arange(head_dim // 2, dtype=torch.float64) - low) / max(high - low, 0.001)).clamp(0, 1)
         extra = 1 - ramp                     # 1: keep the original frequency, 0: interpolate
         out = (inv / factor) * (1 - extra) + inv * extra
         return out, att
@@ -493,27 +491,50 @@ def rotate_interleaved(v: torch.Tensor, positions: torch.Tensor, base: float, di
     return out
 
 
+def rotate_table(v: torch.Tensor, positions: torch.Tensor, table) -> torch.Tensor:
+    """Rotary embedding from a frequency table (``ops/latent.py`` ``RotaryTable``) on the leading
+    2 * len(freq) entries of the last axis: pairs (i, i + len(freq)) or (2i, 2i + 1), cos and sin
+    times the table's magnitude."""
+    vf = v.float()
+    if table.freq is None:
+        return vf
+    r = table.freq.numel()
+    a = positions.float().view(-1, *([1] * (v.dim() - 1))) * table.freq
+    c, s = torch.cos(a) * table.mag, torch.sin(a) * table.mag
+    at = (slice(0, r), slice(r, 2 * r)) if table.halves else (slice(0, 2 * r, 2), slice(1, 2 * r, 2))
+    u, w = vf[..., at[0]], vf[..., at[1]]
+    out = vf.clone()
+    out[..., at[0]] = u * c - w * s
+    out[..., at[1]] = w * c + u * s
+    return out
+
+
 def latent_prep(proj, q_rank, kv_rank, rot_dim, wq, wkv, eps, positions, rot_base, rot_dims, cache_rows,
-                slot_mapping, out_dtype):
-    """From the fused input projection ``proj`` [T, >= q_rank + kv_rank + rot_dim]: the normed
-    query latent (returned) and the cache row (normed latent | rotated shared key part), written
-    at ``slot_mapping`` into ``cache_rows`` [num_blocks, block_size, kv_rank + rot_dim]."""
-    cq = rms_norm(proj[:, :q_rank].float(), wq.float(), eps).to(out_dtype)
-    c = rms_norm(proj[:, q_rank:q_rank + kv_rank].float(), wkv.float(), eps)
-    kr = rotate_interleaved(proj[:, q_rank + kv_rank:q_rank + kv_rank + rot_dim], positions, rot_base, rot_dims)
+                slot_mapping, out_dtype, kv_off=None, table=None):
+    """From the fused input projection ``proj`` [T, >= kv_off + kv_rank + rot_dim]: the normed
+    query latent (columns 0 .. q_rank; returned, None when q_rank is 0) and the cache row (normed
+    latent | rotated shared key part, from column ``kv_off`` on: q_rank by default), written at ``slot_mapping`` into
+    ``cache_rows`` [num_blocks, block_size, kv_rank + rot_dim]. ``table``: a rotary table (halves,
+    rescaled frequencies) instead of interleaved pairs of ``rot_base``."""
+    kv_off = q_rank if kv_off is None else kv_off
+    cq = rms_norm(proj[:, :q_rank].float(), wq.float(), eps).to(out_dtype) if q_rank else None
+    c = rms_norm(proj[:, kv_off:kv_off + kv_rank].float(), wkv.float(), eps)
+    kr = proj[:, kv_off + kv_rank:kv_off + kv_rank + rot_dim]
+    kr = rotate_interleaved(kr, positions, rot_base, rot_dims) if table is None else rotate_table(kr, positions, table)
     flat = cache_rows.view(-1, cache_rows.shape[-1])
     flat[slot_mapping.long()] = torch.cat([c, kr], -1).to(cache_rows.dtype)
     return cq
 
 
 def latent_attention(q_lat, q, rot_off, cache_rows, block_tables, cu_q, start_pos, sink, scale, rot_base,
-                     rot_dims, out_dtype):
+                     rot_dims, out_dtype, table=None, window=0):
     """Causal attention over the cached rows with the query folded into the latent space.
 
     ``q_lat`` [H, T, C] (the unrotated query of each head times its key up-projection), ``q``
     [T, H, Dq] whose entries ``rot_off:`` are the un-rotated rotary part (rotated here, by the
     row's position). Key t = cached row, value t = its first C entries. The softmax denominator
-    also holds exp(sink_h). Returns [H, T, C]."""
+    also holds exp(sink_h) (``sink`` None: it does not). ``window`` > 0: position i sees only keys
+    j with i - j < window. Returns [H, T, C]."""
     H, T, C = q_lat.shape
     out = torch.zeros(H, T, C, dtype=torch.float32, device=q.device)
     cq, sp = cu_q.tolist(), start_pos.tolist()
@@ -526,11 +547,16 @@ def latent_attention(q_lat, q, rot_off, cache_rows, block_tables, cu_q, start_po
         nb = (n + BS - 1) // BS
         K = cache_rows[block_tables[s, :nb].long()].reshape(nb * BS, -1)[:n].float()
         pos = torch.arange(sp[s], n, device=q.device)
-        qr = rotate_interleaved(q[r0:r1, :, rot_off:], pos, rot_base, rot_dims)          # [n_q, H, R]
+        qr = q[r0:r1, :, rot_off:]                                                       # [n_q, H, R]
+        qr = rotate_interleaved(qr, pos, rot_base, rot_dims) if table is None else rotate_table(qr, pos, table)
         Q = torch.cat([q_lat[:, r0:r1].float(), qr.transpose(0, 1)], -1)                 # [H, n_q, C + R]
         sc = torch.einsum("hqd,kd->hqk", Q, K) * scale
-        mask = torch.arange(n, device=q.device).view(1, 1, n) > pos.view(1, -1, 1)
+        dist = pos.view(1, -1, 1) - torch.arange(n, device=q.device).view(1, 1, n)
+        mask = (dist < 0) | (dist >= window) if window > 0 else dist < 0
         sc = sc.masked_fill(mask, float("-inf"))
+        if sink is None:
+            out[:, r0:r1] = torch.einsum("hqk,kc->hqc", torch.softmax(sc, -1), K[:, :C])
+            continue
         sk = sink.float().view(H, 1, 1)
         m = torch.maximum(sc.max(-1, keepdim=True).values, sk)
         e = torch.exp(sc - m)
