@@ -238,38 +238,50 @@ class StatefulPagedCache(PagedKVCache):
 
 
 class LatentKVCache(StatefulPagedCache):
-    """Paged cache of latent-attention layers plus the input-convolution states.
+    """Paged cache of latent-attention layers plus per-sequence running states.
 
     Per layer ``l`` one tensor ``rows[l]`` ``[num_blocks, block_size, row_l]``: token ``t`` of a
     sequence keeps ``row_l = kv_rank + rot_dim`` numbers (its normed latent, then the rotated key
     part all heads share) at ``slot = block * block_size + offset`` — keys AND values of every
     head are read from that one row, so a layer's cache line is 1 / (2 * heads) of a per-head
-    K/V cache's. Layers may differ in row width.
+    K/V cache's. Layers may differ in row width. A layer that reads another layer's rows
+    (``shared[l]`` = that layer) has the same tensor; a layer without attention gives None as its
+    row width and has none: its memory per sequence is its state alone.
 
-    ``conv[l]`` ``[n_slots, 2, taps - 1, width]`` fp32: for each state slot the last ``taps - 1``
-    inputs of layer ``l``'s two input convolutions (mixer, feed-forward), oldest first. The state
-    belongs to exactly ``state_len`` tokens of its sequence: rolling a sequence back to any other
-    length drops it, and the sequence restarts from position 0."""
+    States, fp32, one row per slot. ``conv[l]`` ``[n_slots, 2, taps - 1, width]`` (``taps`` 0: no
+    input convolutions): the last ``taps - 1`` inputs of layer ``l``'s two input convolutions (mixer,
+    feed-forward), oldest first. ``rec[l]`` ``[n_slots, rec_widths[l]]``: the flattened matrix state
+    of a recurrent mixer (None for a layer without one). The state belongs to exactly ``state_len``
+    tokens of its sequence: rolling a sequence back to any other length drops it, and the sequence
+    restarts from position 0. A sequence at position 0 never reads its slot, so a reused slot needs
+    no clearing."""
 
     def __init__(self, row_dims, conv_width: int, taps: int, num_blocks: int, block_size: int, device,
-                 dtype=torch.bfloat16, n_slots: int = 16):
+                 dtype=torch.bfloat16, n_slots: int = 16, shared=None, rec_widths=None):
         self.n_layers = len(row_dims)
         self.row_dims = list(row_dims)
-        self.n_kv_heads, self.head_dim = 1, max(row_dims)
+        self.shared = list(shared) if shared is not None else [None] * self.n_layers
+        self.n_kv_heads, self.head_dim = 1, max([r for r in row_dims if r] + [1])
         self.block_size, self.num_blocks = block_size, num_blocks
         self.device, self.dtype = device, dtype
         # zero-init: tail rows of a partial block are masked, never skipped, so they must be finite
-        self.rows = [torch.zeros(num_blocks, block_size, r, dtype=dtype, device=device) for r in row_dims]
+        self.rows = [torch.zeros(num_blocks, block_size, r, dtype=dtype, device=device) if r and src is None else None
+                     for r, src in zip(row_dims, self.shared)]
+        for l, src in enumerate(self.shared):
+            if src is not None:
+                self.rows[l] = self.rows[src]
         self.alloc = BlockAllocator(num_blocks)
         self.seqs = {}
         self.taps = taps
         self.state = StateSlots(n_slots)
         self.conv = [torch.zeros(n_slots, 2, max(taps - 1, 1), conv_width, dtype=torch.float32, device=device)
-                     for _ in row_dims]
+                     for _ in row_dims] if taps > 0 else []
+        self.rec = [torch.zeros(n_slots, w, dtype=torch.float32, device=device) if w else None
+                    for w in (rec_widths if rec_widths is not None else [0] * self.n_layers)]
 
     @staticmethod
     def bytes_per_block(row_dims, block_size, dtype_bytes=2) -> int:   # type: ignore[override]
-        return sum(row_dims) * block_size * dtype_bytes
+        return sum(r for r in row_dims if r) * block_size * dtype_bytes
 
     def layer_rows(self, l: int) -> torch.Tensor:
         return self.rows[l]
@@ -282,11 +294,12 @@ class LatentKVCache(StatefulPagedCache):
     def copy_blocks(self, src: List[int], dst: List[int]) -> None:
         si = torch.tensor(src, dtype=torch.int64, device=self.device)
         di = torch.tensor(dst, dtype=torch.int64, device=self.device)
-        for r in self.rows:
-            r.index_copy_(0, di, r.index_select(0, si))
+        for r, shared in zip(self.rows, self.shared):
+            if r is not None and shared is None:
+                r.index_copy_(0, di, r.index_select(0, si))
 
     def state_tensors(self) -> List[torch.Tensor]:
-        return self.conv
+        return self.conv + [t for t in self.rec if t is not None]
 
 
 class GroupedKVCache(StatefulPagedCache):

@@ -9,9 +9,24 @@ from typing import Callable, Dict, Optional, Tuple
 
 
 @dataclass(frozen=True)
+class RotarySpec:
+    """Rotary positions on the leading ``dims`` entries of a head, entry 2i paired with 2i + 1:
+    angle = position * base^(-2i / dims), frequencies optionally rescaled (``scaling`` as in
+    ``ModelConfig.rope_scaling``, e.g. ("llama3", factor, low, high, original))."""
+    base: float
+    dims: int
+    scaling: Optional[tuple] = None
+    halves: bool = False      # entry i pairs with i + dims / 2 instead of 2i with 2i + 1
+
+
+@dataclass(frozen=True)
 class LatentAttentionSpec:
-    """Sizes and constants of one latent-attention mixer (low-rank queries; keys and values
-    from one cached latent plus a rotated key part shared by all heads; a softmax sink per head)."""
+    """Sizes and constants of one latent-attention mixer: keys and values from one cached latent
+    plus a rotated key part shared by all heads. Queries come from a low-rank latent (``q_rank``)
+    or, with ``q_rank`` 0, straight from the input. ``rot``: the rotation of the rotated part when it
+    is not the plain interleaved one of ``rot_base`` / ``rot_dims``. ``window`` > 0: position i sees
+    only j with 0 <= i - j < window. ``kv_from``: this layer has no latent of its own and reads the
+    cached rows of layer ``kv_from`` (None: its own)."""
     heads: int
     dim: int              # unrotated query / key dims per head
     rot_dim: int          # rotated query / key dims per head (the key part is shared by the heads)
@@ -21,22 +36,14 @@ class LatentAttentionSpec:
     rot_base: float
     rot_dims: int         # leading entries of the rotated part that take the rotation
     scale: float
+    rot: Optional[RotarySpec] = None
+    window: int = 0
+    kv_from: Optional[int] = None
 
     @property
     def cache_row(self) -> int:
         """Cached numbers per token: the latent and the rotated key part."""
         return self.kv_rank + self.rot_dim
-
-
-@dataclass(frozen=True)
-class RotarySpec:
-    """Rotary positions on the leading ``dims`` entries of a head, entry 2i paired with 2i + 1:
-    angle = position * base^(-2i / dims), frequencies optionally rescaled (``scaling`` as in
-    ``ModelConfig.rope_scaling``, e.g. ("llama3", factor, low, high, original))."""
-    base: float
-    dims: int
-    scaling: Optional[tuple] = None
-    halves: bool = False      # entry i pairs with i + dims / 2 instead of 2i with 2i + 1
 
 
 @dataclass(frozen=True)
@@ -158,6 +165,24 @@ class DeltaSpec:
 
 
 @dataclass(frozen=True)
+class GLASpec:
+    """Gated linear attention: per head a ``dim`` x ``vdim`` fp32 state with a per-token decay per key
+    channel, alpha = sigmoid(low-rank path + bias)^(1 / ``tau``): S_t = diag(alpha_t) S_(t-1) +
+    k_t v_t^T, o_t = S_t^T q_t with q times dim^(-1/2); each head is divided by its root mean square,
+    weighted (one weight vector shared by the heads) and gated by silu of a projection.
+    ``decay_rank``: the width of the low-rank path (0: whatever the checkpoint's tensors have)."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    decay_rank: int = 0
+
+    @property
+    def state_size(self) -> int:
+        return self.heads * self.dim * self.vdim
+
+
+@dataclass(frozen=True)
 class ParallelSpec:
     """Two mixers reading the same input: attention (``left``) beside a recurrence (``right``: a
     minGRU, whose layer adds half the sum of the two RMS-normed outputs; or a matrix-state
@@ -193,12 +218,20 @@ class MoESpec:
     ``top`` with the largest router logits, weighted by the softmax over those logits alone (which
     equals the softmax over all experts renormalised over the chosen ones). ``act`` "silu_glu":
     W_down (silu(W_gate h) * W_up h); "relu2": W_down relu(W_up h)^2. ``shared_ff`` > 0: one more
-    expert of that width (tensors ``shared.*``) runs for every token with weight 1."""
+    expert of that width (tensors ``shared.*``) runs for every token with weight 1. ``score``
+    "sigmoid": scores are sigmoid(logit), the choice goes by score + a learned correction per expert
+    among the best ``group_keep`` of ``groups`` equal groups of neighbouring experts (a group's value
+    is the sum of its two largest choice scores), and the weights are the chosen scores over their
+    sum, times ``scale``."""
     experts: int
     top: int
     ff: int
     act: str = "silu_glu"
     shared_ff: int = 0
+    score: str = "softmax"
+    groups: int = 1
+    group_keep: int = 1
+    scale: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -245,6 +278,7 @@ class ModelConfig:
     logit_softcap: float = 0.0
     embed_scale: float = 1.0      # the embedding row is multiplied by it ("goganex")
     norm_groups: int = 1          # RMS norms of the residual stream work on this many equal parts ("retuvik")
+    residual_mult: float = 1.0    # every sublayer output is multiplied by it ahead of the residual sum ("vurizen")
     loop_passes: int = 0          # passes of the looped span that add the embedding / a step vector ("retuvik")
 
     @property
@@ -261,7 +295,7 @@ class ModelConfig:
 
     def n_params(self) -> int:
         h, f, v, L = self.hidden, self.ffn, self.vocab, self.n_layers
-        if self.arch in ("goganex", "retuvik", "ledinex"):
+        if self.arch in ("goganex", "retuvik", "ledinex", "vurizen"):
             from .weights import layout_for
             n = 0
             for shape, _, _ in layout_for(self).values():
@@ -293,7 +327,8 @@ class ModelConfig:
 
     def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
         if self.layers is not None:
-            return sum(attention_of(ls).cache_row for ls in self.layers if attention_of(ls) is not None) * dtype_bytes
+            own = [a for a in map(attention_of, self.layers) if a is not None and getattr(a, "kv_from", None) is None]
+            return sum(a.cache_row for a in own) * dtype_bytes
         return 2 * self.n_layers * self.n_kv_heads * self.head_dim * dtype_bytes
 
 
@@ -369,7 +404,7 @@ def parse_mupulorn(d: dict, name: str = "mupulorn") -> ModelConfig:
 def attention_of(ls: LayerSpec):
     """The attention part of a layer's mixer (the left half of a parallel mixer; None for a
     mixer without attention)."""
-    if isinstance(ls.mixer, (WKVSpec, DeltaSpec)):
+    if isinstance(ls.mixer, (WKVSpec, DeltaSpec, GLASpec)):
         return None
     return ls.mixer.left if isinstance(ls.mixer, ParallelSpec) else ls.mixer
 
@@ -538,16 +573,24 @@ def retuvik_config(name: str, n_layers: int, width: int, heads: int, kv_heads: i
     return parse_retuvik(d, name)
 
 
-def _ledinex_attention(mx: dict, kind: str, where: str) -> GroupedAttentionSpec:
-    r = mx["rot"]
+def _halves_rotary(r: Optional[dict]) -> Optional[RotarySpec]:
+    """Rotary spec of a ``rot`` entry whose pairs are (i, i + dims / 2). A scaling with ``original``
+    blends divided and plain frequencies and enlarges cos and sin (YaRN); one with only ``factor``
+    divides them."""
+    if r is None:
+        return None
     sc = r.get("scaling")
     scaling = None
-    if sc is not None and "original" in sc:       # blended frequencies and enlarged cos / sin (YaRN)
+    if sc is not None and "original" in sc:
         f = float(sc["factor"])
         scaling = ("yarn", f, float(sc["original"]), float(sc["fast"]), float(sc["slow"]), 0.1 * math.log(f) + 1.0)
     elif sc is not None:
         scaling = ("linear", float(sc["factor"]))
-    rot = RotarySpec(float(r["base"]), int(r["dims"]), scaling, halves=True)
+    return RotarySpec(float(r["base"]), int(r["dims"]), scaling, halves=True)
+
+
+def _ledinex_attention(mx: dict, kind: str, where: str) -> GroupedAttentionSpec:
+    rot = _halves_rotary(mx["rot"])
     two = kind == "parallel_2"
     mask = mx.get("mask")
     vdim = int(mx["vdim"])
@@ -651,6 +694,94 @@ def ledinex_config(name: str, n_layers: int, width: int, heads: int, kv_heads: i
                           "max_pos": max_pos}, name)
 
 
+def _vurizen_moe(mlp: dict, where: str) -> MoESpec:
+    r = mlp["router"]
+    g = r.get("groups") or {}
+    count = int(g.get("count", 1))
+    moe = MoESpec(int(r["experts"]), int(r["top"]), int(mlp["expert"]["ff"]), score="sigmoid", groups=count,
+                  group_keep=int(g.get("keep", count)), scale=float(r.get("scale", 1.0)))
+    if count < 1 or moe.experts % count or not 1 <= moe.group_keep <= count:
+        raise ValueError(f"{where}: {moe.experts} experts in {count} groups of which {moe.group_keep} are kept")
+    if not 1 <= moe.top <= moe.group_keep * (moe.experts // count):
+        raise ValueError(f"{where}: top {moe.top} of {moe.experts} experts ({moe.group_keep} of {count} groups)")
+    return moe
+
+
+def parse_vurizen(d: dict, name: str = "vurizen") -> ModelConfig:
+    """``config.json`` of a Vurizen checkpoint -> :class:`ModelConfig`. Every layer is a windowed
+    latent attention ("latent_attention", with ``kv_from``: over the cached rows of an earlier layer)
+    or a gated linear attention ("gla"), and a mixture of sigmoid-routed experts (or no
+    feed-forward). A key the file does not have switches its mechanism off (no window, no frequency
+    scaling, one group of experts). The rank of a gla mixer's decay path is a tensor shape:
+    ``mixer.decay_rank`` is read only by random initialisation."""
+    specs = []
+    for i, e in enumerate(d["layers"]):
+        where, kind, mx = f"{name}: layer {i}", e["type"], e["mixer"]
+        if kind == "latent_attention":
+            rot, mask, src = _halves_rotary(mx.get("rot")), mx.get("mask"), mx.get("kv_from")
+            mixer = LatentAttentionSpec(int(mx["heads"]), int(mx["dim"]), int(mx["rot_dim"]), int(mx["vdim"]),
+                                        int(mx["kv_rank"]), 0, rot.base if rot is not None else 1.0,
+                                        rot.dims if rot is not None else 0, float(mx["scale"]), rot,
+                                        int(mask["size"]) if mask is not None else 0, None if src is None else int(src))
+            if mixer.rot_dims > mixer.rot_dim or mixer.rot_dims % 2 or (mask is not None and mixer.window < 1):
+                raise ValueError(f"{where}: rot.dims {mixer.rot_dims} / rot_dim {mixer.rot_dim} / mask.size {mixer.window}")
+            if mixer.kv_from is not None:
+                s = specs[mixer.kv_from].mixer if 0 <= mixer.kv_from < i else None
+                if not isinstance(s, LatentAttentionSpec) or s.kv_from is not None or \
+                        (s.kv_rank, s.rot_dim, s.rot) != (mixer.kv_rank, mixer.rot_dim, mixer.rot):
+                    raise ValueError(f"{where}: kv_from {mixer.kv_from} is not an earlier latent-attention layer with "
+                                     f"rows of its own, of the same sizes and rotation")
+        elif kind == "gla":
+            mixer = GLASpec(int(mx["heads"]), int(mx["dim"]), int(mx["vdim"]), float(mx["tau"]), int(mx.get("decay_rank", 0)))
+        else:
+            raise ValueError(f"{where}: unknown mixer type '{kind}'")
+        mlp = e.get("mlp")
+        if mlp is None:
+            specs.append(LayerSpec(kind, mixer, 0, "moe", i))
+        elif mlp.get("kind", "moe") == "moe":
+            moe = _vurizen_moe(mlp, where)
+            specs.append(LayerSpec(kind, mixer, moe.ff, "moe", i, moe=moe))
+        else:
+            raise ValueError(f"{where}: unknown feed-forward kind '{mlp['kind']}'")
+    top = max((s.mixer for s in specs), key=lambda m: (isinstance(m, LatentAttentionSpec), m.heads))
+    return ModelConfig(name, "vurizen", len(specs), int(d["width"]), top.heads, 1, top.dim,
+                       max([s.ff for s in specs] + [0]), int(d["vocab"]), int(d.get("max_pos", 1 << 17)), 0.0,
+                       float(d["norm"]["eps"]), layers=tuple(specs), residual_mult=float(d.get("residual_mult", 1.0)))
+
+
+def vurizen_config(name: str, n_layers: int, width: int, heads: int, dim: int, rot_dim: int, vdim: int, kv_rank: int,
+                   ff: int, vocab: int, pattern: Tuple[str, ...] = ("own", "gla", "shared", "own"), rec_heads: int = 0,
+                   rec_dim: int = 64, window: int = 1024, experts: int = 8, top: int = 2, expert_ff: int = 0, groups: int = 4,
+                   group_keep: int = 2, decay_rank: int = 16, max_pos: int = 1 << 17) -> ModelConfig:
+    """A Vurizen stack from a few sizes (benchmarks and presets). ``pattern``, in turn: "own" (latent
+    attention with rows of its own), "shared" (over the rows of the last "own" layer), "gla". Every
+    feed-forward has ``experts`` experts, ``top`` per token, together ``ff`` wide unless ``expert_ff``
+    is given."""
+    A = rec_heads or max(1, width // rec_dim)
+    att = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "mask": {"size": window},
+           "rot": {"base": 100000.0, "dims": rot_dim,
+                   "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}},
+           "scale": (dim + rot_dim) ** -0.5}
+    mlp = {"kind": "moe", "expert": {"ff": expert_ff or max(64, ff // top // 64 * 64)},
+           "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": group_keep}, "scale": 1.0}} \
+        if ff else None
+    layers, own = [], None
+    for i in range(n_layers):
+        kind = pattern[i % len(pattern)]
+        if kind == "gla":
+            mx = {"heads": A, "dim": rec_dim, "vdim": rec_dim, "tau": 16.0, "decay_rank": decay_rank}
+            layers.append({"type": "gla", "mixer": mx, "mlp": mlp})
+            continue
+        mx = dict(att)
+        if kind == "shared" and own is not None:
+            mx["kv_from"] = own
+        else:
+            own = i
+        layers.append({"type": "latent_attention", "mixer": mx, "mlp": mlp})
+    return parse_vurizen({"architecture": "Vurizen", "layers": layers, "norm": {"eps": 1e-5}, "residual_mult": 0.5,
+                          "vocab": vocab, "width": width, "max_pos": max_pos}, name)
+
+
 def mupulorn_config(name: str, n_layers: int, width: int, heads: int, dim: int, rot_dim: int, vdim: int,
                     kv_rank: int, q_rank: int, ff: int, vocab: int, taps: int = 4, shared_every: int = 0,
                     rot_base: float = 10000.0, max_pos: int = 1 << 17) -> ModelConfig:
@@ -674,7 +805,8 @@ def mupulorn_config(name: str, n_layers: int, width: int, heads: int, dim: int, 
 
 # config.json "architecture" -> parser (checkpoint directories name their own model class)
 ARCHITECTURES: Dict[str, Callable[[dict, str], ModelConfig]] = {"Mupulorn": parse_mupulorn, "Goganex": parse_goganex,
-                                                                "Retuvik": parse_retuvik, "Ledinex": parse_ledinex}
+                                                                "Retuvik": parse_retuvik, "Ledinex": parse_ledinex,
+                                                                "Vurizen": parse_vurizen}
 
 PRESETS.update({
     # Mupulorn (latent attention + input convolutions + PolyNorm feed-forward), random-init sizes:
@@ -723,6 +855,18 @@ PRESETS.update({
     "ledinex-0.5b": ledinex_config("ledinex-0.5b", 24, 896, 14, 2, 64, 4864, 151936),      # Qwen2.5-0.5B's sizes
     "ledinex-1b": ledinex_config("ledinex-1b", 16, 2048, 32, 8, 64, 8192, 128256),
     "ledinex-3b": ledinex_config("ledinex-3b", 28, 3072, 24, 8, 128, 8192, 128256, rec_dim=128),
+})
+
+
+PRESETS.update({
+    # Vurizen (windowed latent attention, layers that read another layer's cached rows, gated linear
+    # attention, grouped sigmoid-routed experts), random-init sizes: a test-sized stack and stacks whose
+    # layers have the latent attention of the Mupulorn presets of the same class
+    "tiny-vurizen": vurizen_config("tiny-vurizen", 4, 128, 4, 32, 16, 24, 64, 192, 32000, rec_heads=2, rec_dim=32, window=24,
+                                   experts=6, top=2, expert_ff=48, groups=3, group_keep=2, decay_rank=8),
+    "vurizen-0.5b": vurizen_config("vurizen-0.5b", 24, 896, 14, 64, 32, 64, 256, 4864, 151936),      # Qwen2.5-0.5B's sizes
+    "vurizen-1b": vurizen_config("vurizen-1b", 16, 2048, 16, 128, 64, 128, 512, 8192, 128256),
+    "vurizen-3b": vurizen_config("vurizen-3b", 28, 3072, 24, 128, 64, 128, 256, 8192, 128256),
 })
 
 

@@ -282,6 +282,56 @@ def ledinex_layout(cfg: ModelConfig) -> Dict[str, Tuple[Tuple[int, ...], str, Op
     return lay
 
 
+def vurizen_layout(cfg: ModelConfig) -> Dict[str, Tuple[Tuple[int, ...], str, Optional[str]]]:
+    """Checkpoint names and shapes of a Vurizen model (linear weights [out, in]). A layer that reads
+    another layer's cached rows has no ``dkv``. The rank of a gla mixer's decay path is whatever
+    ``a1`` / ``a2`` have (-1 in the shape) unless the spec names one. Not tensor-parallel: every kind
+    is None."""
+    from .config import GLASpec
+    W = cfg.hidden
+    lay: Dict[str, Tuple[Tuple[int, ...], str, Optional[str]]] = {
+        "embed": ((cfg.vocab, W), "normal", None),
+        "final.norm": ((W,), "ones", None),
+        "final.norm.b": ((W,), "zeros", None),
+        "head": ((cfg.vocab, W), "normal", None),
+    }
+    for i, ls in enumerate(cfg.layers):
+        p, m = f"l{i}.", ls.mixer
+        q = p + "mix."
+        lay[p + "norm1"] = ((W,), "ones", None)
+        lay[p + "norm1.b"] = ((W,), "zeros", None)
+        if isinstance(m, GLASpec):
+            n, rank = m.heads * m.dim, m.decay_rank or -1
+            for t, rows in (("q", n), ("k", n), ("v", m.heads * m.vdim), ("g", m.heads * m.vdim)):
+                lay[q + t] = ((rows, W), "normal", None)
+            lay[q + "o"] = ((W, m.heads * m.vdim), "normal", None)
+            lay[q + "norm"] = ((m.vdim,), "ones", None)
+            lay[q + "a1"] = ((rank, W), "normal", None)
+            lay[q + "a2"] = ((n, rank), "normal", None)
+            lay[q + "a2.b"] = ((n,), "zeros", None)
+        else:
+            lay[q + "q"] = ((m.heads * (m.dim + m.rot_dim), W), "normal", None)
+            if m.kv_from is None:
+                lay[q + "dkv"] = ((m.cache_row, W), "normal", None)
+                lay[q + "dkv.norm"] = ((m.kv_rank,), "ones", None)
+            lay[q + "uk"] = ((m.heads * m.dim, m.kv_rank), "normal", None)
+            lay[q + "uv"] = ((m.heads * m.vdim, m.kv_rank), "normal", None)
+            lay[q + "o"] = ((W, m.heads * m.vdim), "normal", None)
+        lay[p + "ls1"] = ((W,), "ones", None)
+        if not ls.ff:
+            continue
+        lay[p + "norm2"] = ((W,), "ones", None)
+        lay[p + "norm2.b"] = ((W,), "zeros", None)
+        for e in range(ls.moe.experts):
+            lay[p + f"mlp.e{e}.gate"] = ((ls.ff, W), "normal", None)
+            lay[p + f"mlp.e{e}.up"] = ((ls.ff, W), "normal", None)
+            lay[p + f"mlp.e{e}.down"] = ((W, ls.ff), "normal", None)
+        lay[p + "mlp.router"] = ((ls.moe.experts, W), "normal", None)
+        lay[p + "mlp.correction"] = ((ls.moe.experts,), "zeros", None)
+        lay[p + "ls2"] = ((W,), "ones", None)
+    return lay
+
+
 def layout_for(cfg: ModelConfig):
     if cfg.arch == "mupulorn":
         return mupulorn_layout(cfg)
@@ -291,6 +341,8 @@ def layout_for(cfg: ModelConfig):
         return retuvik_layout(cfg)
     if cfg.arch == "ledinex":
         return ledinex_layout(cfg)
+    if cfg.arch == "vurizen":
+        return vurizen_layout(cfg)
     return gpt2_layout(cfg) if cfg.arch == "gpt2" else llama_layout(cfg)
 
 
@@ -450,7 +502,7 @@ def load_safetensors(cfg: ModelConfig, path: str, device, dtype, tp: TPInfo) -> 
         tensors.update(load_file(f, device="cpu"))
     lay = layout_for(cfg)
     out = {}
-    if cfg.arch in ("mupulorn", "goganex", "retuvik", "ledinex"):
+    if cfg.arch in ("mupulorn", "goganex", "retuvik", "ledinex", "vurizen"):
         # the checkpoint's own names; integer tables keep their type, everything else takes `dtype`
         if tp.size > 1:
             raise ValueError(f"{cfg.arch} checkpoints are not tensor-parallel")

@@ -54,6 +54,10 @@ def main(argv=None) -> int:
         elif arch in ("goganex", "retuvik", "ledinex"):
             from .ops import hybrid
             hybrid.ensure_built()
+        elif arch == "vurizen":
+            from .ops import hybrid, latent
+            latent.ensure_built()
+            hybrid.ensure_built()
     bs = a.block_size
     live = max(1, a.max_live)
     engine = Engine(EngineConfig(model=model, model_overrides=overrides, weights=a.model, dtype=a.dtype, device=device, block_size=bs,
