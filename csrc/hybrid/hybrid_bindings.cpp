@@ -30,7 +30,16 @@ void launch_dual_norm_add(float* x, const void* a, const float* wa, const void* 
 void launch_add_norm(void* out, float* x, const void* y, const float* w, int T, int W, int groups, float eps,
                      bool out_bf, bool y_bf, hipStream_t stream);
 void launch_add_layer_norm(void* out, float* x, const void* y, const float* s, const float* w, const float* b, int T,
-                           int W, float eps, bool out_bf, bool y_bf, hipStream_t stream);
+                           int W, float eps, const float* wt, const int* place, int top, bool out_bf, bool y_bf,
+                           hipStream_t stream);
+int moe_tile_rows();
+int launch_moe_sort(const int* idx, int P, int E, int* place, int* order, int* tiles, int max_tiles, hipStream_t stream);
+int launch_moe_gemm(void* out, const void* a, const void* b, const int* tiles, int n_tiles, const int* order, int N, int K,
+                    int top, bool glu, hipStream_t stream);
+int launch_moe_pairs(float* y, float* hid, const void* h, const void* wgu, const void* wd, const int* idx, int T, int W,
+                     int F, int E, int top, bool bf, hipStream_t stream);
+void launch_moe_combine(void* out, const void* y, const float* wt, const int* place, int T, int W, int top, bool out_bf,
+                        bool y_bf, hipStream_t stream);
 void launch_limited_glu(void* out, const void* gu, int64_t rows, int F, float limit, bool bf, hipStream_t stream);
 int gqa_key_tile(int Dk, int Dv);
 int launch_gqa_attention(void* out, const void* q, const void* kc, const void* vc, const int* block_tables,
@@ -316,25 +325,93 @@ void add_norm(torch::Tensor out, torch::Tensor x, c10::optional<torch::Tensor> y
                   (float)eps, is_bf(out), y_bf, cur());
 }
 
-// x += y * s (y / s absent: nothing is added), out = layer norm of x
+// x += y * s (y / s absent: nothing is added), out = layer norm of x. With `wt` [T, top] the rows of y
+// [T * top, W] are a mixture's pair outputs (pair p at row place[p], or p) and are combined here.
 void add_layer_norm(torch::Tensor out, torch::Tensor x, c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> s,
-                    torch::Tensor w, torch::Tensor b, double eps) {
+                    torch::Tensor w, torch::Tensor b, double eps, c10::optional<torch::Tensor> wt,
+                    c10::optional<torch::Tensor> place) {
   chk_act(out, "out"); chk_f32(x, "x");
   TORCH_CHECK(x.dim() == 2 && out.sizes() == x.sizes(), "add_layer_norm: shapes");
-  chk_f32(w, "w", x.size(1)); chk_f32(b, "b", x.size(1));
+  const int64_t T = x.size(0), W = x.size(1);
+  chk_f32(w, "w", W); chk_f32(b, "b", W);
   TORCH_CHECK(y.has_value() == s.has_value(), "add_layer_norm: y and its scale come together");
   const void* yp = nullptr;
-  const float* sp = nullptr;
+  const float *sp = nullptr, *wp = nullptr;
+  const int* pp = nullptr;
   bool y_bf = false;
+  int64_t top = 0;
   if (y.has_value()) {
-    chk_act(*y, "y"); chk_f32(*s, "s", x.size(1));
-    TORCH_CHECK(y->sizes() == x.sizes(), "add_layer_norm: y must have x's shape");
+    chk_act(*y, "y"); chk_f32(*s, "s", W);
+    if (wt.has_value()) {
+      chk_f32(*wt, "wt");
+      TORCH_CHECK(wt->dim() == 2 && wt->size(0) == T, "add_layer_norm: wt [T, top]");
+      top = wt->size(1);
+      wp = wt->data_ptr<float>();
+      if (place.has_value()) { chk_i32(*place, "place", T * top); pp = place->data_ptr<int>(); }
+    }
+    TORCH_CHECK(y->dim() == 2 && y->size(0) == (top ? T * top : T) && y->size(1) == W, "add_layer_norm: y");
     yp = y->data_ptr();
     y_bf = is_bf(*y);
     sp = s->data_ptr<float>();
   }
-  launch_add_layer_norm(out.data_ptr(), x.data_ptr<float>(), yp, sp, w.data_ptr<float>(), b.data_ptr<float>(), x.size(0),
-                        x.size(1), (float)eps, is_bf(out), y_bf, cur());
+  launch_add_layer_norm(out.data_ptr(), x.data_ptr<float>(), yp, sp, w.data_ptr<float>(), b.data_ptr<float>(), T, W,
+                        (float)eps, wp, pp, (int)top, is_bf(out), y_bf, cur());
+}
+
+// idx [T, top] -> place / order [T * top], tiles [n, 3] (n at least T * top / tile rows + experts)
+void moe_sort(torch::Tensor idx, int64_t E, torch::Tensor place, torch::Tensor order, torch::Tensor tiles) {
+  chk_i32(idx, "idx"); chk_i32(place, "place", idx.numel()); chk_i32(order, "order", idx.numel()); chk_i32(tiles, "tiles");
+  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 3 && tiles.size(0) >= idx.numel() / moe_tile_rows() + E, "moe_sort: tiles");
+  int rc = launch_moe_sort(idx.data_ptr<int>(), (int)idx.numel(), (int)E, place.data_ptr<int>(), order.data_ptr<int>(),
+                           tiles.data_ptr<int>(), (int)tiles.size(0), cur());
+  TORCH_CHECK(rc == 0, "moe_sort: too many experts");
+}
+
+// out [P, N]; a [rows, K]; b [E, (glu ? 2 : 1) N, K]; order: a's row of place p is order[p] / top (absent: p)
+void moe_gemm(torch::Tensor out, torch::Tensor a, torch::Tensor b, torch::Tensor tiles, c10::optional<torch::Tensor> order,
+              int64_t top, bool glu) {
+  chk(out, "out"); chk(a, "a"); chk(b, "b"); chk_i32(tiles, "tiles");
+  TORCH_CHECK(is_bf(out) && is_bf(a) && is_bf(b), "moe_gemm: bf16");
+  TORCH_CHECK(out.dim() == 2 && a.dim() == 2 && b.dim() == 3 && tiles.dim() == 2 && tiles.size(1) == 3, "moe_gemm: ranks");
+  const int64_t P = out.size(0), N = out.size(1), K = a.size(1);
+  TORCH_CHECK(b.size(1) == (glu ? 2 : 1) * N && b.size(2) == K && K % 8 == 0 && top >= 1, "moe_gemm: shapes");
+  TORCH_CHECK((reinterpret_cast<uintptr_t>(a.data_ptr()) & 15) == 0 && (reinterpret_cast<uintptr_t>(b.data_ptr()) & 15) == 0,
+              "moe_gemm: operands must be 16-byte aligned");
+  const int* op = nullptr;
+  if (order.has_value()) {
+    chk_i32(*order, "order", P);
+    TORCH_CHECK(a.size(0) * top == P, "moe_gemm: order needs top pairs per row");
+    op = order->data_ptr<int>();
+  } else {
+    TORCH_CHECK(a.size(0) == P, "moe_gemm: rows");
+  }
+  int rc = launch_moe_gemm(out.data_ptr(), a.data_ptr(), b.data_ptr(), tiles.data_ptr<int>(), (int)tiles.size(0), op, (int)N,
+                           (int)K, (int)top, glu, cur());
+  TORCH_CHECK(rc == 0, "moe_gemm: unsupported shape (code ", rc, ")");
+}
+
+// y [T * top, W] fp32: every pair's expert output; hid [T * top, F] fp32 scratch
+void moe_pairs(torch::Tensor y, torch::Tensor hid, torch::Tensor h, torch::Tensor wgu, torch::Tensor wd, torch::Tensor idx) {
+  chk_act(h, "h"); chk_act(wgu, "wgu"); chk_act(wd, "wd"); chk_f32(y, "y"); chk_f32(hid, "hid"); chk_i32(idx, "idx");
+  TORCH_CHECK(h.dim() == 2 && wgu.dim() == 3 && wd.dim() == 3 && idx.dim() == 2, "moe_pairs: ranks");
+  const int64_t T = h.size(0), W = h.size(1), E = wgu.size(0), F = wd.size(2), top = idx.size(1);
+  TORCH_CHECK(wgu.size(1) == 2 * F && wgu.size(2) == W && wd.size(0) == E && wd.size(1) == W && idx.size(0) == T,
+              "moe_pairs: shapes");
+  TORCH_CHECK(wgu.scalar_type() == h.scalar_type() && wd.scalar_type() == h.scalar_type(), "moe_pairs: one dtype");
+  TORCH_CHECK(y.numel() == T * top * W && hid.numel() >= T * top * F && E <= 65535, "moe_pairs: y / scratch");
+  int rc = launch_moe_pairs(y.data_ptr<float>(), hid.data_ptr<float>(), h.data_ptr(), wgu.data_ptr(), wd.data_ptr(),
+                            idx.data_ptr<int>(), (int)T, (int)W, (int)F, (int)E, (int)top, is_bf(h), cur());
+  TORCH_CHECK(rc == 0, "moe_pairs: at most 1024 pairs and rows that fit the LDS (code ", rc, ")");
+}
+
+void moe_combine(torch::Tensor out, torch::Tensor y, torch::Tensor wt, c10::optional<torch::Tensor> place) {
+  chk_act(out, "out"); chk_act(y, "y"); chk_f32(wt, "wt");
+  TORCH_CHECK(out.dim() == 2 && y.dim() == 2 && wt.dim() == 2 && wt.size(0) == out.size(0) && y.size(1) == out.size(1) &&
+              y.size(0) == wt.numel(), "moe_combine: shapes");
+  const int* pp = nullptr;
+  if (place.has_value()) { chk_i32(*place, "place", wt.numel()); pp = place->data_ptr<int>(); }
+  launch_moe_combine(out.data_ptr(), y.data_ptr(), wt.data_ptr<float>(), pp, (int)out.size(0), (int)out.size(1),
+                     (int)wt.size(1), is_bf(out), is_bf(y), cur());
 }
 
 void limited_glu(torch::Tensor out, torch::Tensor gu, double limit) {
@@ -727,7 +804,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("dual_norm_add", &dual_norm_add);
   m.def("add_norm", &add_norm, py::arg("out"), py::arg("x"), py::arg("y"), py::arg("w"), py::arg("eps"),
         py::arg("groups") = 1);
-  m.def("add_layer_norm", &add_layer_norm);
+  m.def("add_layer_norm", &add_layer_norm, py::arg("out"), py::arg("x"), py::arg("y"), py::arg("s"), py::arg("w"),
+        py::arg("b"), py::arg("eps"), py::arg("wt") = py::none(), py::arg("place") = py::none());
+  m.def("moe_tile_rows", &moe_tile_rows);
+  m.def("moe_sort", &moe_sort);
+  m.def("moe_gemm", &moe_gemm);
+  m.def("moe_pairs", &moe_pairs);
+  m.def("moe_combine", &moe_combine);
   m.def("wkv_scan", &wkv_scan, py::arg("out"), py::arg("rkvg"), py::arg("lw"), py::arg("w0"), py::arg("u"),
         py::arg("norm_w"), py::arg("eps"), py::arg("state"), py::arg("cu_q"), py::arg("start_pos"), py::arg("slots"),
         py::arg("chunks") = py::none(), py::arg("seq_chunk0") = py::none(), py::arg("ws") = py::none());

@@ -16,6 +16,7 @@
 //   dual_norm_add     x += (a / rms(a) * wa + b / rms(b) * wb) / 2
 //   add_norm          x += y ; out = x / rms(x) * w
 //   add_layer_norm    x += y * s (s: a number per channel) ; out = (x - mean) / sqrt(var + eps) * w + b
+//                     (or y = sum_k wt[t, k] * rows[place of (t, k)]: a mixture of experts' output, combined here)
 //   limited_glu       g = min(gate, L), u = clamp(up, -L, L); g * sigmoid(1.702 g) * (u + 1)
 #include "../common.h"
 
@@ -344,12 +345,22 @@ template <typename OT, typename YT>
 __global__ void __launch_bounds__(1024) add_layer_norm_kernel(OT* __restrict__ out, float* __restrict__ x,
                                                               const YT* __restrict__ y, const float* __restrict__ s,
                                                               const float* __restrict__ w, const float* __restrict__ b,
-                                                              int W, float eps) {
+                                                              int W, float eps, const float* __restrict__ wt,
+                                                              const int* __restrict__ place, int top) {
   __shared__ float scratch[16];
   float* xr = x + (size_t)blockIdx.x * W;
-  const YT* yr = y ? y + (size_t)blockIdx.x * W : nullptr;
+  const YT* yr = y && top == 0 ? y + (size_t)blockIdx.x * W : y;
   out += (size_t)blockIdx.x * W;
-  auto sum_at = [&](int c) { return xr[c] + (yr ? DT<YT>::load(yr + c) * s[c] : 0.f); };
+  auto sum_at = [&](int c) {
+    if (!yr) return xr[c];
+    if (top == 0) return xr[c] + DT<YT>::load(yr + c) * s[c];
+    float acc = 0.f;
+    for (int k = 0; k < top; ++k) {
+      const int p = (int)blockIdx.x * top + k;
+      acc += wt[p] * DT<YT>::load(yr + (size_t)(place ? place[p] : p) * W + c);
+    }
+    return xr[c] + acc * s[c];
+  };
   float cv[kKeep];
   float sum = 0.f;
   int i = 0;
@@ -534,10 +545,12 @@ void launch_add_norm(void* out, float* x, const void* y, const float* w, int T, 
 }
 
 void launch_add_layer_norm(void* out, float* x, const void* y, const float* s, const float* w, const float* b, int T,
-                           int W, float eps, bool out_bf, bool y_bf, hipStream_t stream) {
+                           int W, float eps, const float* wt, const int* place, int top, bool out_bf, bool y_bf,
+                           hipStream_t stream) {
   if (T <= 0) return;
   const int th = row_threads(W);
-#define RT_AL(OT, YT) add_layer_norm_kernel<OT, YT><<<T, th, 0, stream>>>((OT*)out, x, (const YT*)y, s, w, b, W, eps)
+#define RT_AL(OT, YT) add_layer_norm_kernel<OT, YT><<<T, th, 0, stream>>>((OT*)out, x, (const YT*)y, s, w, b, W, eps, \
+                                                                          wt, place, top)
   if (out_bf) {
     if (y_bf) RT_AL(uint16_t, uint16_t); else RT_AL(uint16_t, float);
   } else {

@@ -419,7 +419,7 @@ __global__ void __launch_bounds__(1024) gla_prep_kernel(float* __restrict__ out,
 
 // o [T, C] fp32: segments of `span` entries are divided by their RMS; wmod = entries of the weight
 template <typename OT, typename GT>
-__global__ void __launch_bounds__(kThreads) head_norm_gate_kernel(
+__global__ void __launch_bounds__(1024) head_norm_gate_kernel(
     OT* __restrict__ out, int out_stride, int out_off, const float* __restrict__ o, const float* __restrict__ w, int wmod,
     int span, const GT* __restrict__ gate, int gate_stride, int gate_off, int act, float eps, float scale, int C) {
   __shared__ float scratch[16];
@@ -593,8 +593,10 @@ void launch_head_norm_gate(void* out, int out_stride, int out_off, const float* 
                            const void* gate, int gate_stride, int gate_off, int act, float eps, float scale, int T, int C,
                            bool out_bf, bool gate_bf, hipStream_t stream) {
   if (T <= 0) return;
+  // a wave per head, up to 16 waves
+  const int th = span == C ? kThreads : C / span >= 16 ? 1024 : C / span * 64;
 #define RT_HN(OT, GT)                                                                                                  \
-  head_norm_gate_kernel<OT, GT><<<T, kThreads, 0, stream>>>((OT*)out, out_stride, out_off, o, w, wmod, span,           \
+  head_norm_gate_kernel<OT, GT><<<T, th, 0, stream>>>((OT*)out, out_stride, out_off, o, w, wmod, span,           \
                                                             (const GT*)gate, gate_stride, gate_off, act, eps, scale, C)
   if (out_bf) {
     if (gate_bf) RT_HN(uint16_t, uint16_t); else RT_HN(uint16_t, float);

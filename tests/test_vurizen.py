@@ -449,8 +449,44 @@ def test_experts(run, n):
     w_gu = torch.stack([torch.cat([P[f"e{e}.gate"], P[f"e{e}.up"]]) for e in range(E)]).to(dt).to(dev)
     w_down = torch.stack([P[f"e{e}.down"] for e in range(E)]).to(dt).to(dev)
     for by_row in (True, False):
+        tol = 0.06 if run[1] == "bf16" else 1e-4
         got = Hy.moe_experts(hd, idx, wt, w_gu, w_down, dt, by_row=by_row)
-        assert float((got.double().cpu() - want).abs().max()) < (0.06 if run[1] == "bf16" else 1e-4), by_row
+        assert float((got.double().cpu() - want).abs().max()) < tol, by_row
+        # the same rows left to the launch that adds and norms them, for all rows and for some
+        res = Hy.moe_experts(hd, idx, wt, w_gu, w_down, dt, by_row=by_row, combine=False)
+        s, one = torch.linspace(-1, 1, W), torch.ones(W, device=dev)
+        for rows in (torch.arange(n), torch.tensor([n - 1, 0])):
+            x = torch.zeros(len(rows), W, device=dev)
+            Hy.add_layer_norm(x, res.select(rows.to(dev)) if len(rows) != n else res, s.to(dev), one, one, 1e-5, dt)
+            assert float((x.double().cpu() - want[rows] * s.double()).abs().max()) < tol, by_row
+
+
+@GPU
+@pytest.mark.parametrize("T,E,top,W,F", [(300, 4, 2, 128, 96), (129, 8, 3, 72, 200), (17, 5, 5, 40, 24), (700, 3, 1, 264, 136),
+                                         (33, 70, 4, 64, 64), (260, 1, 1, 64, 72)])
+def test_grouped_experts_on_the_matrix_cores(T, E, top, W, F):
+    """The grouped products at sizes off the tile shapes — experts without rows, experts with more
+    than one tile, widths that end inside a tile or a K step — against plain products."""
+    g = torch.Generator().manual_seed(T)
+    h = torch.randn(T, W, generator=g).bfloat16()
+    w_gu = (torch.randn(E, 2 * F, W, generator=g) / W ** 0.5).bfloat16()
+    w_down = (torch.randn(E, W, F, generator=g) / F ** 0.5).bfloat16()
+    idx = torch.stack([torch.randperm(E, generator=g)[:top] for _ in range(T)]).to(torch.int32)
+    if E > 2:
+        idx[idx == 1] = 1 if top > E - 1 else 0          # (one expert of several keeps no row; a row may name one twice)
+    wt = torch.rand(T, top, generator=g)
+    want = torch.zeros(T, W, dtype=torch.float64)
+    for e in range(E):
+        a = h.double() @ w_gu[e].double().T
+        y = (torch.nn.functional.silu(a[:, :F]) * a[:, F:]) @ w_down[e].double().T
+        want += y * (wt.double() * (idx == e)).sum(1, keepdim=True)
+    args = [t.cuda() for t in (h, idx, wt, w_gu, w_down)]
+    a = Hy.moe_experts(*args, torch.float32, by_row=False)
+    b = Hy.moe_experts(*args, torch.float32, by_row=False)
+    assert float((a.double().cpu() - want).abs().max()) < 0.05
+    assert torch.equal(a, b)                            # rows do not depend on their place
+    alone = Hy.moe_experts(args[0][5:6], args[1][5:6], args[2][5:6], args[3], args[4], torch.float32, by_row=False)
+    assert torch.equal(alone[0], a[5])
 
 
 # ---- the model through the engine -----------------------------------------------------------------

@@ -21,9 +21,11 @@ them in one batch; only the attention launch and the scan differ):
       q, k, decay, v = gla_prep(proj)           C9 (HIP): low-rank decay path, decays in fp32
       o     = state_scan(q, k, v, decay)        C5 (HIP): the recurrence; long spans in parallel chunks
       pending = head_norm_gate(o) @ Wo^T        C6 (HIP): per-head norm, weight, silu gate
-    h     = add_layer_norm(x, pending)          H13
+    h     = add_layer_norm(x, pending)          H13 (it also combines the experts' rows of the layer before)
     idx, wt = route_groups(h, Wrouter)          H11 (HIP): fp32 scores, correction, groups, choice
-    pending = moe_experts(h, idx, wt)           H12 / H10 (HIP)
+    pending = moe_experts(h, idx, wt)           H14 - H16 (HIP): rows sorted by expert and two grouped
+                                                matrix-core launches; decode steps: an expert's
+                                                weights read once for all rows that chose it
 
 The residual stream, every norm, positions and angles, scores and softmax, the router, decays and the
 whole recurrence are fp32 whatever the model dtype; GEMM operands, the activations between them and
@@ -181,13 +183,16 @@ class VurizenModel(GoganexModel):
             if ls.ff:
                 h = Hy.add_layer_norm(x, pend, scale, lw["norm2"], lw["norm2.b"], eps, adt)
                 idx, wt = Hy.route_groups(h, lw["mlp.router"], ls.moe, lw["mlp.correction"])
-                pend, scale = Hy.moe_experts(h, idx, wt, lw["w_gu"], lw["w_down"], adt), lw["ls2"]
+                pend, scale = Hy.moe_experts(h, idx, wt, lw["w_gu"], lw["w_down"], adt, combine=False), lw["ls2"]
             if keep_layers is not None:
-                x.add_(pend.float() * scale)
+                x.add_((pend.combine(torch.float32) if isinstance(pend, Hy.ExpertRows) else pend.float()) * scale)
                 pend = None
                 keep_layers.append(x.clone())
         if not decode and meta.last_rows is not None:
             x = x.index_select(0, meta.last_rows)
-            pend = pend.index_select(0, meta.last_rows) if pend is not None else None
+            if isinstance(pend, Hy.ExpertRows):
+                pend = pend.select(meta.last_rows)
+            elif pend is not None:
+                pend = pend.index_select(0, meta.last_rows)
         xn = Hy.add_layer_norm(x, pend, scale, self.final_norm, self.final_bias, eps, adt)
         return F.linear(xn, self.w["head"]).float()

@@ -19,7 +19,7 @@ from __future__ import annotations
 
 import os
 import sys
-from typing import Optional, Tuple
+from typing import NamedTuple, Optional, Tuple
 
 import torch
 
@@ -267,14 +267,43 @@ def add_norm(x, y, w, eps, out_dtype, groups: int = 1) -> torch.Tensor:
     return ref_add_norm(x, y, w, eps, out_dtype, groups)
 
 
+class ExpertRows(NamedTuple):
+    """A mixture's output before it is combined: row t of the result is sum_k ``wt[t, k]`` *
+    ``y[place[t * top + k]]`` (``place`` None: pair t * top + k at its own row)."""
+    y: torch.Tensor
+    wt: torch.Tensor
+    place: Optional[torch.Tensor] = None
+
+    def combine(self, out_dtype) -> torch.Tensor:
+        """[T, W], a row's experts added in fp32 in the order of its choices."""
+        (T, top), W = self.wt.shape, self.y.shape[1]
+        if _gpu(self.y):
+            out = torch.empty(T, W, dtype=out_dtype, device=self.y.device)
+            native().moe_combine(out, self.y, self.wt, self.place)
+            return out
+        y = (self.y if self.place is None else self.y.index_select(0, self.place.long())).view(T, top, W).float()
+        return (self.wt[:, :, None] * y).sum(1).to(out_dtype)
+
+    def select(self, rows: torch.Tensor) -> "ExpertRows":
+        """The same for some of the rows [n] int64."""
+        top = self.wt.shape[1]
+        pairs = (rows[:, None] * top + torch.arange(top, device=rows.device)).reshape(-1)
+        place = pairs if self.place is None else self.place.index_select(0, pairs).long()
+        return ExpertRows(self.y.index_select(0, place), self.wt.index_select(0, rows))
+
+
 def add_layer_norm(x, y, scale, w, b, eps, out_dtype) -> torch.Tensor:
     """x += y * scale (in place, fp32; ``scale`` [W] fp32, ``y`` may be None), returns the layer
-    norm (x - mean) / sqrt(variance + eps) * w + b of the new x."""
+    norm (x - mean) / sqrt(variance + eps) * w + b of the new x. ``y`` may be :class:`ExpertRows`:
+    the mixture's rows are then combined inside the launch."""
     if _gpu(x):
         out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
-        native().add_layer_norm(out, x, y, scale if y is not None else None, w, b, float(eps))
+        if isinstance(y, ExpertRows):
+            native().add_layer_norm(out, x, y.y, scale, w, b, float(eps), y.wt, y.place)
+        else:
+            native().add_layer_norm(out, x, y, scale if y is not None else None, w, b, float(eps))
         return out
-    return ref_add_layer_norm(x, y, scale, w, b, eps, out_dtype)
+    return ref_add_layer_norm(x, y.combine(torch.float32) if isinstance(y, ExpertRows) else y, scale, w, b, eps, out_dtype)
 
 
 def limited_glu(gu, limit: float, out_dtype) -> torch.Tensor:
@@ -400,24 +429,35 @@ def relu2(a, out_dtype) -> torch.Tensor:
     return ref_relu2(a, out_dtype)
 
 
-def moe_experts(h, idx, wt, w_gu, w_down, out_dtype, by_row: Optional[bool] = None, act: str = "silu_glu") -> torch.Tensor:
+def moe_experts(h, idx, wt, w_gu, w_down, out_dtype, by_row: Optional[bool] = None, act: str = "silu_glu",
+                combine: bool = True):
     """Mixture of experts: ``h`` [T, W]; row t runs experts ``idx[t]`` [top] and adds their
     outputs W_down[e] (silu(W_gate[e] h) * (W_up[e] h)) with the weights ``wt[t]``. ``w_gu``
     [E, 2F, W] = every expert's gate rows, then up rows; ``w_down`` [E, W, F]. ``act`` "relu2":
-    the experts are W_down[e] relu(W_up[e] h)^2 and ``w_gu`` is [E, F, W]. Two forms: row by row
-    (GPU steps of a few rows: two launches, no host round trip, so a captured decode step can hold
-    them) and expert by expert (the rows of each expert gathered for library GEMMs, one host read of
-    the expert counts; a row's experts are added in fp32 in the order of its choices whatever else is
-    in the batch)."""
+    the experts are W_down[e] relu(W_up[e] h)^2 and ``w_gu`` is [E, F, W]. ``combine`` False: returns
+    the experts' rows as :class:`ExpertRows`, for a launch that combines them itself. A row's experts
+    are added in fp32 in the order of its choices whatever else is in the batch. Forms: row by row
+    (GPU steps of a few rows, no host round trip, so a captured decode step can hold them);
+    grouped (bf16 prompts of gated experts: rows sorted by expert on the GPU, two grouped matrix-core
+    launches); expert by expert (everything else: the rows of each expert gathered for library GEMMs,
+    one host read of the expert counts)."""
     T, top = idx.shape
+    E, W, F = w_gu.shape[0], h.shape[1], w_down.shape[2]
     if by_row is None:
         by_row = _gpu(h) and T <= MOE_ROWS
     if by_row and _gpu(h):
+        if act == "silu_glu" and not combine and T * top <= 1024:
+            y = torch.empty(T * top, W, dtype=torch.float32, device=h.device)
+            native().moe_pairs(y, torch.empty(T * top, F, dtype=torch.float32, device=h.device), h.contiguous(), w_gu, w_down,
+                               idx)
+            return ExpertRows(y, wt)
         out = torch.empty(h.shape, dtype=out_dtype, device=h.device)
-        hid = torch.empty(T * top * w_down.shape[2], dtype=torch.float32, device=h.device)
+        hid = torch.empty(T * top * F, dtype=torch.float32, device=h.device)
         native().moe_rows(out, hid, h.contiguous(), w_gu, w_down, idx, wt, 1 if act == "relu2" else 0)
-        return out
-    E, W = w_gu.shape[0], h.shape[1]
+        return out if combine else ExpertRows(out, torch.ones_like(wt[:, :1]))
+    if _gpu(h) and act == "silu_glu" and h.dtype == torch.bfloat16 and W % 8 == 0 and F % 8 == 0 and E <= 4096:
+        res = _moe_grouped(h.contiguous(), idx, wt, w_gu, w_down)
+        return res.combine(out_dtype) if combine else res
     flat = idx.reshape(-1).long()
     order = torch.argsort(flat, stable=True)            # (row, choice) pairs, expert by expert
     counts = torch.bincount(flat, minlength=E).tolist()
@@ -430,11 +470,23 @@ def moe_experts(h, idx, wt, w_gu, w_down, out_dtype, by_row: Optional[bool] = No
             a = relu2(a, h.dtype) if act == "relu2" else silu_glu(a, h.dtype)
             torch.mm(a, w_down[e].t(), out=ys[at:at + n])
             at += n
-    back = torch.empty_like(order)
-    back[order] = torch.arange(T * top, device=h.device)
-    y = ys.index_select(0, back).view(T, top, W).float()
-    # a row's experts are added in the order of its choices, in fp32, whatever else is in the batch
-    return torch.bmm(wt.view(T, 1, top), y).view(T, W).to(out_dtype)
+    back = torch.empty(T * top, dtype=torch.int32, device=h.device)
+    back[order] = torch.arange(T * top, dtype=torch.int32, device=h.device)
+    res = ExpertRows(ys, wt, back)
+    return res.combine(out_dtype) if combine else res
+
+
+def _moe_grouped(h, idx, wt, w_gu, w_down) -> ExpertRows:
+    nat = native()
+    (T, top), E, W, F, dev = idx.shape, w_gu.shape[0], h.shape[1], w_down.shape[2], h.device
+    place, order = (torch.empty(T * top, dtype=torch.int32, device=dev) for _ in range(2))
+    tiles = torch.empty(T * top // nat.moe_tile_rows() + E, 3, dtype=torch.int32, device=dev)
+    nat.moe_sort(idx, E, place, order, tiles)
+    hid = torch.empty(T * top, F, dtype=h.dtype, device=dev)
+    nat.moe_gemm(hid, h, w_gu, tiles, order, top, True)
+    ys = torch.empty(T * top, W, dtype=h.dtype, device=dev)
+    nat.moe_gemm(ys, hid, w_down, tiles, None, top, False)
+    return ExpertRows(ys, wt, place)
 
 
 # ---- the PyTorch statements (CPU tensors; what the kernels are tested against) ---------------------
