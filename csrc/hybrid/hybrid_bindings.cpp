@@ -36,8 +36,8 @@ int moe_tile_rows();
 int launch_moe_sort(const int* idx, int P, int E, int* place, int* order, int* tiles, int max_tiles, hipStream_t stream);
 int launch_moe_gemm(void* out, const void* a, const void* b, const int* tiles, int n_tiles, const int* order, int N, int K,
                     int top, bool glu, hipStream_t stream);
-int launch_moe_pairs(float* y, float* hid, const void* h, const void* wgu, const void* wd, const int* idx, int T, int W,
-                     int F, int E, int top, bool bf, hipStream_t stream);
+int launch_moe_pairs(float* y, void* hid, const void* h, const void* wgu, const void* wd, const int* idx, int T, int W,
+                     int F, int E, int top, hipStream_t stream);
 void launch_moe_combine(void* out, const void* y, const float* wt, const int* place, int T, int W, int top, bool out_bf,
                         bool y_bf, hipStream_t stream);
 void launch_limited_glu(void* out, const void* gu, int64_t rows, int F, float limit, bool bf, hipStream_t stream);
@@ -390,18 +390,20 @@ void moe_gemm(torch::Tensor out, torch::Tensor a, torch::Tensor b, torch::Tensor
   TORCH_CHECK(rc == 0, "moe_gemm: unsupported shape (code ", rc, ")");
 }
 
-// y [T * top, W] fp32: every pair's expert output; hid [T * top, F] fp32 scratch
+// bf16. y [T * top, W] fp32: every pair's expert output; hid [T * top, F] bf16 scratch
 void moe_pairs(torch::Tensor y, torch::Tensor hid, torch::Tensor h, torch::Tensor wgu, torch::Tensor wd, torch::Tensor idx) {
-  chk_act(h, "h"); chk_act(wgu, "wgu"); chk_act(wd, "wd"); chk_f32(y, "y"); chk_f32(hid, "hid"); chk_i32(idx, "idx");
+  chk(h, "h"); chk(wgu, "wgu"); chk(wd, "wd"); chk(hid, "hid"); chk_f32(y, "y"); chk_i32(idx, "idx");
   TORCH_CHECK(h.dim() == 2 && wgu.dim() == 3 && wd.dim() == 3 && idx.dim() == 2, "moe_pairs: ranks");
   const int64_t T = h.size(0), W = h.size(1), E = wgu.size(0), F = wd.size(2), top = idx.size(1);
   TORCH_CHECK(wgu.size(1) == 2 * F && wgu.size(2) == W && wd.size(0) == E && wd.size(1) == W && idx.size(0) == T,
               "moe_pairs: shapes");
-  TORCH_CHECK(wgu.scalar_type() == h.scalar_type() && wd.scalar_type() == h.scalar_type(), "moe_pairs: one dtype");
+  TORCH_CHECK(is_bf(h) && is_bf(wgu) && is_bf(wd) && is_bf(hid), "moe_pairs: bf16");
   TORCH_CHECK(y.numel() == T * top * W && hid.numel() >= T * top * F && E <= 65535, "moe_pairs: y / scratch");
-  int rc = launch_moe_pairs(y.data_ptr<float>(), hid.data_ptr<float>(), h.data_ptr(), wgu.data_ptr(), wd.data_ptr(),
-                            idx.data_ptr<int>(), (int)T, (int)W, (int)F, (int)E, (int)top, is_bf(h), cur());
-  TORCH_CHECK(rc == 0, "moe_pairs: at most 1024 pairs and rows that fit the LDS (code ", rc, ")");
+  for (const torch::Tensor* t : {&h, &wgu, &wd, &hid})
+    TORCH_CHECK((reinterpret_cast<uintptr_t>(t->data_ptr()) & 15) == 0, "moe_pairs: operands must be 16-byte aligned");
+  int rc = launch_moe_pairs(y.data_ptr<float>(), hid.data_ptr(), h.data_ptr(), wgu.data_ptr(), wd.data_ptr(),
+                            idx.data_ptr<int>(), (int)T, (int)W, (int)F, (int)E, (int)top, cur());
+  TORCH_CHECK(rc == 0, "moe_pairs: at most 1024 pairs, sizes that are multiples of 8 (code ", rc, ")");
 }
 
 void moe_combine(torch::Tensor out, torch::Tensor y, torch::Tensor wt, c10::optional<torch::Tensor> place) {

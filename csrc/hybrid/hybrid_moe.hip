@@ -7,8 +7,8 @@
 //                  tiles on mfma_f32_32x32x16_bf16; the first product gathers its rows through the
 //                  sorted pairs and writes silu(gate) * up (a tile holds the gate and the up columns of
 //                  the same 64 hidden entries), the second writes every pair's output row.
-//   moe_pairs      decode steps: a workgroup takes 16 output entries of ONE expert and all rows routed
-//                  to it, so an expert's weights are read once however many rows chose it.
+//   moe_pairs      decode steps, bf16: a workgroup takes 16 output entries of ONE expert and all rows
+//                  routed to it, so an expert's weights are read once for up to 16 rows that chose it.
 //   moe_combine    out[t] = sum_k wt[t, k] * y[place of pair (t, k)], in the order of the choices
 //
 // A row's result does not depend on its place or on the other rows.
@@ -215,72 +215,7 @@ __global__ void __launch_bounds__(256, 2) moe_gemm_kernel(GroupedArgs g) {
 
 // ---- decode steps: one expert's weights, every row that chose it ----------------------------------
 
-// R weight rows (w, w + rs, ..; the first `ok` are real) against PR input rows (fp32 in LDS, xs apart),
-// n entries each, for the whole wave: the next step's weight chunks are in flight while the current
-// ones are used, and each is used for all PR rows.
-template <typename T, int R, int PR>
-RT_DEVICE void dot_block(const T* __restrict__ w, size_t rs, int ok, const float* __restrict__ x, int xs, int n, int lane,
-                         float (&acc)[R][PR]) {
-  constexpr int V = 16 / sizeof(T);
-#pragma unroll
-  for (int i = 0; i < R; ++i)
-#pragma unroll
-    for (int p = 0; p < PR; ++p) acc[i][p] = 0.f;
-  if (n % V == 0 && rs % V == 0 && (reinterpret_cast<uintptr_t>(w) & 15) == 0) {
-    rt::u32x4 cur[R], nxt[R];
-    int c = lane * V;
-    auto fetch = [&](rt::u32x4* d, int at) {
-#pragma unroll
-      for (int i = 0; i < R; ++i)
-        d[i] = at < n ? *reinterpret_cast<const rt::u32x4*>(w + (size_t)(i < ok ? i : 0) * rs + at) : rt::u32x4{0u, 0u, 0u, 0u};
-    };
-    fetch(cur, c);
-    for (; c < n; c += 64 * V) {
-      fetch(nxt, c + 64 * V);
-      float wf[R][V];
-#pragma unroll
-      for (int i = 0; i < R; ++i) {
-        if constexpr (V == 8) {
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            wf[i][2 * e] = __uint_as_float(cur[i][e] << 16);
-            wf[i][2 * e + 1] = __uint_as_float(cur[i][e] & 0xffff0000u);
-          }
-        } else {
-#pragma unroll
-          for (int e = 0; e < V; ++e) wf[i][e] = __uint_as_float(cur[i][e]);
-        }
-      }
-#pragma unroll
-      for (int p = 0; p < PR; ++p) {
-        const float4* xp = reinterpret_cast<const float4*>(x + (size_t)p * xs + c);
-#pragma unroll
-        for (int e4 = 0; e4 < V / 4; ++e4) {
-          const float4 xv = xp[e4];
-#pragma unroll
-          for (int i = 0; i < R; ++i)
-            acc[i][p] += wf[i][4 * e4] * xv.x + wf[i][4 * e4 + 1] * xv.y + wf[i][4 * e4 + 2] * xv.z + wf[i][4 * e4 + 3] * xv.w;
-        }
-      }
-#pragma unroll
-      for (int i = 0; i < R; ++i) cur[i] = nxt[i];
-    }
-  } else {
-    for (int c = lane; c < n; c += 64)
-#pragma unroll
-      for (int i = 0; i < R; ++i) {
-        const float wv = DT<T>::load(w + (size_t)(i < ok ? i : 0) * rs + c);
-#pragma unroll
-        for (int p = 0; p < PR; ++p) acc[i][p] += wv * x[(size_t)p * xs + c];
-      }
-  }
-#pragma unroll
-  for (int i = 0; i < R; ++i)
-#pragma unroll
-    for (int p = 0; p < PR; ++p) acc[i][p] = rt::wave_sum(acc[i][p]);
-}
-
-constexpr int kPairWaves = 4, kPairRows = 4, kPairBlock = kPairWaves * kPairRows;
+constexpr int kPairWaves = 4, kPairBlock = 16;      // output entries of one workgroup
 constexpr int kMaxPairs = 1024;
 
 // the pairs that chose `expert`, in order (wave 0); returns their number
@@ -300,44 +235,82 @@ RT_DEVICE int list_pairs(const int* __restrict__ idx, int P, int expert, int* li
   return *count;
 }
 
-// grid (blocks of 16 output entries, experts). GLU: w [E][2N][K] (gate rows, up rows), x = row pair / top
-// of h [T][K], out [pairs][N] = silu(gate) * up; else w [E][N][K], x = row `pair` of the hidden rows.
-// xs is K rounded up to a multiple of 4.
-template <typename T, typename XT, int PR, bool GLU>
-__global__ void __launch_bounds__(64 * kPairWaves) moe_pairs_kernel(float* __restrict__ out, const XT* __restrict__ x,
-                                                                    const T* __restrict__ w, const int* __restrict__ idx,
-                                                                    int P, int top, int K, int N, int xs) {
-  extern __shared__ float4 x4[];
-  float* xl = reinterpret_cast<float*>(x4);      // [PR][xs]
+typedef float f4v __attribute__((ext_vector_type(4)));
+
+// grid (blocks of 16 output entries, experts). GLU: w [E][2N][K] (gate rows, up rows), input row of
+// pair p = row p / top of x [T][K], out bf16 [pairs][N] = silu(gate) * up; else w [E][N][K], input
+// row p of x, out fp32 [pairs][N]. The four waves take a quarter of K each: a wave streams its part of
+// the 16 (32) weight rows straight into mfma_f32_16x16x32_bf16 operands — up to kUnroll steps of
+// loads in flight, no LDS — against up to 16 input rows (the columns); the quarters are added
+// through LDS.
+template <bool GLU>
+__global__ void __launch_bounds__(64 * kPairWaves) moe_pairs_kernel(void* __restrict__ out, const uint16_t* __restrict__ x,
+                                                                    const uint16_t* __restrict__ w,
+                                                                    const int* __restrict__ idx, int P, int top, int K,
+                                                                    int N) {
+  constexpr int NW = GLU ? 2 : 1;
+  constexpr int kUnroll = GLU ? 4 : 8;
   __shared__ int list[kMaxPairs];
   __shared__ int count;
+  __shared__ float part[kPairWaves][NW][16 * 17];      // [input row][entry], rows padded
   const int expert = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int n = list_pairs(idx, P, expert, list, &count);
   if (n == 0) return;
-  const int f = blockIdx.x * kPairBlock + wave * kPairRows;
-  const int ok = min(kPairRows, N - f);
-  const T* we = w + (size_t)expert * (GLU ? 2 : 1) * N * K;
-  for (int b = 0; b < n; b += PR) {
-    const int m = min(PR, n - b);
-    __syncthreads();      // the previous rows' readers are done
-    for (int p = 0; p < PR; ++p) {
-      const XT* xr = x + (size_t)(GLU ? list[b + min(p, m - 1)] / top : list[b + min(p, m - 1)]) * K;
-      for (int c = threadIdx.x; c < K; c += blockDim.x) xl[(size_t)p * xs + c] = p < m ? DT<XT>::load(xr + c) : 0.f;
+  const int c = lane & 15, h = lane >> 4;              // weight row / input row of this lane, its 8 entries of a step
+  const int f0 = blockIdx.x * kPairBlock;
+  const int frow = min(f0 + c, N - 1);
+  const uint16_t* wp[NW];
+#pragma unroll
+  for (int j = 0; j < NW; ++j) wp[j] = w + ((size_t)expert * NW * N + (size_t)j * N + frow) * K + 8 * h;
+  const int kq = ((K + 32 * kPairWaves - 1) / (32 * kPairWaves)) * 32;     // a wave's part of K: whole steps of 32
+  const int kb = wave * kq, ke = min(K, kb + kq);
+  for (int b = 0; b < n; b += 16) {
+    const int m = min(16, n - b);
+    const int pair = list[b + min(c, m - 1)];
+    const uint16_t* xp = x + (size_t)(GLU ? pair / top : pair) * K + 8 * h;
+    f4v acc[NW];
+#pragma unroll
+    for (int j = 0; j < NW; ++j) acc[j] = f4v{0.f, 0.f, 0.f, 0.f};
+    for (int k = kb; k < ke; k += 32 * kUnroll) {
+      rt::u32x4 wv[kUnroll][NW], xv[kUnroll];
+#pragma unroll
+      for (int u = 0; u < kUnroll; ++u) {
+        const bool ok = k + 32 * u + 8 * h < ke;          // K is a multiple of 8
+#pragma unroll
+        for (int j = 0; j < NW; ++j) {
+          wv[u][j] = rt::u32x4{0u, 0u, 0u, 0u};
+          if (ok) wv[u][j] = *reinterpret_cast<const rt::u32x4*>(wp[j] + k + 32 * u);
+        }
+        xv[u] = rt::u32x4{0u, 0u, 0u, 0u};
+        if (ok) xv[u] = *reinterpret_cast<const rt::u32x4*>(xp + k + 32 * u);
+      }
+#pragma unroll
+      for (int u = 0; u < kUnroll; ++u)
+#pragma unroll
+        for (int j = 0; j < NW; ++j)
+          acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(rt::bf16x8, wv[u][j]),
+                                                           __builtin_bit_cast(rt::bf16x8, xv[u]), acc[j], 0, 0, 0);
+    }
+    // lane: column c (input row), rows 4 h + e (weight rows)
+#pragma unroll
+    for (int j = 0; j < NW; ++j)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) part[wave][j][c * 17 + 4 * h + e] = acc[j][e];
+    __syncthreads();
+    const int row = threadIdx.x >> 4, ent = threadIdx.x & 15;
+    if (row < m && f0 + ent < N) {
+      float v[NW];
+#pragma unroll
+      for (int j = 0; j < NW; ++j) {
+        v[j] = 0.f;
+#pragma unroll
+        for (int q = 0; q < kPairWaves; ++q) v[j] += part[q][j][row * 17 + ent];
+      }
+      const size_t at = (size_t)list[b + row] * N + f0 + ent;
+      if constexpr (GLU) ((uint16_t*)out)[at] = rt::f2bf(v[0] * sigm(v[0]) * v[1]);
+      else ((float*)out)[at] = v[0];
     }
     __syncthreads();
-    if (ok <= 0) continue;
-    float a[kPairRows][PR], u[kPairRows][PR];
-    dot_block<T, kPairRows, PR>(we + (size_t)f * K, (size_t)K, ok, xl, xs, K, lane, a);
-    if (GLU) dot_block<T, kPairRows, PR>(we + (size_t)(N + f) * K, (size_t)K, ok, xl, xs, K, lane, u);
-    // lane 4 p + i writes entry f + i of row p
-#pragma unroll
-    for (int p = 0; p < PR; ++p)
-#pragma unroll
-      for (int i = 0; i < kPairRows; ++i)
-        if (lane == p * kPairRows + i && p < m && i < ok) {
-          const float v = a[i][p];
-          out[(size_t)list[b + p] * N + f + i] = GLU ? v * sigm(v) * u[i][p] : v;
-        }
   }
 }
 
@@ -392,46 +365,18 @@ int launch_moe_gemm(void* out, const void* a, const void* b, const int* tiles, i
   return 0;
 }
 
-// hid [P][F] fp32, y [P][W] fp32: every pair's output row, P = T * top <= 1024
-int launch_moe_pairs(float* y, float* hid, const void* h, const void* wgu, const void* wd, const int* idx, int T, int W,
-                     int F, int E, int top, bool bf, hipStream_t stream) {
+// bf16: hid [P][F] bf16 scratch, y [P][W] fp32 = every pair's output row, P = T * top <= 1024; W and F
+// multiples of 8
+int launch_moe_pairs(float* y, void* hid, const void* h, const void* wgu, const void* wd, const int* idx, int T, int W,
+                     int F, int E, int top, hipStream_t stream) {
   if (T <= 0) return 0;
   const int P = T * top;
   if (P > kMaxPairs) return -1;
-  auto pick = [&](int K) {      // input rows held at a time: up to four, 64 KB of LDS
-    const int rows = T >= 3 ? 4 : T;
-    for (int r = rows; r > 1; r >>= 1)
-      if ((size_t)r * ((K + 3) & ~3) * 4 <= 64 * 1024) return r;
-    return (size_t)((K + 3) & ~3) * 4 <= 150 * 1024 ? 1 : 0;
-  };
-  const int p1 = pick(W), p2 = pick(F);
-  if (p1 == 0 || p2 == 0) return -2;
-#define RT_PAIRS(TT, XT, PRV, GLUV, OUT, X, WP, KK, NN)                                                                \
-  do {                                                                                                                 \
-    auto kern = moe_pairs_kernel<TT, XT, PRV, GLUV>;                                                                   \
-    const int xs = ((KK) + 3) & ~3;                                                                                    \
-    const size_t shm = sizeof(float) * (size_t)(PRV) * xs;                                                             \
-    if (shm > 48 * 1024 &&                                                                                             \
-        hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm) != hipSuccess)    \
-      return -3;                                                                                                       \
-    kern<<<dim3(((NN) + kPairBlock - 1) / kPairBlock, E), 64 * kPairWaves, shm, stream>>>(                             \
-        OUT, (const XT*)(X), (const TT*)(WP), idx, P, top, KK, NN, xs);                                                \
-  } while (0)
-#define RT_PAIRS_R(TT, XT, R, GLUV, OUT, X, WP, KK, NN)                                                                \
-  do {                                                                                                                 \
-    if (R == 4) RT_PAIRS(TT, XT, 4, GLUV, OUT, X, WP, KK, NN);                                                         \
-    else if (R >= 2) RT_PAIRS(TT, XT, 2, GLUV, OUT, X, WP, KK, NN);                                                    \
-    else RT_PAIRS(TT, XT, 1, GLUV, OUT, X, WP, KK, NN);                                                                \
-  } while (0)
-  if (bf) {
-    RT_PAIRS_R(uint16_t, uint16_t, p1, true, hid, h, wgu, W, F);
-    RT_PAIRS_R(uint16_t, float, p2, false, y, hid, wd, F, W);
-  } else {
-    RT_PAIRS_R(float, float, p1, true, hid, h, wgu, W, F);
-    RT_PAIRS_R(float, float, p2, false, y, hid, wd, F, W);
-  }
-#undef RT_PAIRS_R
-#undef RT_PAIRS
+  if (W % 8 || F % 8) return -2;
+  moe_pairs_kernel<true><<<dim3((F + kPairBlock - 1) / kPairBlock, E), 64 * kPairWaves, 0, stream>>>(
+      hid, (const uint16_t*)h, (const uint16_t*)wgu, idx, P, top, W, F);
+  moe_pairs_kernel<false><<<dim3((W + kPairBlock - 1) / kPairBlock, E), 64 * kPairWaves, 0, stream>>>(
+      y, (const uint16_t*)hid, (const uint16_t*)wd, idx, P, top, F, W);
   return 0;
 }
 

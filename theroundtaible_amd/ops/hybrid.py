@@ -436,8 +436,9 @@ def moe_experts(h, idx, wt, w_gu, w_down, out_dtype, by_row: Optional[bool] = No
     [E, 2F, W] = every expert's gate rows, then up rows; ``w_down`` [E, W, F]. ``act`` "relu2":
     the experts are W_down[e] relu(W_up[e] h)^2 and ``w_gu`` is [E, F, W]. ``combine`` False: returns
     the experts' rows as :class:`ExpertRows`, for a launch that combines them itself. A row's experts
-    are added in fp32 in the order of its choices whatever else is in the batch. Forms: row by row
-    (GPU steps of a few rows, no host round trip, so a captured decode step can hold them);
+    are added in fp32 in the order of its choices whatever else is in the batch. Forms: a few rows
+    (GPU steps of up to ``MOE_ROWS``, no host round trip, so a captured decode step can hold them;
+    bf16 gated experts: an expert's weights read once for all rows that chose it, else row by row);
     grouped (bf16 prompts of gated experts: rows sorted by expert on the GPU, two grouped matrix-core
     launches); expert by expert (everything else: the rows of each expert gathered for library GEMMs,
     one host read of the expert counts)."""
@@ -446,11 +447,12 @@ def moe_experts(h, idx, wt, w_gu, w_down, out_dtype, by_row: Optional[bool] = No
     if by_row is None:
         by_row = _gpu(h) and T <= MOE_ROWS
     if by_row and _gpu(h):
-        if act == "silu_glu" and not combine and T * top <= 1024:
+        if act == "silu_glu" and h.dtype == torch.bfloat16 and T * top <= 1024 and W % 8 == 0 and F % 8 == 0:
             y = torch.empty(T * top, W, dtype=torch.float32, device=h.device)
-            native().moe_pairs(y, torch.empty(T * top, F, dtype=torch.float32, device=h.device), h.contiguous(), w_gu, w_down,
-                               idx)
-            return ExpertRows(y, wt)
+            hid = torch.empty(T * top, F, dtype=h.dtype, device=h.device)
+            native().moe_pairs(y, hid, h.contiguous(), w_gu, w_down, idx)
+            res = ExpertRows(y, wt)
+            return res.combine(out_dtype) if combine else res
         out = torch.empty(h.shape, dtype=out_dtype, device=h.device)
         hid = torch.empty(T * top * F, dtype=torch.float32, device=h.device)
         native().moe_rows(out, hid, h.contiguous(), w_gu, w_down, idx, wt, 1 if act == "relu2" else 0)
