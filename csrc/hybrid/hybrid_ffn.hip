@@ -203,11 +203,24 @@ __global__ void __launch_bounds__(256) route_topk_kernel(int* __restrict__ idx, 
         for (int j = 0; j < kRouteBatch; ++j) acc[j] += wr[(size_t)min(e0 + j, E - 1) * W + c] * x;
       }
     }
+    // the eight sums together: each exchange halves the values a lane still carries, after three of
+    // them lane l holds expert l >> 3
+    static_assert(kRouteBatch == 8, "eight lanes groups");
 #pragma unroll
-    for (int j = 0; j < kRouteBatch; ++j) {
-      const float v = rt::wave_sum(acc[j]);
-      if (lane == 0 && e0 + j < E) part[(e0 + j) * nw + wave] = v;
+    for (int half = 4, o = 32; half; half >>= 1, o >>= 1) {
+      const bool up = (lane & o) != 0;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (j < half) {
+          const float send = up ? acc[j] : acc[j + half], keep = up ? acc[j + half] : acc[j];
+          acc[j] = keep + __shfl_xor(send, o, 64);
+        }
     }
+    float v = acc[0];
+    v += __shfl_xor(v, 4, 64);
+    v += __shfl_xor(v, 2, 64);
+    v += __shfl_xor(v, 1, 64);
+    if ((lane & 7) == 0 && e0 + (lane >> 3) < E) part[(e0 + (lane >> 3)) * nw + wave] = v;
   }
   __syncthreads();
   for (int e = threadIdx.x; e < E; e += blockDim.x) {

@@ -339,9 +339,37 @@ __global__ void __launch_bounds__(1024) add_norm_kernel(OT* __restrict__ out, fl
   }
 }
 
-// the variance is the mean of the squared deviations (a second sum, over the entries kept in
-// registers), not E[x^2] - mean^2
-template <typename OT, typename YT>
+// The variance is the mean of the squared deviations (a second sum, over the entries kept in
+// registers), not E[x^2] - mean^2. A lane takes V neighbouring entries at a time (4, 16-byte loads,
+// when the width allows) and keeps its first kKeepLN groups. MIX: y holds a mixture's pair rows.
+constexpr int kKeepLN = 2;
+template <typename T, int V>
+RT_DEVICE void load_v(float (&d)[V], const T* p) {
+  if constexpr (V == 4 && sizeof(T) == 4) {
+    const float4 t = *reinterpret_cast<const float4*>(p);
+    d[0] = t.x; d[1] = t.y; d[2] = t.z; d[3] = t.w;
+  } else if constexpr (V == 4) {
+    const uint2 t = *reinterpret_cast<const uint2*>(p);
+    d[0] = __uint_as_float(t.x << 16); d[1] = __uint_as_float(t.x & 0xffff0000u);
+    d[2] = __uint_as_float(t.y << 16); d[3] = __uint_as_float(t.y & 0xffff0000u);
+  } else {
+#pragma unroll
+    for (int i = 0; i < V; ++i) d[i] = DT<T>::load(p + i);
+  }
+}
+template <typename T, int V>
+RT_DEVICE void store_v(T* p, const float (&d)[V]) {
+  if constexpr (V == 4 && sizeof(T) == 4) {
+    *reinterpret_cast<float4*>(p) = float4{d[0], d[1], d[2], d[3]};
+  } else if constexpr (V == 4) {
+    *reinterpret_cast<uint2*>(p) = uint2{rt::pack2(d[0], d[1]), rt::pack2(d[2], d[3])};
+  } else {
+#pragma unroll
+    for (int i = 0; i < V; ++i) DT<T>::store(p + i, d[i]);
+  }
+}
+
+template <typename OT, typename YT, int V, bool MIX>
 __global__ void __launch_bounds__(1024) add_layer_norm_kernel(OT* __restrict__ out, float* __restrict__ x,
                                                               const YT* __restrict__ y, const float* __restrict__ s,
                                                               const float* __restrict__ w, const float* __restrict__ b,
@@ -349,49 +377,81 @@ __global__ void __launch_bounds__(1024) add_layer_norm_kernel(OT* __restrict__ o
                                                               const int* __restrict__ place, int top) {
   __shared__ float scratch[16];
   float* xr = x + (size_t)blockIdx.x * W;
-  const YT* yr = y && top == 0 ? y + (size_t)blockIdx.x * W : y;
   out += (size_t)blockIdx.x * W;
-  auto sum_at = [&](int c) {
-    if (!yr) return xr[c];
-    if (top == 0) return xr[c] + DT<YT>::load(yr + c) * s[c];
-    float acc = 0.f;
-    for (int k = 0; k < top; ++k) {
-      const int p = (int)blockIdx.x * top + k;
-      acc += wt[p] * DT<YT>::load(yr + (size_t)(place ? place[p] : p) * W + c);
+  auto sum_at = [&](int c, float (&v)[V]) {
+    load_v<float, V>(v, xr + c);
+    if (!y) return;
+    float add[V], sc[V];
+    load_v<float, V>(sc, s + c);
+    if (MIX) {
+#pragma unroll
+      for (int i = 0; i < V; ++i) add[i] = 0.f;
+#pragma unroll 2
+      for (int k = 0; k < top; ++k) {
+        const int p = (int)blockIdx.x * top + k;
+        float t[V];
+        load_v<YT, V>(t, y + (size_t)(place ? place[p] : p) * W + c);
+        const float wk = wt[p];
+#pragma unroll
+        for (int i = 0; i < V; ++i) add[i] += wk * t[i];
+      }
+    } else {
+      load_v<YT, V>(add, y + (size_t)blockIdx.x * W + c);
     }
-    return xr[c] + acc * s[c];
+#pragma unroll
+    for (int i = 0; i < V; ++i) v[i] += add[i] * sc[i];
   };
-  float cv[kKeep];
+  float cv[kKeepLN][V];
   float sum = 0.f;
-  int i = 0;
-  for (int c = threadIdx.x; c < W; c += blockDim.x, ++i) {
-    const float v = sum_at(c);
-    sum += v;
 #pragma unroll
-    for (int j = 0; j < kKeep; ++j)
-      if (j == i) cv[j] = v;
+  for (int j = 0; j < kKeepLN; ++j) {
+    const int c = (threadIdx.x + j * blockDim.x) * V;
+    if (c < W) {
+      sum_at(c, cv[j]);
+#pragma unroll
+      for (int i = 0; i < V; ++i) sum += cv[j][i];
+    }
   }
-  auto kept = [&](int idx, int c) {
-    if (idx >= kKeep) return sum_at(c);
-    float v = 0.f;
+  const int rest = (threadIdx.x + kKeepLN * blockDim.x) * V, step = blockDim.x * V;
+  for (int c = rest; c < W; c += step) {
+    float v[V];
+    sum_at(c, v);
 #pragma unroll
-    for (int j = 0; j < kKeep; ++j)
-      if (j == idx) v = cv[j];
-    return v;
-  };
+    for (int i = 0; i < V; ++i) sum += v[i];
+  }
   const float mean = rt::block_sum(sum, scratch) / (float)W;
   float ss = 0.f;
-  i = 0;
-  for (int c = threadIdx.x; c < W; c += blockDim.x, ++i) {
-    const float d = kept(i, c) - mean;
-    ss += d * d;
+  auto dev = [&](const float (&v)[V]) {
+#pragma unroll
+    for (int i = 0; i < V; ++i) ss += (v[i] - mean) * (v[i] - mean);
+  };
+#pragma unroll
+  for (int j = 0; j < kKeepLN; ++j)
+    if ((int)(threadIdx.x + j * blockDim.x) * V < W) dev(cv[j]);
+  for (int c = rest; c < W; c += step) {
+    float v[V];
+    sum_at(c, v);
+    dev(v);
   }
   const float k = inv_rms(rt::block_sum(ss, scratch), W, eps);
-  i = 0;
-  for (int c = threadIdx.x; c < W; c += blockDim.x, ++i) {
-    const float v = kept(i, c);
-    if (yr) xr[c] = v;
-    DT<OT>::store(out + c, (v - mean) * k * w[c] + b[c]);
+  auto put = [&](int c, const float (&v)[V]) {
+    float wv[V], bv[V], o[V];
+    load_v<float, V>(wv, w + c);
+    load_v<float, V>(bv, b + c);
+#pragma unroll
+    for (int i = 0; i < V; ++i) o[i] = (v[i] - mean) * k * wv[i] + bv[i];
+    if (y) store_v<float, V>(xr + c, v);
+    store_v<OT, V>(out + c, o);
+  };
+#pragma unroll
+  for (int j = 0; j < kKeepLN; ++j) {
+    const int c = (threadIdx.x + j * blockDim.x) * V;
+    if (c < W) put(c, cv[j]);
+  }
+  for (int c = rest; c < W; c += step) {
+    float v[V];
+    sum_at(c, v);
+    put(c, v);
   }
 }
 
@@ -548,14 +608,23 @@ void launch_add_layer_norm(void* out, float* x, const void* y, const float* s, c
                            int W, float eps, const float* wt, const int* place, int top, bool out_bf, bool y_bf,
                            hipStream_t stream) {
   if (T <= 0) return;
-  const int th = row_threads(W);
-#define RT_AL(OT, YT) add_layer_norm_kernel<OT, YT><<<T, th, 0, stream>>>((OT*)out, x, (const YT*)y, s, w, b, W, eps, \
-                                                                          wt, place, top)
+  auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = W % 4 == 0 && al(out) && al(x) && al(y) && al(s) && al(w) && al(b);
+  const int groups = vec ? W / 4 : W;
+  const int th = groups >= 1024 ? 1024 : groups <= 64 ? 64 : (groups + 63) / 64 * 64;
+#define RT_AL3(OT, YT, V, MIX)                                                                                         \
+  add_layer_norm_kernel<OT, YT, V, MIX><<<T, th, 0, stream>>>((OT*)out, x, (const YT*)y, s, w, b, W, eps, wt, place, top)
+#define RT_AL(OT, YT)                                                                                                  \
+  do {                                                                                                                 \
+    if (vec) { if (top > 0) RT_AL3(OT, YT, 4, true); else RT_AL3(OT, YT, 4, false); }                                   \
+    else { if (top > 0) RT_AL3(OT, YT, 1, true); else RT_AL3(OT, YT, 1, false); }                                       \
+  } while (0)
   if (out_bf) {
     if (y_bf) RT_AL(uint16_t, uint16_t); else RT_AL(uint16_t, float);
   } else {
     if (y_bf) RT_AL(float, uint16_t); else RT_AL(float, float);
   }
+#undef RT_AL3
 #undef RT_AL
 }
 

@@ -237,7 +237,9 @@ __global__ void __launch_bounds__(kThreads) latent_attn_kernel(AttnArgs a) {
 }
 
 // one workgroup per (row, head): merge the split partials and the sink. The splits' weights are
-// formed once (LDS), then every lane sums its columns over the splits with coalesced loads.
+// formed once (LDS). C4 = C / 4 lanes of 16-byte columns times `blockDim.x / C4` shares of the splits,
+// added through LDS, several splits' loads in flight per lane; C not a multiple of 4: a lane per column.
+// (An empty split has weight zero.)
 template <typename OT>
 __global__ void __launch_bounds__(256) latent_combine_kernel(OT* __restrict__ out, const float* __restrict__ part_o,
                                                              const float* __restrict__ part_ml,
@@ -245,6 +247,7 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(OT* __restrict__ ou
                                                              int splits) {
   __shared__ float wgt[64];
   __shared__ float inv_s;
+  __shared__ float4 share[256];
   const int t = blockIdx.x, h = blockIdx.y;
   const float* ml = part_ml + ((size_t)t * H + h) * splits * 2;
   if (threadIdx.x < 64) {
@@ -261,6 +264,33 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(OT* __restrict__ ou
   const float inv = inv_s;
   const float* po = part_o + ((size_t)t * H + h) * splits * C;
   OT* orow = out + ((size_t)h * T + t) * C;
+  const int C4 = C >> 2;
+  if ((C & 3) == 0 && C4 <= (int)blockDim.x) {
+    const int G = blockDim.x / C4;                 // shares of the splits
+    const int g = threadIdx.x / C4, c4 = threadIdx.x - g * C4;
+    float4 acc = {0.f, 0.f, 0.f, 0.f};
+    if (g < G) {
+#pragma unroll 4
+      for (int s = g; s < splits; s += G) {
+        const float4 v = *reinterpret_cast<const float4*>(po + (size_t)s * C + 4 * c4);
+        const float w = wgt[s];
+        acc.x += v.x * w; acc.y += v.y * w; acc.z += v.z * w; acc.w += v.w * w;
+      }
+    }
+    share[threadIdx.x] = acc;
+    __syncthreads();
+    if (g == 0) {
+      for (int j = 1; j < G; ++j) {
+        const float4 v = share[j * C4 + c4];
+        acc.x += v.x; acc.y += v.y; acc.z += v.z; acc.w += v.w;
+      }
+      DT<OT>::store(orow + 4 * c4, acc.x * inv);
+      DT<OT>::store(orow + 4 * c4 + 1, acc.y * inv);
+      DT<OT>::store(orow + 4 * c4 + 2, acc.z * inv);
+      DT<OT>::store(orow + 4 * c4 + 3, acc.w * inv);
+    }
+    return;
+  }
   for (int c = threadIdx.x; c < C; c += blockDim.x) {
     float acc = 0.f;
     for (int s = 0; s < splits; ++s) {
@@ -603,8 +633,8 @@ int launch_latent_attention(void* out, const void* q_lat, const void* q, const v
 #undef RT_ATTN
   }
   if (rc == 0 && num_splits > 1) {
-    if (bf) hipLaunchKernelGGL((latent_combine_kernel<uint16_t>), dim3(T, H), dim3(C >= 256 ? 256 : 64), 0, stream, (uint16_t*)out, part_o, part_ml, sink, T, H, C, num_splits);
-    else hipLaunchKernelGGL((latent_combine_kernel<float>), dim3(T, H), dim3(C >= 256 ? 256 : 64), 0, stream, (float*)out, part_o, part_ml, sink, T, H, C, num_splits);
+    if (bf) hipLaunchKernelGGL((latent_combine_kernel<uint16_t>), dim3(T, H), dim3(256), 0, stream, (uint16_t*)out, part_o, part_ml, sink, T, H, C, num_splits);
+    else hipLaunchKernelGGL((latent_combine_kernel<float>), dim3(T, H), dim3(256), 0, stream, (float*)out, part_o, part_ml, sink, T, H, C, num_splits);
   }
   return rc;
 }

@@ -21,6 +21,8 @@ void launch_latent_prep(void* cq, const void* proj, int proj_stride, int T, int 
                         const int64_t* slot_mapping, bool bf, hipStream_t stream);
 void launch_gate_mul(void* out, const void* o, const void* proj, int proj_stride, int g_off, int T, int H, int Dv,
                      bool bf, hipStream_t stream);
+void launch_head_product(void* out, const void* x, const void* w, int T, int H, int N, int K, int64_t x_row, int64_t x_head,
+                         int64_t o_row, int64_t o_head, hipStream_t stream);
 void launch_poly_norm(void* out, const void* z, const float* coef, int rows, int F, float eps, bool bf,
                       hipStream_t stream);
 void launch_softcap(float* out, const void* x, int64_t n, float scale, float cap, bool bf, hipStream_t stream);
@@ -207,6 +209,20 @@ void gate_mul(torch::Tensor out, torch::Tensor o, torch::Tensor proj, int64_t g_
   launch_gate_mul(out.data_ptr(), o.data_ptr(), proj.data_ptr(), proj.size(1), g_off, T, H, Dv, is_bf(out), cur());
 }
 
+// bf16: out [T, H, N] and x [T, H, K] with any row and head stride (entries in one piece), w [H, N, K]
+void head_product(torch::Tensor out, torch::Tensor x, torch::Tensor w) {
+  chk(out, "out", false); chk(x, "x", false); chk(w, "w");
+  TORCH_CHECK(is_bf(out) && is_bf(x) && is_bf(w), "head_product: bf16");
+  TORCH_CHECK(out.dim() == 3 && x.dim() == 3 && w.dim() == 3 && x.size(0) == out.size(0) && x.size(1) == out.size(1) &&
+              w.size(0) == x.size(1) && w.size(1) == out.size(2) && w.size(2) == x.size(2), "head_product: shapes");
+  TORCH_CHECK((out.stride(2) == 1 || out.size(2) == 1) && (x.stride(2) == 1 || x.size(2) == 1), "head_product: strides");
+  TORCH_CHECK(x.size(2) % 8 == 0 && x.stride(0) % 8 == 0 && x.stride(1) % 8 == 0 &&
+              (reinterpret_cast<uintptr_t>(x.data_ptr()) & 15) == 0 && (reinterpret_cast<uintptr_t>(w.data_ptr()) & 15) == 0,
+              "head_product: rows must lie on 16-byte boundaries");
+  launch_head_product(out.data_ptr(), x.data_ptr(), w.data_ptr(), (int)x.size(0), (int)x.size(1), (int)out.size(2),
+                      (int)x.size(2), x.stride(0), x.stride(1), out.stride(0), out.stride(1), cur());
+}
+
 void poly_norm(torch::Tensor out, torch::Tensor z, torch::Tensor coef, double eps) {
   chk_act(out, "out"); chk_act(z, "z"); chk_f32(coef, "coef");
   TORCH_CHECK(z.dim() == 2 && out.sizes() == z.sizes() && coef.numel() == 4 && out.scalar_type() == z.scalar_type(),
@@ -233,6 +249,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   });
   m.def("latent_attention", &latent_attention);
   m.def("gate_mul", &gate_mul);
+  m.def("head_product", &head_product);
   m.def("poly_norm", &poly_norm);
   m.def("logit_softcap", &logit_softcap);
 }

@@ -11,6 +11,7 @@
 //   latent_prep       query-latent norm (if the layer has one); KV-latent norm + rotary shared key
 //                     part -> paged cache row
 //   gate_mul          [H, T, Dv] head-major -> [T, H * Dv], times sigmoid(gate)
+//   head_product      a few rows through per-head weights: out[t, h] = W[h] x[t, h] (bf16, MFMA)
 //   poly_norm         a N(z) + b N(z^2) + c N(z^3) + e,  N(u) = u / rms(u)
 //   logit_softcap     cap * tanh(scale * x / cap)
 #include "../common.h"
@@ -210,6 +211,46 @@ __global__ void __launch_bounds__(1024) gate_mul_kernel(OT* __restrict__ out, co
   }
 }
 
+// grid (blocks of 64 entries, heads): a wave takes 16 entries (the rows of mfma_f32_16x16x32_bf16) and
+// up to 16 input rows (its columns) at a time; weights and inputs go straight into the operands, up
+// to four K steps of loads in flight. K a multiple of 8, every row on a 16-byte boundary.
+typedef float f4v __attribute__((ext_vector_type(4)));
+__global__ void __launch_bounds__(256) head_product_kernel(uint16_t* __restrict__ out, const uint16_t* __restrict__ x,
+                                                           const uint16_t* __restrict__ w, int T, int N, int K, int64_t x_row,
+                                                           int64_t x_head, int64_t o_row, int64_t o_head) {
+  const int head = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int n0 = blockIdx.x * 64 + wave * 16;
+  if (n0 >= N) return;
+  const int c = lane & 15, h = lane >> 4;
+  const uint16_t* wp = w + ((size_t)head * N + min(n0 + c, N - 1)) * K + 8 * h;
+  for (int t0 = 0; t0 < T; t0 += 16) {
+    const uint16_t* xp = x + (size_t)min(t0 + c, T - 1) * x_row + head * x_head + 8 * h;
+    f4v acc = {0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < K; k += 128) {
+      rt::u32x4 wv[4], xv[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        wv[u] = rt::u32x4{0u, 0u, 0u, 0u};
+        xv[u] = rt::u32x4{0u, 0u, 0u, 0u};
+        if (k + 32 * u + 8 * h < K) {
+          wv[u] = *reinterpret_cast<const rt::u32x4*>(wp + k + 32 * u);
+          xv[u] = *reinterpret_cast<const rt::u32x4*>(xp + k + 32 * u);
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(rt::bf16x8, wv[u]),
+                                                      __builtin_bit_cast(rt::bf16x8, xv[u]), acc, 0, 0, 0);
+    }
+    if (t0 + c < T) {       // column c: input row; entries n0 + 4 h ..
+      uint16_t* o = out + (size_t)(t0 + c) * o_row + head * o_head + n0 + 4 * h;
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (n0 + 4 * h + e < N) o[e] = rt::f2bf(acc[e]);
+    }
+  }
+}
+
 template <typename IT, typename OT>
 __global__ void __launch_bounds__(1024) poly_norm_kernel(OT* __restrict__ out, const IT* __restrict__ z,
                                                              const float* __restrict__ coef, int F, float eps) {
@@ -305,6 +346,13 @@ void launch_gate_mul(void* out, const void* o, const void* proj, int proj_stride
   if (T <= 0) return;
   if (bf) RT_LAUNCH_W((gate_mul_kernel<uint16_t, uint16_t, uint16_t>), T, H * Dv, (uint16_t*)out, (const uint16_t*)o, (const uint16_t*)proj, proj_stride, g_off, T, H, Dv);
   else RT_LAUNCH_W((gate_mul_kernel<float, float, float>), T, H * Dv, (float*)out, (const float*)o, (const float*)proj, proj_stride, g_off, T, H, Dv);
+}
+
+void launch_head_product(void* out, const void* x, const void* w, int T, int H, int N, int K, int64_t x_row, int64_t x_head,
+                         int64_t o_row, int64_t o_head, hipStream_t stream) {
+  if (T <= 0 || H <= 0 || N <= 0) return;
+  hipLaunchKernelGGL(head_product_kernel, dim3((N + 63) / 64, H), dim3(256), 0, stream, (uint16_t*)out, (const uint16_t*)x,
+                     (const uint16_t*)w, T, N, K, x_row, x_head, o_row, o_head);
 }
 
 void launch_poly_norm(void* out, const void* z, const float* coef, int rows, int F, float eps, bool bf,

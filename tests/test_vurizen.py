@@ -489,6 +489,29 @@ def test_grouped_experts_on_the_matrix_cores(T, E, top, W, F):
     assert torch.equal(alone[0], a[5])
 
 
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("T,H,K,N", [(1, 3, 8, 5), (8, 4, 64, 192), (17, 2, 40, 16), (32, 5, 200, 70)])
+def test_head_product(run, T, H, K, N):
+    """Per-head products of a few rows, from a column range of a wider projection into head-major
+    rows and back."""
+    dev, dt = dev_of(run), dt_of(run)
+    g = torch.Generator().manual_seed(K)
+    proj = torch.randn(T, H * (K + 8) + 16, generator=g).to(dt).to(dev)
+    w = (torch.randn(H, N, K, generator=g) / K ** 0.5).to(dt).to(dev)
+    x = proj[:, :H * (K + 8)].unflatten(1, (H, K + 8))[:, :, :K]
+    want = torch.einsum("thk,hnk->thn", x.double().cpu(), w.double().cpu())
+    if run == ("cuda:0", "fp32"):
+        assert not L.head_product_fits(x, w)        # fp32 layers use library products
+        return
+    a = torch.full((H, T, N), 9.0, dtype=dt, device=dev)
+    L.head_product(x, w, a.transpose(0, 1))
+    b = torch.full((T, H, N), 9.0, dtype=dt, device=dev)
+    L.head_product(x, w, b)
+    tol = 0.03 if run[1] == "bf16" else 1e-4
+    assert float((a.double().cpu().transpose(0, 1) - want).abs().max()) < tol
+    assert float((b.double().cpu() - want).abs().max()) < tol
+
+
 # ---- the model through the engine -----------------------------------------------------------------
 
 def test_registry_and_config():

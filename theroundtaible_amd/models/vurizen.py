@@ -12,11 +12,12 @@ them in one batch; only the attention launch and the scan differ):
     latent_attention:
       latent_prep(proj)                         L2 (HIP): latent norm, rotated key part -> the paged
                                                 cache (not in a layer that reads another's rows)
-      q_lat = q_nope . Wuk                      hipBLASLt (batched over heads): the query moves into
-                                                latent space, so keys are the cached rows
+      q_lat = q_nope . Wuk                      hipBLASLt (batched over heads; decode steps: L7 (HIP)):
+                                                the query moves into latent space, so keys are the
+                                                cached rows
       o_lat = latent_attention(q_lat, q_rot)    L3 (HIP): sliding window, all heads of a row share
                                                 each staged key tile (bf16: MFMA)
-      pending = (o_lat . Wuv) @ Wo^T
+      pending = (o_lat . Wuv) @ Wo^T            as q_lat, then the output GEMM
     gla:
       q, k, decay, v = gla_prep(proj)           C9 (HIP): low-rank decay path, decays in fp32
       o     = state_scan(q, k, v, decay)        C5 (HIP): the recurrence; long spans in parallel chunks
@@ -83,7 +84,8 @@ class VurizenModel(GoganexModel):
             else:
                 # per-head up-projections: q_lat[h] = q_nope[h] @ uk_h[h], o[h] = o_lat[h] @ uv_ht[h]
                 lw["uk_h"] = lw.pop("mix.uk").view(m.heads, m.dim, m.kv_rank).contiguous()
-                lw["uv_ht"] = lw.pop("mix.uv").view(m.heads, m.vdim, m.kv_rank).transpose(1, 2).contiguous()
+                lw["uv_h"] = lw.pop("mix.uv").view(m.heads, m.vdim, m.kv_rank).contiguous()
+                lw["uk_ht"], lw["uv_ht"] = (lw[n].transpose(1, 2).contiguous() for n in ("uk_h", "uv_h"))
                 lw["rot"] = L.rotary_table(m.rot, self.device)
             if ls.ff:
                 E = ls.moe.experts
@@ -137,7 +139,13 @@ class VurizenModel(GoganexModel):
             L.latent_prep(proj, m, None, lw["mix.dkv.norm"], self.cfg.norm_eps, positions, rows, meta.slot_mapping, adt,
                           kv_off=lw["off"]["dkv"], table=lw["rot"])
         q = proj[:, :m.heads * (m.dim + m.rot_dim)].unflatten(1, (m.heads, m.dim + m.rot_dim))
-        q_lat = torch.bmm(q[:, :, :m.dim].transpose(0, 1), lw["uk_h"])
+        qn = q[:, :, :m.dim]
+        few = decode and L.head_product_fits(qn, lw["uk_ht"]) and m.kv_rank % 8 == 0
+        if few:
+            q_lat = torch.empty(m.heads, T, m.kv_rank, dtype=adt, device=proj.device)
+            L.head_product(qn, lw["uk_ht"], q_lat.transpose(0, 1))
+        else:
+            q_lat = torch.bmm(qn.transpose(0, 1), lw["uk_h"])
         splits = L.window_splits(self.decode_splits(T, 1), m.window) if decode else 1
         tiles = None
         if proj.is_cuda:
@@ -145,7 +153,10 @@ class VurizenModel(GoganexModel):
         o_lat = L.latent_attention(q_lat, q, m, rows, meta.block_tables, b.cu_q, b.start_pos, None, tiles=tiles,
                                    num_splits=splits, workspace=self._workspace(T, m, splits), out_dtype=adt, table=lw["rot"])
         o = torch.empty(T, m.heads, m.vdim, dtype=adt, device=proj.device)
-        torch.bmm(o_lat, lw["uv_ht"], out=o.transpose(0, 1))
+        if few:
+            L.head_product(o_lat.transpose(0, 1), lw["uv_h"], o)
+        else:
+            torch.bmm(o_lat, lw["uv_ht"], out=o.transpose(0, 1))
         return o.view(T, m.heads * m.vdim)
 
     def _gla(self, proj, m: GLASpec, lw, l, kv, meta, b, decode):

@@ -202,6 +202,24 @@ def window_splits(splits: int, window: int) -> int:
     return splits if window <= 0 else max(1, min(splits, (window + KEY_TILE - 1) // KEY_TILE + 1))
 
 
+HEAD_PRODUCT_ROWS = 32   # decode steps of up to this many rows
+
+
+def head_product_fits(x, w) -> bool:
+    """Whether :func:`head_product` takes these operands (bf16 GPU rows on 16-byte boundaries)."""
+    return (_gpu(x) and x.dtype == torch.bfloat16 and x.shape[0] <= HEAD_PRODUCT_ROWS and x.shape[2] % 8 == 0
+            and x.stride(0) % 8 == 0 and x.stride(1) % 8 == 0 and x.stride(2) == 1 and x.data_ptr() % 16 == 0)
+
+
+def head_product(x, w, out) -> None:
+    """A few rows through per-head weights: ``out[t, h]`` [N] = ``w[h]`` [N, K] . ``x[t, h]`` [K]; ``x``
+    [T, H, K] and ``out`` [T, H, N] may be views with any row and head stride."""
+    if _gpu(x):
+        native().head_product(out, x, w)
+        return
+    out.copy_(torch.einsum("thk,hnk->thn", x.float(), w.float()))
+
+
 def gate_mul(o, proj, g_off, out_dtype):
     if _gpu(o):
         H, T, Dv = o.shape
