@@ -406,7 +406,7 @@ ROUTERS = [(6, 2, 3, 2, 1.7), (8, 3, 4, 3, 0.5), (5, 2, 1, 1, 1.0), (4, 1, 4, 2,
 @pytest.mark.parametrize("E,top,count,keep,scale", ROUTERS)
 def test_router(run, E, top, count, keep, scale):
     """Choices by score + correction within the best groups, weights by the score alone; choice
-    scores of both signs (an excluded expert is minus infinity, not zero), groups of one expert, one
+    scores of both signs (a masked expert must lose to any negative score too), groups of one expert, one
     group, more experts than a wave has lanes."""
     dev, dt = dev_of(run), dt_of(run)
     g = torch.Generator().manual_seed(E)

@@ -26,7 +26,8 @@ of them in one batch; only the attention launch differs):
     h       = add_norm(x, pending)                  H6 (HIP)
     dense:      pending = xielu(h @ Wup^T + b) @ Wdown^T + b     H9 (HIP) between two GEMMs
     experts:    idx, wt = topk_softmax(h @ Wrouter^T + b)        fp32 GEMM, H11 (HIP)
-                pending = moe_experts(h, idx, wt)   a few rows: H12 (HIP), two launches; more rows:
+                pending = moe_experts(h, idx, wt)   bf16: H14 - H17 (HIP), grouped products / expert rows;
+                                                    fp32: a few rows H12 (HIP), two launches; more rows:
                                                     each expert's rows through library GEMMs, H10
 
 The residual stream, every norm, positions, scores and softmax, the router, the token-shift state,
