@@ -82,7 +82,7 @@ def _build_family(name: str, out: str, verbose: bool = False, jobs: int = 8) -> 
     os.makedirs(bdir, exist_ok=True)
     incs, torch_lib, abi = torch_paths()
     py_inc = sysconfig.get_paths()["include"]
-    headers = glob.glob(os.path.join(HERE, "*.h"))
+    headers = glob.glob(os.path.join(HERE, "*.h")) + glob.glob(os.path.join(src_dir, "*.h"))
     common = ["-O3", "-fPIC", "-std=c++17", f"-D_GLIBCXX_USE_CXX11_ABI={abi}", "-D__HIP_PLATFORM_AMD__=1",
               "-DUSE_ROCM=1", "-Wno-unused-result", "-Wno-deprecated-declarations", "-Wno-unused-command-line-argument"]
     jobs_list, objs = [], []
@@ -94,7 +94,7 @@ def _build_family(name: str, out: str, verbose: bool = False, jobs: int = 8) -> 
     bsrc = os.path.join(src_dir, f"{name}_bindings.cpp")
     bobj = os.path.join(bdir, f"{name}_bindings.cpp.o")
     objs.append(bobj)
-    if _newer(bsrc, bobj, []):
+    if _newer(bsrc, bobj, headers):
         jobs_list.append([HIPCC, *common, "-I", py_inc, *sum((["-I", i] for i in incs), []),
                           f"-DTORCH_EXTENSION_NAME=_C_{name}", "-DTORCH_API_INCLUDE_EXTENSION_H", "-c", bsrc, "-o", bobj])
     with cf.ThreadPoolExecutor(max_workers=jobs) as ex:

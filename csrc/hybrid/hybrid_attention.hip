@@ -4,9 +4,10 @@
 //   K cache [num_blocks, G, BS, Dk], V cache [num_blocks, G, BS, Dv], q [T, H, Dk], out [T, H * Dv]
 //   (layout 1: the matrix-core kernels' cache — keys chunk-major per block, V [num_blocks, G, Dv, BS])
 //   score(i, j) = q_i . k_j * scale * temp[h] - slopes[h] * (i - j), j <= position(i),
-//                 and i - j < window when a window is given (tiles wholly ahead of it are skipped)
-//   weight_j   = exp(s_j) / (sink + sum_j exp(s_j))        (sink: a key of score 0 without a value)
-//   out       *= sigmoid(gate[row, h * Dv + col])          when a gate is given
+//                 and i - j < window (or j < keep) when a window is given, j in i's chunk when chunks
+//                 are (tiles that no row sees are skipped)
+//   weight_j   = exp(s_j) / (sink + exp(sinks[h]) + sum_j exp(s_j))   (sink: a key of score 0 without a value)
+//   out       *= sigmoid(gate[row, h * Dv + col]), or sigmoid(gate[row, h])   when a gate is given
 //   with a soft cap c the scaled score becomes c * tanh(score / c) ahead of the distance term; the
 //   result is multiplied by out_scale and may land in a column range of a wider buffer
 //
@@ -21,6 +22,7 @@
 // Split launch (one row per sequence: a decode step): gridDim.z key ranges per work item, each
 // writes (o, m, l) partials; gqa_combine_kernel merges them and adds the sink once.
 #include "../common.h"
+#include "hybrid_args.h"
 
 namespace {
 
@@ -38,8 +40,8 @@ __global__ void __launch_bounds__(256) gqa_attention_kernel(
     const int* __restrict__ block_tables, const int* __restrict__ cu_q, const int* __restrict__ start_pos,
     const int* __restrict__ tiles, const float* __restrict__ temp, float* __restrict__ part_o,
     float* __restrict__ part_ml, int H, int G, int Dk, int Dv, int BS, int max_blocks, int R, int KT, int hchunks,
-    float scale, float sink, int window, const float* __restrict__ slopes, const T* __restrict__ gate,
-    int gate_stride, int layout, float softcap, float out_scale, int out_stride, int out_off) {
+    float scale, float sink, AttnMask mask, const float* __restrict__ slopes, const T* __restrict__ gate,
+    int gate_stride, int gate_heads, int layout, float softcap, float out_scale, int out_stride, int out_off) {
   extern __shared__ float lds[];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int seq = tiles[2 * blockIdx.x], row0 = tiles[2 * blockIdx.x + 1];
@@ -50,13 +52,12 @@ __global__ void __launch_bounds__(256) gqa_attention_kernel(
   const int P = nrows * nh;
   const int pos0 = start_pos[seq] + (row0 - cu_q[seq]);           // position of the tile's first row
   const int kend = pos0 + nrows;                                  // keys 0 .. kend - 1 are visible to the tile
-  // this workgroup's key range (whole tiles of KT keys, counted from key 0; with a window the
-  // tiles that end before the first row's oldest visible key are left out: every weight in them is 0)
+  // this workgroup's key range (whole tiles of KT keys, counted from key 0; tiles between the kept
+  // first keys and the first row's oldest visible key are left out: every weight in them is 0)
   const int S = gridDim.z;
-  const int ntile = (kend + KT - 1) / KT;
-  const int t0 = window > 0 ? max(0, pos0 - window + 1) / KT : 0;
-  const int per = (ntile - t0 + S - 1) / S;
-  const int t_lo = t0 + blockIdx.z * per, t_hi = min(ntile, t_lo + per);
+  const TileRange tr = mask_tiles(mask, pos0, kend, KT);
+  const int per = (tr.n + S - 1) / S;
+  const int t_lo = blockIdx.z * per, t_hi = min(tr.n, t_lo + per);
 
   float* qs = lds;                              // [kWaves * kPW][Dk]
   float* ks = qs + kWaves * kPW * Dk;           // [KT][Dk + 1]
@@ -70,7 +71,7 @@ __global__ void __launch_bounds__(256) gqa_attention_kernel(
     qs[i] = DT<T>::load(q + ((size_t)(row0 + r) * H + h) * Dk + d);
   }
   float m[kPW], l[kPW], hs[kPW], sl[kPW], o[kPW][DVL];
-  int qpos[kPW];
+  int qpos[kPW], qlow[kPW];
 #pragma unroll
   for (int i = 0; i < kPW; ++i) {
     const int p = wave + kWaves * i;
@@ -78,14 +79,15 @@ __global__ void __launch_bounds__(256) gqa_attention_kernel(
     l[i] = 0.f;
     const int r = p / nh, h = g * group + h_lo + (p - r * nh);
     qpos[i] = p < P ? pos0 + r : -1;
+    qlow[i] = mask_low(mask, max(qpos[i], 0));
     hs[i] = p < P ? scale * (temp ? temp[h] : 1.0f) : 0.f;
     sl[i] = p < P && slopes ? slopes[h] : 0.f;
 #pragma unroll
     for (int c = 0; c < DVL; ++c) o[i][c] = 0.f;
   }
 
-  for (int kt = t_lo; kt < t_hi; ++kt) {
-    const int kb = kt * KT;
+  for (int tv = t_lo; tv < t_hi; ++tv) {
+    const int kb = tr.at(tv) * KT;
     __syncthreads();        // the previous tile's readers are done (and qs is written)
     for (int i = threadIdx.x; i < KT * Dk; i += blockDim.x) {
       const int j = i / Dk, d = i - j * Dk;
@@ -122,7 +124,7 @@ __global__ void __launch_bounds__(256) gqa_attention_kernel(
 #pragma unroll
     for (int i = 0; i < kPW; ++i) {
       const int dist = qpos[i] - (kb + lane);
-      const bool ok = lane < KT && dist >= 0 && (window <= 0 || dist < window);
+      const bool ok = lane < KT && mask_sees(mask, qlow[i], qpos[i], kb + lane);
       float raw = s[i] * hs[i];
       if (softcap > 0.f) raw = softcap * tanhf(raw / softcap);
       const float sc = ok ? raw - sl[i] * (float)dist : kNeg;
@@ -160,14 +162,21 @@ __global__ void __launch_bounds__(256) gqa_attention_kernel(
     const int r = p / nh, h = g * group + h_lo + (p - r * nh);
     const size_t rh = (size_t)(row0 + r) * H + h;
     if (S == 1) {
-      const float den = l[i] + sink * __expf(-m[i]);
-      const float inv = den > 0.f ? 1.0f / den : 0.f;
+      float den = l[i] + (sink > 0.f ? sink * __expf(-m[i]) : 0.f), num = 1.0f;
+      if (mask.sinks) {      // relative to the larger of the two, so a sink far above the scores stays finite
+        const float M = fmaxf(m[i], mask.sinks[h]);
+        num = __expf(m[i] - M);
+        den = den * num + __expf(mask.sinks[h] - M);
+      }
+      float inv = den > 0.f ? num / den : 0.f;
+      if (gate && gate_heads) inv *= 1.0f / (1.0f + __expf(-DT<T>::load(gate + (size_t)(row0 + r) * gate_stride + h)));
 #pragma unroll
       for (int c = 0; c < DVL; ++c) {
         const int col = lane + 64 * c;
         if (col < Dv) {
           float v = o[i][c] * inv * out_scale;
-          if (gate) v *= 1.0f / (1.0f + __expf(-DT<T>::load(gate + (size_t)(row0 + r) * gate_stride + h * Dv + col)));
+          if (gate && !gate_heads)
+            v *= 1.0f / (1.0f + __expf(-DT<T>::load(gate + (size_t)(row0 + r) * gate_stride + h * Dv + col)));
           DT<T>::store(out + (size_t)(row0 + r) * out_stride + out_off + h * Dv + col, v);
         }
       }
@@ -191,19 +200,21 @@ template <typename T>
 __global__ void __launch_bounds__(64) gqa_combine_kernel(T* __restrict__ out, const float* __restrict__ part_o,
                                                          const float* __restrict__ part_ml, int S, int Dv, float sink,
                                                          int H, const T* __restrict__ gate, int gate_stride,
+                                                         int gate_heads, const float* __restrict__ sinks,
                                                          float out_scale, int out_stride, int out_off) {
   const size_t rh = blockIdx.x;
   const int lane = threadIdx.x;
-  float M = kNeg;
+  float M = sinks ? sinks[rh % H] : kNeg;
   for (int s = 0; s < S; ++s) M = fmaxf(M, part_ml[(rh * S + s) * 2]);
-  float den = sink * __expf(-M);
+  float den = (sink > 0.f ? sink * __expf(-M) : 0.f) + (sinks ? __expf(sinks[rh % H] - M) : 0.f);
   for (int s = 0; s < S; ++s) den += part_ml[(rh * S + s) * 2 + 1] * __expf(part_ml[(rh * S + s) * 2] - M);
-  const float inv = den > 0.f ? 1.0f / den : 0.f;
+  float inv = den > 0.f ? 1.0f / den : 0.f;
+  if (gate && gate_heads) inv *= 1.0f / (1.0f + __expf(-DT<T>::load(gate + (rh / H) * gate_stride + rh % H)));
   for (int col = lane; col < Dv; col += 64) {
     float acc = 0.f;
     for (int s = 0; s < S; ++s) acc += part_o[(rh * S + s) * Dv + col] * __expf(part_ml[(rh * S + s) * 2] - M);
     float v = acc * inv * out_scale;
-    if (gate) v *= 1.0f / (1.0f + __expf(-DT<T>::load(gate + (rh / H) * gate_stride + (rh % H) * Dv + col)));
+    if (gate && !gate_heads) v *= 1.0f / (1.0f + __expf(-DT<T>::load(gate + (rh / H) * gate_stride + (rh % H) * Dv + col)));
     DT<T>::store(out + (rh / H) * out_stride + out_off + (rh % H) * Dv + col, v);
   }
 }
@@ -224,9 +235,9 @@ int gqa_key_tile(int Dk, int Dv) {
 int launch_gqa_attention(void* out, const void* q, const void* kc, const void* vc, const int* block_tables,
                          const int* cu_q, const int* start_pos, const int* tiles, int n_tiles, const float* temp,
                          float* part_o, float* part_ml, int T, int H, int G, int Dk, int Dv, int BS, int max_blocks,
-                         int rows, int num_splits, float scale, float sink, int window, const float* slopes,
-                         const void* gate, int gate_stride, int layout, float softcap, float out_scale, int out_stride,
-                         int out_off, bool bf, hipStream_t stream) {
+                         int rows, int num_splits, float scale, float sink, const AttnMask& mask, const float* slopes,
+                         const void* gate, int gate_stride, bool gate_heads, int layout, float softcap, float out_scale,
+                         int out_stride, int out_off, bool bf, hipStream_t stream) {
   if (n_tiles <= 0 || T <= 0) return 0;
   const int KT = gqa_key_tile(Dk, Dv);
   if (KT == 0 || Dv > 256 || Dk > 256 || H % G) return -1;
@@ -250,8 +261,8 @@ int launch_gqa_attention(void* out, const void* q, const void* kc, const void* v
       return -3;                                                                                                     \
     kern<<<grid, 256, shm, stream>>>((TT*)out, (const TT*)q, (const TT*)kc, (const TT*)vc, block_tables, cu_q,      \
                                      start_pos, tiles, temp, part_o, part_ml, H, G, Dk, Dv, BS, max_blocks, rows,   \
-                                     KT, hchunks, scale, sink, window, slopes, (const TT*)gate, gate_stride, layout, \
-                                     softcap, out_scale, out_stride, out_off);                                      \
+                                     KT, hchunks, scale, sink, mask, slopes, (const TT*)gate, gate_stride,           \
+                                     gate_heads ? 1 : 0, layout, softcap, out_scale, out_stride, out_off);           \
   } while (0)
   if (bf) {
     if (dvl == 1) RT_GQA(uint16_t, 1); else if (dvl == 2) RT_GQA(uint16_t, 2); else RT_GQA(uint16_t, 4);
@@ -262,11 +273,11 @@ int launch_gqa_attention(void* out, const void* q, const void* kc, const void* v
 #undef RT_GQA2
   if (num_splits > 1) {
     if (bf) gqa_combine_kernel<uint16_t><<<T * H, 64, 0, stream>>>((uint16_t*)out, part_o, part_ml, num_splits, Dv, sink, H,
-                                                                   (const uint16_t*)gate, gate_stride, out_scale,
-                                                                   out_stride, out_off);
+                                                                   (const uint16_t*)gate, gate_stride, gate_heads ? 1 : 0,
+                                                                   mask.sinks, out_scale, out_stride, out_off);
     else gqa_combine_kernel<float><<<T * H, 64, 0, stream>>>((float*)out, part_o, part_ml, num_splits, Dv, sink, H,
-                                                             (const float*)gate, gate_stride, out_scale, out_stride,
-                                                             out_off);
+                                                             (const float*)gate, gate_stride, gate_heads ? 1 : 0,
+                                                             mask.sinks, out_scale, out_stride, out_off);
   }
   return 0;
 }

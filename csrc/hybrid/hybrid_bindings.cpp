@@ -5,6 +5,7 @@
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
 #include <hip/hip_runtime.h>
+#include "hybrid_args.h"
 
 void launch_shift_norm(void* out, float* xs, const float* x, const void* y, const float* w, const float* mu,
                        float* state, const int* row_seq, const int64_t* positions, const int* start_pos,
@@ -16,7 +17,17 @@ void launch_qk_prep(void* q, const void* proj, int stride, int q_off, int k_off,
                     const float* inv_freq, int rot_dims, float eps, const int64_t* positions, void* kc, void* vc,
                     const int64_t* slot_mapping, int T, int H, int G, int Dk, int Dv, int BS, bool bf, int layout,
                     const float* q_scale, const float* q_w, const float* k_w, bool v_norm, float qt_coef, int qt_every,
-                    hipStream_t stream);
+                    const QkExtra& ex, hipStream_t stream);
+void launch_add_tanh_norm(void* out, float* x, const void* y, float alpha, const float* w, const float* b, int T, int W,
+                          bool out_bf, bool y_bf, hipStream_t stream);
+int launch_channel_delta(float* out, float* vout, const void* proj, int stride, int q_off, int b_off, int a_off, int rank,
+                         const float* a2, const float* cw, float* state, const float* neg_rate, const float* dt_bias, int T,
+                         int A, int G, int D, int E, int taps, int keep, const int* row_seq, const int64_t* positions,
+                         const int* start_pos, const int* slots, bool shift_state, bool bf, hipStream_t stream);
+int launch_memory_prep(float* out, float* gates, const void* proj, int stride, int q_off, int k_off, int v_off, int i_off,
+                       int f_off, const float* ib, const float* fb, float cap, float* gmax, const int* cu_q,
+                       const int* start_pos, const int* slots, float q_scale, int S, int T, int A, int D, int E, bool step,
+                       bool bf, hipStream_t stream);
 void launch_mingru_scan(void* out, const void* proj, int stride, int z_off, int x_off, int g_off, int width,
                         const float* bz, const float* bx, float* state, const int* cu_q, const int* start_pos,
                         const int* slots, int S, bool bf, hipStream_t stream);
@@ -45,9 +56,9 @@ int gqa_key_tile(int Dk, int Dv);
 int launch_gqa_attention(void* out, const void* q, const void* kc, const void* vc, const int* block_tables,
                          const int* cu_q, const int* start_pos, const int* tiles, int n_tiles, const float* temp,
                          float* part_o, float* part_ml, int T, int H, int G, int Dk, int Dv, int BS, int max_blocks,
-                         int rows, int num_splits, float scale, float sink, int window, const float* slopes,
-                         const void* gate, int gate_stride, int layout, float softcap, float out_scale, int out_stride,
-                         int out_off, bool bf, hipStream_t stream);
+                         int rows, int num_splits, float scale, float sink, const AttnMask& mask, const float* slopes,
+                         const void* gate, int gate_stride, bool gate_heads, int layout, float softcap, float out_scale,
+                         int out_stride, int out_off, bool bf, hipStream_t stream);
 int wkv_scan_chunk();
 int launch_wkv_scan(void* out, const void* r, const void* k, const void* v, const void* g, const void* lw, int stride,
                     int lw_stride, const float* w0, const float* u, const float* norm_w, float* state, const int* cu_q,
@@ -89,7 +100,7 @@ int launch_gla_prep(float* out, const void* proj, int stride, int q_off, int k_o
                     hipStream_t stream);
 void launch_head_norm_gate(void* out, int out_stride, int out_off, const float* o, const float* w, int wmod, int span,
                            const void* gate, int gate_stride, int gate_off, int act, float eps, float scale, int T, int C,
-                           bool out_bf, bool gate_bf, hipStream_t stream);
+                           const float* floors, bool out_bf, bool gate_bf, hipStream_t stream);
 int launch_state_scan(float* out, const float* q, const float* k, const float* v, const float* w, const float* a,
                       const float* b, int sq, int sk, int sv, int sw, int sa, int sb, const float* decay, float* state,
                       const int* cu_q, const int* start_pos, const int* slots, int S, int T, int A, int D, int E,
@@ -171,7 +182,9 @@ void qk_prep(torch::Tensor q, torch::Tensor proj, int64_t q_off, int64_t k_off, 
              c10::optional<torch::Tensor> inv_freq, double eps, torch::Tensor positions, torch::Tensor kc,
              torch::Tensor vc, torch::Tensor slot_mapping, int64_t layout, c10::optional<torch::Tensor> q_scale,
              c10::optional<torch::Tensor> q_w, c10::optional<torch::Tensor> k_w, bool v_norm, double qt_coef,
-             int64_t qt_every) {
+             int64_t qt_every, bool halves, c10::optional<torch::Tensor> q_b, c10::optional<torch::Tensor> k_b,
+             c10::optional<torch::Tensor> v_b, c10::optional<torch::Tensor> mix, int64_t mix_off,
+             c10::optional<torch::Tensor> mix_b, double mix_w) {
   chk_act(q, "q"); chk_act(proj, "proj"); chk_act(kc, "k_cache"); chk_act(vc, "v_cache");
   TORCH_CHECK(q.scalar_type() == proj.scalar_type() && kc.scalar_type() == proj.scalar_type() &&
               vc.scalar_type() == proj.scalar_type(), "qk_prep: one dtype for proj, q and the cache");
@@ -204,9 +217,38 @@ void qk_prep(torch::Tensor q, torch::Tensor proj, int64_t q_off, int64_t k_off, 
   if (q_w.has_value()) { chk_f32(*q_w, "q_w", Dk); qw = q_w->data_ptr<float>(); }
   if (k_w.has_value()) { chk_f32(*k_w, "k_w", Dk); kw = k_w->data_ptr<float>(); }
   TORCH_CHECK(qt_every >= 0 && qt_every < (int64_t(1) << 31), "qk_prep: q_temp every");
+  QkExtra ex;
+  ex.halves = halves ? 1 : 0;
+  if (q_b.has_value()) { chk_f32(*q_b, "q_b", H * Dk); ex.q_b = q_b->data_ptr<float>(); }
+  if (k_b.has_value()) { chk_f32(*k_b, "k_b", G * Dk); ex.k_b = k_b->data_ptr<float>(); }
+  if (v_b.has_value()) { chk_f32(*v_b, "v_b", G * Dv); ex.v_b = v_b->data_ptr<float>(); }
+  if (mix.has_value()) {      // the values of another projection [T, N'], its columns mix_off .. mix_off + G * Dv
+    chk_act(*mix, "mix");
+    TORCH_CHECK(mix->dim() == 2 && mix->size(0) == T && mix->scalar_type() == proj.scalar_type() && mix_off >= 0 &&
+                mix_off + G * Dv <= mix->size(1), "qk_prep: mixed value columns");
+    ex.mix = static_cast<const char*>(mix->data_ptr()) + mix_off * mix->element_size();
+    ex.mix_stride = (int)mix->size(1);
+    ex.mix_w = (float)mix_w;
+    if (mix_b.has_value()) { chk_f32(*mix_b, "mix_b", G * Dv); ex.mix_b = mix_b->data_ptr<float>(); }
+  }
+  TORCH_CHECK(!((v_b.has_value() || mix.has_value()) && (v_norm || v_from_k)),
+              "qk_prep: biased or mixed values exclude normed values and values taken from the keys");
   launch_qk_prep(q.data_ptr(), proj.data_ptr(), N, q_off, k_off, v_off, v_from_k, fr, rot_dims, (float)eps,
                  positions.data_ptr<int64_t>(), kc.data_ptr(), vc.data_ptr(), slot_mapping.data_ptr<int64_t>(), T, H, G,
-                 Dk, Dv, BS, is_bf(q), (int)layout, qs, qw, kw, v_norm, (float)qt_coef, (int)qt_every, cur());
+                 Dk, Dv, BS, is_bf(q), (int)layout, qs, qw, kw, v_norm, (float)qt_coef, (int)qt_every, ex, cur());
+}
+
+AttnMask mask_of(int64_t window, int64_t keep, int64_t chunk, const c10::optional<torch::Tensor>& sinks, int64_t H) {
+  const int64_t top = int64_t(1) << 30;
+  TORCH_CHECK(window >= 0 && window < top && keep >= 0 && keep < top && chunk >= 0 && chunk < top,
+              "attention: window / keep / chunk out of range");
+  TORCH_CHECK(!(window > 0 && chunk > 0) && (keep == 0 || window > 0), "attention: kept keys go with a window, chunks with none");
+  AttnMask m;
+  m.window = (int)window;
+  m.keep = (int)keep;
+  m.chunk = (int)chunk;
+  if (sinks.has_value()) { chk_f32(*sinks, "sinks", H); m.sinks = sinks->data_ptr<float>(); }
+  return m;
 }
 
 void gqa_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch::Tensor vc, torch::Tensor block_tables,
@@ -214,7 +256,7 @@ void gqa_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch::
                    double scale, double sink, int64_t rows, int64_t num_splits, c10::optional<torch::Tensor> part_o,
                    c10::optional<torch::Tensor> part_ml, int64_t window, c10::optional<torch::Tensor> slopes,
                    c10::optional<torch::Tensor> gate, int64_t gate_off, int64_t layout, double softcap, double out_scale,
-                   int64_t out_off) {
+                   int64_t out_off, int64_t keep, int64_t chunk, c10::optional<torch::Tensor> sinks, bool gate_heads) {
   chk_act(out, "out"); chk_act(q, "q"); chk_act(kc, "k_cache"); chk_act(vc, "v_cache");
   TORCH_CHECK(out.scalar_type() == q.scalar_type() && kc.scalar_type() == q.scalar_type() &&
               vc.scalar_type() == q.scalar_type(), "gqa_attention: one dtype for q, the cache and out");
@@ -250,20 +292,20 @@ void gqa_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch::
   }
   const float* sl = nullptr;
   if (slopes.has_value()) { chk_f32(*slopes, "slopes", H); sl = slopes->data_ptr<float>(); }
-  TORCH_CHECK(window >= 0 && window < (int64_t(1) << 31), "gqa_attention: window");
+  const AttnMask mask = mask_of(window, keep, chunk, sinks, H);
   const char* gp = nullptr;
   int64_t gstride = 0;
   if (gate.has_value()) {      // columns gate_off .. gate_off + H * Dv of a [T, N] tensor
     chk_act(*gate, "gate");
     TORCH_CHECK(gate->dim() == 2 && gate->size(0) == T && gate->scalar_type() == q.scalar_type() && gate_off >= 0 &&
-                gate_off + H * Dv <= gate->size(1), "gqa_attention: gate columns");
+                gate_off + H * (gate_heads ? 1 : Dv) <= gate->size(1), "gqa_attention: gate columns");
     gstride = gate->size(1);
     gp = static_cast<const char*>(gate->data_ptr()) + gate_off * gate->element_size();
   }
   int rc = launch_gqa_attention(out.data_ptr(), q.data_ptr(), kc.data_ptr(), vc.data_ptr(), block_tables.data_ptr<int>(),
                                 cu_q.data_ptr<int>(), start_pos.data_ptr<int>(), tiles.data_ptr<int>(), tiles.size(0), tp,
                                 po, pml, T, H, G, Dk, Dv, BS, block_tables.size(1), rows, num_splits, (float)scale,
-                                (float)sink, (int)window, sl, gp, (int)gstride, (int)layout, (float)softcap,
+                                (float)sink, mask, sl, gp, (int)gstride, gate_heads, (int)layout, (float)softcap,
                                 (float)out_scale, (int)out.size(1), (int)out_off, is_bf(q), cur());
   TORCH_CHECK(rc == 0, "gqa_attention: unsupported shape (code ", rc, ": -1 head sizes beyond 256 or the LDS tile, "
               "-2 rows per tile, -3 LDS size refused)");
@@ -356,6 +398,20 @@ void add_layer_norm(torch::Tensor out, torch::Tensor x, c10::optional<torch::Ten
   }
   launch_add_layer_norm(out.data_ptr(), x.data_ptr<float>(), yp, sp, w.data_ptr<float>(), b.data_ptr<float>(), T, W,
                         (float)eps, wp, pp, (int)top, is_bf(out), y_bf, cur());
+}
+
+void add_tanh_norm(torch::Tensor out, torch::Tensor x, c10::optional<torch::Tensor> y, double alpha, torch::Tensor w,
+                   torch::Tensor b) {
+  chk_act(out, "out"); chk_f32(x, "x");
+  TORCH_CHECK(x.dim() == 2 && out.sizes() == x.sizes(), "add_tanh_norm: shapes");
+  chk_f32(w, "w", x.size(1)); chk_f32(b, "b", x.size(1));
+  if (y.has_value()) {
+    chk_act(*y, "y");
+    TORCH_CHECK(y->sizes() == x.sizes(), "add_tanh_norm: y must have x's shape");
+  }
+  launch_add_tanh_norm(out.data_ptr(), x.data_ptr<float>(), y.has_value() ? y->data_ptr() : nullptr, (float)alpha,
+                       w.data_ptr<float>(), b.data_ptr<float>(), (int)x.size(0), (int)x.size(1), is_bf(out),
+                       y.has_value() && is_bf(*y), cur());
 }
 
 // idx [T, top] -> place / order [T * top], tiles [n, 3] (n at least T * top / tile rows + experts)
@@ -700,6 +756,60 @@ void delta_prep(torch::Tensor five, torch::Tensor vout, torch::Tensor proj, int6
   TORCH_CHECK(rc == 0, "delta_prep: a row does not fit the LDS (code ", rc, ")");
 }
 
+// out [4, T, A * D], v [T, A * E]; proj columns q_off (q, k, v), b_off (A), a_off (rank); a2 [rank, A * D]
+void channel_delta_prep(torch::Tensor out, torch::Tensor vout, torch::Tensor proj, int64_t q_off, int64_t b_off,
+                        int64_t a_off, torch::Tensor a2, torch::Tensor cw, torch::Tensor state, torch::Tensor neg_rate,
+                        torch::Tensor dt_bias, int64_t A, int64_t G, int64_t D, int64_t E, torch::Tensor row_seq,
+                        torch::Tensor positions, torch::Tensor start_pos, torch::Tensor slots, bool shift_state) {
+  chk_act(proj, "proj"); chk_f32(a2, "a2");
+  TORCH_CHECK(proj.dim() == 2 && A >= 1 && G >= 1 && A % G == 0 && D >= 1 && E >= 1, "channel_delta_prep: sizes");
+  TORCH_CHECK(a2.dim() == 2 && a2.size(0) >= 1 && a2.size(1) == A * D, "channel_delta_prep: a2 [rank, heads * dim]");
+  const int64_t T = proj.size(0), N = proj.size(1), C = 2 * G * D + A * E, rank = a2.size(0);
+  chk_f32(out, "out", 4 * T * A * D); chk_f32(vout, "v", T * A * E);
+  TORCH_CHECK(q_off >= 0 && q_off + C <= N && b_off >= 0 && b_off + A <= N && a_off >= 0 && a_off + rank <= N,
+              "channel_delta_prep: columns");
+  chk_f32(cw, "conv_w");
+  TORCH_CHECK(cw.dim() == 2 && cw.size(0) == C && cw.size(1) >= 1 && cw.size(1) <= 16,
+              "channel_delta_prep: conv_w [C, taps <= 16]");
+  const int taps = (int)cw.size(1);
+  chk_f32(state, "state");
+  TORCH_CHECK(state.dim() == 3 && state.size(2) == C && state.size(1) == std::max(taps - 1, 1),
+              "channel_delta_prep: state [slots, taps - 1, C]");
+  chk_f32(neg_rate, "neg_rate", A); chk_f32(dt_bias, "dt_bias", A * D);
+  chk_rows(row_seq, positions, start_pos, slots, T, state.size(0));
+  TORCH_CHECK(!shift_state || start_pos.numel() == T, "channel_delta_prep: shift_state needs one row per sequence");
+  int rc = launch_channel_delta(out.data_ptr<float>(), vout.data_ptr<float>(), proj.data_ptr(), (int)N, (int)q_off,
+                                (int)b_off, (int)a_off, (int)rank, a2.data_ptr<float>(), cw.data_ptr<float>(),
+                                state.data_ptr<float>(), neg_rate.data_ptr<float>(), dt_bias.data_ptr<float>(), (int)T,
+                                (int)A, (int)G, (int)D, (int)E, taps, (int)state.size(1), row_seq.data_ptr<int>(),
+                                positions.data_ptr<int64_t>(), start_pos.data_ptr<int>(), slots.data_ptr<int>(),
+                                shift_state, is_bf(proj), cur());
+  TORCH_CHECK(rc == 0, "channel_delta_prep: a row does not fit the LDS (code ", rc, ")");
+}
+
+// out [T, 3 A D + A (E + 1)], gates [3, T, A]; proj columns q_off, k_off (A D), v_off (A E), i_off, f_off (A)
+void memory_prep(torch::Tensor out, torch::Tensor gates, torch::Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off,
+                 int64_t i_off, int64_t f_off, torch::Tensor ib, torch::Tensor fb, double cap, torch::Tensor gmax,
+                 torch::Tensor cu_q, torch::Tensor start_pos, torch::Tensor slots, double q_scale, int64_t A, int64_t D,
+                 int64_t E, bool step) {
+  chk_act(proj, "proj");
+  TORCH_CHECK(proj.dim() == 2 && A >= 1 && D >= 1 && E >= 1 && cap > 0, "memory_prep: sizes");
+  const int64_t T = proj.size(0), N = proj.size(1), S = cu_q.numel() - 1;
+  chk_f32(out, "out", T * (3 * A * D + A * (E + 1))); chk_f32(gates, "gates", 3 * T * A);
+  TORCH_CHECK(q_off >= 0 && q_off + A * D <= N && k_off >= 0 && k_off + A * D <= N && v_off >= 0 && v_off + A * E <= N &&
+              i_off >= 0 && i_off + A <= N && f_off >= 0 && f_off + A <= N, "memory_prep: columns");
+  chk_f32(ib, "i_b", A); chk_f32(fb, "f_b", A); chk_f32(gmax, "gmax");
+  TORCH_CHECK(gmax.dim() == 2 && gmax.size(1) == A, "memory_prep: gmax [slots, heads]");
+  chk_i32(cu_q, "cu_q"); chk_i32(start_pos, "start_pos", S); chk_i32(slots, "slots", S);
+  TORCH_CHECK(!step || S == T, "memory_prep: step needs one row per sequence");
+  int rc = launch_memory_prep(out.data_ptr<float>(), gates.data_ptr<float>(), proj.data_ptr(), (int)N, (int)q_off, (int)k_off,
+                              (int)v_off, (int)i_off, (int)f_off, ib.data_ptr<float>(), fb.data_ptr<float>(), (float)cap,
+                              gmax.data_ptr<float>(), cu_q.data_ptr<int>(), start_pos.data_ptr<int>(),
+                              slots.data_ptr<int>(), (float)q_scale, (int)S, (int)T, (int)A, (int)D, (int)E, step,
+                              is_bf(proj), cur());
+  TORCH_CHECK(rc == 0, "memory_prep: too many heads (code ", rc, ")");
+}
+
 // an fp32 row stream [T, >= A * n] with unit column stride: pointer and row stride
 const float* stream_of(const OptT& t, const char* name, int64_t T, int64_t n, int& stride) {
   stride = 0;
@@ -768,17 +878,24 @@ void gla_prep(torch::Tensor out, torch::Tensor proj, int64_t q_off, int64_t k_of
 }
 
 void head_norm_gate(torch::Tensor out, int64_t out_off, torch::Tensor o, torch::Tensor w, int64_t span, torch::Tensor gate,
-                    int64_t gate_off, int64_t act, double eps, double scale) {
+                    int64_t gate_off, int64_t act, double eps, double scale, OptT floors) {
   chk_act(out, "out"); chk_f32(o, "o"); chk_act(gate, "gate"); chk_f32(w, "norm_w");
   TORCH_CHECK(out.dim() == 2 && o.dim() == 2 && gate.dim() == 2 && out.size(0) == o.size(0) && gate.size(0) == o.size(0),
               "head_norm_gate: ranks");
-  const int64_t T = o.size(0), C = o.size(1);
+  // floors [T, heads]: o has one more entry per head (n . q of a matrix memory)
+  const int64_t T = o.size(0), heads = floors.has_value() && floors->dim() == 2 ? floors->size(1) : 0;
+  const int64_t C = floors.has_value() ? heads * span : o.size(1);
+  if (floors.has_value()) {
+    chk_f32(*floors, "floors", T * heads);
+    TORCH_CHECK(heads >= 1 && o.size(1) == heads * (span + 1), "head_norm_gate: o [T, heads * (span + 1)] with floors");
+  }
   TORCH_CHECK(span >= 1 && C % span == 0 && (w.numel() == C || w.numel() == span), "head_norm_gate: span / weight");
   TORCH_CHECK(out_off >= 0 && out_off + C <= out.size(1) && gate_off >= 0 && gate_off + C <= gate.size(1),
               "head_norm_gate: columns");
   launch_head_norm_gate(out.data_ptr(), (int)out.size(1), (int)out_off, o.data_ptr<float>(), w.data_ptr<float>(),
                         (int)w.numel(), (int)span, gate.data_ptr(), (int)gate.size(1), (int)gate_off, (int)act, (float)eps,
-                        (float)scale, (int)T, (int)C, is_bf(out), is_bf(gate), cur());
+                        (float)scale, (int)T, (int)C, floors.has_value() ? floors->data_ptr<float>() : nullptr, is_bf(out),
+                        is_bf(gate), cur());
 }
 
 }  // namespace
@@ -792,13 +909,16 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("qk_prep", &qk_prep, py::arg("q"), py::arg("proj"), py::arg("q_off"), py::arg("k_off"), py::arg("v_off"),
         py::arg("v_from_k"), py::arg("inv_freq"), py::arg("eps"), py::arg("positions"), py::arg("kc"), py::arg("vc"),
         py::arg("slot_mapping"), py::arg("layout"), py::arg("q_scale"), py::arg("q_w") = py::none(),
-        py::arg("k_w") = py::none(), py::arg("v_norm") = false, py::arg("qt_coef") = 0.0, py::arg("qt_every") = 0);
+        py::arg("k_w") = py::none(), py::arg("v_norm") = false, py::arg("qt_coef") = 0.0, py::arg("qt_every") = 0,
+        py::arg("halves") = false, py::arg("q_b") = py::none(), py::arg("k_b") = py::none(), py::arg("v_b") = py::none(),
+        py::arg("mix") = py::none(), py::arg("mix_off") = 0, py::arg("mix_b") = py::none(), py::arg("mix_w") = 0.0);
   m.def("gqa_key_tile", [](int64_t Dk, int64_t Dv) { return gqa_key_tile((int)Dk, (int)Dv); });
   m.def("gqa_attention", &gqa_attention, py::arg("out"), py::arg("q"), py::arg("kc"), py::arg("vc"),
         py::arg("block_tables"), py::arg("cu_q"), py::arg("start_pos"), py::arg("tiles"), py::arg("temp"), py::arg("scale"),
         py::arg("sink"), py::arg("rows"), py::arg("num_splits"), py::arg("part_o"), py::arg("part_ml"),
         py::arg("window") = 0, py::arg("slopes") = py::none(), py::arg("gate") = py::none(), py::arg("gate_off") = 0,
-        py::arg("layout") = 0, py::arg("softcap") = 0.0, py::arg("out_scale") = 1.0, py::arg("out_off") = 0);
+        py::arg("layout") = 0, py::arg("softcap") = 0.0, py::arg("out_scale") = 1.0, py::arg("out_off") = 0,
+        py::arg("keep") = 0, py::arg("chunk") = 0, py::arg("sinks") = py::none(), py::arg("gate_heads") = false);
   m.def("mingru_scan", &mingru_scan, py::arg("out"), py::arg("proj"), py::arg("z_off"), py::arg("x_off"), py::arg("g_off"),
         py::arg("bz"), py::arg("bx"), py::arg("state"), py::arg("cu_q"), py::arg("start_pos"), py::arg("slots"),
         py::arg("chunks") = py::none(), py::arg("seq_chunk0") = py::none(), py::arg("ws") = py::none());
@@ -808,6 +928,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("groups") = 1);
   m.def("add_layer_norm", &add_layer_norm, py::arg("out"), py::arg("x"), py::arg("y"), py::arg("s"), py::arg("w"),
         py::arg("b"), py::arg("eps"), py::arg("wt") = py::none(), py::arg("place") = py::none());
+  m.def("add_tanh_norm", &add_tanh_norm);
   m.def("moe_tile_rows", &moe_tile_rows);
   m.def("moe_sort", &moe_sort);
   m.def("moe_gemm", &moe_gemm);
@@ -834,10 +955,14 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("relu2", &relu2);
   m.def("removal_prep", &removal_prep);
   m.def("delta_prep", &delta_prep);
+  m.def("channel_delta_prep", &channel_delta_prep);
+  m.def("memory_prep", &memory_prep);
   m.def("gla_prep", &gla_prep);
   m.def("state_scan", &state_scan, py::arg("out"), py::arg("q"), py::arg("k"), py::arg("v"), py::arg("w"), py::arg("a"),
         py::arg("b"), py::arg("decay"), py::arg("state"), py::arg("cu_q"), py::arg("start_pos"), py::arg("slots"),
         py::arg("heads"), py::arg("dim"), py::arg("vdim"), py::arg("chunks") = py::none(),
         py::arg("seq_chunk0") = py::none(), py::arg("ws") = py::none(), py::arg("chunk_rows") = 0);
-  m.def("head_norm_gate", &head_norm_gate);
+  m.def("head_norm_gate", &head_norm_gate, py::arg("out"), py::arg("out_off"), py::arg("o"), py::arg("w"), py::arg("span"),
+        py::arg("gate"), py::arg("gate_off"), py::arg("act"), py::arg("eps"), py::arg("scale"),
+        py::arg("floors") = py::none());
 }

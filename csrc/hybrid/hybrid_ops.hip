@@ -11,14 +11,17 @@
 //   shift_state       state[slot] = normed last row of every span
 //   qk_prep           rotary pairs (2i, 2i + 1), per-head x / rms(x) (* a weight per channel; queries
 //                     * 1 + coef ln(floor((p + 1) / every) + 1)); values optionally / rms(v);
-//                     keys, values -> paged cache
+//                     keys, values -> paged cache. Optionally: pairs (i, i + dims / 2), biases ahead of
+//                     everything else, values mixed with another tensor's
 //   mingru_scan       z = sigmoid(.), c = u + 1/2 | sigmoid(u); S = (1 - z) S + z c; out = S silu(g)
 //   dual_norm_add     x += (a / rms(a) * wa + b / rms(b) * wb) / 2
 //   add_norm          x += y ; out = x / rms(x) * w
 //   add_layer_norm    x += y * s (s: a number per channel) ; out = (x - mean) / sqrt(var + eps) * w + b
 //                     (or y = sum_k wt[t, k] * rows[place of (t, k)]: a mixture of experts' output, combined here)
+//   add_tanh_norm     x += y ; out = tanh(alpha x) * w + b
 //   limited_glu       g = min(gate, L), u = clamp(up, -L, L); g * sigmoid(1.702 g) * (u + 1)
 #include "../common.h"
+#include "hybrid_args.h"
 
 namespace {
 
@@ -131,7 +134,7 @@ __global__ void __launch_bounds__(1024) qk_prep_kernel(
     const float* __restrict__ inv_freq, int rot_dims, float eps, const int64_t* __restrict__ positions,
     T* __restrict__ kc, T* __restrict__ vc, const int64_t* __restrict__ slot_mapping, int H, int G, int Dk, int Dv,
     int BS, int layout, const float* __restrict__ q_scale, const float* __restrict__ q_w,
-    const float* __restrict__ k_w, int v_norm, float qt_coef, int qt_every) {
+    const float* __restrict__ k_w, int v_norm, float qt_coef, int qt_every, QkExtra ex) {
   __shared__ float cs_tab[256];      // (cos, sin) of the row's angles, once for all its heads
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
   const float pos = (float)positions[t];
@@ -149,6 +152,8 @@ __global__ void __launch_bounds__(1024) qk_prep_kernel(
   for (int u = wave; u < H + G; u += nw) {
     const bool is_q = u < H;
     const T* src = row + (is_q ? q_off + u * Dk : k_off + (u - H) * Dk);
+    const float* bias = is_q ? (ex.q_b ? ex.q_b + u * Dk : nullptr) : (ex.k_b ? ex.k_b + (u - H) * Dk : nullptr);
+    const int half = rot_dims >> 1;
     float val[4];
     float ss = 0.f;
 #pragma unroll
@@ -156,12 +161,15 @@ __global__ void __launch_bounds__(1024) qk_prep_kernel(
       const int d = lane + 64 * j;
       float r = 0.f;
       if (d < Dk) {
-        const float a = DT<T>::load(src + d);
+        const float a = DT<T>::load(src + d) + (bias ? bias[d] : 0.f);
         r = a;
         if (d < rot_dims) {
-          const float b = DT<T>::load(src + (d ^ 1));
-          const float cs = cs_tab[d & ~1], sn = cs_tab[d | 1];
-          r = (d & 1) ? a * cs + b * sn : a * cs - b * sn;
+          // the pair's other entry, the pair's number, and whether d is its second entry
+          const int o = ex.halves ? (d < half ? d + half : d - half) : d ^ 1;
+          const int pi = ex.halves ? (d < half ? d : d - half) : d >> 1;
+          const float b = DT<T>::load(src + o) + (bias ? bias[o] : 0.f);
+          const float cs = cs_tab[2 * pi], sn = cs_tab[2 * pi + 1];
+          r = d > o ? a * cs + b * sn : a * cs - b * sn;
         }
       }
       val[j] = r;
@@ -194,6 +202,13 @@ __global__ void __launch_bounds__(1024) qk_prep_kernel(
         const float kv = inv_rms(rt::wave_sum(sv), Dv, eps);
         for (int d = lane; d < Dv; d += 64)
           DT<T>::store(vd + (layout ? (size_t)d * BS + off : (size_t)off * Dv + d), DT<T>::load(vs + d) * kv);
+      } else if (ex.v_b || ex.mix) {                     // biased values, mixed with the ones given
+        const T* ms = ex.mix ? static_cast<const T*>(ex.mix) + (size_t)t * ex.mix_stride + g * Dv : nullptr;
+        for (int d = lane; d < Dv; d += 64) {
+          float a = DT<T>::load(vs + d) + (ex.v_b ? ex.v_b[g * Dv + d] : 0.f);
+          if (ms) a = (1.0f - ex.mix_w) * a + ex.mix_w * (DT<T>::load(ms + d) + (ex.mix_b ? ex.mix_b[g * Dv + d] : 0.f));
+          DT<T>::store(vd + (layout ? (size_t)d * BS + off : (size_t)off * Dv + d), a);
+        }
       } else if (layout) for (int d = lane; d < Dv; d += 64) vd[(size_t)d * BS + off] = vs[d];
       else for (int d = lane; d < Dv; d += 64) vd[(size_t)off * Dv + d] = vs[d];
     }
@@ -455,6 +470,31 @@ __global__ void __launch_bounds__(1024) add_layer_norm_kernel(OT* __restrict__ o
   }
 }
 
+// no reduction: entry by entry, V neighbouring entries per lane
+template <typename OT, typename YT, int V>
+__global__ void __launch_bounds__(256) add_tanh_norm_kernel(OT* __restrict__ out, float* __restrict__ x,
+                                                            const YT* __restrict__ y, float alpha,
+                                                            const float* __restrict__ w, const float* __restrict__ b,
+                                                            int64_t groups, int W) {
+  const int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x);
+  if (i >= groups) return;
+  const int c = (int)((i * V) % W);
+  float v[V], wv[V], bv[V], o[V];
+  load_v<float, V>(v, x + i * V);
+  load_v<float, V>(wv, w + c);
+  load_v<float, V>(bv, b + c);
+  if (y) {
+    float a[V];
+    load_v<YT, V>(a, y + i * V);
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] += a[j];
+    store_v<float, V>(x + i * V, v);
+  }
+#pragma unroll
+  for (int j = 0; j < V; ++j) o[j] = tanhf(alpha * v[j]) * wv[j] + bv[j];
+  store_v<OT, V>(out + i * V, o);
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256) limited_glu_kernel(T* __restrict__ out, const T* __restrict__ gu, int64_t rows,
                                                           int F, float limit) {
@@ -525,7 +565,7 @@ void launch_qk_prep(void* q, const void* proj, int stride, int q_off, int k_off,
                     const float* inv_freq, int rot_dims, float eps, const int64_t* positions, void* kc, void* vc,
                     const int64_t* slot_mapping, int T, int H, int G, int Dk, int Dv, int BS, bool bf, int layout,
                     const float* q_scale, const float* q_w, const float* k_w, bool v_norm, float qt_coef, int qt_every,
-                    hipStream_t stream) {
+                    const QkExtra& ex, hipStream_t stream) {
   if (T <= 0) return;
   // one wave per head unit, up to 16 waves a row: a decode step's few rows spread over whole workgroups
   const int th = T > 64 ? 256 : 64 * (H + G < 4 ? 4 : H + G > 16 ? 16 : H + G);
@@ -533,12 +573,12 @@ void launch_qk_prep(void* q, const void* proj, int stride, int q_off, int k_off,
     qk_prep_kernel<uint16_t><<<T, th, 0, stream>>>((uint16_t*)q, (const uint16_t*)proj, stride, q_off, k_off, v_off,
                                                     v_from_k, inv_freq, rot_dims, eps, positions, (uint16_t*)kc,
                                                     (uint16_t*)vc, slot_mapping, H, G, Dk, Dv, BS, layout, q_scale,
-                                                    q_w, k_w, v_norm ? 1 : 0, qt_coef, qt_every);
+                                                    q_w, k_w, v_norm ? 1 : 0, qt_coef, qt_every, ex);
   else
     qk_prep_kernel<float><<<T, th, 0, stream>>>((float*)q, (const float*)proj, stride, q_off, k_off, v_off, v_from_k,
                                                  inv_freq, rot_dims, eps, positions, (float*)kc, (float*)vc,
                                                  slot_mapping, H, G, Dk, Dv, BS, layout, q_scale, q_w, k_w,
-                                                 v_norm ? 1 : 0, qt_coef, qt_every);
+                                                 v_norm ? 1 : 0, qt_coef, qt_every, ex);
 }
 
 void launch_mingru_scan(void* out, const void* proj, int stride, int z_off, int x_off, int g_off, int width,
@@ -626,6 +666,28 @@ void launch_add_layer_norm(void* out, float* x, const void* y, const float* s, c
   }
 #undef RT_AL3
 #undef RT_AL
+}
+
+void launch_add_tanh_norm(void* out, float* x, const void* y, float alpha, const float* w, const float* b, int T, int W,
+                          bool out_bf, bool y_bf, hipStream_t stream) {
+  if (T <= 0) return;
+  auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = W % 4 == 0 && al(out) && al(x) && al(y) && al(w) && al(b);
+  const int64_t groups = (int64_t)T * W / (vec ? 4 : 1);
+  const int th = groups >= 256 * 256 ? 256 : 64;
+#define RT_AT(OT, YT)                                                                                                  \
+  do {                                                                                                                 \
+    if (vec) add_tanh_norm_kernel<OT, YT, 4><<<(int)((groups + th - 1) / th), th, 0, stream>>>((OT*)out, x, (const YT*)y, \
+                                                                                           alpha, w, b, groups, W);    \
+    else add_tanh_norm_kernel<OT, YT, 1><<<(int)((groups + th - 1) / th), th, 0, stream>>>((OT*)out, x, (const YT*)y,  \
+                                                                                           alpha, w, b, groups, W);    \
+  } while (0)
+  if (out_bf) {
+    if (y_bf) RT_AT(uint16_t, uint16_t); else RT_AT(uint16_t, float);
+  } else {
+    if (y_bf) RT_AT(float, uint16_t); else RT_AT(float, float);
+  }
+#undef RT_AT
 }
 
 void launch_limited_glu(void* out, const void* gu, int64_t rows, int F, float limit, bool bf, hipStream_t stream) {

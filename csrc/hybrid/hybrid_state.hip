@@ -15,7 +15,11 @@
 //   delta_prep       short convolutions + silu, unit q / k, step size and decay of a gated delta rule
 //   gla_prep         scaled q, k, v and the decay sigmoid(low-rank path + bias)^(1 / tau) of a gated
 //                    linear attention
-//   head_norm_gate   per-head or whole-row RMS norm, weight, sigmoid / silu gate, scale
+//   channel_delta    as delta_prep, with one decay per head and key channel from a low-rank path
+//   memory_gates     log input / forget gates of a matrix memory and their running maximum over a span
+//   memory_prep      scaled q, weighted k, decay, v (and the column of ones that carries n)
+//   head_norm_gate   per-head or whole-row RMS norm, weight, sigmoid / silu gate, scale; optionally a
+//                    matrix memory's read-out, divided by max(|n . q|, exp(-m)) + 1e-6 first
 //   relu2            relu(a)^2
 #include "../common.h"
 
@@ -278,6 +282,21 @@ __global__ void __launch_bounds__(kThreads) relu2_kernel(T* __restrict__ out, co
   DT<T>::store(out + i, v * v);
 }
 
+// bf16, a multiple of 8 entries: 16-byte loads and stores
+__global__ void __launch_bounds__(kThreads) relu2_8_kernel(uint16_t* __restrict__ out, const uint16_t* __restrict__ a,
+                                                           int64_t groups) {
+  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= groups) return;
+  const rt::short8 v = *reinterpret_cast<const rt::short8*>(a + i * 8);
+  rt::short8 o;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const float f = fmaxf(rt::bf2f((uint16_t)v[j]), 0.f);
+    o[j] = (short)rt::f2bf(f * f);
+  }
+  *reinterpret_cast<rt::short8*>(out + i * 8) = o;
+}
+
 // out [6][T][A * D] = r, k, v, w, a * u, u; one wave per head
 template <typename T>
 __global__ void __launch_bounds__(kThreads) removal_prep_kernel(
@@ -417,17 +436,207 @@ __global__ void __launch_bounds__(1024) gla_prep_kernel(float* __restrict__ out,
       out[(size_t)(t0 + r) * os + 3 * (size_t)n + c] = DT<T>::load(proj + (size_t)(t0 + r) * stride + v_off + c);
 }
 
-// o [T, C] fp32: segments of `span` entries are divided by their RMS; wmod = entries of the weight
+RT_DEVICE float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+
+// out [4][T][n] = q, beta k, g, g k per value head (n = A * D), vout [T][A * E]; a2 [rank][n]. ROWS rows per
+// workgroup share a pass over a2. dynamic LDS: low [ROWS][rank], dec [ROWS][n], z [C], unit factors [2 G].
+template <typename T, int ROWS>
+__global__ void __launch_bounds__(1024) channel_delta_kernel(
+    float* __restrict__ out, float* __restrict__ vout, const T* __restrict__ proj, int stride, int q_off, int b_off,
+    int a_off, int rank, const float* __restrict__ a2, const float* __restrict__ cw, float* __restrict__ state,
+    const float* __restrict__ neg_rate, const float* __restrict__ dt_bias, int Tn, int A, int G, int D, int E, int taps,
+    int keep, const int* __restrict__ row_seq, const int64_t* __restrict__ positions, const int* __restrict__ start_pos,
+    const int* __restrict__ slots, int shift_state) {
+  extern __shared__ float lds[];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+  const int n = A * D, C = 2 * G * D + A * E, rep = A / G;
+  float* low = lds;
+  float* dec = low + ROWS * rank;
+  float* z = dec + ROWS * n;
+  float* unit = z + C;
+  const int t0 = blockIdx.x * ROWS;
+  const int rows = min(ROWS, Tn - t0);
+  for (int i = threadIdx.x; i < ROWS * rank; i += blockDim.x) {
+    const int r = i / rank;
+    low[i] = r < rows ? DT<T>::load(proj + (size_t)(t0 + r) * stride + a_off + (i - r * rank)) : 0.f;
+  }
+  __syncthreads();
+  for (int c = threadIdx.x; c < n; c += blockDim.x) {
+    float x[ROWS];
+    const float bc = dt_bias[c];
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) x[r] = bc;
+#pragma unroll 8
+    for (int j = 0; j < rank; ++j) {
+      const float wv = a2[(size_t)j * n + c];
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r) x[r] += wv * low[r * rank + j];
+    }
+    const float nr = neg_rate[c / D];
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) dec[r * n + c] = expf(nr * softplus(x[r]));
+  }
+  const size_t plane = (size_t)Tn * n;
+  const float qs = 1.0f / sqrtf((float)D);
+  for (int r = 0; r < rows; ++r) {
+    const int t = t0 + r;
+    const int s = row_seq[t];
+    const int64_t pos = positions[t];
+    const int local = (int)(pos - start_pos[s]);
+    float* st = state + (size_t)slots[s] * keep * C;
+    const T* pr = proj + (size_t)t * stride;
+    __syncthreads();      // the previous row's readers of z and unit are done (and dec is written)
+    for (int c = threadIdx.x; c < C; c += blockDim.x) {
+      float acc = 0.f, v0 = 0.f;
+      for (int k = 0; k < taps; ++k) {
+        const Tap tp = tap_of(k, t, local, pos, taps);
+        float v = 0.f;
+        if (tp.kind == 1) v = DT<T>::load(proj + tp.at * stride + q_off + c);
+        else if (tp.kind == 2) v = st[tp.at * C + c];
+        if (k == 0) v0 = v;
+        acc += cw[(size_t)c * taps + (taps - 1 - k)] * v;
+      }
+      const float sv = silu(acc);
+      z[c] = sv;
+      if (c >= 2 * G * D) vout[(size_t)t * A * E + (c - 2 * G * D)] = sv;
+      if (shift_state && taps > 1) {
+        for (int i = 0; i + 2 < taps; ++i)
+          st[(size_t)i * C + c] = (pos - (taps - 2 - i) >= 0) ? st[(size_t)(i + 1) * C + c] : 0.f;
+        st[(size_t)(taps - 2) * C + c] = v0;
+      }
+    }
+    __syncthreads();
+    for (int j = wave; j < 2 * G; j += nw) {     // q heads, then k heads
+      float ss = 0.f;
+      for (int d = lane; d < D; d += 64) ss += z[j * D + d] * z[j * D + d];
+      const float iv = 1.0f / sqrtf(rt::wave_sum(ss) + 1e-6f);
+      if (lane == 0) unit[j] = iv;
+    }
+    __syncthreads();
+    for (int c = threadIdx.x; c < n; c += blockDim.x) {
+      const int a = c / D, g = a / rep, d = c - a * D;
+      const float beta = 1.0f / (1.0f + expf(-DT<T>::load(pr + b_off + a)));
+      const float kv = z[(G + g) * D + d] * unit[G + g], gd = dec[r * n + c];
+      float* o = out + (size_t)t * n + c;
+      o[0] = z[g * D + d] * unit[g] * qs;
+      o[plane] = beta * kv;
+      o[2 * plane] = gd;
+      o[3 * plane] = gd * kv;
+    }
+  }
+}
+
+// the gates of one (token, head): the capped log input gate and the log of the capped forget gate
+template <typename T>
+RT_DEVICE void memory_gate(const T* pr, int i_off, int f_off, int a, const float* ib, const float* fb, float cap, float& gi,
+                           float& gf) {
+  gi = cap * tanhf((DT<T>::load(pr + i_off + a) + ib[a]) / cap);
+  gf = -softplus(-cap * tanhf((DT<T>::load(pr + f_off + a) + fb[a]) / cap));
+}
+
+// gates [3][T][A] = exp(f_t + m_(t-1) - m_t), exp(i_t - m_t), exp(-m_t) with m_t = max(f_t + m_(t-1), i_t), m
+// from gmax[slot] (0 at position 0). One wave per (sequence, head): 64 tokens at a time by a scan over
+// the maps m -> max(m + a, b), of which two in a row are (a1 + a2, max(b1 + a2, b2)).
+template <typename T>
+__global__ void __launch_bounds__(64) memory_gates_kernel(float* __restrict__ gates, const T* __restrict__ proj, int stride,
+                                                          int i_off, int f_off, const float* __restrict__ ib,
+                                                          const float* __restrict__ fb, float cap, float* __restrict__ gmax,
+                                                          const int* __restrict__ cu_q, const int* __restrict__ start_pos,
+                                                          const int* __restrict__ slots, int Tn, int A) {
+  const int s = blockIdx.x, a = blockIdx.y, lane = threadIdx.x;
+  const int r0 = cu_q[s], n = cu_q[s + 1] - r0;
+  if (n <= 0) return;
+  float* mp = gmax + (size_t)slots[s] * A + a;
+  float m = start_pos[s] > 0 ? *mp : 0.f;
+  const size_t plane = (size_t)Tn * A;
+  for (int c0 = 0; c0 < n; c0 += 64) {
+    const int t = c0 + lane;
+    float gi = -INFINITY, gf = 0.f;
+    if (t < n) memory_gate(proj + (size_t)(r0 + t) * stride, i_off, f_off, a, ib, fb, cap, gi, gf);
+    float sa = gf, sb = gi;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float pa = __shfl_up(sa, o, 64), pb = __shfl_up(sb, o, 64);
+      if (lane >= o) {
+        sb = fmaxf(pb + sa, sb);
+        sa = pa + sa;
+      }
+    }
+    const float mt = fmaxf(m + sa, sb);
+    float before = __shfl_up(mt, 1, 64);
+    if (lane == 0) before = m;
+    if (t < n) {
+      float* g = gates + (size_t)(r0 + t) * A + a;
+      g[0] = expf(gf + before - mt);
+      g[plane] = expf(gi - mt);
+      g[2 * plane] = expf(-mt);
+    }
+    m = __shfl(mt, min(63, n - 1 - c0), 64);
+  }
+  if (lane == 0) *mp = m;
+}
+
+// out [T][3 n + A (E + 1)] = q * q_scale, weight * k, decay (n = A * D columns each), per head v and a one.
+// gates as written by memory_gates; STEP: one row per sequence, the gates are formed here from gmax
+template <typename T, bool STEP>
+__global__ void __launch_bounds__(1024) memory_prep_kernel(float* __restrict__ out, float* __restrict__ gates,
+                                                           const T* __restrict__ proj, int stride, int q_off, int k_off,
+                                                           int v_off, int i_off, int f_off, const float* __restrict__ ib,
+                                                           const float* __restrict__ fb, float cap,
+                                                           float* __restrict__ gmax, const int* __restrict__ start_pos,
+                                                           const int* __restrict__ slots, float q_scale, int Tn, int A, int D,
+                                                           int E) {
+  extern __shared__ float lds[];      // [2][A]: decay, weight
+  const int t = blockIdx.x;
+  const T* pr = proj + (size_t)t * stride;
+  const size_t plane = (size_t)Tn * A;
+  const int n = A * D;
+  for (int a = threadIdx.x; a < A; a += blockDim.x) {
+    float* g = gates + (size_t)t * A + a;
+    if (STEP) {
+      float* mp = gmax + (size_t)slots[t] * A + a;
+      const float m = start_pos[t] > 0 ? *mp : 0.f;
+      float gi, gf;
+      memory_gate(pr, i_off, f_off, a, ib, fb, cap, gi, gf);
+      const float mt = fmaxf(gf + m, gi);
+      *mp = mt;
+      lds[a] = expf(gf + m - mt);
+      lds[A + a] = expf(gi - mt);
+      g[2 * plane] = expf(-mt);
+    } else {
+      lds[a] = g[0];
+      lds[A + a] = g[plane];
+    }
+  }
+  __syncthreads();
+  float* o = out + (size_t)t * (3 * (size_t)n + (size_t)A * (E + 1));
+  for (int c = threadIdx.x; c < n; c += blockDim.x) {
+    const int a = c / D;
+    o[c] = DT<T>::load(pr + q_off + c) * q_scale;
+    o[n + c] = DT<T>::load(pr + k_off + c) * lds[A + a];
+    o[2 * (size_t)n + c] = lds[a];
+  }
+  for (int c = threadIdx.x; c < A * (E + 1); c += blockDim.x) {
+    const int a = c / (E + 1), e = c - a * (E + 1);
+    o[3 * (size_t)n + c] = e < E ? DT<T>::load(pr + v_off + a * E + e) : 1.0f;
+  }
+}
+
+// o [T, C] fp32: segments of `span` entries are divided by their RMS; wmod = entries of the weight.
+// floors [T, C / span]: o has one more entry per segment, n . q, and a segment is divided by
+// max(|n . q|, floor) + 1e-6 first.
 template <typename OT, typename GT>
 __global__ void __launch_bounds__(1024) head_norm_gate_kernel(
     OT* __restrict__ out, int out_stride, int out_off, const float* __restrict__ o, const float* __restrict__ w, int wmod,
-    int span, const GT* __restrict__ gate, int gate_stride, int gate_off, int act, float eps, float scale, int C) {
+    int span, const GT* __restrict__ gate, int gate_stride, int gate_off, int act, float eps, float scale, int C,
+    const float* __restrict__ floors) {
   __shared__ float scratch[16];
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
-  const float* orow = o + (size_t)t * C;
+  const int heads = C / span, seg = floors ? span + 1 : span;
+  const float* orow = o + (size_t)t * heads * seg;
   const GT* grow = gate + (size_t)t * gate_stride + gate_off;
   OT* dst = out + (size_t)t * out_stride + out_off;
-  if (span == C) {
+  if (span == C && !floors) {
     float ss = 0.f;
     for (int c = threadIdx.x; c < C; c += blockDim.x) ss += orow[c] * orow[c];
     const float iv = rsqrtf(rt::block_sum(ss, scratch) / C + eps);
@@ -437,14 +646,16 @@ __global__ void __launch_bounds__(1024) head_norm_gate_kernel(
     }
     return;
   }
-  for (int h = wave; h < C / span; h += nw) {
+  for (int h = wave; h < heads; h += nw) {
+    const float* os = orow + h * seg;
+    const float den = floors ? 1.0f / (fmaxf(fabsf(os[span]), floors[(size_t)t * heads + h]) + 1e-6f) : 1.0f;
     float ss = 0.f;
-    for (int d = lane; d < span; d += 64) ss += orow[h * span + d] * orow[h * span + d];
-    const float iv = rsqrtf(rt::wave_sum(ss) / span + eps);
+    for (int d = lane; d < span; d += 64) ss += os[d] * os[d];
+    const float iv = den * rsqrtf(rt::wave_sum(ss) * den * den / span + eps);
     for (int d = lane; d < span; d += 64) {
       const int c = h * span + d;
       const float g = DT<GT>::load(grow + c);
-      DT<OT>::store(dst + c, orow[c] * iv * w[c % wmod] * (act ? silu(g) : sigm(g)) * scale);
+      DT<OT>::store(dst + c, os[d] * iv * w[c % wmod] * (act ? silu(g) : sigm(g)) * scale);
     }
   }
 }
@@ -529,6 +740,12 @@ void launch_silu_cols(float* out, const void* proj, int stride, int off, int n, 
 
 void launch_relu2(void* out, const void* a, int64_t total, bool bf, hipStream_t stream) {
   if (total <= 0) return;
+  if (bf && total % 8 == 0 && ((reinterpret_cast<uintptr_t>(a) | reinterpret_cast<uintptr_t>(out)) & 15) == 0) {
+    const int64_t groups = total / 8;
+    relu2_8_kernel<<<(int)((groups + kThreads - 1) / kThreads), kThreads, 0, stream>>>((uint16_t*)out, (const uint16_t*)a,
+                                                                                      groups);
+    return;
+  }
   const int blocks = (int)((total + kThreads - 1) / kThreads);
   if (bf) relu2_kernel<uint16_t><<<blocks, kThreads, 0, stream>>>((uint16_t*)out, (const uint16_t*)a, total);
   else relu2_kernel<float><<<blocks, kThreads, 0, stream>>>((float*)out, (const float*)a, total);
@@ -589,15 +806,72 @@ int launch_gla_prep(float* out, const void* proj, int stride, int q_off, int k_o
   return 0;
 }
 
+int launch_channel_delta(float* out, float* vout, const void* proj, int stride, int q_off, int b_off, int a_off, int rank,
+                         const float* a2, const float* cw, float* state, const float* neg_rate, const float* dt_bias, int T,
+                         int A, int G, int D, int E, int taps, int keep, const int* row_seq, const int64_t* positions,
+                         const int* start_pos, const int* slots, bool shift_state, bool bf, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (taps > kMaxTaps) return -1;
+  const int C = 2 * G * D + A * E;
+  auto lds_of = [&](int rows) { return sizeof(float) * ((size_t)rows * (rank + A * D) + C + 2 * G); };
+  const int rows = T >= 256 && lds_of(4) <= 80 * 1024 ? 4 : 1;    // many rows: the low-rank factor is read once for four
+  const size_t shm = lds_of(rows);
+  if (shm > 150 * 1024) return -1;
+  const int th = C >= 1024 ? 1024 : C <= 256 ? 256 : (C + 63) / 64 * 64;
+#define RT_CD(TT, R)                                                                                                   \
+  do {                                                                                                                 \
+    auto kern = channel_delta_kernel<TT, R>;                                                                           \
+    if (shm > 48 * 1024 &&                                                                                             \
+        hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm) != hipSuccess)    \
+      return -2;                                                                                                       \
+    kern<<<(T + R - 1) / R, th, shm, stream>>>(out, vout, (const TT*)proj, stride, q_off, b_off, a_off, rank, a2, cw,  \
+                                               state, neg_rate, dt_bias, T, A, G, D, E, taps, keep, row_seq,           \
+                                               positions, start_pos, slots, shift_state ? 1 : 0);                      \
+  } while (0)
+  if (bf) {
+    if (rows == 4) RT_CD(uint16_t, 4); else RT_CD(uint16_t, 1);
+  } else {
+    if (rows == 4) RT_CD(float, 4); else RT_CD(float, 1);
+  }
+#undef RT_CD
+  return 0;
+}
+
+int launch_memory_prep(float* out, float* gates, const void* proj, int stride, int q_off, int k_off, int v_off, int i_off,
+                       int f_off, const float* ib, const float* fb, float cap, float* gmax, const int* cu_q,
+                       const int* start_pos, const int* slots, float q_scale, int S, int T, int A, int D, int E, bool step,
+                       bool bf, hipStream_t stream) {
+  if (T <= 0 || S <= 0) return 0;
+  const size_t shm = sizeof(float) * 2 * (size_t)A;
+  if (shm > 48 * 1024) return -1;
+  const int m = A * (D > E + 1 ? D : E + 1);
+  const int th = m >= 1024 ? 1024 : m <= 64 ? 64 : (m + 63) / 64 * 64;
+#define RT_MP(TT)                                                                                                      \
+  do {                                                                                                                 \
+    if (!step)                                                                                                         \
+      memory_gates_kernel<TT><<<dim3(S, A), 64, 0, stream>>>(gates, (const TT*)proj, stride, i_off, f_off, ib, fb, cap, \
+                                                             gmax, cu_q, start_pos, slots, T, A);                      \
+    if (step) memory_prep_kernel<TT, true><<<T, th, shm, stream>>>(out, gates, (const TT*)proj, stride, q_off, k_off,  \
+                                                                   v_off, i_off, f_off, ib, fb, cap, gmax, start_pos,  \
+                                                                   slots, q_scale, T, A, D, E);                        \
+    else memory_prep_kernel<TT, false><<<T, th, shm, stream>>>(out, gates, (const TT*)proj, stride, q_off, k_off,      \
+                                                               v_off, i_off, f_off, ib, fb, cap, gmax, start_pos,      \
+                                                               slots, q_scale, T, A, D, E);                            \
+  } while (0)
+  if (bf) RT_MP(uint16_t); else RT_MP(float);
+#undef RT_MP
+  return 0;
+}
+
 void launch_head_norm_gate(void* out, int out_stride, int out_off, const float* o, const float* w, int wmod, int span,
                            const void* gate, int gate_stride, int gate_off, int act, float eps, float scale, int T, int C,
-                           bool out_bf, bool gate_bf, hipStream_t stream) {
+                           const float* floors, bool out_bf, bool gate_bf, hipStream_t stream) {
   if (T <= 0) return;
   // a wave per head, up to 16 waves
-  const int th = span == C ? kThreads : C / span >= 16 ? 1024 : C / span * 64;
+  const int th = span == C && !floors ? kThreads : C / span >= 16 ? 1024 : C / span * 64;
 #define RT_HN(OT, GT)                                                                                                  \
   head_norm_gate_kernel<OT, GT><<<T, th, 0, stream>>>((OT*)out, out_stride, out_off, o, w, wmod, span,           \
-                                                            (const GT*)gate, gate_stride, gate_off, act, eps, scale, C)
+                                                            (const GT*)gate, gate_stride, gate_off, act, eps, scale, C, floors)
   if (out_bf) {
     if (gate_bf) RT_HN(uint16_t, uint16_t); else RT_HN(uint16_t, float);
   } else {

@@ -324,11 +324,13 @@ class GroupedKVCache(StatefulPagedCache):
     inputs of the layer's two input convolutions (mixer, feed-forward), oldest first.
     ``short_conv[l]`` = (channels, taps): ``sconv[l]`` ``[n_slots, taps - 1, channels]`` holds the
     last inputs of a short convolution inside the mixer (None for a layer without one).
+    ``gate_heads[l]`` = n: ``gmax[l]`` ``[n_slots, n]`` holds the running maximum of a matrix memory's
+    exponential gates per head (None for a layer without one).
     A sequence at position 0 never reads its slot, so a reused slot needs no clearing."""
 
     def __init__(self, shapes, width: int, rec_widths, num_blocks: int, block_size: int, device,
                  dtype=torch.bfloat16, n_slots: int = 16, matrix_layout=None, shift_layers=None,
-                 canon_taps: int = 0, short_conv=None):
+                 canon_taps: int = 0, short_conv=None, gate_heads=None):
         shapes = [sh if sh is not None else (0, 0, 0) for sh in shapes]
         self.n_layers = len(shapes)
         # per run: the layout of the framework's matrix-core attention kernels (keys chunk-major
@@ -357,6 +359,8 @@ class GroupedKVCache(StatefulPagedCache):
         short_conv = list(short_conv) if short_conv is not None else [None] * len(self.shapes)
         self.sconv = [torch.zeros(n_slots, max(sc[1] - 1, 1), sc[0], dtype=torch.float32, device=device)
                       if sc is not None else None for sc in short_conv]
+        gate_heads = list(gate_heads) if gate_heads is not None else [0] * len(self.shapes)
+        self.gmax = [torch.zeros(n_slots, n, dtype=torch.float32, device=device) if n else None for n in gate_heads]
 
     @staticmethod
     def bytes_per_block(shapes, block_size, dtype_bytes=2) -> int:   # type: ignore[override]
@@ -376,4 +380,4 @@ class GroupedKVCache(StatefulPagedCache):
                 t.index_copy_(0, di, t.index_select(0, si))
 
     def state_tensors(self) -> List[torch.Tensor]:
-        return [t for t in self.shift + self.rec + self.conv + self.sconv if t is not None]
+        return [t for t in self.shift + self.rec + self.conv + self.sconv + self.gmax if t is not None]

@@ -68,7 +68,14 @@ class GroupedAttentionSpec:
     ``q.norm`` / ``k.norm`` of the projection's size), BEFORE the rotation. ``bias``: the query and
     key projections add a bias (tensors ``q.b`` / ``k.b``). ``value_rot``: the value of position j
     is turned by j over all its entries before it is cached (pair m by j * base^(-2m / vdim), the
-    pairs laid out as the key rotation's), and each head's output at position i is turned back by i."""
+    pairs laid out as the key rotation's), and each head's output at position i is turned back by i.
+    ``chunk`` > 0: position i sees only j with j // chunk == i // chunk (chunks are counted from the
+    start of the sequence). ``keep_first`` (with a window): the first that many positions stay
+    visible. ``head_sink``: a learned number per head (tensor ``sink``) joins the softmax denominator
+    as exp(sink). ``v_bias``: the value projection adds a bias too (tensor ``v.b``). ``v_mix``: the
+    cached value is (1 - lambda) v + lambda v_first, lambda the tensor ``vmix`` and v_first the same
+    token's value in the first layer of the stack that has the flag (which keeps its own).
+    ``head_gate``: head h's output is multiplied by sigmoid(W_g h)_h ahead of the output projection."""
     heads: int
     kv_heads: int
     dim: int
@@ -88,6 +95,12 @@ class GroupedAttentionSpec:
     wide_norm: bool = False
     bias: bool = False
     value_rot: Optional[RotarySpec] = None
+    chunk: int = 0
+    keep_first: int = 0
+    head_sink: bool = False
+    v_bias: bool = False
+    v_mix: bool = False
+    head_gate: bool = False
 
     @property
     def group(self) -> int:
@@ -148,12 +161,17 @@ class DeltaSpec:
     of size ``dim``; q, k, v pass a causal convolution of ``conv`` taps per channel and silu, q and
     k are made unit vectors (q also times dim^(-1/2)); one decay g and one step size beta per head
     and token: S <- g S; S <- S + k (beta (v - S^T k))^T; o = S^T q. Each head is divided by its
-    root mean square, weighted (one weight vector shared by the heads), gated by silu of a projection."""
+    root mean square, weighted (one weight vector shared by the heads), gated by silu of a projection.
+    ``channel_decay``: g is one number per head and KEY CHANNEL, exp(-exp(A_log) softplus(W_a2 W_a1 h +
+    dt_bias)), and the output gate is sigmoid of a low-rank path too (W_g2 W_g1 h). ``rank``: the width
+    of both paths (0: whatever the checkpoint's tensors have)."""
     heads: int
     kv_heads: int
     dim: int
     vdim: int
     conv: int
+    channel_decay: bool = False
+    rank: int = 0
 
     @property
     def state_size(self) -> int:
@@ -180,6 +198,25 @@ class GLASpec:
     @property
     def state_size(self) -> int:
         return self.heads * self.dim * self.vdim
+
+
+@dataclass(frozen=True)
+class MatrixMemorySpec:
+    """Matrix memory with exponential gates (mLSTM): per head a ``dim`` x ``vdim`` fp32 state S and a
+    vector n of ``dim`` numbers, a log input gate i = cap tanh((W_i h + b) / cap) and a log forget gate
+    f = logsigmoid(cap tanh((W_f h + b) / cap)) with ``gate_cap`` = cap, under a running maximum m that
+    starts at 0: m_t = max(f_t + m_(t-1), i_t), S_t = exp(f_t + m_(t-1) - m_t) S_(t-1) +
+    exp(i_t - m_t) k_t v_t^T (n_t the same with k alone), o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t))
+    + 1e-6), q times dim^(-1/2). Each head is divided by its root mean square, weighted (a weight per
+    head and channel), gated by sigmoid of a projection. n is kept as one more column of S."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+    @property
+    def state_size(self) -> int:
+        return self.heads * self.dim * (self.vdim + 1)
 
 
 @dataclass(frozen=True)
@@ -295,7 +332,7 @@ class ModelConfig:
 
     def n_params(self) -> int:
         h, f, v, L = self.hidden, self.ffn, self.vocab, self.n_layers
-        if self.arch in ("goganex", "retuvik", "ledinex", "vurizen"):
+        if self.arch in ("goganex", "retuvik", "ledinex", "vurizen", "lizesun"):
             from .weights import layout_for
             n = 0
             for shape, _, _ in layout_for(self).values():
@@ -404,7 +441,7 @@ def parse_mupulorn(d: dict, name: str = "mupulorn") -> ModelConfig:
 def attention_of(ls: LayerSpec):
     """The attention part of a layer's mixer (the left half of a parallel mixer; None for a
     mixer without attention)."""
-    if isinstance(ls.mixer, (WKVSpec, DeltaSpec, GLASpec)):
+    if isinstance(ls.mixer, (WKVSpec, DeltaSpec, GLASpec, MatrixMemorySpec)):
         return None
     return ls.mixer.left if isinstance(ls.mixer, ParallelSpec) else ls.mixer
 
@@ -782,6 +819,89 @@ def vurizen_config(name: str, n_layers: int, width: int, heads: int, dim: int, r
                           "vocab": vocab, "width": width, "max_pos": max_pos}, name)
 
 
+def _lizesun_attention(mx: dict, kind: str, where: str) -> GroupedAttentionSpec:
+    rot, mask = _halves_rotary(mx.get("rot")), mx.get("mask") or {}
+    own = kind == "attention"
+    size, keep = int(mask.get("size") or 0), int(mask.get("keep_first") or 0)
+    a = GroupedAttentionSpec(int(mx["heads"]), int(mx["kv_heads"]), int(mx["dim"]), int(mx["vdim"]), float(mx["scale"]),
+                             None if own else rot, softcap=float(mx.get("softcap") or 0.0) if own else 0.0,
+                             qk_weight=own, bias=own, v_bias=own, head_gate=own, v_mix=own and bool(mx.get("v_mix")),
+                             chunk=size if own else 0, window=0 if own else size, keep_first=0 if own or not size else keep,
+                             head_sink=not own)
+    if a.heads % a.kv_heads:
+        raise ValueError(f"{where}: {a.heads} query heads do not divide over {a.kv_heads} key/value heads")
+    if a.rot is not None and (a.rot.dims > a.dim or a.rot.dims % 2):
+        raise ValueError(f"{where}: rot.dims {a.rot.dims} does not fit dim {a.dim}")
+    if size < 0 or keep < 0:
+        raise ValueError(f"{where}: mask.size {size} / mask.keep_first {keep} out of range")
+    return a
+
+
+def parse_lizesun(d: dict, name: str = "lizesun") -> ModelConfig:
+    """``config.json`` of a Lizesun checkpoint -> :class:`ModelConfig`. Every layer has a mixer of type
+    "channel_delta" (a gated delta rule with a decay per key channel), "attention" (attention inside
+    chunks of the sequence, soft-capped scores, values mixed with the first such layer's) or "parallel"
+    (windowed attention with kept first tokens and a learned sink, beside a matrix memory), and a
+    squared-ReLU feed-forward (or none). A key the file does not have switches its mechanism off (no
+    mask, no soft cap, no mixing, no rotation). The ranks of a channel_delta mixer's low-rank paths are
+    tensor shapes: ``mixer.rank`` is read only by random initialisation."""
+    specs, first = [], None
+    for i, e in enumerate(d["layers"]):
+        where, kind, mx = f"{name}: layer {i}", e["type"], e["mixer"]
+        if kind == "channel_delta":
+            mixer = DeltaSpec(int(mx["heads"]), int(mx["kv_heads"]), int(mx["dim"]), int(mx["vdim"]), int(mx["conv"]),
+                              channel_decay=True, rank=int(mx.get("rank", 0)))
+            if mixer.heads % mixer.kv_heads or not 1 <= mixer.conv <= 16:
+                raise ValueError(f"{where}: heads {mixer.heads} / kv_heads {mixer.kv_heads} / conv {mixer.conv}")
+        elif kind == "attention":
+            mixer = _lizesun_attention(mx, kind, where)
+            if mixer.v_mix:
+                first = first if first is not None else mixer
+                if (first.kv_heads, first.vdim) != (mixer.kv_heads, mixer.vdim):
+                    raise ValueError(f"{where}: values of {mixer.kv_heads} x {mixer.vdim} cannot be mixed with the first "
+                                     f"layer's {first.kv_heads} x {first.vdim}")
+        elif kind == "parallel":
+            rx = mx["right"]
+            mixer = ParallelSpec(_lizesun_attention(mx["left"], kind, where),
+                                 MatrixMemorySpec(int(rx["heads"]), int(rx["dim"]), int(rx["vdim"]), float(rx["gate_cap"])),
+                                 float(mx["left_scale"]), float(mx["right_scale"]))
+        else:
+            raise ValueError(f"{where}: unknown mixer type '{kind}'")
+        mlp = e.get("mlp")
+        if mlp is not None and mlp.get("kind", "dense") != "dense":
+            raise ValueError(f"{where}: unknown feed-forward kind '{mlp['kind']}'")
+        specs.append(LayerSpec(kind, mixer, int(mlp["ff"]) if mlp is not None else 0, "dense", i))
+    atts = [attention_of(s) for s in specs if attention_of(s) is not None]
+    top = max(atts, key=lambda m: m.heads) if atts else None
+    any_mixer = specs[0].mixer
+    return ModelConfig(name, "lizesun", len(specs), int(d["width"]), top.heads if top else any_mixer.heads,
+                       top.kv_heads if top else any_mixer.heads, top.dim if top else any_mixer.dim,
+                       max([s.ff for s in specs] + [0]), int(d["vocab"]), int(d.get("max_pos", 1 << 17)), 0.0,
+                       float(d["norm"]["eps"]), layers=tuple(specs),
+                       embed_scale=float(d.get("embedding", {}).get("scale", 1.0)))
+
+
+def lizesun_config(name: str, n_layers: int, width: int, heads: int, kv_heads: int, dim: int, ff: int, vocab: int,
+                   pattern: Tuple[str, ...] = ("channel_delta", "attention", "parallel", "attention"), rec_heads: int = 0,
+                   rec_dim: int = 64, rec_vdim: int = 0, chunk: int = 2048, window: int = 1024, keep_first: int = 4,
+                   conv: int = 4, rank: int = 64, max_pos: int = 1 << 17) -> ModelConfig:
+    """A Lizesun stack from a few sizes (benchmarks and presets): the mixer types of ``pattern`` in turn."""
+    A, E = rec_heads or max(1, width // rec_dim), rec_vdim or rec_dim
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5}
+    kinds = {
+        "channel_delta": {"heads": A, "kv_heads": A, "dim": rec_dim, "vdim": E, "conv": conv, "rank": rank},
+        "attention": dict(att, mask={"size": chunk}, softcap=30.0, v_mix=True),
+        "parallel": {"left": dict(att, mask={"size": window, "keep_first": keep_first},
+                                  rot={"base": 500000.0, "dims": dim // 2}),
+                     "left_scale": 0.7, "right_scale": 0.7,
+                     "right": {"heads": A, "dim": rec_dim, "vdim": E, "gate_cap": 15.0}},
+    }
+    layers = [{"type": pattern[i % len(pattern)], "mixer": kinds[pattern[i % len(pattern)]],
+               "mlp": {"kind": "dense", "ff": ff} if ff else None} for i in range(n_layers)]
+    return parse_lizesun({"architecture": "Lizesun", "embedding": {"scale": 1.0}, "layers": layers, "norm": {"eps": 1e-5},
+                          "vocab": vocab, "width": width, "max_pos": max_pos}, name)
+
+
 def mupulorn_config(name: str, n_layers: int, width: int, heads: int, dim: int, rot_dim: int, vdim: int,
                     kv_rank: int, q_rank: int, ff: int, vocab: int, taps: int = 4, shared_every: int = 0,
                     rot_base: float = 10000.0, max_pos: int = 1 << 17) -> ModelConfig:
@@ -806,7 +926,7 @@ def mupulorn_config(name: str, n_layers: int, width: int, heads: int, dim: int, 
 # config.json "architecture" -> parser (checkpoint directories name their own model class)
 ARCHITECTURES: Dict[str, Callable[[dict, str], ModelConfig]] = {"Mupulorn": parse_mupulorn, "Goganex": parse_goganex,
                                                                 "Retuvik": parse_retuvik, "Ledinex": parse_ledinex,
-                                                                "Vurizen": parse_vurizen}
+                                                                "Vurizen": parse_vurizen, "Lizesun": parse_lizesun}
 
 PRESETS.update({
     # Mupulorn (latent attention + input convolutions + PolyNorm feed-forward), random-init sizes:
@@ -867,6 +987,19 @@ PRESETS.update({
     "vurizen-0.5b": vurizen_config("vurizen-0.5b", 24, 896, 14, 64, 32, 64, 256, 4864, 151936),      # Qwen2.5-0.5B's sizes
     "vurizen-1b": vurizen_config("vurizen-1b", 16, 2048, 16, 128, 64, 128, 512, 8192, 128256),
     "vurizen-3b": vurizen_config("vurizen-3b", 28, 3072, 24, 128, 64, 128, 256, 8192, 128256),
+})
+
+
+PRESETS.update({
+    # Lizesun (Dynamic Tanh norms, delta rule with a decay per key channel, attention in chunks with mixed
+    # values, windowed attention beside a matrix memory, squared-ReLU feed-forward), random-init sizes: a
+    # test-sized stack and stacks whose layers have the shapes of 0.5B (Qwen2.5) / 1B / 3B-class models
+    # (the two-matrix feed-forward is 1.5x as wide as a gated three-matrix one, so it holds as many weights)
+    "tiny-lizesun": lizesun_config("tiny-lizesun", 4, 128, 4, 2, 32, 192, 32000, rec_heads=2, rec_dim=32, rec_vdim=48,
+                                   chunk=40, window=24, keep_first=3, rank=16),
+    "lizesun-0.5b": lizesun_config("lizesun-0.5b", 24, 896, 14, 2, 64, 7296, 151936),      # Qwen2.5-0.5B's sizes
+    "lizesun-1b": lizesun_config("lizesun-1b", 16, 2048, 32, 8, 64, 12288, 128256),
+    "lizesun-3b": lizesun_config("lizesun-3b", 28, 3072, 24, 8, 128, 12288, 128256, rec_dim=128),
 })
 
 

@@ -101,5 +101,8 @@ def build_model(cfg: ModelConfig, weights, device, dtype=torch.bfloat16, tp: Opt
     if cfg.arch == "vurizen":
         from .vurizen import VurizenModel
         return VurizenModel(cfg, weights, device, dtype, tp)
+    if cfg.arch == "lizesun":
+        from .lizesun import LizesunModel
+        return LizesunModel(cfg, weights, device, dtype, tp)
     from .llama import LlamaModel
     return LlamaModel(cfg, weights, device, dtype, tp)

@@ -332,6 +332,74 @@ def vurizen_layout(cfg: ModelConfig) -> Dict[str, Tuple[Tuple[int, ...], str, Op
     return lay
 
 
+def lizesun_layout(cfg: ModelConfig) -> Dict[str, Tuple[Tuple[int, ...], str, Optional[str]]]:
+    """Checkpoint names and shapes of a Lizesun model (linear weights [out, in]). The ranks of a
+    channel_delta mixer's low-rank paths are whatever ``a1`` / ``a2`` and ``g1`` / ``g2`` have (-1 in the
+    shape) unless the spec names one. Not tensor-parallel: every kind is None."""
+    from .config import DeltaSpec, ParallelSpec
+    W = cfg.hidden
+    lay: Dict[str, Tuple[Tuple[int, ...], str, Optional[str]]] = {}
+
+    def norm(name):
+        lay[name] = ((W,), "ones", None)
+        lay[name + ".b"] = ((W,), "zeros", None)
+        lay[name + ".alpha"] = ((), "ones", None)
+
+    def attention(q, a):
+        for n, rows in (("q", a.heads * a.dim), ("k", a.kv_heads * a.dim), ("v", a.kv_heads * a.vdim)):
+            lay[q + n] = ((rows, W), "normal", None)
+            if a.v_bias if n == "v" else a.bias:
+                lay[q + n + ".b"] = ((rows,), "zeros", None)
+        if a.qk_weight:
+            lay[q + "q.norm"] = ((a.dim,), "ones", None)
+            lay[q + "k.norm"] = ((a.dim,), "ones", None)
+        if a.v_mix:
+            lay[q + "vmix"] = ((), "half", None)
+        if a.head_gate:
+            lay[q + "g"] = ((a.heads, W), "normal", None)
+        if a.head_sink:
+            lay[q + "sink"] = ((a.heads,), "zeros", None)
+        lay[q + "o"] = ((W, a.heads * a.vdim), "normal", None)
+
+    lay["embed"] = ((cfg.vocab, W), "normal", None)
+    norm("final.norm")
+    lay["head"] = ((cfg.vocab, W), "normal", None)
+    for i, ls in enumerate(cfg.layers):
+        p, m = f"l{i}.", ls.mixer
+        q = p + "mix."
+        norm(p + "norm1")
+        if isinstance(m, DeltaSpec):
+            rank = m.rank or -1
+            for n, rows in (("q", m.kv_heads * m.dim), ("k", m.kv_heads * m.dim), ("v", m.heads * m.vdim)):
+                lay[q + n] = ((rows, W), "normal", None)
+                lay[q + n + ".conv"] = ((rows, m.conv), "conv", None)
+            lay[q + "b"] = ((m.heads, W), "normal", None)
+            lay[q + "A_log"] = ((m.heads,), "zeros", None)
+            lay[q + "dt_bias"] = ((m.heads * m.dim,), "zeros", None)
+            lay[q + "norm"] = ((m.vdim,), "ones", None)
+            for n, rows in (("a", m.heads * m.dim), ("g", m.heads * m.vdim)):
+                lay[q + n + "1"] = ((rank, W), "normal", None)
+                lay[q + n + "2"] = ((rows, rank), "normal", None)
+            lay[q + "o"] = ((W, m.heads * m.vdim), "normal", None)
+        elif isinstance(m, ParallelSpec):
+            attention(q + "left.", m.left)
+            r, q = m.right, q + "right."
+            for n, rows in (("q", r.heads * r.dim), ("k", r.heads * r.dim), ("v", r.heads * r.vdim), ("g", r.heads * r.vdim),
+                            ("i", r.heads), ("f", r.heads)):
+                lay[q + n] = ((rows, W), "normal", None)
+            lay[q + "i.b"] = ((r.heads,), "zeros", None)
+            lay[q + "f.b"] = ((r.heads,), "ones", None)
+            lay[q + "norm"] = ((r.heads * r.vdim,), "ones", None)
+            lay[q + "o"] = ((W, r.heads * r.vdim), "normal", None)
+        else:
+            attention(q, m)
+        if ls.ff:
+            norm(p + "norm2")
+            lay[p + "mlp.up"] = ((ls.ff, W), "normal", None)
+            lay[p + "mlp.down"] = ((W, ls.ff), "normal", None)
+    return lay
+
+
 def layout_for(cfg: ModelConfig):
     if cfg.arch == "mupulorn":
         return mupulorn_layout(cfg)
@@ -343,6 +411,8 @@ def layout_for(cfg: ModelConfig):
         return ledinex_layout(cfg)
     if cfg.arch == "vurizen":
         return vurizen_layout(cfg)
+    if cfg.arch == "lizesun":
+        return lizesun_layout(cfg)
     return gpt2_layout(cfg) if cfg.arch == "gpt2" else llama_layout(cfg)
 
 
@@ -502,7 +572,7 @@ def load_safetensors(cfg: ModelConfig, path: str, device, dtype, tp: TPInfo) -> 
         tensors.update(load_file(f, device="cpu"))
     lay = layout_for(cfg)
     out = {}
-    if cfg.arch in ("mupulorn", "goganex", "retuvik", "ledinex", "vurizen"):
+    if cfg.arch in ("mupulorn", "goganex", "retuvik", "ledinex", "vurizen", "lizesun"):
         # the checkpoint's own names; integer tables keep their type, everything else takes `dtype`
         if tp.size > 1:
             raise ValueError(f"{cfg.arch} checkpoints are not tensor-parallel")

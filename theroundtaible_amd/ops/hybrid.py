@@ -4,8 +4,9 @@ equal parts of it), query / key preparation (rotary pairs, per-head unit RMS, op
 query factor that grows with the position, unit-RMS values) with the paged cache write,
 grouped-query attention with an optional softmax sink, per-head temperature, sliding window,
 distance penalty and output gate, the minGRU scan, the wkv scan (linear attention with a per-token
-decay), the two-branch normed residual add, residual add + RMS norm, the clamped gated, xIELU and
-silu-gated feed-forward activations, and a routed mixture of experts.
+decay), the two-branch normed residual add, residual add + RMS norm, layer norm or Dynamic Tanh, the
+inputs and norms of matrix-state recurrences (constant, per-token and per-channel decays, delta rules,
+exponential gates under a running maximum), the clamped gated, xIELU, squared-ReLU and silu-gated feed-forward activations, and a routed mixture of experts.
 
 GPU tensors go to the HIP kernels of ``theroundtaible_amd._C_hybrid`` (``csrc/hybrid/``, built
 in-tree by ``csrc/build.py``; :func:`ensure_built` compiles it on first use in a fresh checkout);
@@ -106,7 +107,7 @@ def rotary_table(rot, device) -> Optional[torch.Tensor]:
 
 def qk_prep(proj, spec, q_off: int, k_off: int, v_off: int, inv_freq, eps, positions, k_cache, v_cache,
             slot_mapping, out_dtype, matrix_layout: bool = False, q_scale=None, q_weight=None,
-            k_weight=None) -> torch.Tensor:
+            k_weight=None, q_bias=None, k_bias=None, v_bias=None, mix=None) -> torch.Tensor:
     """``proj`` [T, N]: columns ``q_off ..`` hold the projected queries (heads x dim), ``k_off ..``
     the keys (kv_heads x dim), ``v_off ..`` the values (kv_heads x vdim; ignored when the values
     are the keys). Rotates the leading ``2 * len(inv_freq)`` entries of every query / key head
@@ -117,21 +118,28 @@ def qk_prep(proj, spec, q_off: int, k_off: int, v_off: int, inv_freq, eps, posit
     ``q_scale`` [heads] fp32 multiplies each query head (a per-head temperature moved into q).
     ``q_weight`` / ``k_weight`` [dim] fp32 multiply the normed queries / keys channel by channel.
     ``spec.q_temp`` = (coef, every): queries of position p times 1 + coef ln(floor((p + 1) / every) + 1);
-    ``spec.value_norm``: every value head is divided by its root mean square before it is cached."""
+    ``spec.value_norm``: every value head is divided by its root mean square before it is cached.
+    ``spec.rot.halves``: entry i turns with entry i + dims / 2 instead. ``q_bias`` [heads * dim],
+    ``k_bias`` [kv_heads * dim], ``v_bias`` [kv_heads * vdim] fp32 join the projections first.
+    ``mix`` = (proj' [T, N'], offset, bias', lam): the cached values are (1 - lam) v + lam v', v' the
+    same rows' values in the columns of another projection."""
+    halves = spec.rot is not None and spec.rot.halves
     if _gpu(proj):
         T = proj.shape[0]
         q = torch.empty(T, spec.heads, spec.dim, dtype=out_dtype, device=proj.device)
         qt = spec.q_temp or (0.0, 0)
+        mp, mo, mb, lam = mix if mix is not None else (None, 0, None, 0.0)
         native().qk_prep(q, proj, int(q_off), int(k_off), int(v_off), bool(spec.value_from_key), inv_freq, float(eps),
                          positions, k_cache, v_cache, slot_mapping, 1 if matrix_layout else 0, q_scale, q_weight, k_weight,
-                         bool(spec.value_norm), float(qt[0]), int(qt[1]))
+                         bool(spec.value_norm), float(qt[0]), int(qt[1]), bool(halves), q_bias, k_bias, v_bias, mp,
+                         int(mo), mb, float(lam))
         return q
     if matrix_layout:
         raise ValueError("qk_prep: the matrix-core cache layout exists on the GPU only")
     if q_scale is not None:
         raise ValueError("qk_prep: q_scale is a GPU-path option (the CPU statement keeps the temperature in the scores)")
     return ref_qk_prep(proj, spec, q_off, k_off, v_off, inv_freq, eps, positions, k_cache, v_cache, slot_mapping,
-                       out_dtype, q_weight, k_weight)
+                       out_dtype, q_weight, k_weight, q_bias, k_bias, v_bias, mix)
 
 
 def rows_per_tile(group: int) -> int:
@@ -164,7 +172,8 @@ def gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale: flo
                   tiles=None, num_splits: int = 1, workspace: Optional[SplitWorkspace] = None,
                   out_dtype=None, window: int = 0, slopes=None, gate=None, gate_off: int = 0,
                   matrix_layout: bool = False, softcap: float = 0.0, out_scale: float = 1.0, out_buf=None,
-                  out_off: int = 0) -> torch.Tensor:
+                  out_off: int = 0, keep_first: int = 0, chunk: int = 0, sinks=None,
+                  gate_heads: bool = False) -> torch.Tensor:
     """Causal attention of the rows ``q`` [T, H, Dk] (span s = rows ``cu_q[s] .. cu_q[s + 1]`` at
     positions ``start_pos[s] ..`` of sequence s) over the paged keys ``k_cache`` [nb, G, BS, Dk]
     and values ``v_cache`` [nb, G, BS, Dv]: score = q . k * scale (* ``temp[h]``), weights
@@ -177,7 +186,10 @@ def gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale: flo
     kernels (see :func:`qk_prep`), e.g. decode rows of a layer whose prompts run on those kernels.
     ``softcap`` > 0: scaled scores become softcap * tanh(score / softcap). ``out_scale`` multiplies
     the result. ``out_buf`` [T, N]: the result goes to its columns ``out_off ..`` (a wider
-    activation buffer that another branch fills beside it) and ``out_buf`` is returned."""
+    activation buffer that another branch fills beside it) and ``out_buf`` is returned. ``keep_first``:
+    with a window, keys j < keep_first stay visible. ``chunk`` > 0 (no window): row i sees only keys j
+    with j // chunk == i // chunk. ``sinks`` [H] fp32: exp(sinks[h]) joins the denominator.
+    ``gate_heads``: the gate is one column per head, ``gate_off .. gate_off + H``."""
     out_dtype = out_dtype or q.dtype
     if _gpu(q):
         T, H, _ = q.shape
@@ -192,12 +204,14 @@ def gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale: flo
                                float(sink), rows, int(num_splits),
                                workspace.part_o if num_splits > 1 else None,
                                workspace.part_ml if num_splits > 1 else None, int(window), slopes, gate, int(gate_off),
-                               1 if matrix_layout else 0, float(softcap), float(out_scale), int(out_off))
+                               1 if matrix_layout else 0, float(softcap), float(out_scale), int(out_off),
+                               int(keep_first), int(chunk), sinks, bool(gate_heads))
         return out
     if matrix_layout:
         raise ValueError("gqa_attention: the matrix-core cache layout exists on the GPU only")
     o = ref_gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale, temp, sink,
-                          torch.float32 if out_scale != 1.0 else out_dtype, window, slopes, gate, gate_off, softcap)
+                          torch.float32 if out_scale != 1.0 else out_dtype, window, slopes, gate, gate_off, softcap,
+                          keep_first, chunk, sinks, gate_heads)
     if out_scale != 1.0:
         o = (o * out_scale).to(out_dtype)
     if out_buf is not None:
@@ -304,6 +318,17 @@ def add_layer_norm(x, y, scale, w, b, eps, out_dtype) -> torch.Tensor:
             native().add_layer_norm(out, x, y, scale if y is not None else None, w, b, float(eps))
         return out
     return ref_add_layer_norm(x, y.combine(torch.float32) if isinstance(y, ExpertRows) else y, scale, w, b, eps, out_dtype)
+
+
+def add_tanh_norm(x, y, alpha: float, w, b, out_dtype) -> torch.Tensor:
+    """Dynamic Tanh: x += y (in place, fp32; ``y`` may be None), returns tanh(alpha x) * w + b."""
+    if _gpu(x):
+        out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+        native().add_tanh_norm(out, x, y, float(alpha), w, b)
+        return out
+    if y is not None:
+        x.add_(y.float())
+    return (torch.tanh(alpha * x) * w + b).to(out_dtype)
 
 
 def limited_glu(gu, limit: float, out_dtype) -> torch.Tensor:
@@ -533,13 +558,19 @@ def _rotate_pairs(t, positions, inv_freq):
 
 
 def ref_qk_prep(proj, spec, q_off, k_off, v_off, inv_freq, eps, positions, k_cache, v_cache, slot_mapping, out_dtype,
-                q_weight=None, k_weight=None):
+                q_weight=None, k_weight=None, q_bias=None, k_bias=None, v_bias=None, mix=None):
     T = proj.shape[0]
     H, G, Dk, Dv = spec.heads, spec.kv_heads, spec.dim, spec.vdim
     q = proj[:, q_off:q_off + H * Dk].float().reshape(T, H, Dk)
     k = proj[:, k_off:k_off + G * Dk].float().reshape(T, G, Dk)
     v = proj[:, k_off:k_off + G * Dk] if spec.value_from_key else proj[:, v_off:v_off + G * Dv]
-    if inv_freq is not None:
+    if q_bias is not None:
+        q = q + q_bias.reshape(H, Dk)
+    if k_bias is not None:
+        k = k + k_bias.reshape(G, Dk)
+    if inv_freq is not None and spec.rot.halves:
+        q, k = _rotate_halves(q, positions, inv_freq, 1.0), _rotate_halves(k, positions, inv_freq, 1.0)
+    elif inv_freq is not None:
         q, k = _rotate_pairs(q, positions, inv_freq), _rotate_pairs(k, positions, inv_freq)
     q, k = _rms(q, eps), _rms(k, eps)
     if q_weight is not None:
@@ -551,6 +582,12 @@ def ref_qk_prep(proj, spec, q_off, k_off, v_off, inv_freq, eps, positions, k_cac
         steps = torch.div(positions.long() + 1, every, rounding_mode="floor").to(torch.float32)
         q = q * (1.0 + coef * torch.log(steps + 1.0))[:, None, None]
     v = v.reshape(T, G, Dv)
+    if v_bias is not None:
+        v = v.float() + v_bias.reshape(G, Dv)
+    if mix is not None:
+        mp, mo, mb, lam = mix
+        first = mp[:, mo:mo + G * Dv].float() + (mb if mb is not None else 0.0)
+        v = (1.0 - lam) * v.float() + lam * first.reshape(T, G, Dv)
     if spec.value_norm:
         v = _rms(v.float(), eps)
     BS = k_cache.shape[2]
@@ -561,7 +598,8 @@ def ref_qk_prep(proj, spec, q_off, k_off, v_off, inv_freq, eps, positions, k_cac
 
 
 def ref_gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale, temp, sink, out_dtype,
-                      window=0, slopes=None, gate=None, gate_off=0, softcap=0.0):
+                      window=0, slopes=None, gate=None, gate_off=0, softcap=0.0, keep_first=0, chunk=0, sinks=None,
+                      gate_heads=False):
     T, H, Dk = q.shape
     G, BS, Dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[3]
     out = torch.empty(T, H, Dv, dtype=torch.float32, device=q.device)
@@ -585,16 +623,26 @@ def ref_gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale,
         dist = qpos[:, None] - torch.arange(ctx, device=q.device)[None, :]
         mask = dist >= 0
         if window > 0:
-            mask = mask & (dist < window)
+            mask = mask & ((dist < window) | (torch.arange(ctx, device=q.device) < keep_first)[None, :])
+        if chunk > 0:
+            mask = mask & (qpos[:, None] // chunk == (torch.arange(ctx, device=q.device) // chunk)[None, :])
         if slopes is not None:
             sc = sc - slopes.float()[:, None, None] * dist.to(torch.float32)[None]
         sc = sc.masked_fill(~mask[None], float("-inf"))
         m = sc.max(-1, keepdim=True).values
+        if sinks is not None:
+            m = torch.maximum(m, sinks.float()[:, None, None])
         e = torch.exp(sc - m)
-        den = e.sum(-1, keepdim=True) + sink * torch.exp(-m)
+        den = e.sum(-1, keepdim=True)
+        if sink:
+            den = den + sink * torch.exp(-m)
+        if sinks is not None:
+            den = den + torch.exp(sinks.float()[:, None, None] - m)
         out[r0:r1] = torch.einsum("hnk,hkd->hnd", e / den, V.repeat_interleave(H // G, 0)).permute(1, 0, 2)
+    if gate is not None and gate_heads:
+        out = out * torch.sigmoid(gate[:, gate_off:gate_off + H].float())[:, :, None]
     out = out.reshape(T, H * Dv)
-    if gate is not None:
+    if gate is not None and not gate_heads:
         out = out * torch.sigmoid(gate[:, gate_off:gate_off + H * Dv].float())
     return out.to(out_dtype)
 
@@ -819,6 +867,65 @@ def delta_prep(proj, spec, q_off: int, b_off: int, a_off: int, conv_w, state, ne
                           start_pos, slots, shift_state)
 
 
+def channel_delta_prep(proj, spec, q_off: int, b_off: int, a_off: int, a2, conv_w, state, neg_rate, dt_bias, row_seq,
+                       positions, start_pos, slots, shift_state: bool = False):
+    """As :func:`delta_prep` with one decay per head and key channel: g = exp(neg_rate[head] *
+    softplus(low . a2 + dt_bias)), ``low`` the columns ``a_off ..`` of ``proj``, ``a2`` [rank,
+    heads * dim] fp32, ``dt_bias`` [heads * dim]. Returns fp32 ``(four [4, T, heads * dim], v)`` with
+    four = (q, beta k, g, g k) per value head: :func:`state_scan` with (q, k, w, a, b) = (q, beta k, g,
+    beta k, g k) computes S <- diag(g) S; S <- S + k (beta (v - S^T k))^T; o = S^T q."""
+    if _gpu(proj):
+        T = proj.shape[0]
+        four = torch.empty(4, T, spec.heads * spec.dim, dtype=torch.float32, device=proj.device)
+        v = torch.empty(T, spec.heads * spec.vdim, dtype=torch.float32, device=proj.device)
+        native().channel_delta_prep(four, v, proj, int(q_off), int(b_off), int(a_off), a2, conv_w, state, neg_rate, dt_bias,
+                                    int(spec.heads), int(spec.kv_heads), int(spec.dim), int(spec.vdim), row_seq, positions,
+                                    start_pos, slots, bool(shift_state))
+        return four, v
+    T, A, D = proj.shape[0], spec.heads, spec.dim
+    q, k, v, beta = _delta_inputs(proj, spec, q_off, b_off, conv_w, state, row_seq, positions, start_pos, slots, shift_state)
+    z = proj[:, a_off:a_off + a2.shape[0]].float() @ a2 + dt_bias
+    g = torch.exp(neg_rate[:, None] * torch.nn.functional.softplus(z).reshape(T, A, D))
+    return torch.stack([q, beta * k, g, g * k]).reshape(4, T, A * D), v.contiguous()
+
+
+def memory_prep(proj, spec, q_off: int, k_off: int, v_off: int, i_off: int, f_off: int, i_bias, f_bias, gmax, cu_q,
+                start_pos, slots, step: bool = False) -> Tuple[torch.Tensor, ...]:
+    """Inputs of a matrix memory with exponential gates (``spec``: :class:`MatrixMemorySpec`) from
+    ``proj`` [T, N]: columns of q, k (heads x dim), v (heads x vdim) and the two gates (one number per
+    head, biases fp32 [heads]). With i = cap tanh((p_i + i_bias) / cap), f = logsigmoid(cap tanh((p_f +
+    f_bias) / cap)) and the running maximum m_t = max(f_t + m_(t-1), i_t) from ``gmax[slot]`` [heads] (0 at
+    position 0; every span's last m is left there) returns fp32 rows (q dim^(-1/2), exp(i_t - m_t) k,
+    exp(f_t + m_(t-1) - m_t) repeated over dim, per head v and a column of ones, exp(-m_t) [T, heads]):
+    the (q, k, w, v) of :func:`state_scan` with vdim + 1 columns, whose last one is n . q, and the
+    ``floors`` of :func:`head_norm_gate`. ``step``: one row per sequence, a single launch."""
+    A, D, E = spec.heads, spec.dim, spec.vdim
+    T, n, nv = proj.shape[0], A * D, A * (E + 1)
+    if _gpu(proj):
+        out = torch.empty(T, 3 * n + nv, dtype=torch.float32, device=proj.device)
+        gates = torch.empty(3, T, A, dtype=torch.float32, device=proj.device)
+        native().memory_prep(out, gates, proj, int(q_off), int(k_off), int(v_off), int(i_off), int(f_off), i_bias, f_bias,
+                             float(spec.gate_cap), gmax, cu_q, start_pos, slots, D ** -0.5, A, D, E, bool(step))
+        return out[:, :n], out[:, n:2 * n], out[:, 2 * n:3 * n], out[:, 3 * n:], gates[2]
+    cap = spec.gate_cap
+    gi = cap * torch.tanh((proj[:, i_off:i_off + A].float() + i_bias) / cap)
+    gf = torch.nn.functional.logsigmoid(cap * torch.tanh((proj[:, f_off:f_off + A].float() + f_bias) / cap))
+    keep, write, floor = (torch.empty(T, A, dtype=torch.float32) for _ in range(3))
+    cq, sp, sl = cu_q.tolist(), start_pos.tolist(), slots.tolist()
+    for s in range(len(sp)):
+        if cq[s + 1] == cq[s]:
+            continue
+        m = gmax[sl[s]].clone() if sp[s] > 0 else torch.zeros(A)
+        for t in range(cq[s], cq[s + 1]):
+            new = torch.maximum(gf[t] + m, gi[t])
+            keep[t], write[t], floor[t] = torch.exp(gf[t] + m - new), torch.exp(gi[t] - new), torch.exp(-new)
+            m = new
+        gmax[sl[s]] = m
+    k = (proj[:, k_off:k_off + n].float().reshape(T, A, D) * write[:, :, None]).reshape(T, n)
+    v = torch.cat([proj[:, v_off:v_off + A * E].float().reshape(T, A, E), torch.ones(T, A, 1)], -1).reshape(T, nv)
+    return proj[:, q_off:q_off + n].float() * D ** -0.5, k, keep[:, :, None].expand(T, A, D).reshape(T, n), v, floor
+
+
 def gla_prep(proj, spec, q_off: int, k_off: int, v_off: int, a_off: int, a2, a_bias) -> Tuple[torch.Tensor, ...]:
     """Inputs of a gated linear attention (``spec``: :class:`GLASpec`) from ``proj`` [T, N]: columns of
     q and k (heads x dim), v (heads x vdim) and the input of the decay's low-rank path (``a2``
@@ -864,15 +971,20 @@ def state_scan(q, k, v, w, a, b, decay, state, cu_q, start_pos, slots, heads: in
 
 
 def head_norm_gate(o, norm_w, span: int, gate, gate_off: int, gate_act: str, eps, scale: float, out_buf,
-                   out_off: int) -> torch.Tensor:
+                   out_off: int, floors=None) -> torch.Tensor:
     """``o`` [T, C] fp32: every ``span`` consecutive entries (a head; ``span`` = C: the whole row)
     divided by their root mean square, times ``norm_w`` (fp32 [C], or [span] shared by the heads),
     times sigmoid or silu (``gate_act``) of the columns ``gate_off ..`` of ``gate`` [T, N], times
-    ``scale``, into columns ``out_off ..`` of ``out_buf``."""
+    ``scale``, into columns ``out_off ..`` of ``out_buf``. ``floors`` [T, heads] fp32: ``o`` is
+    [T, heads * (span + 1)], a head's last entry x is no output: the others are divided by
+    max(|x|, floor) + 1e-6 ahead of the norm."""
     if _gpu(o):
         native().head_norm_gate(out_buf, int(out_off), o, norm_w, int(span), gate, int(gate_off),
-                                1 if gate_act == "silu" else 0, float(eps), float(scale))
+                                1 if gate_act == "silu" else 0, float(eps), float(scale), floors)
         return out_buf
+    if floors is not None:
+        oh = o.reshape(o.shape[0], floors.shape[1], span + 1)
+        o = (oh[..., :span] / (torch.maximum(oh[..., span:].abs(), floors[:, :, None]) + 1e-6)).reshape(o.shape[0], -1)
     T, C = o.shape
     n = _rms(o.reshape(T, C // span, span), eps)
     n = (n * norm_w).reshape(T, C) if norm_w.numel() == span else n.reshape(T, C) * norm_w
@@ -997,8 +1109,8 @@ def ref_removal_prep(proj, r_off, k_off, v_off, a_off, lw, w0, a_bias, heads, di
     return torch.stack([r, k, v, w, a * u, u])
 
 
-def ref_delta_prep(proj, spec, q_off, b_off, a_off, conv_w, state, neg_rate, dt_bias, row_seq, positions, start_pos,
-                   slots, shift_state=False):
+def _delta_inputs(proj, spec, q_off, b_off, conv_w, state, row_seq, positions, start_pos, slots, shift_state):
+    """Convolved, unit q and k [T, heads, dim], v [T, heads * vdim], beta [T, heads, 1] of a delta rule."""
     T = proj.shape[0]
     A, G, D, E = spec.heads, spec.kv_heads, spec.dim, spec.vdim
     C = 2 * G * D + A * E
@@ -1013,6 +1125,13 @@ def ref_delta_prep(proj, spec, q_off, b_off, a_off, conv_w, state, neg_rate, dt_
     k = k / torch.sqrt((k * k).sum(-1, keepdim=True) + 1e-6)
     q, k = q.repeat_interleave(A // G, 1), k.repeat_interleave(A // G, 1)           # [T, A, D]
     beta = torch.sigmoid(proj[:, b_off:b_off + A].float())[:, :, None]
+    return q, k, v, beta
+
+
+def ref_delta_prep(proj, spec, q_off, b_off, a_off, conv_w, state, neg_rate, dt_bias, row_seq, positions, start_pos,
+                   slots, shift_state=False):
+    T, A, D = proj.shape[0], spec.heads, spec.dim
+    q, k, v, beta = _delta_inputs(proj, spec, q_off, b_off, conv_w, state, row_seq, positions, start_pos, slots, shift_state)
     g = torch.exp(neg_rate * torch.nn.functional.softplus(proj[:, a_off:a_off + A].float() + dt_bias))[:, :, None]
     five = torch.stack([q, beta * k, g.expand(T, A, D), g * beta * k, k]).reshape(5, T, A * D)
     return five.contiguous(), v.contiguous()

@@ -51,7 +51,7 @@ def main(argv=None) -> int:
         if arch == "mupulorn":
             from .ops import latent
             latent.ensure_built()
-        elif arch in ("goganex", "retuvik", "ledinex"):
+        elif arch in ("goganex", "retuvik", "ledinex", "lizesun"):
             from .ops import hybrid
             hybrid.ensure_built()
         elif arch == "vurizen":
