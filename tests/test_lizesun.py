@@ -1,0 +1,908 @@
+"""Lizesun through the engine (model registry, grouped cache with convolution, matrix and gate states,
+state slots, Engine.step, generation) against the plain float64 statement in ``oracle_lizesun.py``, on
+small random checkpoints of several shapes. Every case runs on the CPU (PyTorch statements of the ops)
+and, marked ``gpu``, on the HIP kernels in fp32 and bf16.
+"""
+import json
+import math
+import os
+
+import pytest
+import torch
+from safetensors.torch import save_file
+
+import oracle_lizesun as O
+from theroundtaible_amd.engine import Engine, EngineConfig, SamplingParams, Turn
+from theroundtaible_amd.engine.kv_cache import KVCacheOOM
+from theroundtaible_amd.models.config import (DeltaSpec, GroupedAttentionSpec, MatrixMemorySpec, ParallelSpec, RotarySpec,
+                                              config_from_dir, get_config, parse_lizesun)
+from theroundtaible_amd.models.weights import layout_for
+from theroundtaible_amd.ops import hybrid as Hy
+
+GPU = pytest.mark.gpu
+RUNS = [("cpu", "fp32"), pytest.param(("cuda:0", "fp32"), marks=GPU), pytest.param(("cuda:0", "bf16"), marks=GPU)]
+RUNS32 = RUNS[:2]
+
+
+def delta(heads=4, kv=2, dim=6, vdim=10, conv=4, ff=40):
+    return {"type": "channel_delta", "mlp": {"kind": "dense", "ff": ff} if ff else None,
+            "mixer": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": conv}}
+
+
+def att(heads=6, kv=2, dim=12, vdim=10, chunk=13, softcap=9.0, v_mix=True, scale=None, ff=56):
+    m = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "scale": 1.3 * dim ** -0.5 if scale is None else scale,
+         "v_mix": v_mix}
+    if chunk:
+        m["mask"] = {"size": chunk}
+    if softcap:
+        m["softcap"] = softcap
+    return {"type": "attention", "mixer": m, "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def left(heads=4, kv=2, dim=12, vdim=10, window=11, keep=3, rot_dims=8, base=5000.0, scale=None):
+    m = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "scale": 1.4 * dim ** -0.5 if scale is None else scale}
+    if rot_dims:
+        m["rot"] = {"base": base, "dims": rot_dims}
+    if window:
+        m["mask"] = {"size": window, "keep_first": keep}
+    return m
+
+
+def par(rheads=3, rdim=8, rvdim=6, cap=7.0, ls=0.7, rs=1.2, ff=48, **kw):
+    return {"type": "parallel", "mlp": {"kind": "dense", "ff": ff} if ff else None,
+            "mixer": {"left": left(**kw), "left_scale": ls, "right_scale": rs,
+                      "right": {"heads": rheads, "dim": rdim, "vdim": rvdim, "gate_cap": cap}}}
+
+
+def make_config(width=40, vocab=97, layers=None, embed_scale=1.7, eps=1e-5):
+    if layers is None:
+        layers = [par(), att(), delta(), att(3, 1, 8, 20, chunk=7, ff=0, v_mix=False),
+                  att(4, 2, 9, 10, chunk=29, softcap=4.0), delta(2, 1, 8, 4, conv=2, ff=0)]
+    return {"architecture": "Lizesun", "embedding": {"scale": embed_scale}, "layers": layers, "norm": {"eps": eps},
+            "vocab": vocab, "width": width}
+
+
+def make_checkpoint(path, cfg, seed=0, edit=None, rank=5, gate_rank=7):
+    """Random weights for ``cfg`` (a config.json dict) written as a checkpoint directory; returns
+    the float64 tensors. ``edit(P)`` may change tensors before they are written."""
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    mc = config_from_dir(path)
+    g = torch.Generator().manual_seed(seed)
+    P = {}
+    for name, (shape, _, _) in layout_for(mc).items():
+        r = gate_rank if name.endswith(("g1", "g2")) else rank      # the two paths' ranks are the checkpoint's
+        shape = tuple(r if n < 0 else n for n in shape)
+        rnd = torch.randn(shape, generator=g)
+        if name.endswith(".alpha"):
+            w = 0.4 + 0.5 * torch.rand(shape, generator=g)
+        elif name.endswith(("norm1.b", "norm2.b", "norm.b")):
+            w = 0.2 * rnd
+        elif name.endswith(("norm1", "norm2", "norm")):
+            w = 0.6 + torch.rand(shape, generator=g)
+        elif name.endswith(".conv"):
+            w = 0.4 * rnd
+            w[:, -1] += 1.0
+        elif name.endswith("A_log"):
+            w = -2.0 + 0.5 * rnd
+        elif name.endswith("vmix"):
+            w = torch.tensor(0.37)
+        elif name.endswith("f.b"):
+            w = 1.0 + rnd
+        elif name.endswith(("sink", "dt_bias", "q.b", "k.b", "v.b", "i.b")):
+            w = 0.8 * rnd
+        elif name == "embed":
+            w = rnd
+        else:
+            w = rnd / math.sqrt(shape[-1])
+        P[name] = w.to(torch.bfloat16).float()      # values both number formats hold exactly
+    if edit is not None:
+        edit(P)
+    save_file({k: v.contiguous() for k, v in P.items()}, os.path.join(path, "model.safetensors"))
+    return {k: v.double() for k, v in P.items()}
+
+
+def engine_for(path, run, tokens=512, block_size=16, slots=4, graphs=False):
+    device, dtype = run
+    if device != "cpu":
+        Hy.native()     # the GPU cases fail loudly when the extension is missing
+    return Engine(EngineConfig(model=str(path), weights=str(path), dtype=dtype, device=device, block_size=block_size,
+                               num_blocks=(tokens + block_size - 1) // block_size + (1 if graphs else 0),
+                               use_graphs=graphs, state_slots=slots, max_batch=slots))
+
+
+def close(got, want, run, what=""):
+    """fp32 runs: every logit within 2e-3 of the oracle. bf16 runs: rows are judged together, since a
+    per-head norm of a read-out that nearly cancels turns rounding into a visible error now and then:
+    the median row error (root mean square over the vocabulary) stays under 2.5 % of the logits' own
+    and at most one row in ten is off by more than 10 %. A wrong kernel misses by about 100 %."""
+    got = got.double().cpu()
+    assert got.shape == want.shape and torch.isfinite(got).all(), what
+    if run[1] != "bf16":
+        torch.testing.assert_close(got, want, msg=lambda m: f"{what}: {m}", rtol=0, atol=2e-3)
+        return
+    err = (got - want).pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()
+    assert float(err.median()) < 0.025 and float((err > 0.1).double().mean()) <= 0.1, \
+        f"{what}: median row error {float(err.median()):.3f}, worst {float(err.max()):.3f}"
+
+
+def toks(n, vocab, seed):
+    return torch.randint(0, vocab, (n,), generator=torch.Generator().manual_seed(seed)).tolist()
+
+
+def dev_of(run):
+    return torch.device(run[0])
+
+
+def dt_of(run):
+    return torch.bfloat16 if run[1] == "bf16" else torch.float32
+
+
+def spans(cuts, slot=1):
+    """Row metadata of ONE sequence fed in portions: yields (rows, row_seq, positions, start_pos, cu_q, slots)."""
+    at = 0
+    for n in cuts:
+        yield (slice(at, at + n), torch.zeros(n, dtype=torch.int32), torch.arange(at, at + n),
+               torch.tensor([at], dtype=torch.int32), torch.tensor([0, n], dtype=torch.int32),
+               torch.tensor([slot], dtype=torch.int32))
+        at += n
+
+
+def config_like(layers, **kw):
+    return parse_lizesun(make_config(layers=layers, **kw), "t")
+
+
+# ---- each mechanism alone (package ops against the oracle's functions) ----------------------------
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("rows,W", [(1, 5), (3, 37), (70, 64), (2, 1000), (300, 260)])
+def test_tanh_norm(run, rows, W):
+    """The residual add and tanh(alpha x) w + b, pending output present or not, far into the tanh's flat
+    parts and close to zero; the sum stays in the fp32 residual."""
+    dev, dt = dev_of(run), dt_of(run)
+    g = torch.Generator().manual_seed(W)
+    x, y = 3 * torch.randn(rows, W, generator=g), torch.randn(rows, W, generator=g).to(dt).float()
+    x[0, :3], y[0, :3] = torch.tensor([60.0, -60.0, 1e-4]), 0.0
+    w, b = torch.randn(W, generator=g), torch.randn(W, generator=g)
+    for pend in (None, y):
+        for alpha in (0.3, 1.0, -2.0):
+            xs = x.clone().to(dev)
+            got = Hy.add_tanh_norm(xs, None if pend is None else pend.to(dt).to(dev), alpha, w.to(dev), b.to(dev), dt)
+            s = x + (pend if pend is not None else 0.0)
+            want = O.tanh_norm(s.double(), alpha, w.double(), b.double())
+            assert got.dtype == dt and torch.equal(xs.cpu(), s)
+            assert float((got.double().cpu() - want).abs().max()) < (0.04 if run[1] == "bf16" else 2e-6)
+
+
+def _attend(run, a, proj, off, P, lam, first, cuts, BS, sinks=None, gate=False, splits=3):
+    """qk_prep + gqa_attention of one sequence in portions through a paged cache on scattered pages
+    whose unused entries are large; single rows past the start are decode rows with split keys."""
+    dev, dt = dev_of(run), dt_of(run)
+    n = proj.shape[0]
+    nb = (n + BS - 1) // BS
+    perm = torch.randperm(nb + 3, generator=torch.Generator().manual_seed(5))[:nb].to(torch.int32)
+    kc = torch.full((nb + 3, a.kv_heads, BS, a.dim), 50.0, dtype=dt, device=dev)
+    vc = torch.full((nb + 3, a.kv_heads, BS, a.vdim), -50.0, dtype=dt, device=dev)
+    freq = Hy.rotary_halves_table(a.rot, dev)[0]
+    on = lambda name: P[name].float().to(dev) if name in P else None
+    out = []
+    for rows, rs, pos, sp, cu, sl in spans(cuts):
+        T = rows.stop - rows.start
+        slot_map = (perm[pos // BS].long() * BS + pos % BS).to(dev)
+        p = proj[rows].to(dt).to(dev)
+        mix = (first[rows].to(dt).to(dev), 2, on("first.b"), lam) if first is not None else None
+        q = Hy.qk_prep(p, a, off["q"], off["k"], off["v"], freq, 1e-5, pos.to(dev), kc, vc, slot_map, dt,
+                       q_weight=on("q.norm"), k_weight=on("k.norm"), q_bias=on("q.b"), k_bias=on("k.b"), v_bias=on("v.b"), mix=mix)
+        one = T == 1 and rows.start > 0
+        buf = torch.zeros(T, a.heads * a.vdim + 5, dtype=dt, device=dev)
+        Hy.gqa_attention(q, kc, vc, perm[None].to(dev), cu.to(dev), sp.to(dev), a.scale, None, 0.0,
+                         num_splits=splits if one and dev.type == "cuda" else 1, out_dtype=dt, window=a.window,
+                         keep_first=a.keep_first, chunk=a.chunk, softcap=a.softcap, out_scale=0.8, out_buf=buf, out_off=5,
+                         sinks=None if sinks is None else sinks.to(dev), gate=p if gate else None,
+                         gate_off=off.get("g", 0), gate_heads=gate)
+        out.append(buf)
+    out = torch.cat(out)
+    assert float(out[:, :5].abs().max()) == 0
+    return out[:, 5:].double().cpu()
+
+
+def _attention_case(run, d, kind, n, seed, edit=None):
+    """Projected columns and small parameters of one attention mixer, and the oracle's result with
+    identity projections (h = the projected columns)."""
+    dt = dt_of(run)
+    g = torch.Generator().manual_seed(seed)
+    H, G, D, E = (int(d[k]) for k in ("heads", "kv_heads", "dim", "vdim"))
+    nq, nk, nv = H * D, G * D, G * E
+    off = {"q": 3, "k": 3 + nq, "v": 3 + nq + nk, "g": 3 + nq + nk + nv}
+    width = nq + nk + nv + (H if kind == "attention" else 0)
+    proj = torch.randn(n, 3 + width, generator=g)
+    if edit is not None:
+        edit(proj, off)
+    proj = proj.to(dt).float()
+    eye = torch.eye(width, dtype=torch.float64)
+    P = {"q": eye[:nq], "k": eye[nq:nq + nk], "v": eye[nq + nk:nq + nk + nv], "o": torch.eye(H * E, dtype=torch.float64)}
+    if kind == "attention":
+        P["g"] = eye[nq + nk + nv:]
+        for nm, size in (("q.b", nq), ("k.b", nk), ("v.b", nv)):
+            P[nm] = 0.3 * torch.randn(size, generator=g).double()
+        for nm in ("q.norm", "k.norm"):
+            P[nm] = (0.6 + torch.rand(D, generator=g)).double()
+    else:
+        P["sink"] = torch.randn(H, generator=g).double()
+    return proj, off, P
+
+
+def spec_of(d, kind):
+    if kind == "attention":
+        return config_like([att(ff=0) | {"mixer": d}]).layers[0].mixer
+    p = par(ff=0)
+    return config_like([p | {"mixer": dict(p["mixer"], left=d)}]).layers[0].mixer.left
+
+
+TOL = {"bf16": 0.09, "fp32": 4e-4}
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("cuts", [[75], [5, 1, 1, 2, 40, 1, 20, 1, 1, 3]])
+@pytest.mark.parametrize("shape", [(4, 2, 12, 10), (6, 1, 32, 32), (2, 2, 70, 130), (5, 5, 64, 48), (40, 1, 16, 16)])
+def test_chunked_attention_mixed_values_and_gate(run, cuts, shape):
+    """Biases, per-head norms with weights, soft cap, chunks, values mixed with another layer's, one gate
+    per head; unequal key and value sizes, one to forty query heads per key / value head; prompts,
+    portions and decoded rows."""
+    H, G, D, E = shape
+    d = att(H, G, D, E, chunk=19, softcap=2.5, scale=2.0 * D ** -0.5)["mixer"]
+    proj, off, P = _attention_case(run, d, "attention", sum(cuts), 1)
+    g = torch.Generator().manual_seed(2)
+    first = torch.randn(sum(cuts), 2 + G * E, generator=g).to(dt_of(run)).float()
+    P["first.b"], P["vmix"] = torch.randn(G * E, generator=g).double(), torch.tensor(0.35).double()
+    v_first = (first[:, 2:].double() + P["first.b"]).reshape(-1, G, E)
+    a = spec_of(d, "attention")
+    for mixed in (False, True):
+        want = O.chunked_attention(proj[:, 3:].double(), P, "", d, 1e-5, v_first if mixed else None)[0]
+        got = _attend(run, a, proj, off, P, 0.35, first if mixed else None, cuts, 8, gate=True)
+        assert float((got - 0.8 * want).abs().max()) < TOL[run[1]], mixed
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("cuts", [[75], [5, 1, 1, 2, 40, 1, 20, 1, 1, 3]])
+@pytest.mark.parametrize("shape", [(4, 2, 12, 10, 8), (6, 1, 32, 32, 32), (2, 2, 70, 130, 2), (6, 2, 96, 80, 64), (40, 1, 16, 16, 0)])
+def test_window_attention_with_kept_keys_and_sink(run, cuts, shape):
+    """Rotation in halves ahead of the unit norms, a sliding window with kept first keys, a learned sink
+    per head."""
+    H, G, D, E, R = shape
+    d = left(H, G, D, E, window=14, keep=5, rot_dims=R, scale=2.0 * D ** -0.5)
+    proj, off, P = _attention_case(run, d, "parallel", sum(cuts), 3)
+    want = 0.8 * O.window_attention(proj[:, 3:].double(), P, "", d, 1e-5)
+    got = _attend(run, spec_of(d, "parallel"), proj, off, P, 0.0, None, cuts, 8, sinks=P["sink"].float())
+    assert float((got - want).abs().max()) < TOL[run[1]]
+
+
+def _standing_keys(n, at, H, G, D):
+    """Queries that all point one way and keys that all point the other, but for the keys ``at``."""
+    def edit(proj, off):
+        proj[:, off["q"]:off["k"]] *= 0.05
+        proj[:, off["q"]:off["k"]:D] = 6.0
+        proj[:, off["k"]:off["v"]] *= 0.05
+        proj[:, off["k"]:off["v"]:D] = -2.0
+        for j in at:
+            proj[j, off["k"]:off["v"]:D] = 6.0
+            proj[j, off["v"]:off["v"] + 1] += 4.0 * (1 + j % 3)
+    return edit
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("D", [8, 32])
+@pytest.mark.parametrize("window,keep", [(1, 0), (2, 1), (6, 3), (16, 1), (17, 20), (32, 4), (33, 8), (64, 65), (65, 64), (130, 2)])
+def test_window_and_kept_key_edges(run, window, keep, D):
+    """Keys that stand out at the last kept position, the first one that is not kept, and far inside: a
+    window or a kept span that is one token off changes the result far beyond the tolerance. In a
+    prompt, in portions cut at the edges, and decoded on split keys."""
+    n, H, G = 210, 2, 1
+    marks = sorted({max(keep - 1, 0), keep, 70, 71})
+    d = left(H, G, D, D, window=window, keep=keep, rot_dims=0, scale=4.0 / D)
+    proj, off, P = _attention_case(run, d, "parallel", n, 4, _standing_keys(n, marks, H, G, D))
+    P["sink"][:] = 0.0
+    h = proj[:, 3:].double()
+    want = 0.8 * O.window_attention(h, P, "", d, 1e-5)
+    for other in (dict(size=window + 1, keep_first=keep), dict(size=window, keep_first=keep + 1)):     # the edges show
+        off_by_one = 0.8 * O.window_attention(h, P, "", dict(d, mask=other), 1e-5)
+        assert float((off_by_one - want).abs().max()) > 0.3
+    edge = 70 + window
+    cuts = [edge - 1, 1, 1] if edge < n - 1 else [n - 3, 1, 1]
+    for c in ([n], cuts + [n - sum(cuts)] if sum(cuts) < n else cuts, [60] + [1] * 30 + [n - 90], [2, 40] + [1] * (n - 42)):
+        got = _attend(run, spec_of(d, "parallel"), proj, off, P, 0.0, None, c, 16, sinks=P["sink"].float())
+        assert float((got - want).abs().max()) < (0.12 if run[1] == "bf16" else 5e-4), c[:4]
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("D", [8, 32])
+@pytest.mark.parametrize("chunk", [1, 2, 15, 16, 17, 32, 64, 65, 130, 1000])
+def test_chunk_edges(run, chunk, D):
+    """Keys that stand out at the last position of a chunk and the first of the next: rows on both sides
+    of every border, in a prompt, in portions cut beside the border, and decoded."""
+    n, H, G = 150, 4, 2
+    first = chunk * max(1, 64 // chunk) if chunk < n else 64
+    marks = sorted({max(first - 1, 0), first, 0, 1})
+    d = att(H, G, D, D, chunk=chunk, softcap=50.0, scale=4.0 / D)["mixer"]
+    proj, off, P = _attention_case(run, d, "attention", n, 6, _standing_keys(n, marks, H, G, D))
+    for nm in ("q.b", "k.b"):
+        P[nm][:] = 0.0
+    for nm in ("q.norm", "k.norm"):
+        P[nm][:] = 1.0
+    h = proj[:, 3:].double()
+    want = O.chunked_attention(h, P, "", d, 1e-5)[0] * 0.8
+    if 1 < chunk < n:
+        for size in (chunk - 1, chunk + 1):
+            assert float((O.chunked_attention(h, P, "", dict(d, mask={"size": size}), 1e-5)[0] * 0.8 - want).abs().max()) > 0.3
+    for c in ([n], [first - 1, 1, 1, n - first - 1] if first > 1 else [1, 1, n - 2], [first, 2, n - first - 2],
+              [33] + [1] * (n - 33)):
+        got = _attend(run, spec_of(d, "attention"), proj, off, P, 0.0, None, c, 16, gate=True)
+        assert float((got - want).abs().max()) < (0.12 if run[1] == "bf16" else 5e-4), c[:4]
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("kind", ["attention", "parallel"])
+def test_a_far_key_among_hundreds(run, kind):
+    """700 keys on scattered pages: one early key (a kept one, or one of the same long chunk) carries
+    almost all the weight of the late queries; losing it (a page, a tile, a split) shows."""
+    n, H, G, D = 700, 4, 2, 32
+    d = (att(H, G, D, D, chunk=699, softcap=50.0, scale=0.3)["mixer"] if kind == "attention"
+         else left(H, G, D, D, window=90, keep=4, rot_dims=0, scale=0.3))
+    proj, off, P = _attention_case(run, d, kind, n, 7, _standing_keys(n, [2], H, G, D))
+    for nm in P:
+        if nm in ("q.b", "k.b", "sink"):
+            P[nm][:] = 0.0
+    h = proj[:, 3:].double()
+    fn = (lambda: O.chunked_attention(h, P, "", d, 1e-5)[0]) if kind == "attention" else (lambda: O.window_attention(h, P, "", d, 1e-5))
+    want = 0.8 * fn()
+    got = _attend(run, spec_of(d, kind), proj, off, P, 0.0, None, [650] + [1] * 50, 16, gate=kind == "attention",
+                  sinks=P["sink"].float() if kind == "parallel" else None, splits=5)
+    assert float((got - want).abs().max()) < (0.1 if run[1] == "bf16" else 4e-4)
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_sinks_far_above_and_below_the_scores(run):
+    """A sink takes its share once per head: none at -1000, half against one key of the same score, all
+    at +300 (the result is zero, not NaN); with the scores themselves far below zero too."""
+    n, H, G, D = 40, 5, 1, 8
+    d = left(H, G, D, D, window=9, keep=2, rot_dims=0, scale=30.0)
+    proj, off, P = _attention_case(run, d, "parallel", n, 8)
+    proj[:, off["q"]:off["q"] + D] = 1.0
+    proj[:, off["k"]:off["v"]] = -1.0          # scores of head 0: -30 * D
+    P["sink"] = torch.tensor([0.0, -1000.0, 0.0, 300.0, 4.0], dtype=torch.float64)
+    want = 0.8 * O.window_attention(proj[:, 3:].double(), P, "", d, 1e-5)
+    assert float(want[:, 3 * D:4 * D].abs().max()) < 1e-6 < float(want[:, D:2 * D].abs().max())
+    for cuts in ([n], [3] + [1] * (n - 3)):
+        got = _attend(run, spec_of(d, "parallel"), proj, off, P, 0.0, None, cuts, 8, sinks=P["sink"].float())
+        assert torch.isfinite(got).all()
+        assert float((got - want).abs().max()) < (0.1 if run[1] == "bf16" else 2e-3)
+
+
+def _delta_mixer(run, spec, cuts, seed, rank=5, edit=None):
+    dev, dt = dev_of(run), dt_of(run)
+    A, G, D, E, C, conv = spec.heads, spec.kv_heads, spec.dim, spec.vdim, spec.conv_channels, spec.conv
+    n = sum(cuts)
+    g = torch.Generator().manual_seed(seed)
+    N = C + A + rank + A * E
+    proj = torch.randn(n, 2 + N, generator=g).to(dt).float()
+    cw = 0.4 * torch.randn(C, conv, generator=g)
+    cw[:, -1] += 1.0
+    A_log, dtb = torch.randn(A, generator=g) * 0.5 - 1.0, torch.randn(A * D, generator=g)
+    nw, a2 = 0.6 + torch.rand(E, generator=g), torch.randn(A * D, rank, generator=g) / rank ** 0.5
+    if edit is not None:
+        edit(A_log, dtb, proj)
+    gq, gk = G * D, 2 * G * D
+    eye = torch.eye(N, dtype=torch.float64)
+    P = {"q": eye[:gq], "k": eye[gq:gk], "v": eye[gk:C], "b": eye[C:C + A], "a1": eye[C + A:C + A + rank],
+         "g1": eye[C + A + rank:], "g2": torch.eye(A * E, dtype=torch.float64), "a2": a2.double(), "q.conv": cw[:gq].double(),
+         "k.conv": cw[gq:gk].double(), "v.conv": cw[gk:].double(), "A_log": A_log.double(), "dt_bias": dtb.double(),
+         "norm": nw.double(), "o": torch.eye(A * E, dtype=torch.float64)}
+    want = O.channel_delta(proj[:, 2:].double(), P, "", {"heads": A, "kv_heads": G, "dim": D, "vdim": E, "conv": conv}, 1e-5)
+    sconv = torch.full((3, max(conv - 1, 1), C), 5.0, device=dev)        # a used slot: never read at position 0
+    rec = torch.full((3, A * D * E), 5.0, device=dev)
+    out = []
+    for rows, rs, pos, sp, cu, sl in spans(cuts):
+        one = rows.stop - rows.start == 1 and rows.start > 0
+        p = proj[rows].to(dt).to(dev)
+        f, v = Hy.channel_delta_prep(p, spec, 2, 2 + C, 2 + C + A, a2.t().contiguous().to(dev), cw.to(dev), sconv,
+                                     (-torch.exp(A_log)).to(dev), dtb.to(dev), rs.to(dev), pos.to(dev), sp.to(dev),
+                                     sl.to(dev), shift_state=one)
+        if not one:
+            Hy.conv_state_update(p, 2, C, sconv, 0, cu.to(dev), sp.to(dev), sl.to(dev))
+        chunks = Hy.scan_chunks(cu, dev) if dev.type == "cuda" else None
+        o = Hy.state_scan(f[0], f[1], v, f[2], f[1], f[3], None, rec, cu.to(dev), sp.to(dev), sl.to(dev), A, D, E, chunks=chunks)
+        buf = torch.zeros(p.shape[0], A * E, dtype=dt, device=dev)
+        out.append(Hy.head_norm_gate(o, nw.to(dev), E, p, 2 + C + A + rank, "sigmoid", 1e-5, 1.0, buf, 0))
+    return torch.cat(out).double().cpu(), want
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("shape", [(4, 2, 6, 10, 4), (3, 3, 32, 16, 2), (2, 1, 72, 132, 1), (1, 1, 64, 64, 5), (2, 2, 130, 8, 3)])
+@pytest.mark.parametrize("cuts", [[24], [5, 1, 2, 1, 1, 14], [300, 1, 1, 2, 70, 1, 65]])
+def test_channel_delta_across_cuts(run, shape, cuts):
+    """Short convolutions (state across portions), silu, unit vectors, step sizes, a decay per head and
+    key channel, the scan in one pass and in chunks, and the gated per-head norm: the whole mixer."""
+    A, G, D, E, conv = shape
+    spec = DeltaSpec(A, G, D, E, conv, channel_decay=True)
+    got, want = _delta_mixer(run, spec, cuts, D, rank=1 if D == 64 else 5)
+    assert float((got - want).abs().max()) < (0.12 if run[1] == "bf16" else 1e-3)
+
+
+@pytest.mark.parametrize("run", RUNS32)
+def test_channel_decays_of_zero_and_one(run):
+    """Channels that forget at once beside channels that keep everything: the decay acts on key channels
+    (the state's rows), and a channel of the first kind holds nothing of an earlier token."""
+    def edit(A_log, dtb, proj):
+        A_log[:] = 3.0
+        dtb[:] = -60.0          # decay exp(-e^3 softplus(-60)) = 1
+        dtb[::3] = 60.0         # decay exp(-e^3 * 60) = 0
+    spec = DeltaSpec(2, 1, 12, 8, 2, channel_decay=True)
+    for cuts in ([150], [70, 1, 1, 8, 70]):
+        got, want = _delta_mixer(run, spec, cuts, 3, edit=edit)
+        assert float((got - want).abs().max()) < 1e-3
+
+
+def _memory_mixer(run, spec, cuts, seed, edit=None):
+    dev, dt = dev_of(run), dt_of(run)
+    A, D, E = spec.heads, spec.dim, spec.vdim
+    n = sum(cuts)
+    g = torch.Generator().manual_seed(seed)
+    N = 2 * A * D + 2 * A * E + 2 * A
+    proj = torch.randn(n, 1 + N, generator=g)
+    ib, fb, nw = torch.randn(A, generator=g), 1 + torch.randn(A, generator=g), 0.6 + torch.rand(A * E, generator=g)
+    off, at = {}, 1
+    for nm, size in (("q", A * D), ("k", A * D), ("v", A * E), ("g", A * E), ("i", A), ("f", A)):
+        off[nm] = at
+        at += size
+    if edit is not None:
+        edit(proj, off, ib, fb)
+    proj = proj.to(dt).float()
+    eye = torch.eye(N, dtype=torch.float64)
+    sizes = {"q": A * D, "k": A * D, "v": A * E, "g": A * E, "i": A, "f": A}
+    P = {nm: eye[off[nm] - 1:off[nm] - 1 + sizes[nm]] for nm in off}
+    P.update({"i.b": ib.double(), "f.b": fb.double(), "norm": nw.double(), "o": torch.eye(A * E, dtype=torch.float64)})
+    m = {"heads": A, "dim": D, "vdim": E, "gate_cap": spec.gate_cap}
+    want = 0.7 * O.memory_mixer(proj[:, 1:].double(), P, "", m, 1e-5)
+    rec = torch.full((3, spec.state_size), 4.0, device=dev)
+    gmax = torch.full((3, A), 9.0, device=dev)
+    out = []
+    for rows, rs, pos, sp, cu, sl in spans(cuts, slot=2):
+        T = rows.stop - rows.start
+        one = T == 1 and rows.start > 0
+        p = proj[rows].to(dt).to(dev)
+        q, k, w, v, fl = Hy.memory_prep(p, spec, off["q"], off["k"], off["v"], off["i"], off["f"], ib.to(dev), fb.to(dev),
+                                        gmax, cu.to(dev), sp.to(dev), sl.to(dev), step=one)
+        chunks = Hy.scan_chunks(cu, dev) if dev.type == "cuda" else None
+        o = Hy.state_scan(q, k, v, w, None, None, None, rec, cu.to(dev), sp.to(dev), sl.to(dev), A, D, E + 1, chunks=chunks)
+        buf = torch.zeros(T, A * E + 3, dtype=dt, device=dev)
+        out.append(Hy.head_norm_gate(o, nw.to(dev), E, p, off["g"], "sigmoid", 1e-5, 0.7, buf, 3, floors=fl))
+    assert float((gmax[:2] - 9.0).abs().max()) == 0 and float((rec[:2] - 4.0).abs().max()) == 0
+    return torch.cat(out)[:, 3:].double().cpu(), want
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("shape", [(3, 8, 6, 7.0), (1, 64, 64, 15.0), (2, 70, 130, 2.0), (5, 32, 40, 11.0)])
+@pytest.mark.parametrize("cuts", [[24], [5, 1, 2, 1, 1, 14], [300, 1, 1, 2, 70, 1, 65]])
+def test_matrix_memory_across_cuts(run, shape, cuts):
+    """Capped exponential gates, the running maximum, state, normaliser, per-head norm, weight and gate;
+    spans below and above a wave's 64 tokens, decoded rows, a used slot."""
+    got, want = _memory_mixer(run, MatrixMemorySpec(*shape), cuts, shape[1])
+    assert float((got - want).abs().max()) < (0.2 if run[1] == "bf16" else 2e-3)
+
+
+@pytest.mark.parametrize("run", RUNS32)
+def test_matrix_memory_gates_at_their_caps(run):
+    """Input gates at the cap on some tokens (the maximum jumps to it and decays with the forget gates),
+    far below zero on all the others, forget gates at both caps; and a sequence whose gates are all far
+    below zero from the first token on, where the maximum's start at 0 and the floor exp(-m) decide."""
+    def jumps(proj, off, ib, fb):
+        proj[:, off["i"]:off["f"]] = -40.0
+        proj[::37, off["i"]:off["f"]] = 60.0
+        proj[:, off["f"]:] = 30.0
+        proj[50::61, off["f"]:] = -30.0
+
+    def quiet(proj, off, ib, fb):
+        proj[:, off["i"]:off["f"]] = -4.0
+        ib[:] = 0.0
+        proj[:, off["f"]:] = 3.0
+    for edit in (jumps, quiet):
+        for cuts in ([200], [3, 1, 1, 90, 2, 103]):
+            got, want = _memory_mixer(run, MatrixMemorySpec(2, 12, 10, 9.0), cuts, 1, edit)
+            assert float((got - want).abs().max()) < 2e-3
+
+
+@pytest.mark.parametrize("run", RUNS32)
+@pytest.mark.parametrize("sizes", [(2, 64, 64), (3, 20, 33), (1, 130, 40)])
+def test_unequal_sequences_in_one_scan(run, sizes):
+    """Delta rule and matrix memory of several sequences in one launch (one starts, one goes on, one has a
+    single row), in chunks where spans are long, against each sequence alone."""
+    dev = dev_of(run)
+    A, D, E = sizes
+    lens, starts = [200, 1, 70, 64, 129], [0, 5, 12, 0, 64]
+    cu = torch.tensor([0] + list(torch.tensor(lens).cumsum(0)), dtype=torch.int32)
+    T = int(cu[-1])
+    g = torch.Generator().manual_seed(D)
+    q, v = torch.randn(T, A * D, generator=g), torch.randn(T, A * E, generator=g)
+    k = O.unit_length(torch.randn(T, A, D, generator=g).double()).float().reshape(T, A * D)
+    w = torch.rand(T, A * D, generator=g) * 0.5 + 0.5
+    beta = torch.rand(T, A, generator=g).repeat_interleave(D, 1)
+    sl = torch.tensor([4, 0, 2, 1, 3], dtype=torch.int32)
+    rec0 = torch.randn(5, A * D * E, generator=g)
+    for ab in (False, True):
+        b = (beta * k, w * k) if ab else (None, None)
+        kk = b[0] if ab else k
+        rec = rec0.clone().to(dev)
+        on = lambda t: None if t is None else t.contiguous().to(dev)
+        got = Hy.state_scan(on(q), on(kk), on(v), on(w), on(b[0]), on(b[1]), None, rec, cu.to(dev),
+                            torch.tensor(starts, dtype=torch.int32, device=dev), sl.to(dev), A, D, E,
+                            chunks=Hy.scan_chunks(cu, dev) if dev.type == "cuda" else None).double().cpu()
+        for s in range(5):
+            r = slice(int(cu[s]), int(cu[s + 1]))
+            S = (rec0[sl[s]].double().reshape(A, E, D).transpose(1, 2).clone() if starts[s] > 0
+                 else torch.zeros(A, D, E, dtype=torch.float64))
+            for t in range(r.start, r.stop):
+                wt, qt, kt, bt = (x[t].double().reshape(A, D) for x in (w, q, k, beta))
+                S = wt[:, :, None] * S
+                u = v[t].double().reshape(A, E)
+                if ab:
+                    u = bt[:, :1] * (u - torch.einsum("ai,aij->aj", kt, S))
+                S = S + kt[:, :, None] * u[:, None, :]
+                want = torch.einsum("ai,aij->aj", qt, S)
+                assert float((got[t].reshape(A, E) - want).abs().max()) < 1e-3 * max(1.0, float(want.abs().max())), (ab, s, t)
+            assert float((rec[sl[s]].double().cpu().reshape(A, E, D).transpose(1, 2) - S).abs().max()) < 2e-3
+
+
+@pytest.mark.parametrize("run", RUNS32)
+def test_a_far_token_in_the_states(run):
+    """One early token that the last query asks for: a matrix memory whose forget gates stay open keeps it
+    over 500 tokens and many portions."""
+    def edit(proj, off, ib, fb):
+        A, D = 2, 16
+        proj[:, off["q"]:off["v"]] *= 0.02
+        proj[4, off["k"] + 3:off["v"]:D] = 5.0
+        proj[-1, off["q"] + 3:off["k"]:D] = 5.0
+        proj[:, off["f"]:] = 20.0
+        proj[:, off["i"]:off["f"]] = 0.0
+    for cuts in ([500], [100, 1, 1, 198] + [1] * 200):
+        got, want = _memory_mixer(run, MatrixMemorySpec(2, 16, 8, 15.0), cuts, 1, edit)
+        assert float((got - want).abs().max()) < 2e-3
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("n", [7, 64, 1000])
+def test_squared_relu(run, n):
+    dev, dt = dev_of(run), dt_of(run)
+    a = torch.randn(3, n, generator=torch.Generator().manual_seed(n)).to(dt)
+    got = Hy.relu2(a.to(dev), dt).double().cpu()
+    assert float((got - torch.relu(a.double()) ** 2).abs().max()) < (0.05 if run[1] == "bf16" else 1e-5)
+
+
+# ---- the model through the engine -----------------------------------------------------------------
+
+def test_config_reader_and_registry(tmp_path):
+    cfg = make_config()
+    make_checkpoint(tmp_path / "m", cfg)
+    mc = get_config(str(tmp_path / "m"))
+    assert mc.arch == "lizesun" and mc.n_layers == 6 and mc.embed_scale == 1.7
+    m0, m1, m2, m3 = (mc.layers[i].mixer for i in range(4))
+    assert isinstance(m0, ParallelSpec) and m0.right == MatrixMemorySpec(3, 8, 6, 7.0) and (m0.left_scale, m0.right_scale) == (0.7, 1.2)
+    assert m0.left.window == 11 and m0.left.keep_first == 3 and m0.left.head_sink and not m0.left.bias and m0.left.chunk == 0
+    assert m0.left.rot == RotarySpec(5000.0, 8, None, True) and m0.left.softcap == 0.0
+    assert isinstance(m1, GroupedAttentionSpec) and m1.chunk == 13 and m1.window == 0 and m1.softcap == 9.0 and m1.v_mix
+    assert m1.bias and m1.v_bias and m1.head_gate and m1.qk_weight and m1.rot is None and not m1.head_sink
+    assert isinstance(m2, DeltaSpec) and m2.channel_decay and m2.conv == 4 and not m3.v_mix and mc.layers[3].ff == 0
+    e = engine_for(tmp_path / "m", ("cpu", "fp32"))
+    assert type(e.model).__name__ == "LizesunModel" and e.model.first_mix == 1
+    assert e.kv.k_layer(2) is None and e.kv.sconv[2].shape == (5, 3, 2 * 2 * 6 + 4 * 10) and e.kv.sconv[0] is None
+    assert e.kv.rec[0].shape == (5, 3 * 8 * 7) and e.kv.gmax[0].shape == (5, 3) and e.kv.gmax[1] is None
+    assert any(t is e.kv.gmax[0] for t in e.kv.state_tensors())
+    for bad in ([dict(par(), type="wkv")], [att(), att(4, 4, 12, 10)], [delta(3, 2)], [par(rot_dims=14)], [par(rot_dims=5)]):
+        with pytest.raises(ValueError):
+            config_like(bad)
+    assert config_like([att(), att(4, 4, 12, 10, v_mix=False)]).n_layers == 2       # only mixing layers must agree
+    assert get_config("tiny-lizesun").arch == "lizesun"
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_whole_prompt_and_layers(tmp_path, run):
+    cfg = make_config()
+    P = make_checkpoint(tmp_path / "m", cfg, seed=1)
+    e = engine_for(tmp_path / "m", run)
+    t = toks(45, cfg["vocab"], 1)
+    layers = []
+    want = O.forward(cfg, P, t, layers)
+    got = e.step([("a", t, list(range(len(t))))])
+    close(got, want, run, "logits")
+    s = e.kv.seq("b")
+    tok, pos, meta = e._varlen_meta([e.reserve(s, t)])
+    keep = []
+    with torch.no_grad():
+        e.model.forward(tok, pos, e.kv, meta, keep_layers=keep)
+    assert len(keep) == len(layers) == 6
+    for i, (a, b) in enumerate(zip(keep, layers)):
+        err = (a.double().cpu() - b).abs().max(-1).values
+        assert float(err.median() if run[1] == "bf16" else err.max()) < (0.2 if run[1] == "bf16" else 1e-3), \
+            f"residual stream after layer {i}"
+
+
+SHAPES = {
+    # one query head per key/value head; one key/value head for all; one recurrence head
+    "groups": [att(3, 3, 8, 8, chunk=5), par(1, 6, 10, heads=5, kv=1, dim=6, vdim=4, rot_dims=6), att(6, 3, 4, 8, chunk=16, ff=0)],
+    # heads wider than a wave's 64 lanes; states of 72 x 132 and 130 x 8
+    "wide": [par(1, 72, 132, heads=2, kv=1, dim=72, vdim=132, rot_dims=40, ff=0), att(1, 1, 68, 70, chunk=33, ff=0),
+             delta(2, 1, 130, 8, conv=3, ff=0)],
+    # more query heads per key/value head than one attention workgroup's pairs
+    "many-heads": [par(2, 4, 4, heads=40, kv=1, dim=4, vdim=4, rot_dims=2), att(40, 1, 4, 4, chunk=9)],
+    # windows, chunks, taps and kept keys of one token, constants that are 1
+    "ones": [par(1, 4, 4, cap=1.0, ls=1.0, rs=1.0, heads=1, kv=1, dim=4, vdim=4, window=1, keep=1, rot_dims=4, scale=1.0, ff=0),
+             att(1, 1, 4, 4, chunk=1, softcap=1.0, scale=1.0), delta(1, 1, 4, 4, conv=1)],
+    # nothing masked, capped, mixed, rotated or kept
+    "off": [att(2, 1, 8, 6, chunk=0, softcap=None, v_mix=False), par(2, 6, 4, heads=2, kv=2, dim=6, vdim=8, window=0, rot_dims=0)],
+    # only recurrences; value heads over fewer key heads; five taps
+    "delta-only": [delta(6, 2, 4, 6, conv=5), delta(2, 2, 10, 4, conv=2, ff=0)],
+    # kept keys beyond the window; the mixing layers are the last ones, and neighbours
+    "kept": [par(2, 8, 8, window=3, keep=9, rot_dims=12), delta(), att(chunk=11), att(heads=2, kv=2, chunk=24), att(heads=4, kv=2, dim=7)],
+}
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("shape", list(SHAPES))
+def test_other_sizes(tmp_path, run, shape):
+    """Sizes, orders of layers and constants that the usual test model does not have, or makes equal or 1."""
+    cfg = make_config(width=24, vocab=61, layers=SHAPES[shape], embed_scale=1.0 if shape == "ones" else 2.1)
+    P = make_checkpoint(tmp_path / "m", cfg, seed=2, rank=1 if shape == "ones" else 6, gate_rank=1 if shape == "ones" else 3)
+    e = engine_for(tmp_path / "m", run, block_size=8)
+    t = toks(70, cfg["vocab"], 2)
+    want = O.forward(cfg, P, t)
+    got = torch.cat([e.step([("a", t[:37], list(range(37)))]), e.step([("a", t[37:39], [0, 1])])] +
+                    [e.step([("a", t[i:i + 1], [0])]) for i in range(39, 70)])
+    close(got, want, run, shape)
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("heads,kv,dim,vdim", [(8, 2, 64, 64), (6, 3, 96, 80), (4, 1, 128, 128)])
+def test_wider_layers(tmp_path, run, heads, kv, dim, vdim):
+    """Rows wide enough for several waves per workgroup, attention and recurrence heads of ordinary sizes, a
+    window and a chunk that cross many key tiles and pages: a prompt in portions (the first spans many
+    scan chunks), then decoded tokens."""
+    layers = [par(4, 64, 64, heads=heads, kv=kv, dim=dim, vdim=vdim, window=200, keep=6, rot_dims=dim // 2, ff=384),
+              att(heads, kv, dim, vdim, chunk=240, ff=384), delta(8, 4, 64, 64, ff=384),
+              att(heads, kv, dim, vdim, chunk=310, softcap=20.0, ff=384)]
+    cfg = make_config(width=512, vocab=331, layers=layers)
+    P = make_checkpoint(tmp_path / "m", cfg, seed=21, rank=24, gate_rank=40)
+    e = engine_for(tmp_path / "m", run, tokens=1024, block_size=32)
+    t = toks(520, cfg["vocab"], 21)
+    want = O.forward(cfg, P, t)
+    got = [e.step([("a", t[:300], [0, 5, 6, 199, 200, 201, 239, 240, 299])]), e.step([("a", t[300:302], [0, 1])]),
+           e.step([("a", t[302:500], [0, 7, 8, 177, 178, 197])])] + [e.step([("a", t[i:i + 1], [0])]) for i in range(500, 520)]
+    rows = [0, 5, 6, 199, 200, 201, 239, 240, 299, 300, 301, 302, 309, 310, 479, 480, 499] + list(range(500, 520))
+    close(torch.cat(got), want[rows], run, "wider layers")
+
+
+# ---- portions, decoding, batches ------------------------------------------------------------------
+
+@pytest.mark.parametrize("run", RUNS)
+def test_prefill_against_token_by_token(tmp_path, run):
+    cfg = make_config()
+    P = make_checkpoint(tmp_path / "m", cfg, seed=3)
+    e = engine_for(tmp_path / "m", run)
+    t = toks(40, cfg["vocab"], 3)
+    want = O.forward(cfg, P, t)
+    one = torch.cat([e.step([("a", [x], [0])]) for x in t])          # from the first token on
+    close(one, want, run, "token by token")
+    whole = e.step([("b", t, list(range(40)))])
+    close(whole, want, run, "whole")
+    if run[1] != "bf16":
+        assert float((one - whole).abs().max()) < 1e-3
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("cuts", [[2, 2, 3, 1, 30, 2, 17, 1, 1, 5], [16, 16, 16, 16], [1, 63], [33, 31], [131, 2, 70], [2] * 32])
+def test_portions(tmp_path, run, cuts):
+    """Portions of several sizes, down to two tokens and one, cut inside and at page borders (pages
+    of 16), inside windows, chunks and the convolutions' reach: every state carries over every cut."""
+    cfg = make_config()
+    P = make_checkpoint(tmp_path / "m", cfg, seed=4)
+    e = engine_for(tmp_path / "m", run)
+    t = toks(sum(cuts), cfg["vocab"], 4)
+    want = O.forward(cfg, P, t)
+    out, at = [], 0
+    for n in cuts:
+        out.append(e.step([("a", t[at:at + n], list(range(n)))]))
+        at += n
+    close(torch.cat(out), want, run, f"portions {cuts}")
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_mixed_batch_equals_each_alone_and_slots_are_reused(tmp_path, run):
+    """Unequal requests in one batch (portions beside single tokens, requests paused for a step),
+    a pool of four state slots and few pages, so both are freed and used again: a request that
+    takes a used slot starts from zero states."""
+    cfg = make_config()
+    P = make_checkpoint(tmp_path / "m", cfg, seed=5)
+    e = engine_for(tmp_path / "m", run, tokens=160, slots=4)
+    V = cfg["vocab"]
+    reqs = {k: toks(n, V, 10 + i) for i, (k, n) in enumerate([("a", 50), ("b", 7), ("c", 33), ("d", 1), ("e", 41), ("f", 20)])}
+    want = {k: O.forward(cfg, P, v) for k, v in reqs.items()}
+    got = {k: [] for k in reqs}
+    at = {k: 0 for k in reqs}
+    plan = [[("a", 20), ("b", 7)], [("a", 1), ("c", 30), ("d", 1)], [("a", 2), ("c", 1)], [("c", 2), ("a", 27), ("e", 3)],
+            [("e", 38), ("f", 5)], [("f", 1)], [("f", 14)]]
+    for step in plan:
+        entries, end = [], []
+        for k, n in step:
+            entries.append((k, reqs[k][at[k]:at[k] + n], list(range(n))))
+            at[k] += n
+            if at[k] == len(reqs[k]):
+                end.append(k)
+        out = e.step(entries, end=end)
+        o = 0
+        for k, n in step:
+            got[k].append(out[o:o + n])
+            o += n
+    if run[1] == "bf16":        # judged together: a request of one row has no median to speak of
+        close(torch.cat([torch.cat(got[k]) for k in reqs]), torch.cat([want[k] for k in reqs]), run, "all requests")
+    else:
+        for k in reqs:
+            close(torch.cat(got[k]), want[k], run, f"request {k}")
+    assert e.kv.alloc.num_free == e.kv.num_blocks and len(e.kv.state.free) == 4
+    with pytest.raises(KVCacheOOM):       # a fifth live request has no slot
+        for i in range(5):
+            e.step([(f"x{i}", [1, 2], [])])
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_long_decoding_past_windows_chunks_and_page_borders(tmp_path, run):
+    """150 tokens, all but five decoded one by one through pages of 8: windows slide over decoded tokens
+    and chunks begin among them many times."""
+    cfg = make_config()
+    P = make_checkpoint(tmp_path / "m", cfg, seed=7)
+    e = engine_for(tmp_path / "m", run, block_size=8)
+    t = toks(150, cfg["vocab"], 7)
+    want = O.forward(cfg, P, t)
+    got = torch.cat([e.step([("a", t[:5], list(range(5)))])] + [e.step([("a", [x], [0])]) for x in t[5:]])
+    close(got, want, run, "long decode")
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_rows_of_a_decode_batch_do_not_depend_on_each_other(tmp_path, run):
+    """Three sequences decoded together (the decode launches) against each decoded alone."""
+    cfg = make_config()
+    P = make_checkpoint(tmp_path / "m", cfg, seed=12)
+    V = cfg["vocab"]
+    reqs = {"a": toks(60, V, 1), "b": toks(31, V, 2), "c": toks(44, V, 3)}
+    e = engine_for(tmp_path / "m", run)
+    for k, t in reqs.items():
+        e.step([(k, t[:-20], [])])
+    got = {k: [] for k in reqs}
+    for i in range(20):
+        out = e.step([(k, [t[len(t) - 20 + i]], [0]) for k, t in reqs.items()])
+        for j, k in enumerate(reqs):
+            got[k].append(out[j:j + 1])
+    close(torch.cat([torch.cat(got[k]) for k in reqs]), torch.cat([O.forward(cfg, P, t)[-20:] for t in reqs.values()]), run)
+
+
+# ---- the engine's own generation path and scheduler -----------------------------------------------
+
+def _greedy_oracle(P, cfg, prompt, n):
+    seq = list(prompt)
+    for _ in range(n):
+        seq.append(int(O.forward(cfg, P, seq)[-1].argmax()))
+    return seq[len(prompt):]
+
+
+@pytest.mark.parametrize("run,graphs", [(("cpu", "fp32"), False), pytest.param(("cuda:0", "fp32"), False, marks=GPU),
+                                        pytest.param(("cuda:0", "fp32"), True, marks=GPU)])
+def test_greedy_generation_through_run_turns(tmp_path, run, graphs):
+    """Greedy decoding through Engine.run_turns (tokenizer, prefix reuse, batched decode loop — the
+    captured graph on the GPU) gives the oracle's tokens, for two requests of unequal length, and for
+    the first one continued."""
+    cfg = make_config(vocab=300, embed_scale=1.5)
+    P = make_checkpoint(tmp_path / "m", cfg, seed=8)
+    e = engine_for(tmp_path / "m", run, tokens=2048, graphs=graphs)
+    sp = SamplingParams(temperature=0.0, max_new_tokens=12, ignore_eos=True, stop_on_consensus=False)
+    prompts = ["De ridders aan de ronde tafel overleggen over het cachebeleid.", "Kort."]
+    outs = e.run_turns([Turn("A", prompts[0], sp), Turn("B", prompts[1], sp)])
+    for o, p in zip(outs, prompts):
+        assert o.error is None, o.error
+        ids = e.encode_prompt(p)
+        assert o.ids == _greedy_oracle(P, cfg, ids, 12)
+    from theroundtaible_amd.prompt import Prompt
+    p2 = Prompt().add(prompts[0]).add(outs[0].text, outs[0].ids, e.tokenizer.family)
+    o2 = e.run_turns([Turn("A", p2, sp)])[0]
+    ids2 = e.encode_prompt(prompts[0]) + outs[0].ids
+    assert o2.ids == _greedy_oracle(P, cfg, ids2, 12)
+
+
+@GPU
+def test_decode_steps_on_the_skinny_gemm(tmp_path):
+    """Sizes the framework's skinny decode GEMM takes (K a multiple of 32; N is padded to a multiple of
+    16): decode steps run their linears on it; the logits match the oracle and the same steps on the
+    library GEMMs."""
+    from theroundtaible_amd import ops
+    if not ops.native_available():
+        pytest.skip("main extension not built")
+    layers = [par(2, 16, 16, heads=4, kv=2, dim=16, vdim=16, rot_dims=8, ff=96), delta(4, 2, 16, 16, ff=64),
+              att(4, 2, 16, 16, ff=64)]
+    cfg = make_config(width=64, vocab=80, layers=layers)
+    P = make_checkpoint(tmp_path / "m", cfg, seed=11, rank=9, gate_rank=32)
+    t = toks(60, cfg["vocab"], 11)
+    want = O.forward(cfg, P, t)
+    outs = []
+    for skinny in (True, False):
+        e = engine_for(tmp_path / "m", ("cuda:0", "bf16"))
+        e.model.use_skinny = skinny
+        got = torch.cat([e.step([("a", t[:20], list(range(20)))])] + [e.step([("a", [x], [0])]) for x in t[20:]])
+        close(got, want, ("cuda:0", "bf16"), f"skinny={skinny}")
+        outs.append(got)
+        if skinny:
+            assert all("w_in" in d and "w_out" in d and "mlp.down" in d for d in e.model._dec.values())
+    err = (outs[0] - outs[1]).double().pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()
+    assert float(err.median()) < 0.03
+
+
+def test_serving_entry_points_match_run_turns():
+    """The continuous-batching entry points (prefill + first token, then decode in chunks while the
+    state follows) give the tokens of a single run_turns call; random-init preset weights."""
+    def eng():
+        return Engine(EngineConfig(model="tiny-lizesun", weights="random:3", dtype="fp32", device="cpu",
+                                   num_blocks=64, use_graphs=False, state_slots=4))
+    sp = SamplingParams(temperature=0.0, max_new_tokens=10, ignore_eos=True, stop_on_consensus=False)
+    turns = [Turn("A", "Eerste ridder spreekt over de cache.", sp), Turn("B", "Tweede.", sp)]
+    want = [o.ids for o in eng().run_turns(turns)]
+    e = eng()
+    started = e.start_turns(turns)
+    seqs = [s for s, _, _ in started]
+    got = [[f] for _, f, _ in started]
+    for steps in (4, 5):
+        new = e.continue_decode(seqs, turns, [g[-1] for g in got], steps)
+        for g, n in zip(got, new):
+            g.extend(n)
+    assert got == want
+    assert all(s.state_len == s.length for s in seqs)
+
+
+def test_fork_copies_every_state(tmp_path):
+    """A forked sequence continues exactly like its source: pages shared, convolution rows, matrix states
+    and gate maxima copied."""
+    cfg = make_config()
+    P = make_checkpoint(tmp_path / "m", cfg, seed=13)
+    e = engine_for(tmp_path / "m", ("cpu", "fp32"))
+    t = toks(50, cfg["vocab"], 13)
+    e.step([("a", t[:30], [])])
+    e.kv.fork("a", "b")
+    want = O.forward(cfg, P, t)[30:]
+    close(e.step([("a", t[30:], list(range(20)))]), want, ("cpu", "fp32"), "source")
+    close(e.step([("b", t[30:], list(range(20)))]), want, ("cpu", "fp32"), "fork")
+
+
+def test_trace_runner_replays_steps(tmp_path):
+    """The trace runner's own entry point on the CPU: steps in, logit files out, pages and slots
+    given back at the end of a request."""
+    import io
+    import sys
+    import numpy as np
+    from theroundtaible_amd import trace_run
+    cfg = make_config(vocab=50)
+    P = make_checkpoint(tmp_path / "m", cfg, seed=9)
+    t = toks(30, 50, 9)
+    want = O.forward(cfg, P, t)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": t[:20], "want": [0, 19]}], "end": []},
+             {"step": 1, "entries": [{"id": "a", "tokens": t[20:22], "want": []}], "end": []},
+             {"step": 2, "entries": [{"id": "a", "tokens": t[22:], "want": [7]}, {"id": "b", "tokens": t[:3], "want": [2]}],
+              "end": ["a", "b"]}]
+    old_in, old_out = sys.stdin, sys.stdout
+    sys.stdin, sys.stdout = io.StringIO("\n".join(json.dumps(s) for s in steps) + "\n"), io.StringIO()
+    try:
+        rc = trace_run.main(["--model", str(tmp_path / "m"), "--dtype", "float32", "--out", str(tmp_path / "o"),
+                             "--max-tokens", "128", "--device", "cpu"])
+        said = sys.stdout.getvalue()
+    finally:
+        sys.stdin, sys.stdout = old_in, old_out
+    assert rc == 0 and [l for l in said.splitlines() if l.startswith("done")] == ["done 0", "done 1", "done 2"]
+    assert not os.path.exists(tmp_path / "o" / "1.f32")
+    a = np.fromfile(tmp_path / "o" / "0.f32", dtype="<f4").reshape(2, 50)
+    b = np.fromfile(tmp_path / "o" / "2.f32", dtype="<f4").reshape(2, 50)
+    got = torch.tensor(np.concatenate([a, b])).double()
+    assert float((got - want[[0, 19, 29, 2]]).abs().max()) < 2e-3
