@@ -105,7 +105,7 @@ int launch_state_scan(float* out, const float* q, const float* k, const float* v
                       const float* b, int sq, int sk, int sv, int sw, int sa, int sb, const float* decay, float* state,
                       const int* cu_q, const int* start_pos, const int* slots, int S, int T, int A, int D, int E,
                       const int* chunks, int n_chunks, int chunk_rows, const int* seq_chunk0, float* ws,
-                      hipStream_t stream);
+                      bool head_decay, hipStream_t stream);
 
 namespace {
 
@@ -787,7 +787,7 @@ void channel_delta_prep(torch::Tensor out, torch::Tensor vout, torch::Tensor pro
   TORCH_CHECK(rc == 0, "channel_delta_prep: a row does not fit the LDS (code ", rc, ")");
 }
 
-// out [T, 3 A D + A (E + 1)], gates [3, T, A]; proj columns q_off, k_off (A D), v_off (A E), i_off, f_off (A)
+// out [T, 2 A D + A (E + 1)], gates [3, T, A]; proj columns q_off, k_off (A D), v_off (A E), i_off, f_off (A)
 void memory_prep(torch::Tensor out, torch::Tensor gates, torch::Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off,
                  int64_t i_off, int64_t f_off, torch::Tensor ib, torch::Tensor fb, double cap, torch::Tensor gmax,
                  torch::Tensor cu_q, torch::Tensor start_pos, torch::Tensor slots, double q_scale, int64_t A, int64_t D,
@@ -795,7 +795,7 @@ void memory_prep(torch::Tensor out, torch::Tensor gates, torch::Tensor proj, int
   chk_act(proj, "proj");
   TORCH_CHECK(proj.dim() == 2 && A >= 1 && D >= 1 && E >= 1 && cap > 0, "memory_prep: sizes");
   const int64_t T = proj.size(0), N = proj.size(1), S = cu_q.numel() - 1;
-  chk_f32(out, "out", T * (3 * A * D + A * (E + 1))); chk_f32(gates, "gates", 3 * T * A);
+  chk_f32(out, "out", T * (2 * A * D + A * (E + 1))); chk_f32(gates, "gates", 3 * T * A);
   TORCH_CHECK(q_off >= 0 && q_off + A * D <= N && k_off >= 0 && k_off + A * D <= N && v_off >= 0 && v_off + A * E <= N &&
               i_off >= 0 && i_off + A <= N && f_off >= 0 && f_off + A <= N, "memory_prep: columns");
   chk_f32(ib, "i_b", A); chk_f32(fb, "f_b", A); chk_f32(gmax, "gmax");
@@ -832,7 +832,8 @@ void state_scan(torch::Tensor out, torch::Tensor q, torch::Tensor k, torch::Tens
   const float* qp = stream_of(q, "q", T, A * D, sq);
   const float* kp = stream_of(k, "k", T, A * D, sk);
   const float* vp = stream_of(v, "v", T, A * E, sv);
-  const float* wp = stream_of(w, "w", T, A * D, sw);
+  const bool head_decay = w.has_value() && w->dim() == 2 && w->size(1) == A && D != 1;      // one decay per head and token
+  const float* wp = stream_of(w, "w", T, head_decay ? A : A * D, sw);
   const float* ap = stream_of(a, "a", T, A * D, sa);
   const float* bp = stream_of(b, "b", T, A * D, sb);
   TORCH_CHECK(a.has_value() == b.has_value(), "state_scan: a and b come together");
@@ -845,12 +846,12 @@ void state_scan(torch::Tensor out, torch::Tensor q, torch::Tensor k, torch::Tens
   float* wsp = nullptr;
   int n_chunks = 0;
   if (chunks.has_value()) {
-    TORCH_CHECK(!a.has_value(), "state_scan: a recurrence that removes cannot be scanned in chunks");
+    TORCH_CHECK(!a.has_value() || !head_decay, "state_scan: a recurrence that removes takes a decay per key channel");
     TORCH_CHECK(seq_chunk0.has_value() && ws.has_value() && chunk_rows >= 1, "state_scan: chunks need their lists and scratch");
     chk_i32(*chunks, "chunks"); chk_i32(*seq_chunk0, "seq_chunk0", S + 1); chk_f32(*ws, "ws");
     TORCH_CHECK(chunks->dim() == 2 && chunks->size(1) == 2, "state_scan: chunks [n, 2]");
     n_chunks = (int)chunks->size(0);
-    TORCH_CHECK(ws->numel() >= (int64_t)n_chunks * A * D * (E + 1), "state_scan: scratch too small");
+    TORCH_CHECK(ws->numel() >= (int64_t)n_chunks * A * D * (a.has_value() ? E + D : E + 1), "state_scan: scratch too small");
     cp = chunks->data_ptr<int>();
     c0p = seq_chunk0->data_ptr<int>();
     wsp = ws->data_ptr<float>();
@@ -858,7 +859,7 @@ void state_scan(torch::Tensor out, torch::Tensor q, torch::Tensor k, torch::Tens
   int rc = launch_state_scan(out.data_ptr<float>(), qp, kp, vp, wp, ap, bp, sq, sk, sv, sw, sa, sb,
                              opt_f32(decay, "decay", A), state.data_ptr<float>(), cu_q.data_ptr<int>(),
                              start_pos.data_ptr<int>(), slots.data_ptr<int>(), (int)S, (int)T, (int)A, (int)D, (int)E,
-                             cp, n_chunks, (int)chunk_rows, c0p, wsp, cur());
+                             cp, n_chunks, (int)chunk_rows, c0p, wsp, head_decay, cur());
   TORCH_CHECK(rc == 0, "state_scan: unsupported shape (code ", rc, ")");
 }
 

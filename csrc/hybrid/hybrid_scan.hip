@@ -2,9 +2,10 @@
 //
 //   s = b_t^T S ;  S <- diag(w_t) S - a_t s^T + k_t v_t^T ;  o_t = S^T q_t
 //
-// (w: a stream per key channel, or one constant per head; a / b: optional removal streams.) This
-// covers a constant-decay linear attention (no a / b), a generalized delta rule (a = rate * unit
-// key, b = unit key) and a gated delta rule (w = g, a = g beta k, b = k, k <- beta k).
+// (w: a stream per key channel, a stream per head, or one constant per head; a / b: optional removal
+// streams.) This covers a constant-decay linear attention (no a / b), a matrix memory with
+// exponential gates (a decay per head and token), a generalized delta rule (a = rate * unit key, b =
+// unit key) and gated delta rules (w = g, a = k <- beta k, b = g k: a and k are one stream then).
 //
 // The token loop is a dependent chain, so its length per token is what counts. The columns of S
 // are independent; a lane owns DR rows of ONE column in registers, the P = D / DR lanes of a
@@ -23,7 +24,9 @@
 // leaving its end state and its decay product; (2) chunk by chunk, an entry of S per lane, the state
 // each chunk starts from (carry = product * carry + end state, written over the end state) and the
 // sequence's new state; (3) every chunk again from its true start state, writing the outputs. There is
-// no division by a decay product, so decays close to zero are harmless.
+// no division by a decay product, so decays close to zero are harmless. With removal streams the effect
+// is a D x D matrix per chunk: launch (1) also runs D columns that start as the identity and get no
+// values, which end as that matrix, and launch (2) multiplies by it.
 #include "../common.h"
 
 namespace {
@@ -59,17 +62,22 @@ RT_DEVICE float4 load4(const float* __restrict__ row, int r, int D, bool vec) {
 // UNROLL: whole chunks run unrolled (prompts); without it the code is a fraction of the size, which is
 // what a launch over single rows (a decode step, cold instruction cache) is timed by
 // MODE 0: whole spans, state in and out of the slots; 1 / 2: launch (1) / (3) of the chunked form
-template <int DR, bool HAS_W, bool HAS_AB, bool UNROLL, int MODE>
+// W: 0 a constant per head, 1 a decay per head and key channel, 2 a decay per head; AB: 0 no removal,
+// 1 streams a and b, 2 a is the stream k. EC: columns kept per chunk and head in ws_e
+template <int DR, int W, int AB, bool UNROLL, int MODE>
 __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
     float* __restrict__ out, const float* __restrict__ q, const float* __restrict__ k, const float* __restrict__ v,
     const float* __restrict__ w, const float* __restrict__ a, const float* __restrict__ b, int sq, int sk, int sv, int sw,
     int sa, int sb, const float* __restrict__ decay, float* __restrict__ state, const int* __restrict__ cu_q,
     const int* __restrict__ start_pos, const int* __restrict__ slots, int A, int D, int E, int P, int lgP, int vec,
-    const int* __restrict__ chunks, int chunk_rows, float* __restrict__ ws_e, float* __restrict__ ws_p) {
+    const int* __restrict__ chunks, int chunk_rows, float* __restrict__ ws_e, float* __restrict__ ws_p, int EC) {
   extern __shared__ float4 lds4[];
+  constexpr bool HAS_W = W == 1, HAS_AB = AB != 0, HAS_A = AB == 1;
+  constexpr bool WIDE = MODE == 1 && HAS_AB;    // the identity's columns run too
+  constexpr bool PROD = MODE == 1 && !HAS_AB;   // the chunk's decay product is kept
   constexpr bool OUT = MODE != 1;               // q is read and outputs are written
   constexpr int NQ = OUT ? 1 : 0;
-  constexpr int NS = NQ + 1 + (HAS_W ? 1 : 0) + (HAS_AB ? 2 : 0);
+  constexpr int NS = NQ + 1 + (HAS_W ? 1 : 0) + (HAS_A ? 1 : 0) + (HAS_AB ? 1 : 0);
   constexpr int NL = (kTT * DR + 63) / 64;      // 16-byte loads per lane, stream and chunk (P <= 16)
   constexpr int R4 = DR / 4;
   const int seq = MODE == 0 ? (int)blockIdx.x : chunks[2 * blockIdx.x], head = blockIdx.y;
@@ -84,11 +92,12 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
   float4* str = lds4;                                             // [kTT][NS][Dp4]
   float* vs = reinterpret_cast<float*>(str + kTT * NS * Dp4);     // [kTT][CB]
   float* os = vs + kTT * CB;                                      // [kTT][256]: every lane's share of q . S
+  float* whs = os + kTT * kScanThreads;                           // [kTT]: W 2's decays
   const int row_lo = part * DR;
-  const bool live = col < E;
+  const bool live = col < (WIDE ? EC : E);
   float S[DR];
-  float* sp = (MODE == 0 ? state + (size_t)slots[seq] * A * E * D : ws_e + (size_t)blockIdx.x * A * E * D) +
-              ((size_t)head * E + (live ? col : 0)) * D + row_lo;
+  float* sp = MODE == 0 ? state + (size_t)slots[seq] * A * E * D + ((size_t)head * E + (live ? col : 0)) * D + row_lo
+                        : ws_e + (((size_t)blockIdx.x * A + head) * EC + (live ? col : 0)) * D + row_lo;
   const bool cont = MODE == 0 ? start_pos[seq] > 0 : MODE == 2;
   const bool svec = (D & 3) == 0;
 #pragma unroll
@@ -97,10 +106,14 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
     if (cont && live) t = load4(sp, i4 * 4, D - row_lo, svec);
     S[i4 * 4] = t.x; S[i4 * 4 + 1] = t.y; S[i4 * 4 + 2] = t.z; S[i4 * 4 + 3] = t.w;
   }
-  float prod[MODE == 1 ? DR : 1];               // MODE 1: product of the chunk's decays, per row
+  if (WIDE) {
 #pragma unroll
-  for (int i = 0; i < (MODE == 1 ? DR : 1); ++i) prod[i] = 1.f;
-  const float dconst = HAS_W ? 1.f : decay[head];
+    for (int i = 0; i < DR; ++i) S[i] = col - E == row_lo + i ? 1.f : 0.f;
+  }
+  float prod[PROD ? DR : 1];                    // product of the chunk's decays, per row
+#pragma unroll
+  for (int i = 0; i < (PROD ? DR : 1); ++i) prod[i] = 1.f;
+  const float dconst = W == 0 ? decay[head] : 1.f;
   const float* src[NS];
   int strides[NS];
   {
@@ -108,10 +121,12 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
     if (OUT) { src[j] = q; strides[j++] = sq; }
     src[j] = k; strides[j++] = sk;
     if (HAS_W) { src[j] = w; strides[j++] = sw; }
-    if (HAS_AB) { src[j] = a; strides[j++] = sa; src[j] = b; strides[j++] = sb; }
+    if (HAS_A) { src[j] = a; strides[j++] = sa; }
+    if (HAS_AB) { src[j] = b; strides[j++] = sb; }
   }
   float4 pre[NS][NL];
   float prev[kTT];        // this lane's share of the chunk's value columns: kTT / P entries
+  float prew = 1.f;
   const int nv = kTT >> lgP;      // 0 when P > kTT cannot happen (P <= 16 = kTT)
   auto fetch = [&](int c0) {
     const int nt = min(kTT, n - c0);
@@ -136,6 +151,7 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
         prev[l] = (tok < nt && gc < E) ? v[(size_t)(r0 + c0 + tok) * sv + head * E + gc] : 0.f;
       }
     }
+    if (W == 2 && (int)threadIdx.x < nt) prew = w[(size_t)(r0 + c0 + threadIdx.x) * sw + head];
   };
   fetch(0);
   for (int c0 = 0; c0 < n; c0 += kTT) {
@@ -153,13 +169,14 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
 #pragma unroll
     for (int l = 0; l < kTT; ++l)
       if (l < nv) vs[threadIdx.x + l * kScanThreads] = prev[l];
+    if (W == 2 && threadIdx.x < kTT) whs[threadIdx.x] = prew;
     __syncthreads();
     if (c0 + kTT < n) fetch(c0 + kTT);      // in flight while this chunk is computed
     // One token: s = b . S (summed over the column's lanes, the only cross-lane step on the chain),
     // the update, and this lane's share of q . S, which goes to LDS as it is: the shares of a
     // column are added when the chunk's outputs are written, not inside the token loop.
     auto step = [&](int tok, const float4* tq, const float4* tk, const float4* tw, const float4* ta, const float4* tb,
-                    float vv) {
+                    float vv, float wh) {
       float sv_ = 0.f;
       if (HAS_AB) {
 #pragma unroll
@@ -169,16 +186,18 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
         }
         sv_ = group_sum(sv_, P);
       }
+      if (AB == 2) vv -= sv_;
       float acc = 0.f;
 #pragma unroll
       for (int i4 = 0; i4 < R4; ++i4) {
         const float4 kk = tk[i4];
         float u0 = kk.x * vv, u1 = kk.y * vv, u2 = kk.z * vv, u3 = kk.w * vv;
-        if (HAS_AB) {
+        if (HAS_A) {
           const float4 aa = ta[i4];
           u0 -= aa.x * sv_; u1 -= aa.y * sv_; u2 -= aa.z * sv_; u3 -= aa.w * sv_;
         }
-        float d0 = dconst, d1 = dconst, d2 = dconst, d3 = dconst;
+        const float dh = W == 2 ? wh : dconst;
+        float d0 = dh, d1 = dh, d2 = dh, d3 = dh;
         if (HAS_W) {
           const float4 ww = tw[i4];
           d0 = ww.x; d1 = ww.y; d2 = ww.z; d3 = ww.w;
@@ -191,48 +210,47 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
           const float4 qq = tq[i4];
           acc += qq.x * S[i4 * 4] + qq.y * S[i4 * 4 + 1] + qq.z * S[i4 * 4 + 2] + qq.w * S[i4 * 4 + 3];
         }
-        if (MODE == 1) {
+        if constexpr (PROD) {
           prod[i4 * 4] *= d0; prod[i4 * 4 + 1] *= d1; prod[i4 * 4 + 2] *= d2; prod[i4 * 4 + 3] *= d3;
         }
       }
       if (OUT) os[tok * kScanThreads + threadIdx.x] = acc;
     };
-    auto read_tok = [&](int tok, float4* tq, float4* tk, float4* tw, float4* ta, float4* tb, float& tv) {
+    auto read_tok = [&](int tok, float4* tq, float4* tk, float4* tw, float4* ta, float4* tb, float& tv, float& th) {
       const float4* qs = str + (tok * NS) * Dp4 + part * R4;
       const float4* ks = qs + NQ * Dp4;
       const float4* ws = ks + Dp4;                              // HAS_W
-      const float4* as = ks + (HAS_W ? 2 : 1) * Dp4;            // HAS_AB
-      const float4* bs = as + Dp4;
+      const float4* as = ks + (HAS_W ? 2 : 1) * Dp4;            // HAS_A
+      const float4* bs = as + (HAS_A ? Dp4 : 0);                // HAS_AB
 #pragma unroll
       for (int i4 = 0; i4 < R4; ++i4) {
         if (OUT) tq[i4] = qs[i4];
         tk[i4] = ks[i4];
         if (HAS_W) tw[i4] = ws[i4];
-        if (HAS_AB) {
-          ta[i4] = as[i4];
-          tb[i4] = bs[i4];
-        }
+        if (HAS_A) ta[i4] = as[i4];
+        if (HAS_AB) tb[i4] = bs[i4];
       }
       tv = vs[tok * CB + cl];
+      if (W == 2) th = whs[tok];
     };
     if (UNROLL && nt == kTT) {
       // a whole chunk: unrolled, two operand sets in turn, so the operands of token tok + 1 are
       // read from LDS while token tok is computed and nothing is copied
       float4 oq[2][R4], ok[2][R4], ow[2][R4], oa[2][R4], ob[2][R4];
-      float ov[2];
-      read_tok(0, oq[0], ok[0], ow[0], oa[0], ob[0], ov[0]);
+      float ov[2], oh[2] = {1.f, 1.f};
+      read_tok(0, oq[0], ok[0], ow[0], oa[0], ob[0], ov[0], oh[0]);
 #pragma unroll
       for (int tok = 0; tok < kTT; ++tok) {
         const int c = tok & 1, nx = c ^ 1;
-        if (tok + 1 < kTT) read_tok(tok + 1, oq[nx], ok[nx], ow[nx], oa[nx], ob[nx], ov[nx]);
-        step(tok, oq[c], ok[c], ow[c], oa[c], ob[c], ov[c]);
+        if (tok + 1 < kTT) read_tok(tok + 1, oq[nx], ok[nx], ow[nx], oa[nx], ob[nx], ov[nx], oh[nx]);
+        step(tok, oq[c], ok[c], ow[c], oa[c], ob[c], ov[c], oh[c]);
       }
     } else {
       float4 tq[R4], tk[R4], tw[R4], ta[R4], tb[R4];
-      float tv;
+      float tv, th = 1.f;
       for (int tok = 0; tok < nt; ++tok) {
-        read_tok(tok, tq, tk, tw, ta, tb, tv);
-        step(tok, tq, tk, tw, ta, tb, tv);
+        read_tok(tok, tq, tk, tw, ta, tb, tv, th);
+        step(tok, tq, tk, tw, ta, tb, tv, th);
       }
     }
     if (!OUT) continue;
@@ -247,11 +265,11 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
     }
   }
   if (MODE == 2) return;      // the sequence's new state came out of the carry
-  if (MODE == 1 && blockIdx.z == 0 && cl == 0) {
+  if (PROD && blockIdx.z == 0 && cl == 0) {
     float* pp = ws_p + ((size_t)blockIdx.x * A + head) * D + row_lo;
 #pragma unroll
     for (int i = 0; i < DR; ++i)
-      if (row_lo + i < D) pp[i] = prod[MODE == 1 ? i : 0];
+      if (row_lo + i < D) pp[i] = prod[PROD ? i : 0];
   }
   if (live) {
     if (svec && row_lo + DR <= D) {
@@ -301,6 +319,112 @@ __global__ void __launch_bounds__(256) state_carry_kernel(float* __restrict__ ws
   *st = S;
 }
 
+// launch (2) with removal: per (sequence, head, 4 * 256 / Dp columns) the chain S <- M_c S + B_c over the
+// chunks, ws_e[chunk][head][E columns of B, then D columns of M][D]; the state a chunk starts from is
+// written over its B. Lane = (row i, a group of 4 columns): it reads row i of M (coalesced over i), the
+// columns of S sit in LDS. DM >= D: the next chunk's row of M is loaded while this one is used.
+template <int DM>
+__global__ void __launch_bounds__(256) state_carry_matrix_kernel(float* __restrict__ ws_e, float* __restrict__ state,
+                                                                 const int* __restrict__ seq_chunk0,
+                                                                 const int* __restrict__ start_pos,
+                                                                 const int* __restrict__ slots, int A, int D, int E, int lgDp) {
+  extern __shared__ float4 cols[];      // [2][D][groups]
+  const int s = blockIdx.x, h = blockIdx.y;
+  const int k0 = seq_chunk0[s], k1 = seq_chunk0[s + 1];
+  if (k1 <= k0) return;
+  const int Dp = 1 << lgDp, groups = 256 >> lgDp;
+  const int i = threadIdx.x & (Dp - 1), g = threadIdx.x >> lgDp;
+  const int col = (blockIdx.z * groups + g) * 4;
+  const int EC = E + D;
+  const bool row = i < D;
+  float* st = state + ((size_t)slots[s] * A + h) * E * D;
+  const bool cont = start_pos[s] > 0;
+  float S[4];
+#pragma unroll
+  for (int c = 0; c < 4; ++c) S[c] = cont && row && col + c < E ? st[(size_t)(col + c) * D + i] : 0.f;
+  auto load = [&](int k, float (&m)[DM], float (&bb)[4]) {
+    const float* base = ws_e + ((size_t)k * A + h) * EC * D;
+#pragma unroll
+    for (int c = 0; c < 4; ++c) bb[c] = row && col + c < E ? base[(size_t)(col + c) * D + i] : 0.f;
+#pragma unroll
+    for (int j = 0; j < DM; ++j) m[j] = row && j < D ? base[(size_t)(E + j) * D + i] : 0.f;
+  };
+  float m[DM], b[4];
+  load(k0, m, b);
+  for (int k = k0; k < k1; ++k) {
+    float4* cur = cols + ((k - k0) & 1) * D * groups;
+    if (row) cur[i * groups + g] = float4{S[0], S[1], S[2], S[3]};
+    __syncthreads();      // (the other buffer's readers are past the barrier of the step before)
+    float mn[DM], bn[4];
+    if (k + 1 < k1) load(k + 1, mn, bn);
+    float acc[4] = {b[0], b[1], b[2], b[3]};
+#pragma unroll
+    for (int j = 0; j < DM; ++j)
+      if (j < D) {
+        const float4 sj = cur[j * groups + g];
+        acc[0] += m[j] * sj.x; acc[1] += m[j] * sj.y; acc[2] += m[j] * sj.z; acc[3] += m[j] * sj.w;
+      }
+    float* base = ws_e + ((size_t)k * A + h) * EC * D;
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      if (row && col + c < E) base[(size_t)(col + c) * D + i] = S[c];
+      S[c] = acc[c];
+    }
+    if (k + 1 < k1) {
+#pragma unroll
+      for (int j = 0; j < DM; ++j) m[j] = mn[j];
+#pragma unroll
+      for (int c = 0; c < 4; ++c) b[c] = bn[c];
+    }
+  }
+#pragma unroll
+  for (int c = 0; c < 4; ++c)
+    if (row && col + c < E) st[(size_t)(col + c) * D + i] = S[c];
+}
+
+// the same for any D <= 256, without the rows in registers
+__global__ void __launch_bounds__(256) state_carry_matrix_any_kernel(float* __restrict__ ws_e, float* __restrict__ state,
+                                                                     const int* __restrict__ seq_chunk0,
+                                                                     const int* __restrict__ start_pos,
+                                                                     const int* __restrict__ slots, int A, int D, int E) {
+  extern __shared__ float4 cols[];      // [2][D]
+  const int s = blockIdx.x, h = blockIdx.y, i = threadIdx.x, col = blockIdx.z * 4;
+  const int k0 = seq_chunk0[s], k1 = seq_chunk0[s + 1];
+  if (k1 <= k0) return;
+  const int EC = E + D;
+  const bool row = i < D;
+  float* st = state + ((size_t)slots[s] * A + h) * E * D;
+  const bool cont = start_pos[s] > 0;
+  float S[4];
+#pragma unroll
+  for (int c = 0; c < 4; ++c) S[c] = cont && row && col + c < E ? st[(size_t)(col + c) * D + i] : 0.f;
+  for (int k = k0; k < k1; ++k) {
+    float4* cur = cols + ((k - k0) & 1) * D;
+    if (row) cur[i] = float4{S[0], S[1], S[2], S[3]};
+    __syncthreads();
+    if (row) {
+      float* base = ws_e + ((size_t)k * A + h) * EC * D;
+      float acc[4];
+#pragma unroll
+      for (int c = 0; c < 4; ++c) acc[c] = col + c < E ? base[(size_t)(col + c) * D + i] : 0.f;
+#pragma unroll 8
+      for (int j = 0; j < D; ++j) {
+        const float4 sj = cur[j];
+        const float mj = base[(size_t)(E + j) * D + i];
+        acc[0] += mj * sj.x; acc[1] += mj * sj.y; acc[2] += mj * sj.z; acc[3] += mj * sj.w;
+      }
+#pragma unroll
+      for (int c = 0; c < 4; ++c) {
+        if (col + c < E) base[(size_t)(col + c) * D + i] = S[c];
+        S[c] = acc[c];
+      }
+    }
+  }
+#pragma unroll
+  for (int c = 0; c < 4; ++c)
+    if (row && col + c < E) st[(size_t)(col + c) * D + i] = S[c];
+}
+
 }  // namespace
 
 // rows of a column one lane keeps, and lanes per column (a power of two <= 16), for D state rows
@@ -318,23 +442,25 @@ int launch_state_scan(float* out, const float* q, const float* k, const float* v
                       const float* b, int sq, int sk, int sv, int sw, int sa, int sb, const float* decay, float* state,
                       const int* cu_q, const int* start_pos, const int* slots, int S, int T, int A, int D, int E,
                       const int* chunks, int n_chunks, int chunk_rows, const int* seq_chunk0, float* ws,
-                      hipStream_t stream) {
+                      bool head_decay, hipStream_t stream) {
   if (S <= 0) return 0;
   if (chunks != nullptr && n_chunks <= 0) return 0;
   const bool unroll = T > 2 * S;      // rows per span on average: single rows take the small kernel
   int DR, P, lgP;
   scan_shape(D, DR, P, lgP);
   if (P > 16 || D < 1 || E < 1) return -1;
-  const bool has_w = w != nullptr, has_ab = a != nullptr && b != nullptr;
-  if (!has_w && decay == nullptr) return -2;
+  const bool has_w = w != nullptr && !head_decay, has_ab = a != nullptr && b != nullptr;
+  const bool a_is_k = has_ab && a == k && sa == sk;
+  if (w == nullptr && decay == nullptr) return -2;
   if (!has_w && has_ab) return -4;
-  const int NS = 2 + (has_w ? 1 : 0) + (has_ab ? 2 : 0);
+  const int NS = 2 + (has_w ? 1 : 0) + (has_ab ? (a_is_k ? 1 : 2) : 0);
   const int CB = kScanThreads / P, Dp = P * DR;
   // 16-byte loads of the streams: every row start and the head offset on a 16-byte boundary
   auto al = [&](const float* p, int st) { return p == nullptr || ((reinterpret_cast<uintptr_t>(p) & 15) == 0 && (st & 3) == 0); };
-  const int vec = (D & 3) == 0 && al(q, sq) && al(k, sk) && al(w, sw) && al(a, sa) && al(b, sb) ? 1 : 0;
-  const size_t shm = sizeof(float) * (size_t)kTT * ((size_t)NS * Dp + CB + kScanThreads);
-  dim3 grid(chunks != nullptr ? n_chunks : S, A, (E + CB - 1) / CB);
+  const int vec = (D & 3) == 0 && al(q, sq) && al(k, sk) && (head_decay || al(w, sw)) && al(a, sa) && al(b, sb) ? 1 : 0;
+  const size_t shm = sizeof(float) * (size_t)kTT * ((size_t)NS * Dp + CB + kScanThreads + 1);
+  const int EC = has_ab ? E + D : E;      // columns per chunk and head in the scratch
+  const dim3 grid_e(chunks != nullptr ? n_chunks : S, A, (E + CB - 1) / CB), grid_w(n_chunks, A, (EC + CB - 1) / CB);
   float* ws_e = ws;
   float* ws_p = ws != nullptr ? ws + (size_t)n_chunks * A * E * D : nullptr;
 #define RT_SCAN(DRV, HW, HAB)                                                                                          \
@@ -347,29 +473,46 @@ int launch_state_scan(float* out, const float* q, const float* k, const float* v
     if (shm > 48 * 1024 &&                                                                                             \
         hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm) != hipSuccess)    \
       return -3;                                                                                                       \
-    kern<<<grid, kScanThreads, shm, stream>>>(out, q, k, v, w, a, b, sq, sk, sv, sw, sa, sb, decay, state, cu_q,       \
-                                              start_pos, slots, A, D, E, P, lgP, vec, chunks, chunk_rows, ws_e, ws_p); \
+    kern<<<MODE == 1 ? grid_w : grid_e, kScanThreads, shm, stream>>>(out, q, k, v, w, a, b, sq, sk, sv, sw, sa, sb,    \
+                                                                     decay, state, cu_q, start_pos, slots, A, D, E, P, \
+                                                                     lgP, vec, chunks, chunk_rows, ws_e, ws_p, EC);    \
   } while (0)
 #define RT_SCAN_DR(HW, HAB)                                                                                            \
   do {                                                                                                                 \
     if (DR == 4) RT_SCAN(4, HW, HAB); else if (DR == 8) RT_SCAN(8, HW, HAB); else RT_SCAN(16, HW, HAB);                \
   } while (0)
-#define RT_CHUNK(HW, MODE)                                                                                             \
+#define RT_CHUNK(HW, HAB, MODE)                                                                                        \
   do {                                                                                                                 \
-    if (DR == 4) RT_SCAN_U(4, HW, false, true, MODE); else if (DR == 8) RT_SCAN_U(8, HW, false, true, MODE);           \
-    else RT_SCAN_U(16, HW, false, true, MODE);                                                                         \
+    if (DR == 4) RT_SCAN_U(4, HW, HAB, true, MODE); else if (DR == 8) RT_SCAN_U(8, HW, HAB, true, MODE);               \
+    else RT_SCAN_U(16, HW, HAB, true, MODE);                                                                           \
+  } while (0)
+#define RT_ANY(LAUNCH, ...)                                                                                            \
+  do {                                                                                                                 \
+    if (has_ab && a_is_k) LAUNCH(1, 2, ##__VA_ARGS__); else if (has_ab) LAUNCH(1, 1, ##__VA_ARGS__);                   \
+    else if (has_w) LAUNCH(1, 0, ##__VA_ARGS__); else if (head_decay) LAUNCH(2, 0, ##__VA_ARGS__);                     \
+    else LAUNCH(0, 0, ##__VA_ARGS__);                                                                                  \
   } while (0)
   if (chunks != nullptr) {
-    if (has_ab) return -5;
-    if (has_w) RT_CHUNK(true, 1); else RT_CHUNK(false, 1);
-    state_carry_kernel<<<dim3(S, A, (D * E + 255) / 256), 256, 0, stream>>>(ws_e, ws_p, state, seq_chunk0, start_pos, slots,
-                                                                            A, D, E);
-    if (has_w) RT_CHUNK(true, 2); else RT_CHUNK(false, 2);
+    RT_ANY(RT_CHUNK, 1);
+    if (has_ab) {
+      int lgDp = 5;
+      while ((1 << lgDp) < D) ++lgDp;
+      const int groups = 256 >> lgDp;
+      const dim3 grid(S, A, (E + 4 * groups - 1) / (4 * groups));
+      const size_t cshm = sizeof(float4) * 2 * (size_t)D * groups;
+      if (D <= 64) state_carry_matrix_kernel<64><<<grid, 256, cshm, stream>>>(ws_e, state, seq_chunk0, start_pos, slots, A, D,
+                                                                              E, lgDp);
+      else state_carry_matrix_any_kernel<<<dim3(S, A, (E + 3) / 4), 256, sizeof(float4) * 2 * (size_t)D, stream>>>(
+          ws_e, state, seq_chunk0, start_pos, slots, A, D, E);
+    } else {
+      state_carry_kernel<<<dim3(S, A, (D * E + 255) / 256), 256, 0, stream>>>(ws_e, ws_p, state, seq_chunk0, start_pos,
+                                                                              slots, A, D, E);
+    }
+    RT_ANY(RT_CHUNK, 2);
     return 0;
   }
-  if (has_w && has_ab) RT_SCAN_DR(true, true);
-  else if (!has_w) RT_SCAN_DR(false, false);
-  else RT_SCAN_DR(true, false);
+  RT_ANY(RT_SCAN_DR);
+#undef RT_ANY
 #undef RT_SCAN_DR
 #undef RT_CHUNK
 #undef RT_SCAN

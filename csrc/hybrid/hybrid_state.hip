@@ -576,7 +576,7 @@ __global__ void __launch_bounds__(64) memory_gates_kernel(float* __restrict__ ga
   if (lane == 0) *mp = m;
 }
 
-// out [T][3 n + A (E + 1)] = q * q_scale, weight * k, decay (n = A * D columns each), per head v and a one.
+// out [T][2 n + A (E + 1)] = q * q_scale, weight * k (n = A * D columns each), per head v and a one.
 // gates as written by memory_gates; STEP: one row per sequence, the gates are formed here from gmax
 template <typename T, bool STEP>
 __global__ void __launch_bounds__(1024) memory_prep_kernel(float* __restrict__ out, float* __restrict__ gates,
@@ -586,7 +586,7 @@ __global__ void __launch_bounds__(1024) memory_prep_kernel(float* __restrict__ o
                                                            float* __restrict__ gmax, const int* __restrict__ start_pos,
                                                            const int* __restrict__ slots, float q_scale, int Tn, int A, int D,
                                                            int E) {
-  extern __shared__ float lds[];      // [2][A]: decay, weight
+  extern __shared__ float lds[];      // [A]: weights
   const int t = blockIdx.x;
   const T* pr = proj + (size_t)t * stride;
   const size_t plane = (size_t)Tn * A;
@@ -600,25 +600,23 @@ __global__ void __launch_bounds__(1024) memory_prep_kernel(float* __restrict__ o
       memory_gate(pr, i_off, f_off, a, ib, fb, cap, gi, gf);
       const float mt = fmaxf(gf + m, gi);
       *mp = mt;
-      lds[a] = expf(gf + m - mt);
-      lds[A + a] = expf(gi - mt);
+      lds[a] = expf(gi - mt);
+      g[0] = expf(gf + m - mt);
       g[2 * plane] = expf(-mt);
     } else {
-      lds[a] = g[0];
-      lds[A + a] = g[plane];
+      lds[a] = g[plane];
     }
   }
   __syncthreads();
-  float* o = out + (size_t)t * (3 * (size_t)n + (size_t)A * (E + 1));
+  float* o = out + (size_t)t * (2 * (size_t)n + (size_t)A * (E + 1));
   for (int c = threadIdx.x; c < n; c += blockDim.x) {
     const int a = c / D;
     o[c] = DT<T>::load(pr + q_off + c) * q_scale;
-    o[n + c] = DT<T>::load(pr + k_off + c) * lds[A + a];
-    o[2 * (size_t)n + c] = lds[a];
+    o[n + c] = DT<T>::load(pr + k_off + c) * lds[a];
   }
   for (int c = threadIdx.x; c < A * (E + 1); c += blockDim.x) {
     const int a = c / (E + 1), e = c - a * (E + 1);
-    o[3 * (size_t)n + c] = e < E ? DT<T>::load(pr + v_off + a * E + e) : 1.0f;
+    o[2 * (size_t)n + c] = e < E ? DT<T>::load(pr + v_off + a * E + e) : 1.0f;
   }
 }
 
@@ -842,7 +840,7 @@ int launch_memory_prep(float* out, float* gates, const void* proj, int stride, i
                        const int* start_pos, const int* slots, float q_scale, int S, int T, int A, int D, int E, bool step,
                        bool bf, hipStream_t stream) {
   if (T <= 0 || S <= 0) return 0;
-  const size_t shm = sizeof(float) * 2 * (size_t)A;
+  const size_t shm = sizeof(float) * (size_t)A;
   if (shm > 48 * 1024) return -1;
   const int m = A * (D > E + 1 ? D : E + 1);
   const int th = m >= 1024 ? 1024 : m <= 64 ? 64 : (m + 63) / 64 * 64;

@@ -539,7 +539,7 @@ def test_unequal_sequences_in_one_scan(run, sizes):
                             chunks=Hy.scan_chunks(cu, dev) if dev.type == "cuda" else None).double().cpu()
         for s in range(5):
             r = slice(int(cu[s]), int(cu[s + 1]))
-            S = (rec0[sl[s]].double().reshape(A, E, D).transpose(1, 2).clone() if starts[s] > 0
+            S = (rec0[int(sl[s])].double().reshape(A, E, D).transpose(1, 2).clone() if starts[s] > 0
                  else torch.zeros(A, D, E, dtype=torch.float64))
             for t in range(r.start, r.stop):
                 wt, qt, kt, bt = (x[t].double().reshape(A, D) for x in (w, q, k, beta))
@@ -550,7 +550,7 @@ def test_unequal_sequences_in_one_scan(run, sizes):
                 S = S + kt[:, :, None] * u[:, None, :]
                 want = torch.einsum("ai,aij->aj", qt, S)
                 assert float((got[t].reshape(A, E) - want).abs().max()) < 1e-3 * max(1.0, float(want.abs().max())), (ab, s, t)
-            assert float((rec[sl[s]].double().cpu().reshape(A, E, D).transpose(1, 2) - S).abs().max()) < 2e-3
+            assert float((rec[int(sl[s])].double().cpu().reshape(A, E, D).transpose(1, 2) - S).abs().max()) < 2e-3
 
 
 @pytest.mark.parametrize("run", RUNS32)

@@ -179,7 +179,7 @@ class LizesunModel(GoganexModel):
         return Hy.head_norm_gate(o, lw["mix.right.norm"], r.vdim, proj, off["right.g"], "sigmoid", self.cfg.norm_eps,
                                  m.right_scale, cat, nl, floors=floors)
 
-    def _delta(self, proj, m: DeltaSpec, lw, l, positions, kv, b, decode, skinny):
+    def _delta(self, proj, m: DeltaSpec, lw, l, positions, kv, meta, b, decode, skinny):
         off = lw["off"]
         four, v = Hy.channel_delta_prep(proj, m, off["q"], off["b"], off["a1"], lw["a2_t"], lw["conv_w"], kv.sconv[l],
                                         lw["neg_rate"], lw["mix.dt_bias"], b.row_seq, positions, b.start_pos, b.slots,
@@ -187,7 +187,7 @@ class LizesunModel(GoganexModel):
         if not decode:
             Hy.conv_state_update(proj, off["q"], m.conv_channels, kv.sconv[l], 0, b.cu_q, b.start_pos, b.slots)
         o = Hy.state_scan(four[0], four[1], v, four[2], four[1], four[3], None, kv.rec[l], b.cu_q, b.start_pos, b.slots,
-                          m.heads, m.dim, m.vdim)
+                          m.heads, m.dim, m.vdim, chunks=self._scan_chunks(meta, b) if proj.is_cuda and not decode else None)
         low = proj[:, off["g1"]:off["g1"] + lw["gate_rank"]]
         gate = self._linear(low.contiguous() if skinny else low, l, "mix.g2", skinny)
         out = torch.empty(proj.shape[0], m.heads * m.vdim, dtype=self.dtype, device=proj.device)
@@ -212,7 +212,7 @@ class LizesunModel(GoganexModel):
             h = Hy.add_tanh_norm(x, pend, lw["norm1.alpha"], lw["norm1"], lw["norm1.b"], adt)
             proj = self._linear(h, l, "w_in", skinny)
             if isinstance(m, DeltaSpec):
-                o = self._delta(proj, m, lw, l, positions, kv, b, decode, skinny)
+                o = self._delta(proj, m, lw, l, positions, kv, meta, b, decode, skinny)
             elif isinstance(m, ParallelSpec):
                 o = self._parallel(proj, m, lw, l, positions, kv, meta, b, decode)
             else:

@@ -568,7 +568,7 @@ def ref_qk_prep(proj, spec, q_off, k_off, v_off, inv_freq, eps, positions, k_cac
         q = q + q_bias.reshape(H, Dk)
     if k_bias is not None:
         k = k + k_bias.reshape(G, Dk)
-    if inv_freq is not None and spec.rot.halves:
+    if inv_freq is not None and spec.rot is not None and spec.rot.halves:
         q, k = _rotate_halves(q, positions, inv_freq, 1.0), _rotate_halves(k, positions, inv_freq, 1.0)
     elif inv_freq is not None:
         q, k = _rotate_pairs(q, positions, inv_freq), _rotate_pairs(k, positions, inv_freq)
@@ -896,17 +896,17 @@ def memory_prep(proj, spec, q_off: int, k_off: int, v_off: int, i_off: int, f_of
     head, biases fp32 [heads]). With i = cap tanh((p_i + i_bias) / cap), f = logsigmoid(cap tanh((p_f +
     f_bias) / cap)) and the running maximum m_t = max(f_t + m_(t-1), i_t) from ``gmax[slot]`` [heads] (0 at
     position 0; every span's last m is left there) returns fp32 rows (q dim^(-1/2), exp(i_t - m_t) k,
-    exp(f_t + m_(t-1) - m_t) repeated over dim, per head v and a column of ones, exp(-m_t) [T, heads]):
+    exp(f_t + m_(t-1) - m_t) [T, heads], per head v and a column of ones, exp(-m_t) [T, heads]):
     the (q, k, w, v) of :func:`state_scan` with vdim + 1 columns, whose last one is n . q, and the
     ``floors`` of :func:`head_norm_gate`. ``step``: one row per sequence, a single launch."""
     A, D, E = spec.heads, spec.dim, spec.vdim
     T, n, nv = proj.shape[0], A * D, A * (E + 1)
     if _gpu(proj):
-        out = torch.empty(T, 3 * n + nv, dtype=torch.float32, device=proj.device)
+        out = torch.empty(T, 2 * n + nv, dtype=torch.float32, device=proj.device)
         gates = torch.empty(3, T, A, dtype=torch.float32, device=proj.device)
         native().memory_prep(out, gates, proj, int(q_off), int(k_off), int(v_off), int(i_off), int(f_off), i_bias, f_bias,
                              float(spec.gate_cap), gmax, cu_q, start_pos, slots, D ** -0.5, A, D, E, bool(step))
-        return out[:, :n], out[:, n:2 * n], out[:, 2 * n:3 * n], out[:, 3 * n:], gates[2]
+        return out[:, :n], out[:, n:2 * n], gates[0], out[:, 2 * n:], gates[2]
     cap = spec.gate_cap
     gi = cap * torch.tanh((proj[:, i_off:i_off + A].float() + i_bias) / cap)
     gf = torch.nn.functional.logsigmoid(cap * torch.tanh((proj[:, f_off:f_off + A].float() + f_bias) / cap))
@@ -923,7 +923,7 @@ def memory_prep(proj, spec, q_off: int, k_off: int, v_off: int, i_off: int, f_of
         gmax[sl[s]] = m
     k = (proj[:, k_off:k_off + n].float().reshape(T, A, D) * write[:, :, None]).reshape(T, n)
     v = torch.cat([proj[:, v_off:v_off + A * E].float().reshape(T, A, E), torch.ones(T, A, 1)], -1).reshape(T, nv)
-    return proj[:, q_off:q_off + n].float() * D ** -0.5, k, keep[:, :, None].expand(T, A, D).reshape(T, n), v, floor
+    return proj[:, q_off:q_off + n].float() * D ** -0.5, k, keep, v, floor
 
 
 def gla_prep(proj, spec, q_off: int, k_off: int, v_off: int, a_off: int, a2, a_bias) -> Tuple[torch.Tensor, ...]:
@@ -952,16 +952,16 @@ def state_scan(q, k, v, w, a, b, decay, state, cu_q, start_pos, slots, heads: in
     from ``state[slot]`` (zeros at position 0), for every token in order:
         s = b_t^T S;   S <- diag(w_t) S - a_t s^T + k_t v_t^T;   o_t = S^T q_t
     ``q, k, w, a, b`` [T, heads * dim] and ``v`` [T, heads * vdim] are fp32 rows (any row stride).
-    ``w`` None: every head decays by its constant ``decay[head]``; ``a`` / ``b`` None: nothing is
-    removed. Returns o [T, heads * vdim] fp32 and leaves every span's last S in ``state``
-    (``[n_slots, heads * vdim * dim]``, each head stored column by column). ``chunks`` (GPU, without
-    a / b): :func:`scan_chunks` of this batch — spans are then scanned in chunks of ``SCAN_CHUNK``
-    rows in parallel (chunk end states and decay products, a carry pass, the outputs from each
-    chunk's true start state); the results differ from the one-launch scan by rounding only."""
+    ``w`` may be [T, heads]: one decay per head and token. ``w`` None: every head decays by its constant
+    ``decay[head]``; ``a`` / ``b`` None: nothing is removed (``a`` may be ``k`` itself). Returns o [T, heads * vdim] fp32 and leaves every span's last S in ``state``
+    (``[n_slots, heads * vdim * dim]``, each head stored column by column). ``chunks`` (GPU):
+    :func:`scan_chunks` of this batch — spans are then scanned in chunks of ``SCAN_CHUNK`` rows in
+    parallel (chunk end states and what a chunk does to a state: decay products, or with a / b a
+    dim x dim matrix per head; a carry pass; the outputs from each chunk's true start state); the results differ from the one-launch scan by rounding only."""
     if _gpu(q):
         out = torch.empty(q.shape[0], heads * vdim, dtype=torch.float32, device=q.device)
         if chunks is not None:
-            ws = torch.empty(chunks[0].shape[0] * heads * dim * (vdim + 1), dtype=torch.float32, device=q.device)
+            ws = torch.empty(chunks[0].shape[0] * heads * dim * (vdim + (dim if a is not None else 1)), dtype=torch.float32, device=q.device)
             native().state_scan(out, q, k, v, w, a, b, decay, state, cu_q, start_pos, slots, int(heads), int(dim), int(vdim),
                                 chunks[0], chunks[1], ws, SCAN_CHUNK)
             return out
@@ -1141,7 +1141,7 @@ def ref_state_scan(q, k, v, w, a, b, decay, state, cu_q, start_pos, slots, heads
     T = q.shape[0]
     A, D, E = heads, dim, vdim
     q, k, v = q.float().reshape(T, A, D), k.float().reshape(T, A, D), v.float().reshape(T, A, E)
-    w = w.float().reshape(T, A, D) if w is not None else None
+    w = w.float().reshape(T, A, -1).expand(T, A, D) if w is not None else None
     a = a.float().reshape(T, A, D) if a is not None else None
     b = b.float().reshape(T, A, D) if b is not None else None
     out = torch.empty(T, A, E, dtype=torch.float32, device=q.device)
