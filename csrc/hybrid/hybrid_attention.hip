@@ -195,7 +195,7 @@ __global__ void __launch_bounds__(256) gqa_attention_kernel(
   }
 }
 
-// one wave per (row, head): merge the S partials, add the sink once
+// one wave per (row, head): merge the S <= 64 partials (lane = split), add the sinks once
 template <typename T>
 __global__ void __launch_bounds__(64) gqa_combine_kernel(T* __restrict__ out, const float* __restrict__ part_o,
                                                          const float* __restrict__ part_ml, int S, int Dv, float sink,
@@ -204,16 +204,24 @@ __global__ void __launch_bounds__(64) gqa_combine_kernel(T* __restrict__ out, co
                                                          float out_scale, int out_stride, int out_off) {
   const size_t rh = blockIdx.x;
   const int lane = threadIdx.x;
-  float M = sinks ? sinks[rh % H] : kNeg;
-  for (int s = 0; s < S; ++s) M = fmaxf(M, part_ml[(rh * S + s) * 2]);
-  float den = (sink > 0.f ? sink * __expf(-M) : 0.f) + (sinks ? __expf(sinks[rh % H] - M) : 0.f);
-  for (int s = 0; s < S; ++s) den += part_ml[(rh * S + s) * 2 + 1] * __expf(part_ml[(rh * S + s) * 2] - M);
-  float inv = den > 0.f ? 1.0f / den : 0.f;
+  const float hs = sinks ? sinks[rh % H] : kNeg;
+  float ml = kNeg, ll = 0.f;
+  if (lane < S) {
+    ml = part_ml[(rh * S + lane) * 2];
+    ll = part_ml[(rh * S + lane) * 2 + 1];
+  }
+  const float M = fmaxf(hs, rt::wave_max(ml));
+  const float wt = lane < S ? __expf(ml - M) : 0.f;
+  const float den = (sink > 0.f ? sink * __expf(-M) : 0.f) + (sinks ? __expf(hs - M) : 0.f) + rt::wave_sum(ll * wt);
+  float inv = (den > 0.f ? 1.0f / den : 0.f) * out_scale;
   if (gate && gate_heads) inv *= 1.0f / (1.0f + __expf(-DT<T>::load(gate + (rh / H) * gate_stride + rh % H)));
-  for (int col = lane; col < Dv; col += 64) {
+  for (int col = lane; col - lane < Dv; col += 64) {
     float acc = 0.f;
-    for (int s = 0; s < S; ++s) acc += part_o[(rh * S + s) * Dv + col] * __expf(part_ml[(rh * S + s) * 2] - M);
-    float v = acc * inv * out_scale;
+    const float* po = part_o + rh * S * Dv + min(col, Dv - 1);
+#pragma unroll 8
+    for (int s = 0; s < S; ++s) acc += po[(size_t)s * Dv] * __shfl(wt, s, 64);
+    if (col >= Dv) continue;
+    float v = acc * inv;
     if (gate && !gate_heads) v *= 1.0f / (1.0f + __expf(-DT<T>::load(gate + (rh / H) * gate_stride + (rh % H) * Dv + col)));
     DT<T>::store(out + (rh / H) * out_stride + out_off + (rh % H) * Dv + col, v);
   }
@@ -224,6 +232,19 @@ size_t lds_bytes(int Dk, int Dv, int KT, int pairs = kPairs) {
 }
 
 }  // namespace
+
+void launch_gqa_combine(void* out, const float* part_o, const float* part_ml, int num_splits, int T, int H, int Dv, float sink,
+                        const AttnMask& mask, const void* gate, int gate_stride, bool gate_heads, float out_scale,
+                        int out_stride, int out_off, bool bf, hipStream_t stream) {
+  if (bf)
+    gqa_combine_kernel<uint16_t><<<T * H, 64, 0, stream>>>((uint16_t*)out, part_o, part_ml, num_splits, Dv, sink, H,
+                                                           (const uint16_t*)gate, gate_stride, gate_heads ? 1 : 0, mask.sinks,
+                                                           out_scale, out_stride, out_off);
+  else
+    gqa_combine_kernel<float><<<T * H, 64, 0, stream>>>((float*)out, part_o, part_ml, num_splits, Dv, sink, H,
+                                                        (const float*)gate, gate_stride, gate_heads ? 1 : 0, mask.sinks,
+                                                        out_scale, out_stride, out_off);
+}
 
 // keys per staged tile: the largest of 64 / 32 / 16 / 8 whose LDS fits; 0 if none does
 int gqa_key_tile(int Dk, int Dv) {
@@ -271,13 +292,8 @@ int launch_gqa_attention(void* out, const void* q, const void* kc, const void* v
   }
 #undef RT_GQA
 #undef RT_GQA2
-  if (num_splits > 1) {
-    if (bf) gqa_combine_kernel<uint16_t><<<T * H, 64, 0, stream>>>((uint16_t*)out, part_o, part_ml, num_splits, Dv, sink, H,
-                                                                   (const uint16_t*)gate, gate_stride, gate_heads ? 1 : 0,
-                                                                   mask.sinks, out_scale, out_stride, out_off);
-    else gqa_combine_kernel<float><<<T * H, 64, 0, stream>>>((float*)out, part_o, part_ml, num_splits, Dv, sink, H,
-                                                             (const float*)gate, gate_stride, gate_heads ? 1 : 0,
-                                                             mask.sinks, out_scale, out_stride, out_off);
-  }
+  if (num_splits > 1)
+    launch_gqa_combine(out, part_o, part_ml, num_splits, T, H, Dv, sink, mask, gate, gate_stride, gate_heads, out_scale,
+                       out_stride, out_off, bf, stream);
   return 0;
 }

@@ -53,6 +53,13 @@ void launch_moe_combine(void* out, const void* y, const float* wt, const int* pl
                         bool y_bf, hipStream_t stream);
 void launch_limited_glu(void* out, const void* gu, int64_t rows, int F, float limit, bool bf, hipStream_t stream);
 int gqa_key_tile(int Dk, int Dv);
+int flash_key_tile();
+bool flash_fits(int Dk, int Dv, int BS);
+int launch_flash_attention(void* out, const void* q, const void* kc, const void* vc, const int* block_tables, const int* cu_q,
+                           const int* start_pos, const int* tiles, int n_tiles, float* part_o, float* part_ml, int T, int H,
+                           int G, int Dk, int Dv, int BS, int max_blocks, int rows, int waves, int num_splits, float scale,
+                           const AttnMask& mask, const void* gate, int gate_stride, float softcap, float out_scale,
+                           int out_stride, int out_off, hipStream_t stream);
 int launch_gqa_attention(void* out, const void* q, const void* kc, const void* vc, const int* block_tables,
                          const int* cu_q, const int* start_pos, const int* tiles, int n_tiles, const float* temp,
                          float* part_o, float* part_ml, int T, int H, int G, int Dk, int Dv, int BS, int max_blocks,
@@ -238,6 +245,20 @@ void qk_prep(torch::Tensor q, torch::Tensor proj, int64_t q_off, int64_t k_off, 
                  Dk, Dv, BS, is_bf(q), (int)layout, qs, qw, kw, v_norm, (float)qt_coef, (int)qt_every, ex, cur());
 }
 
+// scratch of a split launch over the keys, [T * H * num_splits (, Dv | 2)]
+void split_buffers(int64_t num_splits, int64_t rows, const c10::optional<torch::Tensor>& part_o,
+                   const c10::optional<torch::Tensor>& part_ml, int64_t TH, int64_t Dv, float*& po, float*& pml) {
+  TORCH_CHECK(num_splits >= 1 && num_splits <= 64, "attention: num_splits must be 1..64");
+  if (num_splits == 1) return;
+  TORCH_CHECK(rows == 1, "attention: split keys need one row per tile");
+  TORCH_CHECK(part_o.has_value() && part_ml.has_value(), "attention: split keys need the partial buffers");
+  chk_f32(*part_o, "part_o"); chk_f32(*part_ml, "part_ml");
+  TORCH_CHECK(part_o->numel() >= TH * num_splits * Dv && part_ml->numel() >= TH * num_splits * 2,
+              "attention: partial buffers too small");
+  po = part_o->data_ptr<float>();
+  pml = part_ml->data_ptr<float>();
+}
+
 AttnMask mask_of(int64_t window, int64_t keep, int64_t chunk, const c10::optional<torch::Tensor>& sinks, int64_t H) {
   const int64_t top = int64_t(1) << 30;
   TORCH_CHECK(window >= 0 && window < top && keep >= 0 && keep < top && chunk >= 0 && chunk < top,
@@ -273,7 +294,6 @@ void gqa_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch::
   chk_i32(tiles, "tiles");
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(0) == start_pos.numel(), "gqa_attention: block_tables [S, n]");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2, "gqa_attention: tiles [n, 2]");
-  TORCH_CHECK(num_splits >= 1 && num_splits <= 64, "gqa_attention: num_splits must be 1..64");
   TORCH_CHECK(rows >= 1, "gqa_attention: rows per tile");
   const float* tp = nullptr;
   if (temp.has_value()) {
@@ -281,15 +301,7 @@ void gqa_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch::
     tp = temp->data_ptr<float>();
   }
   float *po = nullptr, *pml = nullptr;
-  if (num_splits > 1) {
-    TORCH_CHECK(rows == 1, "gqa_attention: split keys need one row per tile");
-    TORCH_CHECK(part_o.has_value() && part_ml.has_value(), "gqa_attention: split keys need the partial buffers");
-    chk_f32(*part_o, "part_o"); chk_f32(*part_ml, "part_ml");
-    TORCH_CHECK(part_o->numel() >= T * H * num_splits * Dv && part_ml->numel() >= T * H * num_splits * 2,
-                "gqa_attention: partial buffers too small");
-    po = part_o->data_ptr<float>();
-    pml = part_ml->data_ptr<float>();
-  }
+  split_buffers(num_splits, rows, part_o, part_ml, T * H, Dv, po, pml);
   const float* sl = nullptr;
   if (slopes.has_value()) { chk_f32(*slopes, "slopes", H); sl = slopes->data_ptr<float>(); }
   const AttnMask mask = mask_of(window, keep, chunk, sinks, H);
@@ -309,6 +321,48 @@ void gqa_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch::
                                 (float)out_scale, (int)out.size(1), (int)out_off, is_bf(q), cur());
   TORCH_CHECK(rc == 0, "gqa_attention: unsupported shape (code ", rc, ": -1 head sizes beyond 256 or the LDS tile, "
               "-2 rows per tile, -3 LDS size refused)");
+}
+
+// gqa_attention's bf16 form on the matrix cores: rows layout, a gate per head or none
+void flash_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch::Tensor vc, torch::Tensor block_tables,
+                     torch::Tensor cu_q, torch::Tensor start_pos, torch::Tensor tiles, double scale, int64_t rows,
+                     int64_t waves, int64_t num_splits, c10::optional<torch::Tensor> part_o,
+                     c10::optional<torch::Tensor> part_ml, int64_t window, int64_t keep, int64_t chunk,
+                     c10::optional<torch::Tensor> sinks, c10::optional<torch::Tensor> gate, int64_t gate_off, double softcap,
+                     double out_scale, int64_t out_off) {
+  chk(out, "out"); chk(q, "q"); chk(kc, "k_cache"); chk(vc, "v_cache");
+  TORCH_CHECK(is_bf(out) && is_bf(q) && is_bf(kc) && is_bf(vc), "flash_attention: bf16");
+  TORCH_CHECK(q.dim() == 3 && kc.dim() == 4 && vc.dim() == 4 && out.dim() == 2, "flash_attention: ranks");
+  const int64_t T = q.size(0), H = q.size(1), Dk = q.size(2), G = kc.size(1), BS = kc.size(2), Dv = vc.size(3);
+  TORCH_CHECK(kc.size(3) == Dk && vc.size(0) == kc.size(0) && vc.size(1) == G && vc.size(2) == BS && H % G == 0,
+              "flash_attention: cache shapes");
+  auto al = [](const torch::Tensor& t) { return (reinterpret_cast<uintptr_t>(t.data_ptr()) & 15) == 0; };
+  TORCH_CHECK(al(q) && al(kc) && al(vc), "flash_attention: q and the cache must be 16-byte aligned");
+  TORCH_CHECK(out.size(0) == T && out_off >= 0 && out_off + H * Dv <= out.size(1) && softcap >= 0,
+              "flash_attention: out [T, >= out_off + H * Dv]");
+  chk_i32(block_tables, "block_tables"); chk_i32(cu_q, "cu_q"); chk_i32(start_pos, "start_pos", cu_q.numel() - 1);
+  chk_i32(tiles, "tiles");
+  TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(0) == start_pos.numel(), "flash_attention: block_tables [S, n]");
+  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2 && rows >= 1, "flash_attention: tiles [n, 2]");
+  float *po = nullptr, *pml = nullptr;
+  split_buffers(num_splits, rows, part_o, part_ml, T * H, Dv, po, pml);
+  const AttnMask mask = mask_of(window, keep, chunk, sinks, H);
+  const char* gp = nullptr;
+  int64_t gstride = 0;
+  if (gate.has_value()) {
+    chk(*gate, "gate");
+    TORCH_CHECK(is_bf(*gate) && gate->dim() == 2 && gate->size(0) == T && gate_off >= 0 && gate_off + H <= gate->size(1),
+                "flash_attention: gate columns");
+    gstride = gate->size(1);
+    gp = static_cast<const char*>(gate->data_ptr()) + gate_off * gate->element_size();
+  }
+  int rc = launch_flash_attention(out.data_ptr(), q.data_ptr(), kc.data_ptr(), vc.data_ptr(), block_tables.data_ptr<int>(),
+                                  cu_q.data_ptr<int>(), start_pos.data_ptr<int>(), tiles.data_ptr<int>(), (int)tiles.size(0),
+                                  po, pml, (int)T, (int)H, (int)G, (int)Dk, (int)Dv, (int)BS, (int)block_tables.size(1),
+                                  (int)rows, (int)waves, (int)num_splits, (float)scale, mask, gp, (int)gstride, (float)softcap,
+                                  (float)out_scale, (int)out.size(1), (int)out_off, cur());
+  TORCH_CHECK(rc == 0, "flash_attention: unsupported shape (code ", rc, ": -1 head or page sizes, -2 rows per tile, -3 LDS "
+              "size refused)");
 }
 
 void mingru_scan(torch::Tensor out, torch::Tensor proj, int64_t z_off, int64_t x_off, int64_t g_off, torch::Tensor bz,
@@ -914,6 +968,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("halves") = false, py::arg("q_b") = py::none(), py::arg("k_b") = py::none(), py::arg("v_b") = py::none(),
         py::arg("mix") = py::none(), py::arg("mix_off") = 0, py::arg("mix_b") = py::none(), py::arg("mix_w") = 0.0);
   m.def("gqa_key_tile", [](int64_t Dk, int64_t Dv) { return gqa_key_tile((int)Dk, (int)Dv); });
+  m.def("flash_key_tile", &flash_key_tile);
+  m.def("flash_fits", [](int64_t Dk, int64_t Dv, int64_t BS) { return flash_fits((int)Dk, (int)Dv, (int)BS); });
+  m.def("flash_attention", &flash_attention, py::arg("out"), py::arg("q"), py::arg("kc"), py::arg("vc"),
+        py::arg("block_tables"), py::arg("cu_q"), py::arg("start_pos"), py::arg("tiles"), py::arg("scale"), py::arg("rows"),
+        py::arg("waves"), py::arg("num_splits"), py::arg("part_o"), py::arg("part_ml"), py::arg("window") = 0,
+        py::arg("keep") = 0, py::arg("chunk") = 0, py::arg("sinks") = py::none(), py::arg("gate") = py::none(),
+        py::arg("gate_off") = 0, py::arg("softcap") = 0.0, py::arg("out_scale") = 1.0, py::arg("out_off") = 0);
   m.def("gqa_attention", &gqa_attention, py::arg("out"), py::arg("q"), py::arg("kc"), py::arg("vc"),
         py::arg("block_tables"), py::arg("cu_q"), py::arg("start_pos"), py::arg("tiles"), py::arg("temp"), py::arg("scale"),
         py::arg("sink"), py::arg("rows"), py::arg("num_splits"), py::arg("part_o"), py::arg("part_ml"),

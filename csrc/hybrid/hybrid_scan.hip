@@ -328,7 +328,7 @@ __global__ void __launch_bounds__(256) state_carry_matrix_kernel(float* __restri
                                                                  const int* __restrict__ seq_chunk0,
                                                                  const int* __restrict__ start_pos,
                                                                  const int* __restrict__ slots, int A, int D, int E, int lgDp) {
-  extern __shared__ float4 cols[];      // [2][D][groups]
+  extern __shared__ float4 cols[];      // [2][DM][groups], rows from D on stay zero
   const int s = blockIdx.x, h = blockIdx.y;
   const int k0 = seq_chunk0[s], k1 = seq_chunk0[s + 1];
   if (k1 <= k0) return;
@@ -339,31 +339,35 @@ __global__ void __launch_bounds__(256) state_carry_matrix_kernel(float* __restri
   const bool row = i < D;
   float* st = state + ((size_t)slots[s] * A + h) * E * D;
   const bool cont = start_pos[s] > 0;
+  for (int x = threadIdx.x; x < 2 * DM * groups; x += 256) cols[x] = float4{0.f, 0.f, 0.f, 0.f};
+  __syncthreads();
   float S[4];
 #pragma unroll
   for (int c = 0; c < 4; ++c) S[c] = cont && row && col + c < E ? st[(size_t)(col + c) * D + i] : 0.f;
+  // (no branches, so that all of a chunk's loads leave together: indices past the end repeat the last
+  // entry, whose products are with zero rows or are not kept)
+  const int ic = min(i, D - 1);
   auto load = [&](int k, float (&m)[DM], float (&bb)[4]) {
-    const float* base = ws_e + ((size_t)k * A + h) * EC * D;
+    const float* base = ws_e + ((size_t)k * A + h) * EC * D + ic;
 #pragma unroll
-    for (int c = 0; c < 4; ++c) bb[c] = row && col + c < E ? base[(size_t)(col + c) * D + i] : 0.f;
+    for (int c = 0; c < 4; ++c) bb[c] = base[(size_t)min(col + c, E - 1) * D];
 #pragma unroll
-    for (int j = 0; j < DM; ++j) m[j] = row && j < D ? base[(size_t)(E + j) * D + i] : 0.f;
+    for (int j = 0; j < DM; ++j) m[j] = base[(size_t)(E + min(j, D - 1)) * D];
   };
   float m[DM], b[4];
   load(k0, m, b);
   for (int k = k0; k < k1; ++k) {
-    float4* cur = cols + ((k - k0) & 1) * D * groups;
+    float4* cur = cols + ((k - k0) & 1) * DM * groups;
     if (row) cur[i * groups + g] = float4{S[0], S[1], S[2], S[3]};
     __syncthreads();      // (the other buffer's readers are past the barrier of the step before)
     float mn[DM], bn[4];
     if (k + 1 < k1) load(k + 1, mn, bn);
     float acc[4] = {b[0], b[1], b[2], b[3]};
 #pragma unroll
-    for (int j = 0; j < DM; ++j)
-      if (j < D) {
-        const float4 sj = cur[j * groups + g];
-        acc[0] += m[j] * sj.x; acc[1] += m[j] * sj.y; acc[2] += m[j] * sj.z; acc[3] += m[j] * sj.w;
-      }
+    for (int j = 0; j < DM; ++j) {
+      const float4 sj = cur[j * groups + g];
+      acc[0] += m[j] * sj.x; acc[1] += m[j] * sj.y; acc[2] += m[j] * sj.z; acc[3] += m[j] * sj.w;
+    }
     float* base = ws_e + ((size_t)k * A + h) * EC * D;
 #pragma unroll
     for (int c = 0; c < 4; ++c) {
@@ -499,7 +503,7 @@ int launch_state_scan(float* out, const float* q, const float* k, const float* v
       while ((1 << lgDp) < D) ++lgDp;
       const int groups = 256 >> lgDp;
       const dim3 grid(S, A, (E + 4 * groups - 1) / (4 * groups));
-      const size_t cshm = sizeof(float4) * 2 * (size_t)D * groups;
+      const size_t cshm = sizeof(float4) * 2 * 64 * (size_t)groups;
       if (D <= 64) state_carry_matrix_kernel<64><<<grid, 256, cshm, stream>>>(ws_e, state, seq_chunk0, start_pos, slots, A, D,
                                                                               E, lgDp);
       else state_carry_matrix_any_kernel<<<dim3(S, A, (E + 3) / 4), 256, sizeof(float4) * 2 * (size_t)D, stream>>>(

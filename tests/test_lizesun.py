@@ -196,7 +196,8 @@ def _attend(run, a, proj, off, P, lam, first, cuts, BS, sinks=None, gate=False, 
                        q_weight=on("q.norm"), k_weight=on("k.norm"), q_bias=on("q.b"), k_bias=on("k.b"), v_bias=on("v.b"), mix=mix)
         one = T == 1 and rows.start > 0
         buf = torch.zeros(T, a.heads * a.vdim + 5, dtype=dt, device=dev)
-        Hy.gqa_attention(q, kc, vc, perm[None].to(dev), cu.to(dev), sp.to(dev), a.scale, None, 0.0,
+        plan = Hy.attention_plan(a, T, BS, dt, one) if dev.type == "cuda" else None
+        Hy.gqa_attention(q, kc, vc, perm[None].to(dev), cu.to(dev), sp.to(dev), a.scale, None, 0.0, plan=plan,
                          num_splits=splits if one and dev.type == "cuda" else 1, out_dtype=dt, window=a.window,
                          keep_first=a.keep_first, chunk=a.chunk, softcap=a.softcap, out_scale=0.8, out_buf=buf, out_off=5,
                          sinks=None if sinks is None else sinks.to(dev), gate=p if gate else None,
@@ -906,3 +907,39 @@ def test_trace_runner_replays_steps(tmp_path):
     b = np.fromfile(tmp_path / "o" / "2.f32", dtype="<f4").reshape(2, 50)
     got = torch.tensor(np.concatenate([a, b])).double()
     assert float((got - want[[0, 19, 29, 2]]).abs().max()) < 2e-3
+
+
+@GPU
+@pytest.mark.parametrize("waves", [2, 4])
+@pytest.mark.parametrize("shape", [(8, 2, 64, 64), (7, 1, 40, 48), (6, 2, 96, 80), (4, 4, 128, 128), (3, 1, 256, 72), (2, 2, 72, 256),
+                                   (140, 1, 16, 16)])
+@pytest.mark.parametrize("mask", [dict(window=0), dict(window=100, keep_first=70), dict(window=64, keep_first=3), dict(chunk=100)])
+def test_matrix_core_attention_against_the_any_size_kernel(waves, shape, mask):
+    """The bf16 matrix-core kernel and the fp32-FMA kernel on the same queries and cache: several
+    sequences of unequal length and start on scattered pages of 4 to 64 tokens, prompts and split decode
+    rows, with soft cap, sinks, gates, a scaled result in a column range."""
+    H, G, Dk, Dv = shape
+    dev, dt = torch.device("cuda:0"), torch.bfloat16
+    g = torch.Generator().manual_seed(Dk)
+    for BS, lens, starts in ((64, [130, 1, 77], [0, 300, 95]), (4, [2, 65], [31, 0]), (16, [1, 1, 1], [200, 3, 64])):
+        S, T = len(lens), sum(lens)
+        nb = [(a + b + BS - 1) // BS for a, b in zip(lens, starts)]
+        perm = torch.randperm(sum(nb), generator=g).to(torch.int32)
+        bt = torch.zeros(S, max(nb), dtype=torch.int32)
+        for s in range(S):
+            bt[s, :nb[s]] = perm[sum(nb[:s]):sum(nb[:s + 1])]
+        rnd = lambda *sh: torch.randn(*sh, generator=g).to(dt).to(dev)
+        kc, vc, q, gate = rnd(sum(nb), G, BS, Dk), rnd(sum(nb), G, BS, Dv), rnd(T, H, Dk), rnd(T, H + 3)
+        sinks = torch.randn(H, generator=g).to(dev)
+        cu = torch.tensor([0] + list(torch.tensor(lens).cumsum(0)), dtype=torch.int32)
+        sp = torch.tensor(starts, dtype=torch.int32)
+        decode = max(lens) == 1
+        kw = dict(softcap=3.0, sinks=sinks, gate=gate, gate_off=2, gate_heads=True, out_scale=0.7, out_off=4,
+                  num_splits=3 if decode else 1, **mask)
+        rows = 1 if decode else max(1, waves * 32 // (H // G))
+        outs = []
+        for plan in (None, Hy.AttnPlan(waves, rows, 64)):
+            buf = torch.zeros(T, H * Dv + 8, dtype=dt, device=dev)
+            outs.append(Hy.gqa_attention(q, kc, vc, bt.to(dev), cu.to(dev), sp.to(dev), Dk ** -0.5, plan=plan, out_buf=buf, **kw))
+        assert float(outs[0].float().abs().max()) > 0.1
+        assert float((outs[0].float() - outs[1].float()).abs().max()) < 0.03, (BS, lens)

@@ -16,10 +16,10 @@ one batch; only the attention launch and the scan differ):
     attention:
       q     = qk_prep(proj)                     H2 (HIP): biases, per-head norms with weights, values mixed
                                                 with the first such layer's; keys / values -> paged cache
-      pending = gqa_attention(q) @ Wo^T         H3 (HIP): chunks, soft cap, one gate per head
+      pending = gqa_attention(q) @ Wo^T         H19 / H3 (HIP): chunks, soft cap, one gate per head
     parallel:
       q     = qk_prep(proj)                     H2: rotation in halves, then the norms
-      cat[:, :left] = gqa_attention(q)          H3: window, kept first keys, learned sinks, scaled result
+      cat[:, :left] = gqa_attention(q)          H19 / H3: window, kept first keys, learned sinks, scaled result
       s     = memory_prep(proj)                 C11 (HIP): gates, running maximum, weighted keys
       o     = state_scan(s)                     C5: the state and, as one more column, its normaliser
       cat[:, left:] = head_norm_gate(o)         C6: read-out divided, per-head norm, weight, gate, scale
@@ -134,21 +134,21 @@ class LizesunModel(GoganexModel):
         return max(1, sum(sh[0] * (sh[1] + sh[2]) for sh in self.cache_shapes() if sh is not None)) * block_size * dtype_bytes
 
     # ---- forward ----------------------------------------------------------------------------------
-    def _mask_splits(self, a: GroupedAttentionSpec, rows: int) -> int:
+    def _mask_splits(self, a: GroupedAttentionSpec, rows: int, kt: int) -> int:
         """Key ranges per decoded row: as many as fill the chip, but no more than the key tiles a row's
         window (with its kept first keys) or chunk can touch."""
         splits = self.decode_splits(rows, a.kv_heads)
         span = a.window or a.chunk
         if splits > 1 and span > 0:
-            kt = max(1, Hy.native().gqa_key_tile(a.dim, a.vdim))
             splits = max(1, min(splits, (span + kt - 1) // kt + 1 + (a.keep_first + kt - 1) // kt))
         return splits
 
     def _attend(self, q, a: GroupedAttentionSpec, l, kv, meta, b, decode, **kw):
         T = q.shape[0]
-        splits = self._mask_splits(a, T) if decode else 1
+        plan = Hy.attention_plan(a, T, kv.block_size, self.dtype, decode) if q.is_cuda else None
+        splits = self._mask_splits(a, T, plan.key_tile) if decode and plan is not None else 1
         return Hy.gqa_attention(q, kv.k_layer(l), kv.v_layer(l), meta.block_tables, b.cu_q, b.start_pos, a.scale, None, 0.0,
-                                tiles=self._tiles(meta, Hy.rows_per_tile(a.group), b) if q.is_cuda else None,
+                                tiles=self._tiles(meta, plan.rows, b) if plan is not None else None, plan=plan,
                                 num_splits=splits, workspace=self._workspace(T, a, splits), out_dtype=self.dtype,
                                 window=a.window, keep_first=a.keep_first, chunk=a.chunk, softcap=a.softcap, **kw)
 

@@ -147,6 +147,25 @@ def rows_per_tile(group: int) -> int:
     return max(1, PAIRS_PER_TILE // max(1, group))
 
 
+class AttnPlan(NamedTuple):
+    """How :func:`gqa_attention` runs a layer's rows on the GPU: ``waves`` 0 the any-size kernel, else the
+    matrix-core kernel with that many waves per workgroup; query rows per work item; keys per tile."""
+    waves: int
+    rows: int
+    key_tile: int
+
+
+def attention_plan(spec, n_rows: int, block_size: int, dtype, decode: bool = False) -> AttnPlan:
+    """The matrix-core kernel takes bf16 heads of a multiple of 8 entries up to 256 on pages of a power
+    of two; a launch of few rows gets smaller workgroups, so that more of them fill the chip."""
+    if dtype != torch.bfloat16 or not native().flash_fits(spec.dim, spec.vdim, block_size):
+        return AttnPlan(0, 1 if decode else rows_per_tile(spec.group), native().gqa_key_tile(spec.dim, spec.vdim))
+    waves = 4
+    if not decode and n_rows * spec.heads <= 512 * 128 and spec.group <= 64:
+        waves = 2
+    return AttnPlan(waves, 1 if decode else max(1, waves * 32 // spec.group), native().flash_key_tile())
+
+
 def tile_map(cu_q: torch.Tensor, start_pos: torch.Tensor, rows: int) -> torch.Tensor:
     """[n_tiles, 2] int32 (sequence, first row) of the varlen attention launch, heaviest first."""
     items = []
@@ -173,7 +192,7 @@ def gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale: flo
                   out_dtype=None, window: int = 0, slopes=None, gate=None, gate_off: int = 0,
                   matrix_layout: bool = False, softcap: float = 0.0, out_scale: float = 1.0, out_buf=None,
                   out_off: int = 0, keep_first: int = 0, chunk: int = 0, sinks=None,
-                  gate_heads: bool = False) -> torch.Tensor:
+                  gate_heads: bool = False, plan: Optional[AttnPlan] = None) -> torch.Tensor:
     """Causal attention of the rows ``q`` [T, H, Dk] (span s = rows ``cu_q[s] .. cu_q[s + 1]`` at
     positions ``start_pos[s] ..`` of sequence s) over the paged keys ``k_cache`` [nb, G, BS, Dk]
     and values ``v_cache`` [nb, G, BS, Dv]: score = q . k * scale (* ``temp[h]``), weights
@@ -189,17 +208,27 @@ def gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale: flo
     activation buffer that another branch fills beside it) and ``out_buf`` is returned. ``keep_first``:
     with a window, keys j < keep_first stay visible. ``chunk`` > 0 (no window): row i sees only keys j
     with j // chunk == i // chunk. ``sinks`` [H] fp32: exp(sinks[h]) joins the denominator.
-    ``gate_heads``: the gate is one column per head, ``gate_off .. gate_off + H``."""
+    ``gate_heads``: the gate is one column per head, ``gate_off .. gate_off + H``. ``plan`` (GPU):
+    :func:`attention_plan` of these rows (``tiles`` are then its tiles); the matrix-core kernel knows no
+    temperature, constant sink, distance penalty or gate per column."""
     out_dtype = out_dtype or q.dtype
     if _gpu(q):
         T, H, _ = q.shape
         G, Dv = k_cache.shape[1], v_cache.shape[2 if matrix_layout else 3]
         out = out_buf if out_buf is not None else torch.empty(T, H * Dv, dtype=out_dtype, device=q.device)
-        rows = 1 if num_splits > 1 else rows_per_tile(H // G)
+        rows = plan.rows if plan is not None else 1 if num_splits > 1 else rows_per_tile(H // G)
         if tiles is None:
             tiles = tile_map(cu_q.cpu(), start_pos.cpu(), rows).to(q.device)
         if num_splits > 1 and workspace is None:
             workspace = SplitWorkspace(T, H, Dv, num_splits, q.device)
+        if plan is not None and plan.waves:
+            if temp is not None or sink or slopes is not None or matrix_layout or (gate is not None and not gate_heads):
+                raise ValueError("gqa_attention: not an attention of the matrix-core kernel")
+            native().flash_attention(out, q, k_cache, v_cache, block_tables, cu_q, start_pos, tiles, float(scale), rows,
+                                     plan.waves, int(num_splits), workspace.part_o if num_splits > 1 else None,
+                                     workspace.part_ml if num_splits > 1 else None, int(window), int(keep_first), int(chunk),
+                                     sinks, gate, int(gate_off), float(softcap), float(out_scale), int(out_off))
+            return out
         native().gqa_attention(out, q, k_cache, v_cache, block_tables, cu_q, start_pos, tiles, temp, float(scale),
                                float(sink), rows, int(num_splits),
                                workspace.part_o if num_splits > 1 else None,
