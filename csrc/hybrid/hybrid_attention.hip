@@ -205,6 +205,12 @@ __global__ void __launch_bounds__(64) gqa_combine_kernel(T* __restrict__ out, co
   const size_t rh = blockIdx.x;
   const int lane = threadIdx.x;
   const float hs = sinks ? sinks[rh % H] : kNeg;
+  // the first columns' partials leave together with the maxima and sums
+  constexpr int kAhead = 16;
+  const float* p0 = part_o + rh * S * Dv + min(lane, Dv - 1);
+  float pre[kAhead];
+#pragma unroll
+  for (int s = 0; s < kAhead; ++s) pre[s] = p0[(size_t)min(s, S - 1) * Dv];
   float ml = kNeg, ll = 0.f;
   if (lane < S) {
     ml = part_ml[(rh * S + lane) * 2];
@@ -218,8 +224,14 @@ __global__ void __launch_bounds__(64) gqa_combine_kernel(T* __restrict__ out, co
   for (int col = lane; col - lane < Dv; col += 64) {
     float acc = 0.f;
     const float* po = part_o + rh * S * Dv + min(col, Dv - 1);
+    int s = 0;
+    if (col == lane) {
+#pragma unroll
+      for (int j = 0; j < kAhead; ++j) acc += j < S ? pre[j] * __shfl(wt, j, 64) : 0.f;
+      s = kAhead;
+    }
 #pragma unroll 8
-    for (int s = 0; s < S; ++s) acc += po[(size_t)s * Dv] * __shfl(wt, s, 64);
+    for (; s < S; ++s) acc += po[(size_t)s * Dv] * __shfl(wt, s, 64);
     if (col >= Dv) continue;
     float v = acc * inv;
     if (gate && !gate_heads) v *= 1.0f / (1.0f + __expf(-DT<T>::load(gate + (rh / H) * gate_stride + (rh % H) * Dv + col)));

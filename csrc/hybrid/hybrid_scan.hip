@@ -319,74 +319,71 @@ __global__ void __launch_bounds__(256) state_carry_kernel(float* __restrict__ ws
   *st = S;
 }
 
-// launch (2) with removal: per (sequence, head, 4 * 256 / Dp columns) the chain S <- M_c S + B_c over the
+// launch (2) with removal: per (sequence, head, 4 * 256 / D columns) the chain S <- M_c S + B_c over the
 // chunks, ws_e[chunk][head][E columns of B, then D columns of M][D]; the state a chunk starts from is
 // written over its B. Lane = (row i, a group of 4 columns): it reads row i of M (coalesced over i), the
-// columns of S sit in LDS. DM >= D: the next chunk's row of M is loaded while this one is used.
-template <int DM>
-__global__ void __launch_bounds__(256) state_carry_matrix_kernel(float* __restrict__ ws_e, float* __restrict__ state,
-                                                                 const int* __restrict__ seq_chunk0,
-                                                                 const int* __restrict__ start_pos,
-                                                                 const int* __restrict__ slots, int A, int D, int E, int lgDp) {
-  extern __shared__ float4 cols[];      // [2][DM][groups], rows from D on stay zero
+// columns of S sit in LDS. The next chunk's row of M is loaded into registers while this one is used.
+template <int D>
+__global__ void __launch_bounds__(256, 1) state_carry_matrix_kernel(float* __restrict__ ws_e, float* __restrict__ state,
+                                                                    const int* __restrict__ seq_chunk0,
+                                                                    const int* __restrict__ start_pos,
+                                                                    const int* __restrict__ slots, int A, int E) {
+  constexpr int groups = 256 / D;
+  __shared__ float4 cols[2][D][groups];
   const int s = blockIdx.x, h = blockIdx.y;
   const int k0 = seq_chunk0[s], k1 = seq_chunk0[s + 1];
   if (k1 <= k0) return;
-  const int Dp = 1 << lgDp, groups = 256 >> lgDp;
-  const int i = threadIdx.x & (Dp - 1), g = threadIdx.x >> lgDp;
+  const int i = threadIdx.x % D, g = threadIdx.x / D;
   const int col = (blockIdx.z * groups + g) * 4;
-  const int EC = E + D;
-  const bool row = i < D;
+  const size_t step = (size_t)A * (E + D) * D;      // floats from a chunk to the next
+  float* base = ws_e + (size_t)k0 * step + (size_t)h * (E + D) * D;
   float* st = state + ((size_t)slots[s] * A + h) * E * D;
   const bool cont = start_pos[s] > 0;
-  for (int x = threadIdx.x; x < 2 * DM * groups; x += 256) cols[x] = float4{0.f, 0.f, 0.f, 0.f};
-  __syncthreads();
+  int off[4];                                       // this lane's entries of B and of the state
+  bool live[4];
   float S[4];
 #pragma unroll
-  for (int c = 0; c < 4; ++c) S[c] = cont && row && col + c < E ? st[(size_t)(col + c) * D + i] : 0.f;
-  // (no branches, so that all of a chunk's loads leave together: indices past the end repeat the last
-  // entry, whose products are with zero rows or are not kept)
-  const int ic = min(i, D - 1);
-  auto load = [&](int k, float (&m)[DM], float (&bb)[4]) {
-    const float* base = ws_e + ((size_t)k * A + h) * EC * D + ic;
+  for (int c = 0; c < 4; ++c) {
+    live[c] = col + c < E;
+    off[c] = (live[c] ? col + c : E - 1) * D + i;
+    S[c] = cont && live[c] ? st[off[c]] : 0.f;
+  }
+  const int moff = E * D + i;
+  float m[D], b[4], mn[D], bn[4];
+  auto load = [&](const float* at, float (&mm)[D], float (&bb)[4]) {
 #pragma unroll
-    for (int c = 0; c < 4; ++c) bb[c] = base[(size_t)min(col + c, E - 1) * D];
+    for (int c = 0; c < 4; ++c) bb[c] = at[off[c]];
+    const float* row = at + moff;
 #pragma unroll
-    for (int j = 0; j < DM; ++j) m[j] = base[(size_t)(E + min(j, D - 1)) * D];
+    for (int j = 0; j < D; ++j) mm[j] = row[j * D];
   };
-  float m[DM], b[4];
-  load(k0, m, b);
-  for (int k = k0; k < k1; ++k) {
-    float4* cur = cols + ((k - k0) & 1) * DM * groups;
-    if (row) cur[i * groups + g] = float4{S[0], S[1], S[2], S[3]};
+  load(base, m, b);
+  for (int k = k0; k < k1; ++k, base += step) {
+    float4 (*cur)[groups] = cols[(k - k0) & 1];
+    cur[i][g] = float4{S[0], S[1], S[2], S[3]};
     __syncthreads();      // (the other buffer's readers are past the barrier of the step before)
-    float mn[DM], bn[4];
-    if (k + 1 < k1) load(k + 1, mn, bn);
+    load(k + 1 < k1 ? base + step : base, mn, bn);
     float acc[4] = {b[0], b[1], b[2], b[3]};
 #pragma unroll
-    for (int j = 0; j < DM; ++j) {
-      const float4 sj = cur[j * groups + g];
+    for (int j = 0; j < D; ++j) {
+      const float4 sj = cur[j][g];
       acc[0] += m[j] * sj.x; acc[1] += m[j] * sj.y; acc[2] += m[j] * sj.z; acc[3] += m[j] * sj.w;
     }
-    float* base = ws_e + ((size_t)k * A + h) * EC * D;
 #pragma unroll
     for (int c = 0; c < 4; ++c) {
-      if (row && col + c < E) base[(size_t)(col + c) * D + i] = S[c];
+      if (live[c]) base[off[c]] = S[c];
       S[c] = acc[c];
+      b[c] = bn[c];
     }
-    if (k + 1 < k1) {
 #pragma unroll
-      for (int j = 0; j < DM; ++j) m[j] = mn[j];
-#pragma unroll
-      for (int c = 0; c < 4; ++c) b[c] = bn[c];
-    }
+    for (int j = 0; j < D; ++j) m[j] = mn[j];
   }
 #pragma unroll
   for (int c = 0; c < 4; ++c)
-    if (row && col + c < E) st[(size_t)(col + c) * D + i] = S[c];
+    if (live[c]) st[off[c]] = S[c];
 }
 
-// the same for any D <= 256, without the rows in registers
+// the same for any D <= 256, read as it goes
 __global__ void __launch_bounds__(256) state_carry_matrix_any_kernel(float* __restrict__ ws_e, float* __restrict__ state,
                                                                      const int* __restrict__ seq_chunk0,
                                                                      const int* __restrict__ start_pos,
@@ -411,7 +408,7 @@ __global__ void __launch_bounds__(256) state_carry_matrix_any_kernel(float* __re
       float acc[4];
 #pragma unroll
       for (int c = 0; c < 4; ++c) acc[c] = col + c < E ? base[(size_t)(col + c) * D + i] : 0.f;
-#pragma unroll 8
+#pragma unroll 16
       for (int j = 0; j < D; ++j) {
         const float4 sj = cur[j];
         const float mj = base[(size_t)(E + j) * D + i];
@@ -499,13 +496,9 @@ int launch_state_scan(float* out, const float* q, const float* k, const float* v
   if (chunks != nullptr) {
     RT_ANY(RT_CHUNK, 1);
     if (has_ab) {
-      int lgDp = 5;
-      while ((1 << lgDp) < D) ++lgDp;
-      const int groups = 256 >> lgDp;
-      const dim3 grid(S, A, (E + 4 * groups - 1) / (4 * groups));
-      const size_t cshm = sizeof(float4) * 2 * 64 * (size_t)groups;
-      if (D <= 64) state_carry_matrix_kernel<64><<<grid, 256, cshm, stream>>>(ws_e, state, seq_chunk0, start_pos, slots, A, D,
-                                                                              E, lgDp);
+      auto grid = [&](int d) { return dim3(S, A, (E + 1024 / d - 1) / (1024 / d)); };
+      if (D == 64) state_carry_matrix_kernel<64><<<grid(64), 256, 0, stream>>>(ws_e, state, seq_chunk0, start_pos, slots, A, E);
+      else if (D == 32) state_carry_matrix_kernel<32><<<grid(32), 256, 0, stream>>>(ws_e, state, seq_chunk0, start_pos, slots, A, E);
       else state_carry_matrix_any_kernel<<<dim3(S, A, (E + 3) / 4), 256, sizeof(float4) * 2 * (size_t)D, stream>>>(
           ws_e, state, seq_chunk0, start_pos, slots, A, D, E);
     } else {

@@ -130,8 +130,8 @@ __global__ void __launch_bounds__(1024) canon_add_kernel(
   }
 }
 
-// one workgroup per sequence: the last `keep` rows of its span (columns col_off .. col_off + C of
-// x) become its state; a shorter span keeps the newest old rows
+// a workgroup per (sequence, 256 channels): the last `keep` rows of the span (columns col_off .. col_off + C
+// of x) become the sequence's state; a shorter span keeps the newest old rows
 template <typename XT>
 __global__ void __launch_bounds__(kThreads) conv_state_kernel(const XT* __restrict__ x, int stride, int col_off, int C,
                                                               float* __restrict__ state, int sub, int nsub, int keep,
@@ -143,7 +143,8 @@ __global__ void __launch_bounds__(kThreads) conv_state_kernel(const XT* __restri
   if (n <= 0) return;
   float* st = state + ((size_t)slots[s] * nsub + sub) * keep * C;
   const int p0 = start_pos[s];
-  for (int c = threadIdx.x; c < C; c += blockDim.x) {
+  const int c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c < C) {
     float nv[kMaxTaps];
 #pragma unroll
     for (int i = 0; i < kMaxTaps; ++i) {
@@ -438,100 +439,109 @@ __global__ void __launch_bounds__(1024) gla_prep_kernel(float* __restrict__ out,
 
 RT_DEVICE float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 
-// out [4][T][n] = q, beta k, g, g k per value head (n = A * D), vout [T][A * E]; a2 [rank][n]. ROWS rows per
-// workgroup share a pass over a2. dynamic LDS: low [ROWS][rank], dec [ROWS][n], z [C], unit factors [2 G].
+// out [4][T][n] = q, beta k, g, g k per value head (n = A * D), vout [T][A * E]; a2 [rank][n]. A workgroup
+// takes ROWS rows of one query / key head and its value heads (no norm or state crosses heads): all its
+// convolution inputs and low-rank terms are in flight together, which is what few rows wait for, and ROWS
+// rows share a pass over a2. dynamic LDS: low [ROWS][rank], part [parts][ROWS][m] (m = rep * D decay
+// columns, the rank split over `parts` groups of lanes), z [ROWS][Cg], unit factors [ROWS][2].
 template <typename T, int ROWS>
-__global__ void __launch_bounds__(1024) channel_delta_kernel(
+__global__ void __launch_bounds__(kThreads) channel_delta_kernel(
     float* __restrict__ out, float* __restrict__ vout, const T* __restrict__ proj, int stride, int q_off, int b_off,
     int a_off, int rank, const float* __restrict__ a2, const float* __restrict__ cw, float* __restrict__ state,
     const float* __restrict__ neg_rate, const float* __restrict__ dt_bias, int Tn, int A, int G, int D, int E, int taps,
     int keep, const int* __restrict__ row_seq, const int64_t* __restrict__ positions, const int* __restrict__ start_pos,
-    const int* __restrict__ slots, int shift_state) {
+    const int* __restrict__ slots, int shift_state, int parts) {
   extern __shared__ float lds[];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
-  const int n = A * D, C = 2 * G * D + A * E, rep = A / G;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int n = A * D, C = 2 * G * D + A * E, rep = A / G, g = blockIdx.y;
+  const int m = rep * D, Cg = 2 * D + rep * E;
   float* low = lds;
-  float* dec = low + ROWS * rank;
-  float* z = dec + ROWS * n;
-  float* unit = z + C;
+  float* part = low + ROWS * rank;
+  float* z = part + parts * ROWS * m;
+  float* unit = z + ROWS * Cg;
   const int t0 = blockIdx.x * ROWS;
   const int rows = min(ROWS, Tn - t0);
-  for (int i = threadIdx.x; i < ROWS * rank; i += blockDim.x) {
+  for (int i = threadIdx.x; i < ROWS * rank; i += kThreads) {
     const int r = i / rank;
     low[i] = r < rows ? DT<T>::load(proj + (size_t)(t0 + r) * stride + a_off + (i - r * rank)) : 0.f;
   }
-  __syncthreads();
-  for (int c = threadIdx.x; c < n; c += blockDim.x) {
-    float x[ROWS];
-    const float bc = dt_bias[c];
+  for (int c = threadIdx.x; c < Cg; c += kThreads) {
+    // channel of the projection: this head's q, its k, its value heads' v
+    const int ch = c < D ? g * D + c : c < 2 * D ? G * D + g * D + (c - D) : 2 * G * D + g * rep * E + (c - 2 * D);
 #pragma unroll
-    for (int r = 0; r < ROWS; ++r) x[r] = bc;
-#pragma unroll 8
-    for (int j = 0; j < rank; ++j) {
-      const float wv = a2[(size_t)j * n + c];
-#pragma unroll
-      for (int r = 0; r < ROWS; ++r) x[r] += wv * low[r * rank + j];
-    }
-    const float nr = neg_rate[c / D];
-#pragma unroll
-    for (int r = 0; r < ROWS; ++r) dec[r * n + c] = expf(nr * softplus(x[r]));
-  }
-  const size_t plane = (size_t)Tn * n;
-  const float qs = 1.0f / sqrtf((float)D);
-  for (int r = 0; r < rows; ++r) {
-    const int t = t0 + r;
-    const int s = row_seq[t];
-    const int64_t pos = positions[t];
-    const int local = (int)(pos - start_pos[s]);
-    float* st = state + (size_t)slots[s] * keep * C;
-    const T* pr = proj + (size_t)t * stride;
-    __syncthreads();      // the previous row's readers of z and unit are done (and dec is written)
-    for (int c = threadIdx.x; c < C; c += blockDim.x) {
+    for (int r = 0; r < ROWS; ++r) {
+      if (r >= rows) break;
+      const int t = t0 + r, s = row_seq[t];
+      const int64_t pos = positions[t];
+      const int local = (int)(pos - start_pos[s]);
+      float* st = state + (size_t)slots[s] * keep * C + ch;
       float acc = 0.f, v0 = 0.f;
       for (int k = 0; k < taps; ++k) {
         const Tap tp = tap_of(k, t, local, pos, taps);
         float v = 0.f;
-        if (tp.kind == 1) v = DT<T>::load(proj + tp.at * stride + q_off + c);
-        else if (tp.kind == 2) v = st[tp.at * C + c];
+        if (tp.kind == 1) v = DT<T>::load(proj + tp.at * stride + q_off + ch);
+        else if (tp.kind == 2) v = st[tp.at * C];
         if (k == 0) v0 = v;
-        acc += cw[(size_t)c * taps + (taps - 1 - k)] * v;
+        acc += cw[(size_t)ch * taps + (taps - 1 - k)] * v;
       }
       const float sv = silu(acc);
-      z[c] = sv;
-      if (c >= 2 * G * D) vout[(size_t)t * A * E + (c - 2 * G * D)] = sv;
+      z[r * Cg + c] = sv;
+      if (c >= 2 * D) vout[(size_t)t * A * E + g * rep * E + (c - 2 * D)] = sv;
       if (shift_state && taps > 1) {
         for (int i = 0; i + 2 < taps; ++i)
-          st[(size_t)i * C + c] = (pos - (taps - 2 - i) >= 0) ? st[(size_t)(i + 1) * C + c] : 0.f;
-        st[(size_t)(taps - 2) * C + c] = v0;
+          st[(size_t)i * C] = (pos - (taps - 2 - i) >= 0) ? st[(size_t)(i + 1) * C] : 0.f;
+        st[(size_t)(taps - 2) * C] = v0;
       }
     }
-    __syncthreads();
-    for (int j = wave; j < 2 * G; j += nw) {     // q heads, then k heads
-      float ss = 0.f;
-      for (int d = lane; d < D; d += 64) ss += z[j * D + d] * z[j * D + d];
-      const float iv = 1.0f / sqrtf(rt::wave_sum(ss) + 1e-6f);
-      if (lane == 0) unit[j] = iv;
+  }
+  __syncthreads();
+  for (int w = threadIdx.x; w < parts * m; w += kThreads) {
+    const int pt = w / m, c = w - pt * m;
+    const int j0 = rank * pt / parts, j1 = rank * (pt + 1) / parts;
+    const float* col = a2 + g * m + c;
+    float x[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) x[r] = 0.f;
+#pragma unroll 16
+    for (int j = j0; j < j1; ++j) {
+      const float wv = col[(size_t)j * n];
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r) x[r] += wv * low[r * rank + j];
     }
-    __syncthreads();
-    for (int c = threadIdx.x; c < n; c += blockDim.x) {
-      const int a = c / D, g = a / rep, d = c - a * D;
-      const float beta = 1.0f / (1.0f + expf(-DT<T>::load(pr + b_off + a)));
-      const float kv = z[(G + g) * D + d] * unit[G + g], gd = dec[r * n + c];
-      float* o = out + (size_t)t * n + c;
-      o[0] = z[g * D + d] * unit[g] * qs;
-      o[plane] = beta * kv;
-      o[2 * plane] = gd;
-      o[3 * plane] = gd * kv;
-    }
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) part[(pt * ROWS + r) * m + c] = x[r];
+  }
+  for (int j = wave; j < 2 * rows; j += kThreads / 64) {      // (row, q or k)
+    const float* zz = z + (j >> 1) * Cg + (j & 1) * D;
+    float ss = 0.f;
+    for (int d = lane; d < D; d += 64) ss += zz[d] * zz[d];
+    const float iv = 1.0f / sqrtf(rt::wave_sum(ss) + 1e-6f);
+    if (lane == 0) unit[j] = iv;
+  }
+  __syncthreads();
+  const size_t plane = (size_t)Tn * n;
+  const float qs = 1.0f / sqrtf((float)D);
+  for (int w = threadIdx.x; w < rows * m; w += kThreads) {
+    const int r = w / m, c = w - r * m;
+    const int a = g * rep + c / D, d = c % D;
+    const T* pr = proj + (size_t)(t0 + r) * stride;
+    float x = dt_bias[g * m + c];
+    for (int pt = 0; pt < parts; ++pt) x += part[(pt * ROWS + r) * m + c];
+    const float gd = expf(neg_rate[a] * softplus(x));
+    const float beta = 1.0f / (1.0f + expf(-DT<T>::load(pr + b_off + a)));
+    const float kv = z[r * Cg + D + d] * unit[2 * r + 1];
+    float* o = out + (size_t)(t0 + r) * n + g * m + c;
+    o[0] = z[r * Cg + d] * unit[2 * r] * qs;
+    o[plane] = beta * kv;
+    o[2 * plane] = gd;
+    o[3 * plane] = gd * kv;
   }
 }
 
 // the gates of one (token, head): the capped log input gate and the log of the capped forget gate
-template <typename T>
-RT_DEVICE void memory_gate(const T* pr, int i_off, int f_off, int a, const float* ib, const float* fb, float cap, float& gi,
-                           float& gf) {
-  gi = cap * tanhf((DT<T>::load(pr + i_off + a) + ib[a]) / cap);
-  gf = -softplus(-cap * tanhf((DT<T>::load(pr + f_off + a) + fb[a]) / cap));
+RT_DEVICE void memory_gate(float pi, float pf, float cap, float& gi, float& gf) {
+  gi = cap * tanhf(pi / cap);
+  gf = -softplus(-cap * tanhf(pf / cap));
 }
 
 // gates [3][T][A] = exp(f_t + m_(t-1) - m_t), exp(i_t - m_t), exp(-m_t) with m_t = max(f_t + m_(t-1), i_t), m
@@ -549,10 +559,21 @@ __global__ void __launch_bounds__(64) memory_gates_kernel(float* __restrict__ ga
   float* mp = gmax + (size_t)slots[s] * A + a;
   float m = start_pos[s] > 0 ? *mp : 0.f;
   const size_t plane = (size_t)Tn * A;
+  const float bi = ib[a], bf = fb[a];
+  const T* pa0 = proj + (size_t)r0 * stride + a;
+  float ni = DT<T>::load(pa0 + (size_t)min(lane, n - 1) * stride + i_off);      // one block of tokens ahead
+  float nf = DT<T>::load(pa0 + (size_t)min(lane, n - 1) * stride + f_off);
   for (int c0 = 0; c0 < n; c0 += 64) {
     const int t = c0 + lane;
-    float gi = -INFINITY, gf = 0.f;
-    if (t < n) memory_gate(proj + (size_t)(r0 + t) * stride, i_off, f_off, a, ib, fb, cap, gi, gf);
+    float gi, gf;
+    memory_gate(ni + bi, nf + bf, cap, gi, gf);
+    if (t >= n) {
+      gi = -INFINITY;
+      gf = 0.f;
+    }
+    const size_t nt = (size_t)min(t + 64, n - 1) * stride;
+    ni = DT<T>::load(pa0 + nt + i_off);
+    nf = DT<T>::load(pa0 + nt + f_off);
     float sa = gf, sb = gi;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
@@ -597,7 +618,7 @@ __global__ void __launch_bounds__(1024) memory_prep_kernel(float* __restrict__ o
       float* mp = gmax + (size_t)slots[t] * A + a;
       const float m = start_pos[t] > 0 ? *mp : 0.f;
       float gi, gf;
-      memory_gate(pr, i_off, f_off, a, ib, fb, cap, gi, gf);
+      memory_gate(DT<T>::load(pr + i_off + a) + ib[a], DT<T>::load(pr + f_off + a) + fb[a], cap, gi, gf);
       const float mt = fmaxf(gf + m, gi);
       *mp = mt;
       lds[a] = expf(gi - mt);
@@ -690,9 +711,10 @@ void launch_canon_add(void* h, float* xs, const float* x, const void* y, const v
 void launch_conv_state(const void* x, int stride, int col_off, int C, float* state, int sub, int nsub, int keep,
                        const int* cu_q, const int* start_pos, const int* slots, int S, bool bf, hipStream_t stream) {
   if (S <= 0) return;
-  if (bf) conv_state_kernel<uint16_t><<<S, kThreads, 0, stream>>>((const uint16_t*)x, stride, col_off, C, state, sub, nsub,
+  const dim3 grid(S, (C + kThreads - 1) / kThreads);
+  if (bf) conv_state_kernel<uint16_t><<<grid, kThreads, 0, stream>>>((const uint16_t*)x, stride, col_off, C, state, sub, nsub,
                                                                    keep, cu_q, start_pos, slots);
-  else conv_state_kernel<float><<<S, kThreads, 0, stream>>>((const float*)x, stride, col_off, C, state, sub, nsub, keep,
+  else conv_state_kernel<float><<<grid, kThreads, 0, stream>>>((const float*)x, stride, col_off, C, state, sub, nsub, keep,
                                                             cu_q, start_pos, slots);
 }
 
@@ -810,21 +832,22 @@ int launch_channel_delta(float* out, float* vout, const void* proj, int stride, 
                          const int* start_pos, const int* slots, bool shift_state, bool bf, hipStream_t stream) {
   if (T <= 0) return 0;
   if (taps > kMaxTaps) return -1;
-  const int C = 2 * G * D + A * E;
-  auto lds_of = [&](int rows) { return sizeof(float) * ((size_t)rows * (rank + A * D) + C + 2 * G); };
-  const int rows = T >= 256 && lds_of(4) <= 80 * 1024 ? 4 : 1;    // many rows: the low-rank factor is read once for four
+  const int rep = A / G, m = rep * D, Cg = 2 * D + rep * E;
+  const int parts = m >= kThreads ? 1 : kThreads / m < rank ? kThreads / m : rank;
+  auto lds_of = [&](int rows) { return sizeof(float) * (size_t)rows * (rank + parts * m + Cg + 2); };
+  const int rows = T >= 256 && lds_of(4) <= 64 * 1024 ? 4 : 1;    // many rows: the low-rank factor is read once for four
   const size_t shm = lds_of(rows);
   if (shm > 150 * 1024) return -1;
-  const int th = C >= 1024 ? 1024 : C <= 256 ? 256 : (C + 63) / 64 * 64;
 #define RT_CD(TT, R)                                                                                                   \
   do {                                                                                                                 \
     auto kern = channel_delta_kernel<TT, R>;                                                                           \
     if (shm > 48 * 1024 &&                                                                                             \
         hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm) != hipSuccess)    \
       return -2;                                                                                                       \
-    kern<<<(T + R - 1) / R, th, shm, stream>>>(out, vout, (const TT*)proj, stride, q_off, b_off, a_off, rank, a2, cw,  \
-                                               state, neg_rate, dt_bias, T, A, G, D, E, taps, keep, row_seq,           \
-                                               positions, start_pos, slots, shift_state ? 1 : 0);                      \
+    kern<<<dim3((T + R - 1) / R, G), kThreads, shm, stream>>>(out, vout, (const TT*)proj, stride, q_off, b_off, a_off, \
+                                                              rank, a2, cw, state, neg_rate, dt_bias, T, A, G, D, E,   \
+                                                              taps, keep, row_seq, positions, start_pos, slots,        \
+                                                              shift_state ? 1 : 0, parts);                             \
   } while (0)
   if (bf) {
     if (rows == 4) RT_CD(uint16_t, 4); else RT_CD(uint16_t, 1);
