@@ -57,7 +57,7 @@ int flash_key_tile();
 bool flash_fits(int Dk, int Dv, int BS);
 int launch_flash_attention(void* out, const void* q, const void* kc, const void* vc, const int* block_tables, const int* cu_q,
                            const int* start_pos, const int* tiles, int n_tiles, float* part_o, float* part_ml, int T, int H,
-                           int G, int Dk, int Dv, int BS, int max_blocks, int rows, int waves, int num_splits, float scale,
+                           int G, int Dk, int Dv, int BS, int max_blocks, int rows, int pairs, int num_splits, float scale,
                            const AttnMask& mask, const void* gate, int gate_stride, float softcap, float out_scale,
                            int out_stride, int out_off, hipStream_t stream);
 int launch_gqa_attention(void* out, const void* q, const void* kc, const void* vc, const int* block_tables,
@@ -326,7 +326,7 @@ void gqa_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch::
 // gqa_attention's bf16 form on the matrix cores: rows layout, a gate per head or none
 void flash_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch::Tensor vc, torch::Tensor block_tables,
                      torch::Tensor cu_q, torch::Tensor start_pos, torch::Tensor tiles, double scale, int64_t rows,
-                     int64_t waves, int64_t num_splits, c10::optional<torch::Tensor> part_o,
+                     int64_t pairs, int64_t num_splits, c10::optional<torch::Tensor> part_o,
                      c10::optional<torch::Tensor> part_ml, int64_t window, int64_t keep, int64_t chunk,
                      c10::optional<torch::Tensor> sinks, c10::optional<torch::Tensor> gate, int64_t gate_off, double softcap,
                      double out_scale, int64_t out_off) {
@@ -359,7 +359,7 @@ void flash_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kc, torch
   int rc = launch_flash_attention(out.data_ptr(), q.data_ptr(), kc.data_ptr(), vc.data_ptr(), block_tables.data_ptr<int>(),
                                   cu_q.data_ptr<int>(), start_pos.data_ptr<int>(), tiles.data_ptr<int>(), (int)tiles.size(0),
                                   po, pml, (int)T, (int)H, (int)G, (int)Dk, (int)Dv, (int)BS, (int)block_tables.size(1),
-                                  (int)rows, (int)waves, (int)num_splits, (float)scale, mask, gp, (int)gstride, (float)softcap,
+                                  (int)rows, (int)pairs, (int)num_splits, (float)scale, mask, gp, (int)gstride, (float)softcap,
                                   (float)out_scale, (int)out.size(1), (int)out_off, cur());
   TORCH_CHECK(rc == 0, "flash_attention: unsupported shape (code ", rc, ": -1 head or page sizes, -2 rows per tile, -3 LDS "
               "size refused)");
@@ -972,7 +972,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("flash_fits", [](int64_t Dk, int64_t Dv, int64_t BS) { return flash_fits((int)Dk, (int)Dv, (int)BS); });
   m.def("flash_attention", &flash_attention, py::arg("out"), py::arg("q"), py::arg("kc"), py::arg("vc"),
         py::arg("block_tables"), py::arg("cu_q"), py::arg("start_pos"), py::arg("tiles"), py::arg("scale"), py::arg("rows"),
-        py::arg("waves"), py::arg("num_splits"), py::arg("part_o"), py::arg("part_ml"), py::arg("window") = 0,
+        py::arg("pairs"), py::arg("num_splits"), py::arg("part_o"), py::arg("part_ml"), py::arg("window") = 0,
         py::arg("keep") = 0, py::arg("chunk") = 0, py::arg("sinks") = py::none(), py::arg("gate") = py::none(),
         py::arg("gate_off") = 0, py::arg("softcap") = 0.0, py::arg("out_scale") = 1.0, py::arg("out_off") = 0);
   m.def("gqa_attention", &gqa_attention, py::arg("out"), py::arg("q"), py::arg("kc"), py::arg("vc"),

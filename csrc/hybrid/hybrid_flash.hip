@@ -5,8 +5,10 @@
 //
 //   K cache [num_blocks, G, BS, Dk], V cache [num_blocks, G, BS, Dv], q [T, H, Dk]
 //
-// A workgroup of NW waves = one work item (sequence, first row) x one key/value head x one key range: 32
-// (row, head) pairs per wave that all read the same keys, walked in tiles of 64 counted from key 0.
+// A workgroup of 4 waves = one work item (sequence, first row) x one key/value head x one key range: 32
+// (row, head) pairs per wave that all read the same keys, walked in tiles of 64 counted from key 0. KS = 2
+// (launches too small to fill the chip with 128-pair workgroups): two waves share 32 pairs, each takes half
+// of every tile's keys, and their results are merged at the end.
 //
 //   S^T [64 keys x 32 pairs] = K Q^T     mfma_f32_32x32x16_bf16, query fragments in registers; a K row is
 //                                        read with its index bits 2 and 3 exchanged, so that a lane's score
@@ -43,9 +45,9 @@ struct FlashArgs {
 };
 
 // NKD, NVD: head sizes in units of 32 (padded)
-template <int NKD, int NVD, int NW>
-__global__ void __launch_bounds__(NW * 64) flash_kernel(FlashArgs p) {
-  constexpr int NT = NW * 64, kRow = NKD * 64 + 16, CH = NKD * 4;
+template <int NKD, int NVD, int KS>
+__global__ void __launch_bounds__(256) flash_kernel(FlashArgs p) {
+  constexpr int NT = 256, NP = 128 / KS, NB = 2 / KS, kRow = NKD * 64 + 16, CH = NKD * 4;
   constexpr int KI = kKT * CH / NT, VI = NVD * 128 / NT;      // 16-byte key chunks, 4 x 4 value blocks per lane
   constexpr int kStage = kKT * kRow + NVD * 32 * kVRow;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -53,7 +55,7 @@ __global__ void __launch_bounds__(NW * 64) flash_kernel(FlashArgs p) {
   const int seq = p.tiles[2 * blockIdx.x], row0 = p.tiles[2 * blockIdx.x + 1];
   const int g = blockIdx.y / p.hchunks, hc = blockIdx.y - g * p.hchunks;
   const int group = p.H / p.G;
-  const int h_lo = hc * NW * 32, nh = min(group - h_lo, NW * 32);
+  const int h_lo = hc * NP, nh = min(group - h_lo, NP);
   const int q_lo = p.cu_q[seq];
   const int nrows = min(p.rows, p.cu_q[seq + 1] - row0);
   const int P = nrows * nh;
@@ -66,13 +68,14 @@ __global__ void __launch_bounds__(NW * 64) flash_kernel(FlashArgs p) {
   const int BS = 1 << p.lgBS;
 
   // this lane's pair
-  const int pair = wave * 32 + col;
+  const int pw = wave % (NP / 32), kh = wave / (NP / 32);      // pairs and (KS 2) keys of this wave
+  const int pair = pw * 32 + col;
   const bool mine = pair < P;
   const int pr = mine ? pair / nh : 0;
   const int h = g * group + h_lo + (mine ? pair - pr * nh : 0);
   const int row = row0 + pr, qpos = pos0 + pr, qlow = mask_low(p.mask, qpos);
   const int low_last = mask_low(p.mask, kend - 1);
-  const bool busy = wave * 32 < P;
+  const bool busy = pw * 32 < P;
 
   short8 qf[NKD * 2];
   {
@@ -170,15 +173,15 @@ __global__ void __launch_bounds__(NW * 64) flash_kernel(FlashArgs p) {
       const unsigned char* ks = smem + buf * kStage;
       const unsigned char* vs = ks + kKT * kRow;
       const int kb = tr.at(v) * kKT;
-      float s[2][16];
+      float s[NB][16];
 #pragma unroll
-      for (int b = 0; b < 2; ++b) {
+      for (int b = 0; b < NB; ++b) {
         float16_ acc;
 #pragma unroll
         for (int i = 0; i < 16; ++i) acc[i] = 0.f;
 #pragma unroll
         for (int c = 0; c < NKD * 2; ++c) {
-          const short8 a = *reinterpret_cast<const short8*>(ks + (b * 32 + krow) * kRow + c * 32 + hi * 16);
+          const short8 a = *reinterpret_cast<const short8*>(ks + ((kh + b) * 32 + krow) * kRow + c * 32 + hi * 16);
           acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(rt::bf16x8, a), __builtin_bit_cast(rt::bf16x8, qf[c]),
                                                         acc, 0, 0, 0);
         }
@@ -187,7 +190,7 @@ __global__ void __launch_bounds__(NW * 64) flash_kernel(FlashArgs p) {
       }
       if (p.softcap > 0.f) {        // c tanh(x / c) = c (1 - 2 / (1 + e^(2 x / c)))
 #pragma unroll
-        for (int b = 0; b < 2; ++b)
+        for (int b = 0; b < NB; ++b)
 #pragma unroll
           for (int i = 0; i < 16; ++i)
             s[b][i] = cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(1.f + rt::fast_exp2(s[b][i]));
@@ -197,25 +200,25 @@ __global__ void __launch_bounds__(NW * 64) flash_kernel(FlashArgs p) {
       float mx = kNeg;
       if (!whole) {
 #pragma unroll
-        for (int b = 0; b < 2; ++b)
+        for (int b = 0; b < NB; ++b)
 #pragma unroll
           for (int i = 0; i < 16; ++i) {
-            const int key = kb + b * 32 + (i & 7) + hi * 8 + (i >> 3) * 16;
+            const int key = kb + (kh + b) * 32 + (i & 7) + hi * 8 + (i >> 3) * 16;
             if (!mask_sees(p.mask, qlow, qpos, key)) s[b][i] = 2.f * kNeg;
           }
       }
 #pragma unroll
-      for (int b = 0; b < 2; ++b)
+      for (int b = 0; b < NB; ++b)
 #pragma unroll
         for (int i = 0; i < 16; ++i) mx = fmaxf(mx, s[b][i]);
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
       const float mn = fmaxf(m, mx);            // at least kNeg: an unseen key's 2 kNeg - mn stays far below zero
       const float alpha = rt::fast_exp2(m - mn);
       m = mn;
-      short8 pt[4];
+      short8 pt[2 * NB];
       float sum = 0.f;
 #pragma unroll
-      for (int k4 = 0; k4 < 4; ++k4) {
+      for (int k4 = 0; k4 < 2 * NB; ++k4) {
         float e[8];
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
@@ -235,8 +238,8 @@ __global__ void __launch_bounds__(NW * 64) flash_kernel(FlashArgs p) {
 #pragma unroll
       for (int d = 0; d < NVD; ++d)
 #pragma unroll
-        for (int k4 = 0; k4 < 4; ++k4) {
-          const short8 a = *reinterpret_cast<const short8*>(vs + (d * 32 + col) * kVRow + k4 * 32 + hi * 16);
+        for (int k4 = 0; k4 < 2 * NB; ++k4) {
+          const short8 a = *reinterpret_cast<const short8*>(vs + (d * 32 + col) * kVRow + (2 * kh + k4) * 32 + hi * 16);
           o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(rt::bf16x8, a), __builtin_bit_cast(rt::bf16x8, pt[k4]),
                                                          o[d], 0, 0, 0);
         }
@@ -246,6 +249,27 @@ __global__ void __launch_bounds__(NW * 64) flash_kernel(FlashArgs p) {
   }
 
   l += __shfl_xor(l, 32, 64);
+  if (KS == 2) {      // (the last barrier freed the tiles) the second key half's results through LDS
+    float* ex = reinterpret_cast<float*>(smem) + pw * (NVD * 16 + 2) * 64 + lane;
+    if (kh == 1) {
+#pragma unroll
+      for (int d = 0; d < NVD; ++d)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) ex[(d * 16 + i) * 64] = o[d][i];
+      ex[NVD * 16 * 64] = m;
+      ex[(NVD * 16 + 1) * 64] = l;
+    }
+    __syncthreads();
+    if (kh == 1) return;
+    const float m1 = ex[NVD * 16 * 64], M = fmaxf(m, m1);
+    const float e0 = rt::fast_exp2(m - M), e1 = rt::fast_exp2(m1 - M);
+    m = M;
+    l = l * e0 + ex[(NVD * 16 + 1) * 64] * e1;
+#pragma unroll
+    for (int d = 0; d < NVD; ++d)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) o[d][i] = o[d][i] * e0 + ex[(d * 16 + i) * 64] * e1;
+  }
   if (!mine) return;
   if (S == 1) {
     float den = l, num = 1.f;
@@ -307,12 +331,12 @@ bool flash_fits(int Dk, int Dv, int BS) {
 
 int launch_flash_attention(void* out, const void* q, const void* kc, const void* vc, const int* block_tables, const int* cu_q,
                            const int* start_pos, const int* tiles, int n_tiles, float* part_o, float* part_ml, int T, int H,
-                           int G, int Dk, int Dv, int BS, int max_blocks, int rows, int waves, int num_splits, float scale,
+                           int G, int Dk, int Dv, int BS, int max_blocks, int rows, int pairs, int num_splits, float scale,
                            const AttnMask& mask, const void* gate, int gate_stride, float softcap, float out_scale,
                            int out_stride, int out_off, hipStream_t stream) {
   if (n_tiles <= 0 || T <= 0) return 0;
-  if (!flash_fits(Dk, Dv, BS) || H % G || (waves != 2 && waves != 4)) return -1;
-  const int group = H / G, pairs = waves * 32;
+  if (!flash_fits(Dk, Dv, BS) || H % G || (pairs != 64 && pairs != 128)) return -1;
+  const int group = H / G;
   if (rows * (group < pairs ? group : pairs) > pairs) return -2;
   FlashArgs a;
   a.out = (uint16_t*)out; a.q = (const uint16_t*)q; a.kc = (const uint16_t*)kc; a.vc = (const uint16_t*)vc;
@@ -330,24 +354,24 @@ int launch_flash_attention(void* out, const void* q, const void* kc, const void*
   const dim3 grid(n_tiles, G * a.hchunks, num_splits);
   const int nk = pad_k(Dk), nv = pad_v(Dv);
   const size_t shm = flash_lds(nk, nv);
-#define RT_FL(NK, NV, NWV)                                                                                             \
+#define RT_FL(NK, NV, KSV)                                                                                             \
   do {                                                                                                                 \
-    auto kern = flash_kernel<NK, NV, NWV>;                                                                             \
+    auto kern = flash_kernel<NK, NV, KSV>;                                                                             \
     if (shm > 48 * 1024 &&                                                                                             \
         hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm) != hipSuccess)    \
       return -3;                                                                                                       \
-    kern<<<grid, NWV * 64, shm, stream>>>(a);                                                                          \
+    kern<<<grid, 256, shm, stream>>>(a);                                                                               \
   } while (0)
-#define RT_FL_V(NK, NWV)                                                                                               \
+#define RT_FL_V(NK, KSV)                                                                                               \
   do {                                                                                                                 \
-    if (nv == 2) RT_FL(NK, 2, NWV); else if (nv == 4) RT_FL(NK, 4, NWV); else RT_FL(NK, 8, NWV);                       \
+    if (nv == 2) RT_FL(NK, 2, KSV); else if (nv == 4) RT_FL(NK, 4, KSV); else RT_FL(NK, 8, KSV);                       \
   } while (0)
-#define RT_FL_K(NWV)                                                                                                   \
+#define RT_FL_K(KSV)                                                                                                   \
   do {                                                                                                                 \
-    if (nk == 2) RT_FL_V(2, NWV); else if (nk == 3) RT_FL_V(3, NWV); else if (nk == 4) RT_FL_V(4, NWV);                \
-    else RT_FL_V(8, NWV);                                                                                              \
+    if (nk == 2) RT_FL_V(2, KSV); else if (nk == 3) RT_FL_V(3, KSV); else if (nk == 4) RT_FL_V(4, KSV);                \
+    else RT_FL_V(8, KSV);                                                                                              \
   } while (0)
-  if (waves == 4) RT_FL_K(4); else RT_FL_K(2);
+  if (pairs == 128) RT_FL_K(1); else RT_FL_K(2);
 #undef RT_FL
 #undef RT_FL_V
 #undef RT_FL_K

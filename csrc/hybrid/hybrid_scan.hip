@@ -260,7 +260,8 @@ __global__ void __launch_bounds__(kScanThreads) state_scan_kernel(
       const int gc = blockIdx.z * CB + c;
       const float* sh = os + tok * kScanThreads + c * P;      // the column's P shares
       float o = 0.f;
-      for (int j = 0; j < P; ++j) o += sh[j];
+      // (starting at different shares keeps the lanes of a wave on different LDS banks)
+      for (int j = 0; j < P; ++j) o += sh[(j + c + tok) & (P - 1)];
       if (gc < E) out[(size_t)(r0 + c0 + tok) * A * E + head * E + gc] = o;
     }
   }

@@ -444,7 +444,8 @@ RT_DEVICE float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)
 // convolution inputs and low-rank terms are in flight together, which is what few rows wait for, and ROWS
 // rows share a pass over a2. dynamic LDS: low [ROWS][rank], part [parts][ROWS][m] (m = rep * D decay
 // columns, the rank split over `parts` groups of lanes), z [ROWS][Cg], unit factors [ROWS][2].
-template <typename T, int ROWS>
+// TAPS: the taps as a compile-time number, or 0 for any number
+template <typename T, int ROWS, int TAPS>
 __global__ void __launch_bounds__(kThreads) channel_delta_kernel(
     float* __restrict__ out, float* __restrict__ vout, const T* __restrict__ proj, int stride, int q_off, int b_off,
     int a_off, int rank, const float* __restrict__ a2, const float* __restrict__ cw, float* __restrict__ state,
@@ -465,9 +466,30 @@ __global__ void __launch_bounds__(kThreads) channel_delta_kernel(
     const int r = i / rank;
     low[i] = r < rows ? DT<T>::load(proj + (size_t)(t0 + r) * stride + a_off + (i - r * rank)) : 0.f;
   }
+  // rows of one span with all their predecessors in this batch: every row is read once, without branches
+  const bool inner = TAPS > 0 && rows == ROWS && row_seq[t0] == row_seq[t0 + ROWS - 1] &&
+                     positions[t0] - start_pos[row_seq[t0]] >= TAPS - 1;
   for (int c = threadIdx.x; c < Cg; c += kThreads) {
     // channel of the projection: this head's q, its k, its value heads' v
     const int ch = c < D ? g * D + c : c < 2 * D ? G * D + g * D + (c - D) : 2 * G * D + g * rep * E + (c - 2 * D);
+    if (TAPS > 0 && inner) {
+      constexpr int NX = TAPS > 0 ? TAPS : 1;
+      float x[ROWS + NX - 1], wk[NX];
+#pragma unroll
+      for (int i = 0; i < ROWS + NX - 1; ++i) x[i] = DT<T>::load(proj + (size_t)(t0 - (NX - 1) + i) * stride + q_off + ch);
+#pragma unroll
+      for (int k = 0; k < NX; ++k) wk[k] = cw[(size_t)ch * NX + k];
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r) {
+        float acc = 0.f;
+#pragma unroll
+        for (int k = 0; k < NX; ++k) acc += wk[NX - 1 - k] * x[r + NX - 1 - k];
+        const float sv = silu(acc);
+        z[r * Cg + c] = sv;
+        if (c >= 2 * D) vout[(size_t)(t0 + r) * A * E + g * rep * E + (c - 2 * D)] = sv;
+      }
+      continue;
+    }
 #pragma unroll
     for (int r = 0; r < ROWS; ++r) {
       if (r >= rows) break;
@@ -840,7 +862,9 @@ int launch_channel_delta(float* out, float* vout, const void* proj, int stride, 
   if (shm > 150 * 1024) return -1;
 #define RT_CD(TT, R)                                                                                                   \
   do {                                                                                                                 \
-    auto kern = channel_delta_kernel<TT, R>;                                                                           \
+    auto kern = R == 4 && taps == 4 ? channel_delta_kernel<TT, R, 4> : R == 4 && taps == 3                             \
+                    ? channel_delta_kernel<TT, R, 3> : R == 4 && taps == 2 ? channel_delta_kernel<TT, R, 2>            \
+                                                                           : channel_delta_kernel<TT, R, 0>;           \
     if (shm > 48 * 1024 &&                                                                                             \
         hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shm) != hipSuccess)    \
       return -2;                                                                                                       \

@@ -910,11 +910,11 @@ def test_trace_runner_replays_steps(tmp_path):
 
 
 @GPU
-@pytest.mark.parametrize("waves", [2, 4])
+@pytest.mark.parametrize("pairs", [64, 128])
 @pytest.mark.parametrize("shape", [(8, 2, 64, 64), (7, 1, 40, 48), (6, 2, 96, 80), (4, 4, 128, 128), (3, 1, 256, 72), (2, 2, 72, 256),
                                    (140, 1, 16, 16)])
 @pytest.mark.parametrize("mask", [dict(window=0), dict(window=100, keep_first=70), dict(window=64, keep_first=3), dict(chunk=100)])
-def test_matrix_core_attention_against_the_any_size_kernel(waves, shape, mask):
+def test_matrix_core_attention_against_the_any_size_kernel(pairs, shape, mask):
     """The bf16 matrix-core kernel and the fp32-FMA kernel on the same queries and cache: several
     sequences of unequal length and start on scattered pages of 4 to 64 tokens, prompts and split decode
     rows, with soft cap, sinks, gates, a scaled result in a column range."""
@@ -936,9 +936,9 @@ def test_matrix_core_attention_against_the_any_size_kernel(waves, shape, mask):
         decode = max(lens) == 1
         kw = dict(softcap=3.0, sinks=sinks, gate=gate, gate_off=2, gate_heads=True, out_scale=0.7, out_off=4,
                   num_splits=3 if decode else 1, **mask)
-        rows = 1 if decode else max(1, waves * 32 // (H // G))
+        rows = 1 if decode else max(1, pairs // (H // G))
         outs = []
-        for plan in (None, Hy.AttnPlan(waves, rows, 64)):
+        for plan in (None, Hy.AttnPlan(pairs, rows, 64)):
             buf = torch.zeros(T, H * Dv + 8, dtype=dt, device=dev)
             outs.append(Hy.gqa_attention(q, kc, vc, bt.to(dev), cu.to(dev), sp.to(dev), Dk ** -0.5, plan=plan, out_buf=buf, **kw))
         assert float(outs[0].float().abs().max()) > 0.1

@@ -148,9 +148,10 @@ def rows_per_tile(group: int) -> int:
 
 
 class AttnPlan(NamedTuple):
-    """How :func:`gqa_attention` runs a layer's rows on the GPU: ``waves`` 0 the any-size kernel, else the
-    matrix-core kernel with that many waves per workgroup; query rows per work item; keys per tile."""
-    waves: int
+    """How :func:`gqa_attention` runs a layer's rows on the GPU: ``pairs`` 0 the any-size kernel, else the
+    matrix-core kernel with that many (row, head) pairs per workgroup (64 or 128); query rows per work
+    item; keys per tile."""
+    pairs: int
     rows: int
     key_tile: int
 
@@ -160,10 +161,8 @@ def attention_plan(spec, n_rows: int, block_size: int, dtype, decode: bool = Fal
     of two; a launch of few rows gets smaller workgroups, so that more of them fill the chip."""
     if dtype != torch.bfloat16 or not native().flash_fits(spec.dim, spec.vdim, block_size):
         return AttnPlan(0, 1 if decode else rows_per_tile(spec.group), native().gqa_key_tile(spec.dim, spec.vdim))
-    waves = 4
-    if not decode and n_rows * spec.heads <= 512 * 128 and spec.group <= 64:
-        waves = 2
-    return AttnPlan(waves, 1 if decode else max(1, waves * 32 // spec.group), native().flash_key_tile())
+    pairs = 64 if decode or n_rows * spec.heads <= 512 * 128 else 128
+    return AttnPlan(pairs, 1 if decode else max(1, pairs // spec.group), native().flash_key_tile())
 
 
 def tile_map(cu_q: torch.Tensor, start_pos: torch.Tensor, rows: int) -> torch.Tensor:
@@ -221,11 +220,11 @@ def gqa_attention(q, k_cache, v_cache, block_tables, cu_q, start_pos, scale: flo
             tiles = tile_map(cu_q.cpu(), start_pos.cpu(), rows).to(q.device)
         if num_splits > 1 and workspace is None:
             workspace = SplitWorkspace(T, H, Dv, num_splits, q.device)
-        if plan is not None and plan.waves:
+        if plan is not None and plan.pairs:
             if temp is not None or sink or slopes is not None or matrix_layout or (gate is not None and not gate_heads):
                 raise ValueError("gqa_attention: not an attention of the matrix-core kernel")
             native().flash_attention(out, q, k_cache, v_cache, block_tables, cu_q, start_pos, tiles, float(scale), rows,
-                                     plan.waves, int(num_splits), workspace.part_o if num_splits > 1 else None,
+                                     plan.pairs, int(num_splits), workspace.part_o if num_splits > 1 else None,
                                      workspace.part_ml if num_splits > 1 else None, int(window), int(keep_first), int(chunk),
                                      sinks, gate, int(gate_off), float(softcap), float(out_scale), int(out_off))
             return out
