@@ -999,7 +999,7 @@ PRESETS.update({
                                    chunk=40, window=24, keep_first=3, rank=16),
     "lizesun-0.5b": lizesun_config("lizesun-0.5b", 24, 896, 14, 2, 64, 7296, 151936),      # Qwen2.5-0.5B's sizes
     "lizesun-1b": lizesun_config("lizesun-1b", 16, 2048, 32, 8, 64, 12288, 128256),
-    "lizesun-3b": lizesun_config("lizesun-3b", 28, 3072, 24, 8, 128, 12288, 128256, rec_dim=128),
+    "lizesun-3b": lizesun_config("lizesun-3b", 28, 3072, 24, 8, 128, 12288, 128256),
 })
 
 
