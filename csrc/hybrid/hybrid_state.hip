@@ -567,15 +567,17 @@ RT_DEVICE void memory_gate(float pi, float pf, float cap, float& gi, float& gf) 
 }
 
 // gates [3][T][A] = exp(f_t + m_(t-1) - m_t), exp(i_t - m_t), exp(-m_t) with m_t = max(f_t + m_(t-1), i_t), m
-// from gmax[slot] (0 at position 0). One wave per (sequence, head): 64 tokens at a time by a scan over
-// the maps m -> max(m + a, b), of which two in a row are (a1 + a2, max(b1 + a2, b2)).
+// from gmax[slot] (0 at position 0). A workgroup per (sequence, head), 64 tokens per wave: a scan over the
+// maps m -> max(m + a, b), of which two in a row are (a1 + a2, max(b1 + a2, b2)), inside every wave, then
+// over the waves' whole maps.
 template <typename T>
-__global__ void __launch_bounds__(64) memory_gates_kernel(float* __restrict__ gates, const T* __restrict__ proj, int stride,
-                                                          int i_off, int f_off, const float* __restrict__ ib,
-                                                          const float* __restrict__ fb, float cap, float* __restrict__ gmax,
-                                                          const int* __restrict__ cu_q, const int* __restrict__ start_pos,
-                                                          const int* __restrict__ slots, int Tn, int A) {
-  const int s = blockIdx.x, a = blockIdx.y, lane = threadIdx.x;
+__global__ void __launch_bounds__(1024) memory_gates_kernel(float* __restrict__ gates, const T* __restrict__ proj, int stride,
+                                                            int i_off, int f_off, const float* __restrict__ ib,
+                                                            const float* __restrict__ fb, float cap, float* __restrict__ gmax,
+                                                            const int* __restrict__ cu_q, const int* __restrict__ start_pos,
+                                                            const int* __restrict__ slots, int Tn, int A) {
+  __shared__ float wa[2][16], wb[2][16];      // every wave's whole map, two sets in turn
+  const int s = blockIdx.x, a = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
   const int r0 = cu_q[s], n = cu_q[s + 1] - r0;
   if (n <= 0) return;
   float* mp = gmax + (size_t)slots[s] * A + a;
@@ -583,17 +585,18 @@ __global__ void __launch_bounds__(64) memory_gates_kernel(float* __restrict__ ga
   const size_t plane = (size_t)Tn * A;
   const float bi = ib[a], bf = fb[a];
   const T* pa0 = proj + (size_t)r0 * stride + a;
-  float ni = DT<T>::load(pa0 + (size_t)min(lane, n - 1) * stride + i_off);      // one block of tokens ahead
-  float nf = DT<T>::load(pa0 + (size_t)min(lane, n - 1) * stride + f_off);
-  for (int c0 = 0; c0 < n; c0 += 64) {
-    const int t = c0 + lane;
+  float ni = DT<T>::load(pa0 + (size_t)min((int)threadIdx.x, n - 1) * stride + i_off);      // one round ahead
+  float nf = DT<T>::load(pa0 + (size_t)min((int)threadIdx.x, n - 1) * stride + f_off);
+  int set = 0;
+  for (int c0 = 0; c0 < n; c0 += (int)blockDim.x, set ^= 1) {
+    const int t = c0 + threadIdx.x;
     float gi, gf;
     memory_gate(ni + bi, nf + bf, cap, gi, gf);
-    if (t >= n) {
+    if (t >= n) {       // the identity
       gi = -INFINITY;
       gf = 0.f;
     }
-    const size_t nt = (size_t)min(t + 64, n - 1) * stride;
+    const size_t nt = (size_t)min(t + (int)blockDim.x, n - 1) * stride;
     ni = DT<T>::load(pa0 + nt + i_off);
     nf = DT<T>::load(pa0 + nt + f_off);
     float sa = gf, sb = gi;
@@ -605,18 +608,27 @@ __global__ void __launch_bounds__(64) memory_gates_kernel(float* __restrict__ ga
         sa = pa + sa;
       }
     }
-    const float mt = fmaxf(m + sa, sb);
+    if (lane == 63) {
+      wa[set][wave] = sa;
+      wb[set][wave] = sb;
+    }
+    __syncthreads();      // (a set is written again two rounds later, past the next round's barrier)
+    float mw = m;         // the maximum ahead of this wave's tokens
+    for (int w = 0; w < nw; ++w) {
+      if (w == wave) mw = m;
+      m = fmaxf(m + wa[set][w], wb[set][w]);
+    }
+    const float mt = fmaxf(mw + sa, sb);
     float before = __shfl_up(mt, 1, 64);
-    if (lane == 0) before = m;
+    if (lane == 0) before = mw;
     if (t < n) {
       float* g = gates + (size_t)(r0 + t) * A + a;
       g[0] = expf(gf + before - mt);
       g[plane] = expf(gi - mt);
       g[2 * plane] = expf(-mt);
+      if (t == n - 1) *mp = mt;
     }
-    m = __shfl(mt, min(63, n - 1 - c0), 64);
   }
-  if (lane == 0) *mp = m;
 }
 
 // out [T][2 n + A (E + 1)] = q * q_scale, weight * k (n = A * D columns each), per head v and a one.
@@ -890,11 +902,12 @@ int launch_memory_prep(float* out, float* gates, const void* proj, int stride, i
   const size_t shm = sizeof(float) * (size_t)A;
   if (shm > 48 * 1024) return -1;
   const int m = A * (D > E + 1 ? D : E + 1);
+  const int gth = T >= 1024 ? 1024 : (T + 63) / 64 * 64;
   const int th = m >= 1024 ? 1024 : m <= 64 ? 64 : (m + 63) / 64 * 64;
 #define RT_MP(TT)                                                                                                      \
   do {                                                                                                                 \
     if (!step)                                                                                                         \
-      memory_gates_kernel<TT><<<dim3(S, A), 64, 0, stream>>>(gates, (const TT*)proj, stride, i_off, f_off, ib, fb, cap, \
+      memory_gates_kernel<TT><<<dim3(S, A), gth, 0, stream>>>(gates, (const TT*)proj, stride, i_off, f_off, ib, fb, cap, \
                                                              gmax, cu_q, start_pos, slots, T, A);                      \
     if (step) memory_prep_kernel<TT, true><<<T, th, shm, stream>>>(out, gates, (const TT*)proj, stride, q_off, k_off,  \
                                                                    v_off, i_off, f_off, ib, fb, cap, gmax, start_pos,  \

@@ -484,10 +484,10 @@ def _memory_mixer(run, spec, cuts, seed, edit=None):
 
 @pytest.mark.parametrize("run", RUNS)
 @pytest.mark.parametrize("shape", [(3, 8, 6, 7.0), (1, 64, 64, 15.0), (2, 70, 130, 2.0), (5, 32, 40, 11.0)])
-@pytest.mark.parametrize("cuts", [[24], [5, 1, 2, 1, 1, 14], [300, 1, 1, 2, 70, 1, 65]])
+@pytest.mark.parametrize("cuts", [[24], [5, 1, 2, 1, 1, 14], [300, 1, 1, 2, 70, 1, 65], [1300, 2, 1100]])
 def test_matrix_memory_across_cuts(run, shape, cuts):
     """Capped exponential gates, the running maximum, state, normaliser, per-head norm, weight and gate;
-    spans below and above a wave's 64 tokens, decoded rows, a used slot."""
+    spans below and above a wave's 64 tokens and a workgroup's 1024, decoded rows, a used slot."""
     got, want = _memory_mixer(run, MatrixMemorySpec(*shape), cuts, shape[1])
     assert float((got - want).abs().max()) < (0.2 if run[1] == "bf16" else 2e-3)
 
